@@ -39,6 +39,10 @@ extern "C" {
                                       infer_pool_last_error()                                   */
 #define INFER_KV_EBUSY        -7   /* the library's own scratch array is still in use by work
                                       pending on another stream (infer_paged_decode_noalloc_bf16) */
+/* element type of the entry points that take `elem` */
+#define INFER_ELEM_BF16        0
+#define INFER_ELEM_F32         1
+
 #define INFER_KV_ENOTINIT     -6   /* first decode call on this device made while its stream is
                                       being captured: call infer_kv_init() before the capture    */
 
@@ -322,6 +326,101 @@ int infer_rms_norm_splitk_bf16(const float* partial, int64_t splits, int64_t spl
                                const void* weight, void* out, int64_t out_stride0,
                                int64_t n_rows, int64_t hidden, float eps, void* stream);
 
+/* ------------------------------------------------------------------ operators of the hybrid models
+ * Models that mix latent attention (one compressed cache row per token) with recurrent layers (one
+ * fixed-size state per sequence) and keep the residual stream in float32.  No counterpart in the
+ * reference.  `elem` is the element type of the activations, weights and cache rows behind the void
+ * pointers (INFER_ELEM_*); norm weights, tables and recurrent state are float32. */
+
+/* One pass over the rows of the float32 residual stream x[rows][width]:
+ *   x = embed[tokens[row]] * embed_scale                    if tokens,
+ *   x = x + y / sqrt(mean(y^2) + eps) * w_post              if y (element type) or partial (the float32
+ *                                                           pieces of infer_skinny_gemm_partial_bf16),
+ *   h = x / sqrt(mean(x^2) + eps) * w_pre                   if w_pre; h in the element type.
+ * Token ids are clamped to the vocabulary. */
+int infer_residual_norm(int elem, const int64_t* tokens, const void* embed, float embed_scale, int64_t vocab,
+                        const void* y, int64_t y_stride, const float* partial, int64_t splits, int64_t split_stride,
+                        int64_t partial_stride, const float* w_post, float* x, int64_t x_stride, const float* w_pre,
+                        void* h, int64_t h_stride, int64_t n_rows, int64_t width, float eps, void* stream);
+
+/* out[r, j] = gelu_tanh(x[r, j]) * x[r, d + j]. */
+int infer_gelu_tanh_and_mul(int elem, void* out, int64_t out_stride, const void* x, int64_t x_stride,
+                            int64_t n_rows, int64_t d, void* stream);
+
+/* Front end of latent attention.  A token's projection row holds q (heads x [dim | rot]) at column 0 and
+ * [latent: rank | rotated key part: rot] at column kv_off.  The latent is RMS-normed (c_norm), the first
+ * rot_dims of every rotated part turn by the token's position (interleaved pairs; table[pos] = cos, sin per
+ * pair), and the cache row [c | 0 .. rank_pad | rotated part | 0 .. row] is stored at slots[t] (negative:
+ * skipped).  Rows below qx_rows get their rotated queries in qx[t][head][rank_pad .. row), zero padded, the
+ * others in place. */
+int infer_latent_front(int elem, void* proj, int64_t proj_stride, int64_t heads, int64_t dim, int64_t rot,
+                       int64_t rot_dims, int64_t kv_off, int64_t rank, const float* c_norm, float eps,
+                       const float* table, int64_t max_pos, const int64_t* positions, const int32_t* slots,
+                       void* cache, int64_t rank_pad, int64_t row, int64_t num_slots, void* qx, int64_t qx_rows,
+                       int64_t n, void* stream);
+
+/* out[m][h][n] = sum_k x[m][h][k] w[h][n][k] (* sigmoid(gate[m][h]) if gate).  w rows are padded with zeros
+ * to w_row elements (a multiple of 32) and every head to a multiple of 16 rows. */
+int infer_head_matmul(int elem, const void* x, int64_t x_row, int64_t x_head, const void* w, int64_t w_head,
+                      int64_t w_row, void* out, int64_t out_row, int64_t out_head, const void* gate, int64_t gate_row,
+                      int64_t m, int64_t heads, int64_t n, int64_t k, void* stream);
+
+/* Attention of query rows over paged latent rows.  qx[rows][heads][row] is dotted with the first ctx[r] cached
+ * rows of the sequence in block-table row row_seq[r] (row_seq NULL: r), softmax of scale * score, and the
+ * first rank_pad elements of the cached rows are summed: out[rows][heads][rank_pad].  `splits` is the number
+ * of parts the keys are cut into (infer_latent_attention_splits gives a good one; the workspace holds
+ * rows * splits * heads * (rank_pad + 2) floats if it is above 1). */
+int64_t infer_latent_attention_splits(int elem, int64_t rows, int64_t heads, int64_t row, int64_t rank_pad,
+                                      int64_t block_size, int64_t max_keys);
+int infer_latent_attention(int elem, const void* qx, const void* cache, int64_t row, int64_t rank_pad,
+                           const int32_t* block_table, int64_t bt_stride, int64_t table_cols, int64_t block_size,
+                           int64_t num_blocks, const int32_t* row_seq, const int32_t* ctx, int64_t rows, int64_t heads,
+                           float scale, int64_t splits, void* out, float* workspace, int64_t workspace_floats,
+                           void* stream);
+
+/* Cached rows (bf16) of whole sequences as dense rows: sequence s, in block-table row seqs[s], goes to rows
+ * cu_k[s] .. cu_k[s + 1) of out[.][row]. */
+int infer_latent_gather(const void* cache, int64_t row, int64_t block_size, int64_t num_blocks,
+                        const int32_t* block_table, int64_t bt_stride, int64_t table_cols, const int32_t* seqs,
+                        const int32_t* cu_k, int64_t num_seqs, int64_t max_keys, void* out, void* stream);
+
+/* Causal varlen attention over dense keys [plain part per head | rotated part shared by all heads] and values
+ * per head (bf16), output gated by sigmoid(gate[token][head]).  cu_q / cu_k: first token row / key row of each
+ * sequence; query i sees keys 0 .. i + (sk - sq). */
+int infer_latent_prefill_supported(int64_t dim, int64_t rot, int64_t vdim);
+int infer_latent_prefill(const void* q, int64_t q_stride, const void* kp, int64_t kp_stride, const void* kr,
+                         int64_t kr_stride, const void* v, int64_t v_stride, const void* gate, int64_t gate_stride,
+                         void* out, int64_t out_stride, const int32_t* cu_q, const int32_t* cu_k, int64_t num_seqs,
+                         int64_t max_seqlen_q, int64_t heads, int64_t dim, int64_t rot, int64_t vdim, float scale,
+                         void* stream);
+
+/* Gated delta rule with a decay per key channel.  A token's projection row holds the inputs of the short
+ * convolution, q and k (kv_heads x dim each) and v (heads x vdim), from column 0 and the write-strength
+ * logits (heads) at column beta_off; decay[row][heads * dim] and gate[row][heads * vdim] are the outputs of
+ * the low-rank projections before softplus and sigmoid.  conv is [channels][taps], the last tap meeting the
+ * current token.  ring[slots][taps][channels] and state[slots][heads][state rows][state columns] are the
+ * sequence's state (infer_delta_layout: [0] state rows, [1] state columns, [2] floats of a chunk record,
+ * [3] tokens per chunk); a sequence at position 0 starts from zero whatever they hold.
+ *
+ * infer_delta_step: one token per row; rows with a negative slot are padding (zeros come out).
+ * infer_delta_chunks: prompt portions, rows row0 .. row0 + rows - 1.  portions[.][4] = first chunk, chunks, slot,
+ * first position; chunks[.][6] = first row, tokens, first position, first position of the portion, slot, 0;
+ * ring_slot[row][2] (indexed by batch row) = the slot, and how many rows of the portion follow.
+ * records: num_chunks * heads * [2] floats; o: (row0 + rows) * heads * [1] floats. */
+int infer_delta_layout(int64_t dim, int64_t vdim, int64_t* out4);
+int infer_delta_step(int elem, const void* proj, int64_t proj_stride, int64_t beta_off, const void* decay,
+                     int64_t decay_stride, const void* gate, int64_t gate_stride, const float* conv, const float* a_log,
+                     const float* dt_bias, const float* norm, void* ring, float* state, int64_t num_slots, int64_t heads,
+                     int64_t kv_heads, int64_t dim, int64_t vdim, int64_t taps, float eps, const int32_t* slots,
+                     const int64_t* positions, void* out, int64_t out_stride, int64_t rows, void* stream);
+int infer_delta_chunks(int elem, const void* proj, int64_t proj_stride, int64_t beta_off, const void* decay,
+                       int64_t decay_stride, const void* gate, int64_t gate_stride, const float* conv, const float* a_log,
+                       const float* dt_bias, const float* norm, void* ring, float* state, int64_t num_slots, int64_t heads,
+                       int64_t kv_heads, int64_t dim, int64_t vdim, int64_t taps, float eps, const int32_t* portions,
+                       int64_t num_portions, const int32_t* chunks, int64_t num_chunks, float* records, float* o,
+                       const int32_t* ring_slot, const int64_t* positions, void* out, int64_t out_stride, int64_t row0,
+                       int64_t rows, void* stream);
+
 /* ------------------------------------------------------------------ 3. block pool (host only)
  * C view of infer::BlockPool (include/infer_kv/block_pool.hpp), the native counterpart of the
  * reference's Python BlockManager (infer/engine/block_mannager.py:44-133), which is the block
@@ -360,6 +459,11 @@ int64_t infer_pool_may_append(infer_pool* pool, const int64_t* token_ids, int64_
  * hand over the whole sequence. */
 int64_t infer_pool_may_append_block(infer_pool* pool, const int64_t* last_block_tokens, int64_t seq_len,
                                     int32_t* table, int64_t num_blocks, int64_t table_capacity);
+
+/* Takes `count` blocks from the front of the free list without hashing anything (sequences whose cache no
+ * other sequence can share: part of their history is recurrent state).  All or nothing:
+ * INFER_KV_ESTATE if fewer are free.  They go back through infer_pool_deallocate. */
+int infer_pool_acquire(infer_pool* pool, int64_t count, int32_t* ids_out);
 
 /* compute_hash :54-60: xxh64(seed 0) over [prefix hash as 8 LE bytes, if has_prefix] ++ int64 LE ids. */
 uint64_t infer_pool_hash(const int64_t* token_ids, int64_t n, int has_prefix, uint64_t prefix_hash);

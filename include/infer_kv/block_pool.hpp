@@ -64,6 +64,7 @@ public:
     // takes the block at the front of the free FIFO / drops one reference.
     int32_t acquire_block();
     void release_block(int32_t block_id);
+    void acquire_blocks(int64_t count, int32_t* ids_out);   // all or nothing
 
     // introspection for tests and statistics
     int32_t ref_count(int32_t block_id) const;

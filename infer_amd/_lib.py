@@ -48,6 +48,28 @@ SIGNATURES = {
     "infer_skinny_gemm_partial_bf16": (_c.c_int, [_vp, _i64, _vp, _vp, _i64, _i64, _i64, _i64, _vp, _sz, _vp, _vp]),
     "infer_rms_norm_splitk_bf16": (_c.c_int, [_vp, _i64, _i64, _i64, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32,
                                               _vp]),
+    "infer_residual_norm": (_c.c_int, [_c.c_int, _vp, _vp, _f32, _i64, _vp, _i64, _vp, _i64, _i64, _i64, _vp,
+                                       _vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
+    "infer_gelu_tanh_and_mul": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _i64, _i64, _i64, _vp]),
+    "infer_latent_front": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _f32, _vp,
+                                      _i64, _vp, _vp, _vp, _i64, _i64, _i64, _vp, _i64, _i64, _vp]),
+    "infer_head_matmul": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _i64,
+                                     _i64, _i64, _i64, _i64, _vp]),
+    "infer_latent_attention_splits": (_i64, [_c.c_int, _i64, _i64, _i64, _i64, _i64, _i64]),
+    "infer_latent_attention": (_c.c_int, [_c.c_int, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i64, _i64, _vp,
+                                          _vp, _i64, _i64, _f32, _i64, _vp, _vp, _i64, _vp]),
+    "infer_latent_gather": (_c.c_int, [_vp, _i64, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _i64, _i64, _vp, _vp]),
+    "infer_latent_prefill_supported": (_c.c_int, [_i64, _i64, _i64]),
+    "infer_latent_prefill": (_c.c_int, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp,
+                                        _vp, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp]),
+    "infer_delta_layout": (_c.c_int, [_i64, _i64, _vp]),
+    "infer_delta_step": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp,
+                                    _vp, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp, _vp, _vp, _i64, _i64,
+                                    _vp]),
+    "infer_delta_chunks": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp,
+                                      _vp, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp, _i64, _vp, _i64, _vp,
+                                      _vp, _vp, _vp, _vp, _i64, _i64, _i64, _vp]),
+    "infer_pool_acquire": (_c.c_int, [_vp, _i64, _vp]),
     "infer_pool_create": (_vp, [_i32, _i32]),
     "infer_pool_destroy": (None, [_vp]),
     "infer_pool_last_error": (_c.c_char_p, []),

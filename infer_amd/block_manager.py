@@ -6,6 +6,7 @@ Same method names, same arguments (a ``Sequence``), same side effects on the seq
 from __future__ import annotations
 
 import ctypes
+from collections import deque
 
 import numpy as np
 
@@ -83,6 +84,19 @@ class BlockManager:
         seq.num_cached_tokens += int(cached)
         seq.block_table.extend(table.tolist())
 
+    def reserve(self, seq: Sequence, num_tokens: int) -> bool:
+        """Extends the sequence's block table to hold ``num_tokens`` tokens, without hashing (nothing of such a
+        sequence is shared with another one).  False, and nothing taken, if too few blocks are free."""
+        need = -(-num_tokens // self.block_size) - len(seq.block_table)
+        if need <= 0:
+            return True
+        if need > self.num_free_blocks:
+            return False
+        ids = np.empty(need, dtype=np.int32)
+        self._state(self._lib.infer_pool_acquire(self._pool, need, ids.ctypes.data))
+        seq.block_table.extend(ids.tolist())
+        return True
+
     def deallocate(self, seq: Sequence):
         table = np.asarray(seq.block_table, dtype=np.int32)
         self._state(self._lib.infer_pool_deallocate(self._pool, table.ctypes.data, table.size))
@@ -108,3 +122,31 @@ class BlockManager:
             self._pool, ids.ctypes.data if ids is not None else None, len(seq), table.ctypes.data, n, table.size))
         if new_n > n:
             seq.block_table.append(int(table[n]))
+
+
+class SlotPool:
+    """Slots of per-sequence recurrent state: first come, first served; a slot that is given back is handed out
+    last.  Nothing is cleared on the way: a sequence starts from zero by its position."""
+
+    def __init__(self, num_slots: int):
+        assert num_slots > 0
+        self.num_slots = num_slots
+        self._free: deque[int] = deque(range(num_slots))
+        self._used: set[int] = set()
+
+    @property
+    def num_free(self) -> int:
+        return len(self._free)
+
+    def take(self) -> int:
+        if not self._free:
+            raise RuntimeError("no free state slot")
+        slot = self._free.popleft()
+        self._used.add(slot)
+        return slot
+
+    def give_back(self, slot: int) -> None:
+        if slot not in self._used:
+            raise RuntimeError(f"state slot {slot} is not in use")
+        self._used.remove(slot)
+        self._free.append(slot)

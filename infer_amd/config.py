@@ -1,4 +1,4 @@
-"""Engine configuration (mirror of ``infer/config.py:5-27``).
+"""Engine configuration (mirror of ``infer/config.py:5-27``) and the model configurations behind it.
 
 The reference reads the model geometry with ``transformers.AutoConfig`` from a checkpoint
 directory.  Here ``hf_config`` may also be handed in directly (a ``ModelConfig`` or any object with
@@ -8,7 +8,8 @@ from __future__ import annotations
 
 import json
 import os
-from dataclasses import dataclass
+import struct
+from dataclasses import dataclass, field
 
 import torch
 
@@ -28,6 +29,9 @@ class ModelConfig:
     rope_theta: float = 1e6
     tie_word_embeddings: bool = False
     torch_dtype: torch.dtype = torch.bfloat16
+
+    block_multiple = 256          # the paged K/V kernels take blocks of a multiple of this many tokens
+    dtypes = (torch.bfloat16,)
 
     @classmethod
     def from_json(cls, path: str) -> "ModelConfig":
@@ -56,6 +60,88 @@ def qwen3_32b() -> ModelConfig:
                        num_key_value_heads=8)
 
 
+def checkpoint_shapes(directory: str) -> dict[str, tuple[int, ...]]:
+    """Tensor shapes of the ``*.safetensors`` files of a directory, from their headers alone."""
+    shapes = {}
+    for name in sorted(os.listdir(directory)):
+        if not name.endswith(".safetensors"):
+            continue
+        with open(os.path.join(directory, name), "rb") as f:
+            (length,) = struct.unpack("<Q", f.read(8))
+            header = json.loads(f.read(length))
+        shapes.update({k: tuple(v["shape"]) for k, v in header.items() if k != "__metadata__"})
+    return shapes
+
+
+@dataclass
+class LayerSpec:
+    """One layer of a model whose layers differ: the kind of its mixer, the mixer's sizes and constants, the
+    width of its feed-forward (None: it has none) and the layer whose weights it uses (its own index unless
+    weights are shared)."""
+    kind: str
+    mixer: dict
+    ff: int | None
+    owner: int
+
+
+@dataclass
+class MerilornConfig:
+    """Merilorn: ``layers`` in order, each latent attention or a gated delta rule, norms on both sides of every
+    sublayer.  The ranks of the low-rank projections of a delta layer (``decay_rank``, ``gate_rank`` of its mixer)
+    are not in ``config.json``; they are read off the checkpoint's tensors."""
+    vocab_size: int
+    hidden_size: int
+    layers: list[LayerSpec] = field(default_factory=list)
+    norm_eps: float = 1e-6
+    embedding_scale: float = 1.0
+    max_position_embeddings: int = 1 << 20          # the design sets no bound; ``max_model_len`` does
+    torch_dtype: torch.dtype = torch.bfloat16
+
+    block_multiple = 32
+    dtypes = (torch.bfloat16, torch.float32)
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_json(cls, path: str) -> "MerilornConfig":
+        with open(path) as f:
+            raw = json.load(f)
+        shapes = checkpoint_shapes(os.path.dirname(os.path.abspath(path)))
+        layers = []
+        for i, entry in enumerate(raw["layers"]):
+            owner = entry.get("weights_of", i)
+            owner = i if owner is None else int(owner)
+            mixer, mlp = dict(entry["mixer"]), entry.get("mlp")
+            if mlp is not None and mlp["kind"] != "dense":
+                raise ValueError(f"layer {i}: feed-forward kind {mlp['kind']!r} is not known")
+            if entry["type"] == "channel_delta":
+                for key, tensor in (("decay_rank", "a1"), ("gate_rank", "g1")):
+                    name = f"l{owner}.mix.{tensor}"
+                    if name in shapes:
+                        mixer[key] = shapes[name][0]
+            layers.append(LayerSpec(entry["type"], mixer, mlp["ff"] if mlp is not None else None, owner))
+        return cls(vocab_size=raw["vocab"], hidden_size=raw["width"], layers=layers, norm_eps=raw["norm"]["eps"],
+                   embedding_scale=raw["embedding"]["scale"])
+
+
+def load_model_config(directory: str):
+    """The configuration of the model in a directory, of the class its ``config.json`` names (``architecture``, or the
+    ``architectures`` list of the transformers layout; without either it is read as Qwen3)."""
+    path = os.path.join(directory, "config.json")
+    with open(path) as f:
+        raw = json.load(f)
+    names = [raw["architecture"]] if "architecture" in raw else raw.get("architectures") or ["Qwen3ForCausalLM"]
+    for name in names:
+        if name in CONFIG_CLASSES:
+            return CONFIG_CLASSES[name].from_json(path)
+    raise ValueError(f"no model of this package serves {names}; known: {sorted(CONFIG_CLASSES)}")
+
+
+CONFIG_CLASSES = {"Qwen3ForCausalLM": ModelConfig, "Merilorn": MerilornConfig}
+
+
 @dataclass
 class Config:
     model: str = ""
@@ -65,20 +151,26 @@ class Config:
     gpu_memory_utilization: float = 0.9
     tensor_parallel_size: int = 1
     enforce_eager: bool = False
-    hf_config: ModelConfig | None = None
+    hf_config: ModelConfig | MerilornConfig | None = None
     eos: int = -1
     kvcache_block_size: int = 256
     num_kvcache_blocks: int = -1
     # Decode tokens are fed position len(seq) by the reference (``model_runner.py:117``) while its
     # prefill positions are zero-based (``:84``); 1 reproduces that, 0 makes both zero-based.
+    # (Models that run portions of prompts beside decoded tokens have one position per token, zero-based.)
     decode_position_offset: int = 1
     seed: int = 0
+    dtype: str | None = None      # element type of weights and activations; None: the model's
 
     def __post_init__(self):
         if self.hf_config is None:
             assert os.path.isdir(self.model)
-            self.hf_config = ModelConfig.from_json(os.path.join(self.model, "config.json"))
-        assert self.kvcache_block_size % 256 == 0
+            self.hf_config = load_model_config(self.model)
+        if self.dtype is not None:
+            self.hf_config.torch_dtype = getattr(torch, self.dtype)
+        if self.hf_config.torch_dtype not in self.hf_config.dtypes:
+            raise ValueError(f"{type(self.hf_config).__name__} does not run in {self.hf_config.torch_dtype}")
+        assert self.kvcache_block_size > 0 and self.kvcache_block_size % self.hf_config.block_multiple == 0
         assert 1 <= self.tensor_parallel_size <= 8
         self.max_model_len = min(self.max_model_len, self.hf_config.max_position_embeddings)
         assert self.max_num_batched_tokens >= self.max_model_len

@@ -248,6 +248,16 @@ int32_t BlockPool::acquire_block() {
     return id;
 }
 
+void BlockPool::acquire_blocks(int64_t count, int32_t* ids_out) {
+    std::lock_guard<std::mutex> g(mu_);
+    if (free_count_ < count) throw std::logic_error("BlockPool::acquire_blocks: out of blocks");
+    for (int64_t i = 0; i < count; ++i) {
+        const int32_t id = free_head_;
+        take(id);
+        ids_out[i] = id;
+    }
+}
+
 void BlockPool::release_block(int32_t id) {
     std::lock_guard<std::mutex> g(mu_);
     if (id < 0 || id >= num_blocks_ || blocks_[id].ref_count <= 0) throw std::logic_error("BlockPool::release_block: block not held");
@@ -328,6 +338,14 @@ int infer_pool_deallocate(infer_pool* p, const int32_t* table, int64_t num_block
     return (int)guarded([&]() -> int64_t {
         std::vector<int32_t> t(table, table + num_blocks);
         p->pool.deallocate(t);
+        return 0;
+    });
+}
+
+int infer_pool_acquire(infer_pool* p, int64_t count, int32_t* ids_out) {
+    if (!p || count < 0 || (!ids_out && count > 0)) return INFER_KV_EINVAL;
+    return (int)guarded([&]() -> int64_t {
+        p->pool.acquire_blocks(count, ids_out);
         return 0;
     });
 }

@@ -1,0 +1,282 @@
+// Causal attention of long prompt portions whose keys come out of a latent: every head has its own unrotated
+// key part and value (W_uk c and W_uv c, dense rows), and one rotated key part is shared by all heads.  bf16 in,
+// float32 accumulate, output gate in the epilogue.
+//
+// A wavefront owns 32 queries (two MFMA column tiles) of one head, a workgroup four wavefronts = 128
+// consecutive queries, and walks the visible keys in steps of 32 that all four share through LDS (two
+// buffers, the next step's rows travel through registers meanwhile):
+//   S^T[key, query] = [k_plain | k_rot][key, :] . q^T      KS k-steps of 32
+//   O^T[v, query]  += V^T[v, key] . P^T                    VT row tiles of 16
+// Row r of the score tile t is key 8 (r / 4) + 4 t + r % 4, so that a lane's eight scores are the eight
+// consecutive keys the second product wants from it and P never leaves its registers.
+#include "elem.h"
+
+namespace {
+
+typedef short i16x4 __attribute__((ext_vector_type(4)));
+typedef short i16x8 __attribute__((ext_vector_type(8)));
+typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
+
+constexpr int kStep = 32;
+constexpr int kWaves = 4;
+constexpr int kQ = 32 * kWaves;         // queries per workgroup
+constexpr float kLazy = 8.f;            // log2 units a row's maximum may grow before the accumulators are rescaled
+
+struct LatentPrefillArgs {
+    const __bf16* q; int64_t q_stride;        // [token][head * (dim + rot)]
+    const __bf16* kp; int64_t kp_stride;      // [key][head * dim]
+    const __bf16* kr; int64_t kr_stride;      // [key][rot]
+    const __bf16* v; int64_t v_stride;        // [key][head * vdim]
+    const __bf16* gate; int64_t gate_stride;  // [token][head]
+    __bf16* out; int64_t out_stride;          // [token][head * vdim]
+    const int32_t* cu_q;                      // first token row of each sequence (rows of q, gate, out)
+    const int32_t* cu_k;                      // first key row of each
+    int heads, dim, rot, vdim, nseq, qblocks;
+    float scale_log2;
+};
+
+__device__ __forceinline__ float max_xor16_32(float x) {
+    const unsigned u = __builtin_bit_cast(unsigned, x);
+    const auto r = __builtin_amdgcn_permlane16_swap(u, u, false, false);
+    const unsigned a0 = r[0], a1 = r[1];
+    const float y = fmaxf(__builtin_bit_cast(float, a0), __builtin_bit_cast(float, a1));
+    const unsigned w = __builtin_bit_cast(unsigned, y);
+    const auto s = __builtin_amdgcn_permlane32_swap(w, w, false, false);
+    const unsigned b0 = s[0], b1 = s[1];
+    return fmaxf(__builtin_bit_cast(float, b0), __builtin_bit_cast(float, b1));
+}
+
+template <int KS, int VT>
+__global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPrefillArgs a) {
+    constexpr int kKPitch = KS * 64 + 16, kVPitch = VT * 32 + 16;              // bytes
+    constexpr int kBuf = kStep * (kKPitch + kVPitch);
+    constexpr int kNK = KS * 4 * kStep / 256, kNV = (VT * 2 * kStep + 255) / 256;    // 16-byte chunks per thread
+    __shared__ __attribute__((aligned(16))) unsigned char lds[2 * kBuf];
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int g = lane >> 4, n = lane & 15;
+    // Workgroups go to the eight dies round-robin; die k works through the k-th contiguous eighth of the
+    // (head, sequence, query block) space, so that the blocks that read the same keys share an L2.
+    const unsigned total = gridDim.x, id = blockIdx.x;
+    const unsigned die = id & 7u, per_die = total >> 3, extra = total & 7u;
+    const unsigned wg = die * per_die + (die < extra ? die : extra) + (id >> 3);
+    const int qblk = a.qblocks - 1 - (int)(wg % a.qblocks);      // late blocks see the most keys: first
+    const int b = (int)((wg / a.qblocks) % a.nseq), h = (int)(wg / ((unsigned)a.qblocks * a.nseq));
+    const int q_beg = a.cu_q[b], sq = a.cu_q[b + 1] - q_beg;
+    const int k_beg = a.cu_k[b], sk = a.cu_k[b + 1] - k_beg;
+    const int wq0 = qblk * kQ;
+    if (wq0 >= sq) return;
+    const int q0 = wq0 + 32 * wave;
+    const bool live = q0 < sq;
+    const int shift = sk - sq;                                   // query i sees keys 0 .. i + shift
+    const int last_q = wq0 + kQ < sq ? wq0 + kQ - 1 : sq - 1;
+    const int nsteps = (last_q + shift + 1 + kStep - 1) / kStep;
+    const int my_last = q0 + 31 < sq ? q0 + 31 : sq - 1;
+    const int my_steps = live ? (my_last + shift + 1 + kStep - 1) / kStep : 0;
+
+    const int qk = a.dim + a.rot;
+    bf16x8_t qreg[2][KS];
+    int limit[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        const int qi = q0 + 16 * u + n;
+        limit[u] = qi + shift;
+        const __bf16* qp = a.q + (int64_t)(q_beg + (qi < sq ? qi : sq - 1)) * a.q_stride + (int64_t)h * qk + 8 * g;
+#pragma unroll
+        for (int j = 0; j < KS; ++j) {
+            qreg[u][j] = bf16x8_t{};
+            if (32 * j + 8 * g < qk) qreg[u][j] = *reinterpret_cast<const bf16x8_t*>(qp + 32 * j);
+        }
+    }
+
+    // the columns behind the real sizes stay zero in both buffers
+    for (int i = tid; i < 2 * kBuf / 16; i += 256) reinterpret_cast<u32x4_t*>(lds)[i] = u32x4_t{0u, 0u, 0u, 0u};
+
+    // chunk i of this thread of the K and of the V tile: key, source, place
+    const int kc = qk / 8, vc = a.vdim / 8, dc = a.dim / 8;
+    int k_key[kNK], k_lds[kNK], v_key[kNV], v_lds[kNV];
+    const __bf16* k_src[kNK];
+    int64_t k_str[kNK];
+    int v_col[kNV];
+#pragma unroll
+    for (int i = 0; i < kNK; ++i) {
+        const int c = tid + 256 * i, key = c / kc, col = c - key * kc;
+        k_key[i] = key < kStep ? key : -1;
+        k_lds[i] = key * kKPitch + col * 16;
+        const bool plain = col < dc;
+        k_src[i] = plain ? a.kp + (int64_t)h * a.dim + 8 * col : a.kr + 8 * (col - dc);
+        k_str[i] = plain ? a.kp_stride : a.kr_stride;
+    }
+#pragma unroll
+    for (int i = 0; i < kNV; ++i) {
+        const int c = tid + 256 * i, key = c / vc, col = c - key * vc;
+        v_key[i] = key < kStep ? key : -1;
+        v_lds[i] = kStep * kKPitch + key * kVPitch + col * 16;
+        v_col[i] = h * a.vdim + 8 * col;
+    }
+    u32x4_t kst[kNK], vst[kNV];
+    auto fetch = [&](int s) {
+        const int last = sk - 1 - s * kStep;       // keys behind the last one re-read it; their weights are zero
+        const int64_t base = k_beg + s * kStep;
+#pragma unroll
+        for (int i = 0; i < kNK; ++i) {
+            const int r = k_key[i] < last ? k_key[i] : last;
+            if (r >= 0) kst[i] = *reinterpret_cast<const u32x4_t*>(k_src[i] + (base + r) * k_str[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < kNV; ++i) {
+            const int r = v_key[i] < last ? v_key[i] : last;
+            if (r >= 0) vst[i] = *reinterpret_cast<const u32x4_t*>(a.v + (base + r) * a.v_stride + v_col[i]);
+        }
+    };
+    auto put = [&](unsigned char* buf) {
+#pragma unroll
+        for (int i = 0; i < kNK; ++i)
+            if (k_key[i] >= 0) *reinterpret_cast<u32x4_t*>(buf + k_lds[i]) = kst[i];
+#pragma unroll
+        for (int i = 0; i < kNV; ++i)
+            if (v_key[i] >= 0) *reinterpret_cast<u32x4_t*>(buf + v_lds[i]) = vst[i];
+    };
+
+    f32x4_t acc[2][VT], lacc[2];
+    float m_neg[2];
+    bf16x8_t ones;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ones[i] = (__bf16)1.f;
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        m_neg[u] = INFINITY;
+        lacc[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int t = 0; t < VT; ++t) acc[u][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
+
+    fetch(0);
+    __syncthreads();          // the zero fill
+    put(lds);
+    __syncthreads();
+    const int k_addr = (8 * (n >> 2) + (n & 3)) * kKPitch + 16 * g;
+    const int v_addr = kStep * kKPitch + (8 * g + (n >> 2)) * kVPitch + (n & 3) * 8;
+    for (int s = 0; s < nsteps; ++s) {
+        const unsigned char* buf = lds + (s & 1) * kBuf;
+        if (s + 1 < nsteps) fetch(s + 1);
+        if (s < my_steps) {
+            const int tok0 = s * kStep;
+            f32x4_t sc[2][2];
+#pragma unroll
+            for (int u = 0; u < 2; ++u)
+#pragma unroll
+                for (int t = 0; t < 2; ++t) sc[u][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int j = 0; j < KS; ++j)
+#pragma unroll
+                for (int t = 0; t < 2; ++t) {
+                    const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(buf + k_addr + 4 * t * kKPitch + 64 * j);
+#pragma unroll
+                    for (int u = 0; u < 2; ++u) sc[u][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qreg[u][j], sc[u][t], 0, 0, 0);
+                }
+            bf16x8_t pb[2];
+#pragma unroll
+            for (int u = 0; u < 2; ++u) {
+                float sv[8];
+#pragma unroll
+                for (int t = 0; t < 2; ++t)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) sv[4 * t + e] = sc[u][t][e];
+                if (tok0 + kStep - 1 > q0 + 16 * u + shift) {          // the earliest query of the tile does not see all of it
+                    const int rel = limit[u] - tok0 - 8 * g;
+#pragma unroll
+                    for (int i = 0; i < 8; ++i)
+                        if (i > rel) sv[i] = -INFINITY;
+                }
+                float mx = sv[0];
+#pragma unroll
+                for (int i = 1; i < 8; ++i) mx = fmaxf(mx, sv[i]);
+                mx = max_xor16_32(mx) * a.scale_log2;
+                const bool grow = mx + m_neg[u] > kLazy;               // +inf before the first step, whose key 0 everyone sees
+                if (__any(grow)) {
+                    const float alpha = grow ? __builtin_amdgcn_exp2f(-m_neg[u] - mx) : 1.f;
+                    m_neg[u] = grow ? -mx : m_neg[u];
+                    lacc[u] *= alpha;
+#pragma unroll
+                    for (int t = 0; t < VT; ++t) acc[u][t] *= alpha;
+                }
+#pragma unroll
+                for (int i = 0; i < 8; ++i) pb[u][i] = (__bf16)__builtin_amdgcn_exp2f(__builtin_fmaf(sv[i], a.scale_log2, m_neg[u]));
+                lacc[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pb[u], lacc[u], 0, 0, 0);
+            }
+#pragma unroll
+            for (int t = 0; t < VT; ++t) {
+                const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(buf + v_addr + 32 * t));
+                const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(buf + v_addr + 32 * t + 4 * kVPitch));
+                const bf16x8_t vt = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+#pragma unroll
+                for (int u = 0; u < 2; ++u) acc[u][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pb[u], acc[u][t], 0, 0, 0);
+            }
+        }
+        if (s + 1 < nsteps) put(lds + ((s + 1) & 1) * kBuf);
+        __syncthreads();
+    }
+    if (!live) return;
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        const int qi = q0 + 16 * u + n;
+        if (qi >= sq) continue;
+        const float l = lacc[u][0];
+        const float f = (l > 0.f ? 1.f / l : 0.f) * sigmoid_f((float)a.gate[(int64_t)(q_beg + qi) * a.gate_stride + h]);
+        __bf16* o = a.out + (int64_t)(q_beg + qi) * a.out_stride + (int64_t)h * a.vdim + 4 * g;
+#pragma unroll
+        for (int t = 0; t < VT; ++t)
+            if (16 * t + 4 * g < a.vdim) {
+                bf16x4_t v;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[e] = (__bf16)(acc[u][t][e] * f);
+                *reinterpret_cast<bf16x4_t*>(o + 16 * t) = v;
+            }
+    }
+}
+
+// (k-steps, value tiles) the kernel is built for, smallest first
+template <int KS, int VT>
+int go(const LatentPrefillArgs& a, unsigned grid, hipStream_t st) {
+    hipLaunchKernelGGL((latent_prefill_kernel<KS, VT>), dim3(grid), dim3(64 * kWaves), 0, st, a);
+    return (int)hipGetLastError();
+}
+
+}  // namespace
+
+// 1 if the sizes are served by the kernel
+extern "C" int infer_latent_prefill_supported(int64_t dim, int64_t rot, int64_t vdim) {
+    if (dim <= 0 || rot <= 0 || vdim <= 0 || dim % 8 || rot % 8 || vdim % 8) return 0;
+    return dim + rot <= 256 && vdim <= 128;
+}
+
+extern "C" int infer_latent_prefill(const void* q, int64_t q_stride, const void* kp, int64_t kp_stride, const void* kr,
+                                    int64_t kr_stride, const void* v, int64_t v_stride, const void* gate, int64_t gate_stride,
+                                    void* out, int64_t out_stride, const int32_t* cu_q, const int32_t* cu_k, int64_t num_seqs,
+                                    int64_t max_seqlen_q, int64_t heads, int64_t dim, int64_t rot, int64_t vdim, float scale,
+                                    void* stream) {
+    if (num_seqs < 0 || max_seqlen_q < 0) return INFER_KV_EINVAL;
+    if (num_seqs == 0 || max_seqlen_q == 0) return INFER_KV_OK;
+    if (!q || !kp || !kr || !v || !gate || !out || !cu_q || !cu_k || heads < 1 || heads > 4096 || !(scale > 0.f)) return INFER_KV_EINVAL;
+    if (!infer_latent_prefill_supported(dim, rot, vdim)) return INFER_KV_EUNSUPPORTED;
+    if (q_stride < heads * (dim + rot) || kp_stride < heads * dim || kr_stride < rot || v_stride < heads * vdim ||
+        gate_stride < heads || out_stride < heads * vdim)
+        return INFER_KV_EINVAL;
+    if (q_stride % 8 || kp_stride % 8 || kr_stride % 8 || v_stride % 8 || out_stride % 4 || !ptr_aligned(q, 16) || !ptr_aligned(kp, 16) ||
+        !ptr_aligned(kr, 16) || !ptr_aligned(v, 16) || !ptr_aligned(out, 8))
+        return INFER_KV_EALIGN;
+    const int64_t qblocks = (max_seqlen_q + kQ - 1) / kQ, total = qblocks * num_seqs * heads;
+    if (total > 0x7fffffff) return INFER_KV_EINVAL;
+    LatentPrefillArgs a{(const __bf16*)q, q_stride, (const __bf16*)kp, kp_stride, (const __bf16*)kr, kr_stride, (const __bf16*)v,
+                        v_stride, (const __bf16*)gate, gate_stride, (__bf16*)out, out_stride, cu_q, cu_k, (int)heads, (int)dim,
+                        (int)rot, (int)vdim, (int)num_seqs, (int)qblocks, scale * kLog2e};
+    hipStream_t st = (hipStream_t)stream;
+    const int64_t qk = dim + rot;
+    const unsigned grid = (unsigned)total;
+    if (qk <= 64 && vdim <= 64) return go<2, 4>(a, grid, st);
+    if (qk <= 128 && vdim <= 64) return go<4, 4>(a, grid, st);
+    if (qk <= 128) return go<4, 8>(a, grid, st);
+    if (qk <= 192) return go<6, 8>(a, grid, st);
+    return go<8, 8>(a, grid, st);
+}

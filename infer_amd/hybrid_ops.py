@@ -1,0 +1,249 @@
+"""Python entry points of the hybrid-model kernels (latent attention, gated delta rule, float32 residual
+stream), beside ``ops``: shape and type checks on the host, then one call into ``libinfer_kv.so`` on torch's
+current stream.  Activations are bfloat16 or float32; there is no CPU path."""
+from __future__ import annotations
+
+import ctypes
+from functools import lru_cache
+
+import torch
+
+from . import _lib
+from .ops import SplitKSum, _require_gpu, _stream_ptr
+
+ELEM = {torch.bfloat16: 0, torch.float32: 1}
+
+
+def _ptr(t):
+    return None if t is None else t.data_ptr()
+
+
+def _rows(t: torch.Tensor, cols: int) -> int:
+    """Row stride of a 2-D view with contiguous rows of at least ``cols`` elements."""
+    assert t.dim() == 2 and t.stride(1) == 1 and t.shape[1] >= cols, (tuple(t.shape), t.stride(), cols)
+    return max(t.stride(0), t.shape[1])
+
+
+def _f32(t: torch.Tensor, *shape) -> torch.Tensor:
+    assert t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == shape, (t.dtype, tuple(t.shape), shape)
+    return t
+
+
+# ------------------------------------------------------------------ residual stream
+def residual_norm(x: torch.Tensor, eps: float, *, y=None, w_post=None, w_pre=None, tokens=None, embed=None,
+                  embed_scale: float = 1.0, dtype: torch.dtype = torch.bfloat16):
+    """``x`` [rows, width] float32 is updated in place: the embedding of ``tokens`` is stored, or
+    ``rms(y) * w_post`` added (``y`` may be an unreduced ``SplitKSum``).  Returns ``rms(x) * w_pre`` in ``dtype``,
+    or None without ``w_pre``."""
+    n, width = x.shape
+    assert x.dtype == torch.float32
+    y_stride = splits = split_stride = partial_stride = 0
+    partial = None
+    if isinstance(y, SplitKSum):
+        y.check_alive()
+        partial, y = y.partial, None
+        assert partial.dtype == torch.float32 and partial.is_contiguous() and tuple(partial.shape[1:]) == (n, width)
+        splits, split_stride, partial_stride = partial.shape[0], n * width, width
+    elif y is not None:
+        assert y.dtype == dtype and tuple(y.shape) == (n, width)
+        y_stride = _rows(y, width)
+    if y is not None or partial is not None:
+        _f32(w_post, width)
+    if w_pre is not None:
+        _f32(w_pre, width)
+    if tokens is not None:
+        assert tokens.dtype == torch.int64 and tokens.is_contiguous() and tokens.numel() == n
+        assert embed.dtype == dtype and embed.is_contiguous() and embed.shape[1] == width
+    out = torch.empty((n, width), dtype=dtype, device=x.device) if w_pre is not None else None
+    _require_gpu(x, *[t for t in (y, partial, w_post, w_pre, tokens, embed) if t is not None])
+    rc = _lib.load().infer_residual_norm(
+        ELEM[dtype], _ptr(tokens), _ptr(embed), float(embed_scale), embed.shape[0] if embed is not None else 0,
+        _ptr(y), y_stride, _ptr(partial), splits, split_stride, partial_stride, _ptr(w_post), x.data_ptr(),
+        _rows(x, width), _ptr(w_pre), _ptr(out), width, n, width, float(eps), _stream_ptr(x))
+    _lib.check(rc, "residual_norm")
+    return out
+
+
+def gelu_tanh_and_mul(x: torch.Tensor) -> torch.Tensor:
+    """``gelu_tanh(x[:, :d]) * x[:, d:]``."""
+    d = x.shape[1] // 2
+    out = torch.empty((x.shape[0], d), dtype=x.dtype, device=x.device)
+    _require_gpu(x)
+    rc = _lib.load().infer_gelu_tanh_and_mul(ELEM[x.dtype], out.data_ptr(), d, x.data_ptr(), _rows(x, 2 * d), x.shape[0],
+                                             d, _stream_ptr(x))
+    _lib.check(rc, "gelu_tanh_and_mul")
+    return out
+
+
+# ------------------------------------------------------------------ latent attention
+def latent_front(proj, heads, dim, rot, rot_dims, kv_off, rank, c_norm, eps, table, positions, slots, cache, rank_pad,
+                 qx, qx_rows) -> None:
+    """Norm of the latent, rotary positions and the append of one cache row per token; ``cache`` is
+    [blocks, block_size, row], ``qx`` [>= qx_rows, heads, row]."""
+    n = proj.shape[0]
+    row = cache.shape[2]
+    _f32(c_norm, rank)
+    assert table.dtype == torch.float32 and table.is_contiguous() and table.shape[1:] == (rot_dims // 2, 2)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == n
+    assert slots.dtype == torch.int32 and slots.is_contiguous() and slots.numel() == n
+    assert cache.dtype == proj.dtype and cache.is_contiguous()
+    assert qx_rows == 0 or (qx.dtype == proj.dtype and qx.is_contiguous() and tuple(qx.shape[1:]) == (heads, row)
+                            and qx.shape[0] >= qx_rows)
+    _require_gpu(proj, c_norm, table, positions, slots, cache)
+    rc = _lib.load().infer_latent_front(
+        ELEM[proj.dtype], proj.data_ptr(), _rows(proj, kv_off + rank + rot), heads, dim, rot, rot_dims, kv_off, rank,
+        c_norm.data_ptr(), float(eps), table.data_ptr(), table.shape[0], positions.data_ptr(), slots.data_ptr(),
+        cache.data_ptr(), rank_pad, row, cache.shape[0] * cache.shape[1], _ptr(qx) if qx_rows else None, qx_rows, n,
+        _stream_ptr(proj))
+    _lib.check(rc, "latent_front")
+
+
+def head_matmul(x, w, out, n: int, k: int, gate=None) -> None:
+    """``out[m, h, :n] = w[h, :n, :k] x[m, h, :k]`` (times ``sigmoid(gate[m, h])``) on 3-D views with a contiguous last
+    axis; ``w`` [heads, n padded to 16, k padded to 32] is padded with zeros."""
+    m, heads = x.shape[:2]
+    assert x.dtype == w.dtype == out.dtype and out.shape[:2] == (m, heads) and w.shape[0] == heads
+    assert x.stride(2) == 1 and out.stride(2) == 1 and w.is_contiguous()
+    assert x.shape[2] >= k and out.shape[2] >= n and w.shape[1] >= (n + 15) // 16 * 16 and w.shape[2] >= k
+    if gate is not None:
+        assert gate.dtype == x.dtype and gate.shape[0] == m and gate.shape[1] >= heads and gate.stride(1) == 1
+    _require_gpu(x, w, out)
+    rc = _lib.load().infer_head_matmul(
+        ELEM[x.dtype], x.data_ptr(), x.stride(0), x.stride(1), w.data_ptr(), w.stride(0), w.shape[2], out.data_ptr(),
+        out.stride(0), out.stride(1), _ptr(gate), max(gate.stride(0), heads) if gate is not None else 0, m, heads, n, k,
+        _stream_ptr(x))
+    _lib.check(rc, "head_matmul")
+
+
+def latent_attention(qx, cache, block_table, ctx, scale: float, rank_pad: int, row_seq=None, max_keys=None,
+                     splits: int = 0) -> torch.Tensor:
+    """``qx`` [rows, heads, row] against the first ``ctx[r]`` cached rows of the sequence in block-table row
+    ``row_seq[r]`` (default ``r``).  Returns the weighted latents [rows, heads, rank_pad].  ``max_keys`` bounds ``ctx`` for the
+    choice of ``splits`` (default: what a block-table row can address)."""
+    rows, heads, row = qx.shape
+    nblk, bs, crow = cache.shape
+    assert qx.is_contiguous() and cache.is_contiguous() and cache.dtype == qx.dtype and crow == row
+    assert block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.stride(1) == 1
+    assert ctx.dtype == torch.int32 and ctx.is_contiguous() and ctx.numel() == rows
+    if row_seq is None:
+        assert block_table.shape[0] >= rows
+    else:
+        assert row_seq.dtype == torch.int32 and row_seq.is_contiguous() and row_seq.numel() == rows
+    _require_gpu(qx, cache, block_table, ctx)
+    lib = _lib.load()
+    elem, cols = ELEM[qx.dtype], block_table.shape[1]
+    if splits <= 0:
+        splits = lib.infer_latent_attention_splits(elem, rows, heads, row, rank_pad, bs, max_keys or cols * bs)
+    out = torch.empty((rows, heads, rank_pad), dtype=qx.dtype, device=qx.device)
+    need = rows * splits * heads * (rank_pad + 2) if splits > 1 else 0
+    ws = torch.empty(need, dtype=torch.float32, device=qx.device) if need else None
+    rc = lib.infer_latent_attention(elem, qx.data_ptr(), cache.data_ptr(), row, rank_pad, block_table.data_ptr(),
+                                    max(block_table.stride(0), cols), cols, bs, nblk, _ptr(row_seq), ctx.data_ptr(), rows,
+                                    heads, float(scale), splits, out.data_ptr(), _ptr(ws), need, _stream_ptr(qx))
+    _lib.check(rc, "latent_attention")
+    return out
+
+
+def latent_gather(cache, block_table, seqs, cu_k, total: int, max_keys: int) -> torch.Tensor:
+    """The cached rows of the sequences in block-table rows ``seqs`` as dense rows [total, row]."""
+    nblk, bs, row = cache.shape
+    assert cache.dtype == torch.bfloat16 and cache.is_contiguous()
+    assert block_table.dtype == torch.int32 and block_table.stride(1) == 1
+    for t in (seqs, cu_k):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    assert cu_k.numel() == seqs.numel() + 1
+    _require_gpu(cache, block_table, seqs, cu_k)
+    out = torch.empty((total, row), dtype=cache.dtype, device=cache.device)
+    rc = _lib.load().infer_latent_gather(cache.data_ptr(), row, bs, nblk, block_table.data_ptr(),
+                                         max(block_table.stride(0), block_table.shape[1]), block_table.shape[1],
+                                         seqs.data_ptr(), cu_k.data_ptr(), seqs.numel(), max_keys, out.data_ptr(),
+                                         _stream_ptr(cache))
+    _lib.check(rc, "latent_gather")
+    return out
+
+
+def latent_prefill_supported(dim: int, rot: int, vdim: int) -> bool:
+    """Whether the dense-key prefill kernel serves these sizes."""
+    return bool(_lib.load().infer_latent_prefill_supported(dim, rot, vdim))
+
+
+def latent_prefill(q, kp, kr, v, gate, out, cu_q, cu_k, max_seqlen_q: int, heads, dim, rot, vdim, scale) -> None:
+    """Causal attention of whole portions over dense keys and values (all bf16, 2-D views)."""
+    for t in (q, kp, kr, v, gate, out):
+        assert t.dtype == torch.bfloat16
+    for t in (cu_q, cu_k):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    assert cu_q.numel() == cu_k.numel() and kp.shape[0] == kr.shape[0] == v.shape[0]
+    assert q.shape[0] == gate.shape[0] == out.shape[0]
+    _require_gpu(q, kp, kr, v, gate, out, cu_q, cu_k)
+    rc = _lib.load().infer_latent_prefill(
+        q.data_ptr(), _rows(q, heads * (dim + rot)), kp.data_ptr(), kp.stride(0), kr.data_ptr(), kr.stride(0), v.data_ptr(),
+        v.stride(0), gate.data_ptr(), max(gate.stride(0), heads), out.data_ptr(), _rows(out, heads * vdim), cu_q.data_ptr(),
+        cu_k.data_ptr(), cu_q.numel() - 1, int(max_seqlen_q), heads, dim, rot, vdim, float(scale), _stream_ptr(q))
+    _lib.check(rc, "latent_prefill")
+
+
+# ------------------------------------------------------------------ gated delta rule
+@lru_cache(maxsize=None)
+def delta_layout(dim: int, vdim: int) -> tuple[int, int, int, int]:
+    """(state rows, state columns, floats of a chunk record, tokens per chunk) of a head."""
+    out = (ctypes.c_int64 * 4)()
+    _lib.check(_lib.load().infer_delta_layout(dim, vdim, ctypes.addressof(out)), "delta_layout")
+    return tuple(out)
+
+
+class DeltaShape:
+    """Sizes and constants of a delta-rule layer, shared by its two entry points."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, eps: float):
+        assert heads % kv_heads == 0
+        self.heads, self.kv_heads, self.dim, self.vdim, self.taps, self.eps = heads, kv_heads, dim, vdim, taps, eps
+        self.channels = 2 * kv_heads * dim + heads * vdim
+        self.state_rows, self.state_cols, self.record, self.chunk = delta_layout(dim, vdim)
+
+
+def _delta_common(s: DeltaShape, proj, beta_off, decay, gate, conv, a_log, dt_bias, norm, ring, state, out):
+    assert proj.dtype == decay.dtype == gate.dtype == ring.dtype == out.dtype
+    n = proj.shape[0]
+    assert decay.shape[0] == gate.shape[0] == out.shape[0] == n
+    slots = state.shape[0]
+    _f32(conv, s.channels, s.taps)
+    _f32(a_log, s.heads)
+    _f32(dt_bias, s.heads * s.dim)
+    _f32(norm, s.vdim)
+    _f32(state, slots, s.heads, s.state_rows, s.state_cols)
+    assert ring.is_contiguous() and tuple(ring.shape) == (slots, s.taps, s.channels)
+    _require_gpu(proj, decay, gate, conv, a_log, dt_bias, norm, ring, state, out)
+    return [ELEM[proj.dtype], proj.data_ptr(), _rows(proj, beta_off + s.heads), beta_off, decay.data_ptr(),
+            _rows(decay, s.heads * s.dim), gate.data_ptr(), _rows(gate, s.heads * s.vdim), conv.data_ptr(), a_log.data_ptr(),
+            dt_bias.data_ptr(), norm.data_ptr(), ring.data_ptr(), state.data_ptr(), slots, s.heads, s.kv_heads, s.dim, s.vdim,
+            s.taps, float(s.eps)]
+
+
+def delta_step(s: DeltaShape, proj, beta_off, decay, gate, conv, a_log, dt_bias, norm, ring, state, slots, positions, out) -> None:
+    """One token per sequence: row r of the inputs advances the state of slot ``slots[r]`` (negative: padding)."""
+    n = proj.shape[0]
+    args = _delta_common(s, proj, beta_off, decay, gate, conv, a_log, dt_bias, norm, ring, state, out)
+    assert slots.dtype == torch.int32 and slots.is_contiguous() and slots.numel() == n
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == n
+    rc = _lib.load().infer_delta_step(*args, slots.data_ptr(), positions.data_ptr(), out.data_ptr(), _rows(out, s.heads * s.vdim),
+                                      n, _stream_ptr(proj))
+    _lib.check(rc, "delta_step")
+
+
+def delta_chunks(s: DeltaShape, proj, beta_off, decay, gate, conv, a_log, dt_bias, norm, ring, state, portions, chunks, ring_slot,
+                 positions, row0: int, out) -> None:
+    """Prompt portions: batch rows ``row0`` and up.  ``portions`` [.., 4] and ``chunks`` [.., 6] are the int32
+    descriptors of ``infer_kv.h``; ``ring_slot`` and ``positions`` are indexed by batch row."""
+    n = proj.shape[0]
+    args = _delta_common(s, proj, beta_off, decay, gate, conv, a_log, dt_bias, norm, ring, state, out)
+    assert portions.dtype == torch.int32 and portions.is_contiguous() and portions.shape[1] == 4
+    assert chunks.dtype == torch.int32 and chunks.is_contiguous() and chunks.shape[1] == 6
+    assert ring_slot.dtype == torch.int32 and ring_slot.is_contiguous() and tuple(ring_slot.shape) == (n, 2)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == n
+    records = torch.empty(chunks.shape[0] * s.heads * s.record, dtype=torch.float32, device=proj.device)
+    o = torch.empty(n * s.heads * s.state_cols, dtype=torch.float32, device=proj.device)
+    rc = _lib.load().infer_delta_chunks(
+        *args, portions.data_ptr(), portions.shape[0], chunks.data_ptr(), chunks.shape[0], records.data_ptr(), o.data_ptr(),
+        ring_slot.data_ptr(), positions.data_ptr(), out.data_ptr(), _rows(out, s.heads * s.vdim), row0, n - row0, _stream_ptr(proj))
+    _lib.check(rc, "delta_chunks")

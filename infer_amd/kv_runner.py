@@ -52,11 +52,11 @@ def prepare_block_tables(seqs: list[Sequence], device="cuda") -> torch.Tensor:
 
 
 def prepare_prefill(seqs: list[Sequence], device="cuda"):
-    block_size = Sequence.block_size
     input_ids, positions, slot_mapping = [], [], []
     cu_seqlens_q, cu_seqlens_k = [0], [0]
     max_seqlen_q = max_seqlen_k = 0
     for seq in seqs:
+        block_size = seq.block_size
         seqlen = len(seq)
         input_ids.extend(seq[seq.num_cached_tokens:])
         positions.extend(range(seq.num_cached_tokens, seqlen))
@@ -80,13 +80,12 @@ def prepare_prefill(seqs: list[Sequence], device="cuda"):
 
 
 def prepare_decode(seqs: list[Sequence], device="cuda"):
-    block_size = Sequence.block_size
     input_ids, positions, slot_mapping, context_lens = [], [], [], []
     for seq in seqs:
         input_ids.append(seq.last_token)
         positions.append(len(seq))
         context_lens.append(len(seq))
-        slot_mapping.append(seq.block_table[-1] * block_size + seq.last_block_num_tokens - 1)
+        slot_mapping.append(seq.block_table[-1] * seq.block_size + seq.last_block_num_tokens - 1)
     set_context(False, slot_mapping=_to_device(slot_mapping, torch.int32, device),
                 context_lens=_to_device(context_lens, torch.int32, device),
                 block_tables=prepare_block_tables(seqs, device))

@@ -11,16 +11,19 @@ What differs from the reference, by design for this hardware:
   which makes every padding row append to slot 0; here padding rows carry length 0 and get slot -1.
 * The metadata kernel is the first node of the captured graph, so a replay needs nothing from the
   host but that one copy.
+* The model class comes from the configuration (``registry``) and says what it keeps between steps
+  (``cache_layout``).  A model with ``mixed_steps`` runs batches of portions (``run_portions``): single decoded
+  tokens beside parts of prompts; a batch of decoded tokens alone takes the same captured graphs.
 """
 from __future__ import annotations
 
 import torch
 
-from . import kv_runner, ops
+from . import kv_runner, ops, step_plan
 from .config import Config
 from .context import reset_context, set_context
 from .layers import Sampler
-from .qwen3 import QwenForCausalLM, init_random_weights
+from .registry import model_class
 from .sampling_params import SamplingParams
 from .sequence import Sequence
 
@@ -35,8 +38,12 @@ class ModelRunner:
         self.device = torch.device(device)
         torch.cuda.set_device(self.device)
 
-        self.model = QwenForCausalLM(hf_config).to(device=self.device, dtype=hf_config.torch_dtype)
+        self.model = model_class(hf_config).build(hf_config, self.device)
+        self.mixed = self.model.mixed_steps
+        # a token's position is its index; only the reference's decode convention adds to it
+        self.position_offset = 0 if self.mixed else config.decode_position_offset
         self.load_weights()
+        self.model.finish_loading(config.max_model_len)
         self.sampler = Sampler()
         self.graphs: dict = {}
         self.graph_bs: list[int] = []
@@ -53,7 +60,7 @@ class ModelRunner:
         if self.config.model and has_checkpoint(self.config.model):
             load_model(self.model, self.config.model)
         else:
-            init_random_weights(self.model, self.config.seed)
+            self.model.init_random_weights(self.config.seed)
 
     def warmup_model(self):
         """One prefill of the largest batch the scheduler may form, so that the peak of everything
@@ -62,52 +69,68 @@ class ModelRunner:
         torch.cuda.reset_peak_memory_stats(self.device)
         max_tokens, max_len = self.config.max_num_batched_tokens, self.config.max_model_len
         num_seqs = max(1, min(max_tokens // max_len, self.config.max_num_seqs))
-        seqs = [Sequence([0] * max_len, SamplingParams(temperature=0.7, max_tokens=512)) for _ in range(num_seqs)]
-        self.run(seqs, True)
+        seqs = [Sequence([0] * max_len, SamplingParams(temperature=0.7, max_tokens=512), self.block_size)
+                for _ in range(num_seqs)]
+        if not self.mixed:
+            self.run(seqs, True)
+        elif self.config.num_kvcache_blocks <= 0:      # a given pool size needs no measurement
+            self._warmup_portions(seqs)
         torch.cuda.empty_cache()
         # what a decode step needs beyond the model is allocated now, before the pool is sized from what
         # is left: the split-KV workspace for the largest batch and the split-K GEMM's partial sums
-        hf = self.config.hf_config
-        ops.decode_workspace(self.device, min(self.config.max_num_seqs, 512), hf.num_attention_heads,
-                             hf.num_key_value_heads, hf.head_dim)
-        ops._gemm_workspace(self.device, 64 << 20)
+        self.model.prepare_decode(self.device, min(self.config.max_num_seqs, 512))
+
+    def _warmup_portions(self, seqs: list[Sequence]):
+        """The warm-up pass of a model that cannot run without its cache: on a pool of just these sequences."""
+        per_seq = -(-len(seqs[0]) // self.block_size)
+        for i, seq in enumerate(seqs):
+            seq.block_table = list(range(i * per_seq, (i + 1) * per_seq))
+            seq.state_slot = i
+        self.num_slots, self.num_blocks = len(seqs), len(seqs) * per_seq
+        self.max_num_blocks = per_seq
+        self.model.bind_cache(self.model.cache_layout(self.block_size).allocate(self.num_blocks, self.num_slots, self.device))
+        self.run_portions([(seq, len(seq)) for seq in seqs])
+        torch.cuda.synchronize(self.device)
+        self.model.bind_cache([None] * len(self.model.caches))
 
     def allocate_kv_cache(self):
-        config, hf = self.config, self.config.hf_config
+        config = self.config
+        layout = self.model.cache_layout(self.block_size)
+        self.num_slots = config.max_num_seqs if layout.slot_bytes else 0
         if config.num_kvcache_blocks <= 0:
             free, total = torch.cuda.mem_get_info(self.device)
             stats = torch.cuda.memory_stats(self.device)
-            block_bytes = kv_runner.kv_block_bytes(hf.num_hidden_layers, self.block_size, hf.num_key_value_heads,
-                                                   hf.head_dim, hf.torch_dtype.itemsize)
             config.num_kvcache_blocks = kv_runner.num_kvcache_blocks(
-                total, total - free, stats["allocated_bytes.all.peak"], stats["allocated_bytes.all.current"],
-                config.gpu_memory_utilization, block_bytes)
+                total, total - free + self.num_slots * layout.slot_bytes, stats["allocated_bytes.all.peak"],
+                stats["allocated_bytes.all.current"], config.gpu_memory_utilization, max(layout.block_bytes, 1))
+            if layout.block_bytes == 0:      # recurrent layers only: blocks are bookkeeping
+                config.num_kvcache_blocks = -(-config.max_model_len // self.block_size) * config.max_num_seqs
         assert config.num_kvcache_blocks > 0
-        self.kv_cache = kv_runner.allocate_kv_cache(config.num_kvcache_blocks, hf.num_hidden_layers, self.block_size,
-                                                    hf.num_key_value_heads, hf.head_dim, self.device, hf.torch_dtype)
-        assert kv_runner.bind_kv_cache(self.model, self.kv_cache) == hf.num_hidden_layers
+        self.num_blocks = config.num_kvcache_blocks
+        self.kv_cache = layout.allocate(self.num_blocks, self.num_slots, self.device)
+        self.model.bind_cache(self.kv_cache)
 
     def _alloc_step_buffers(self):
         """Static buffers of a decode step.  The staging buffer is one int32 array
-        ``[input_ids | seq_lens | block_table]`` that exists twice, pinned on the host and on the device."""
+        ``[input_ids | seq_lens | state_slots | block_table]`` that exists twice, pinned on the host and on the device."""
         config = self.config
         self.max_bs = min(config.max_num_seqs, 512)
         self.max_num_blocks = (config.max_model_len + self.block_size - 1) // self.block_size
         n, m = self.max_bs, self.max_num_blocks
-        self.stage_host = torch.zeros(n * (2 + m), dtype=torch.int32, pin_memory=True)
-        self.stage_dev = torch.zeros(n * (2 + m), dtype=torch.int32, device=self.device)
+        self.stage_host = torch.zeros(n * (3 + m), dtype=torch.int32, pin_memory=True)
+        self.stage_dev = torch.zeros(n * (3 + m), dtype=torch.int32, device=self.device)
         host = self.stage_host.numpy()
-        self.h_input_ids, self.h_seq_lens = host[:n], host[n:2 * n]
-        self.h_block_tables = host[2 * n:].reshape(n, m)
+        self.h_input_ids, self.h_seq_lens, self.h_state_slots = host[:n], host[n:2 * n], host[2 * n:3 * n]
+        self.h_block_tables = host[3 * n:].reshape(n, m)
         self._staged_tables = [None] * n        # what each host row of the block table currently holds
         self.d_input_ids, self.d_seq_lens = self.stage_dev[:n], self.stage_dev[n:2 * n]
-        self.d_block_tables = self.stage_dev[2 * n:].view(n, m)
+        self.d_state_slots = self.stage_dev[2 * n:3 * n]
+        self.d_block_tables = self.stage_dev[3 * n:].view(n, m)
         self.d_positions = torch.zeros(n, dtype=torch.int64, device=self.device)
         self.d_slot_mapping = torch.full((n,), -1, dtype=torch.int32, device=self.device)
         self.d_context_lens = torch.zeros(n, dtype=torch.int32, device=self.device)
-        # split-KV workspace of the decode kernel for the largest batch, so that no step allocates
-        hf = config.hf_config
-        ops.decode_workspace(self.device, n, hf.num_attention_heads, hf.num_key_value_heads, hf.head_dim)
+        # workspaces of the decode kernels for the largest batch, so that no step allocates
+        self.model.prepare_decode(self.device, n)
 
     # ------------------------------------------------------------------ per-step metadata
     def prepare_block_tables(self, seqs: list[Sequence]):
@@ -124,8 +147,17 @@ class ModelRunner:
             raise RuntimeError(f"decode batch of {bs} exceeds max_num_seqs={self.max_bs}")
         run_bs = bs if self.enforce_eager or not self.graph_bs else next(x for x in self.graph_bs if x >= bs)
         ids, lens, tables = self.h_input_ids, self.h_seq_lens, self.h_block_tables
-        ids[:bs] = [seq.last_token for seq in seqs]
-        lens[:bs] = [len(seq) for seq in seqs]
+        if self.mixed:               # the step's token is the first one not computed yet
+            ids[:bs] = [seq.token_ids[seq.num_computed_tokens] for seq in seqs]
+            lens[:bs] = [seq.num_computed_tokens + 1 for seq in seqs]
+            slots = [seq.state_slot for seq in seqs]
+            if self.num_slots and not all(0 <= s < self.num_slots for s in slots):
+                raise RuntimeError("a sequence's state slot lies outside the pool")
+            self.h_state_slots[:bs] = slots
+            self.h_state_slots[bs:run_bs] = -1
+        else:
+            ids[:bs] = [seq.last_token for seq in seqs]
+            lens[:bs] = [len(seq) for seq in seqs]
         staged = self._staged_tables
         for i, seq in enumerate(seqs):
             bt = tuple(seq.block_table)
@@ -147,10 +179,15 @@ class ModelRunner:
         slot_mapping = self.d_slot_mapping[:run_bs]
         context_lens = self.d_context_lens[:run_bs]
         block_tables = self.d_block_tables[:run_bs]
-        ops.decode_metadata(self.d_seq_lens[:run_bs], block_tables, self.block_size,
-                            self.config.decode_position_offset, positions, slot_mapping, context_lens)
-        set_context(False, slot_mapping=slot_mapping, context_lens=context_lens, block_tables=block_tables)
-        return self.model(self.d_input_ids[:run_bs], positions)
+        ops.decode_metadata(self.d_seq_lens[:run_bs], block_tables, self.block_size, self.position_offset, positions,
+                            slot_mapping, context_lens)
+        input_ids, plan = self.d_input_ids[:run_bs], None
+        if self.mixed:
+            input_ids = input_ids.long()
+            plan = step_plan.StepPlan(input_ids, positions, slot_mapping, block_tables, row_ctx=context_lens,
+                                      state_slots=self.d_state_slots[:run_bs], decode_rows=run_bs, dense_row=run_bs)
+        set_context(False, slot_mapping=slot_mapping, context_lens=context_lens, block_tables=block_tables, step=plan)
+        return self.model(input_ids, positions)
 
     def prepare_sample(self, seqs: list[Sequence]):
         temps = [seq.temperature for seq in seqs]
@@ -185,6 +222,36 @@ class ModelRunner:
         reset_context()
         return token_ids
 
+    # ------------------------------------------------------------------ steps of portions
+    @torch.inference_mode()
+    def portion_logits(self, portions, wanted: list[list[int]]) -> torch.Tensor:
+        """One step over ``portions`` ((sequence, count) pairs).  Returns the logits at ``wanted[i]`` (places inside
+        portion i), in that order, [number wanted, vocab]."""
+        if all(count == 1 for _, count in portions) and hasattr(self, "stage_host"):
+            hidden = self.decode_hidden(self.prepare_decode([seq for seq, _ in portions]))
+            first = range(len(portions))
+        else:
+            plan, first = step_plan.build(portions, self.block_size, self.max_num_blocks, self.num_slots, self.num_blocks,
+                                          self.device)
+            set_context(True, step=plan)
+            hidden = self.model(plan.input_ids, plan.positions)
+        rows = [first[i] + k for i, places in enumerate(wanted) for k in places]
+        if not rows:
+            return hidden[:0]
+        index = torch.tensor(rows, dtype=torch.int64, pin_memory=True).to(self.device, non_blocking=True)
+        return self.model.compute_logits(hidden[index])
+
+    def run_portions(self, portions) -> list[int]:
+        """One step; samples the next token of every portion with which its sequence's known tokens end."""
+        ends = [seq.num_computed_tokens + count == len(seq) for seq, count in portions]
+        logits = self.portion_logits(portions, [[count - 1] if end else [] for (_, count), end in zip(portions, ends)])
+        reset_context()
+        if not any(ends):
+            return []
+        temperatures, all_greedy = self.prepare_sample([seq for (seq, _), end in zip(portions, ends) if end])
+        with torch.inference_mode():
+            return self.sampler(logits, temperatures, all_greedy).tolist()
+
     # ------------------------------------------------------------------ HIP graph capture
     @torch.inference_mode()
     def capture_cudagraph(self):
@@ -195,6 +262,7 @@ class ModelRunner:
                                      dtype=self.config.hf_config.torch_dtype, device=self.device)
         self.h_seq_lens[:] = 0
         self.h_input_ids[:] = 0
+        self.h_state_slots[:] = -1
         self.stage_dev.copy_(self.stage_host)
         for bs in reversed(self.graph_bs):
             graph = torch.cuda.CUDAGraph()

@@ -9,8 +9,9 @@ from __future__ import annotations
 import torch
 from torch import nn
 
-from . import ops
+from . import kv_runner, ops
 from .attention import Attention
+from .cache import PagedKVLayout
 from .context import get_context
 from .layers import MLP, Embedding, Linear, LMHead, QKVLinear, RMSNorm, cos_sin_table
 
@@ -119,6 +120,7 @@ class QwenModel(nn.Module):
 
 
 class QwenForCausalLM(nn.Module):
+    mixed_steps = False           # a step is prefill or decode
     packed_modules_mapping = {
         "q_proj": ("qkv_proj", "q"),
         "k_proj": ("qkv_proj", "k"),
@@ -129,10 +131,34 @@ class QwenForCausalLM(nn.Module):
 
     def __init__(self, config):
         super().__init__()
+        self.config = config
         self.model = QwenModel(config)
         self.lm_head = LMHead(config.vocab_size, config.hidden_size)
         if config.tie_word_embeddings:
             self.lm_head.weight = self.model.embed_tokens.weight
+
+    @classmethod
+    def build(cls, config, device) -> "QwenForCausalLM":
+        return cls(config).to(device=device, dtype=config.torch_dtype)
+
+    def init_random_weights(self, seed: int = 0) -> None:
+        init_random_weights(self, seed)
+
+    def finish_loading(self, max_position: int) -> None:
+        pass
+
+    def cache_layout(self, block_size: int) -> PagedKVLayout:
+        c = self.config
+        return PagedKVLayout(c.num_hidden_layers, block_size, c.num_key_value_heads, c.head_dim, c.torch_dtype)
+
+    def bind_cache(self, kv_cache: torch.Tensor) -> None:
+        assert kv_runner.bind_kv_cache(self, kv_cache) == self.config.num_hidden_layers
+
+    def prepare_decode(self, device, max_batch: int) -> None:
+        """Workspaces of a decode step: split-KV attention for the largest batch, split-K products."""
+        c = self.config
+        ops.decode_workspace(device, max_batch, c.num_attention_heads, c.num_key_value_heads, c.head_dim)
+        ops._gemm_workspace(device, 64 << 20)
 
     def forward(self, input_ids: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
         return self.model(input_ids, positions)

@@ -1,0 +1,13 @@
+"""Which model class serves which configuration."""
+from __future__ import annotations
+
+from .config import MerilornConfig, ModelConfig
+from .merilorn import MerilornForCausalLM
+from .qwen3 import QwenForCausalLM
+
+MODELS = {ModelConfig: QwenForCausalLM, MerilornConfig: MerilornForCausalLM}
+
+
+def model_class(config):
+    """The model class of a configuration (any object with Qwen3's attributes counts as Qwen3's)."""
+    return MODELS.get(type(config), QwenForCausalLM)
