@@ -122,6 +122,7 @@ class ModelRunner:
         host = self.stage_host.numpy()
         self.h_input_ids, self.h_seq_lens, self.h_state_slots = host[:n], host[n:2 * n], host[2 * n:3 * n]
         self.h_block_tables = host[3 * n:].reshape(n, m)
+        self._staged = torch.cuda.Event()       # the last copy of the staging buffer has left the host
         self._staged_tables = [None] * n        # what each host row of the block table currently holds
         self.d_input_ids, self.d_seq_lens = self.stage_dev[:n], self.stage_dev[n:2 * n]
         self.d_state_slots = self.stage_dev[2 * n:3 * n]
@@ -146,6 +147,7 @@ class ModelRunner:
         if bs > self.max_bs:
             raise RuntimeError(f"decode batch of {bs} exceeds max_num_seqs={self.max_bs}")
         run_bs = bs if self.enforce_eager or not self.graph_bs else next(x for x in self.graph_bs if x >= bs)
+        self._staged.synchronize()              # a step whose result nobody has waited for may still be queued
         ids, lens, tables = self.h_input_ids, self.h_seq_lens, self.h_block_tables
         if self.mixed:               # the step's token is the first one not computed yet
             ids[:bs] = [seq.token_ids[seq.num_computed_tokens] for seq in seqs]
@@ -170,6 +172,7 @@ class ModelRunner:
         ids[bs:run_bs] = 0
         lens[bs:run_bs] = 0           # padding rows: no append, no attention
         self.stage_dev.copy_(self.stage_host, non_blocking=True)
+        self._staged.record()
         return run_bs
 
     def _decode_forward(self, run_bs: int) -> torch.Tensor:
