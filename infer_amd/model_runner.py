@@ -96,7 +96,7 @@ class ModelRunner:
     def allocate_kv_cache(self):
         config = self.config
         layout = self.model.cache_layout(self.block_size)
-        self.num_slots = config.max_num_seqs if layout.slot_bytes else 0
+        self.num_slots = config.max_num_seqs      # also where no layer keeps a state: slots are handed out all the same
         if config.num_kvcache_blocks <= 0:
             free, total = torch.cuda.mem_get_info(self.device)
             stats = torch.cuda.memory_stats(self.device)
@@ -153,7 +153,7 @@ class ModelRunner:
             ids[:bs] = [seq.token_ids[seq.num_computed_tokens] for seq in seqs]
             lens[:bs] = [seq.num_computed_tokens + 1 for seq in seqs]
             slots = [seq.state_slot for seq in seqs]
-            if self.num_slots and not all(0 <= s < self.num_slots for s in slots):
+            if not all(0 <= s < self.num_slots for s in slots):
                 raise RuntimeError("a sequence's state slot lies outside the pool")
             self.h_state_slots[:bs] = slots
             self.h_state_slots[bs:run_bs] = -1

@@ -147,8 +147,9 @@ MIXERS = {"latent_attention": latent_attention, "channel_delta": channel_delta}
 
 
 # ------------------------------------------------------------------ the model
-def forward(config, weights, tokens):
-    """Logits [tokens, vocab] and the residual stream after every layer [layers, tokens, width]."""
+def forward(config, weights, tokens, cast=lambda a: a):
+    """Logits [tokens, vocab] and the residual stream after every layer [layers, tokens, width].  ``cast`` is applied to
+    what goes into and comes out of every sublayer: with a rounding function it shows what rounding alone does."""
     eps = config["norm"]["eps"]
     x = weights["embed"][np.asarray(tokens)] * config["embedding"]["scale"]
     stream = []
@@ -162,12 +163,12 @@ def forward(config, weights, tokens):
         def mlp(key):
             return weights[name + "mlp." + key]
 
-        y = MIXERS[layer["type"]](rms_norm(x, weights[name + "norm1"], eps), layer["mixer"], mix, eps)
-        x = x + rms_norm(y, weights[name + "norm1b"], eps)
+        y = MIXERS[layer["type"]](cast(rms_norm(x, weights[name + "norm1"], eps)), layer["mixer"], mix, eps)
+        x = x + rms_norm(cast(y), weights[name + "norm1b"], eps)
         if layer["mlp"] is not None:
             assert layer["mlp"]["kind"] == "dense"
-            y = dense_mlp(rms_norm(x, weights[name + "norm2"], eps), mlp)
-            x = x + rms_norm(y, weights[name + "norm2b"], eps)
+            y = dense_mlp(cast(rms_norm(x, weights[name + "norm2"], eps)), mlp)
+            x = x + rms_norm(cast(y), weights[name + "norm2b"], eps)
         stream.append(x)
-    logits = rms_norm(x, weights["final.norm"], eps) @ weights["head"].T
+    logits = cast(rms_norm(x, weights["final.norm"], eps)) @ weights["head"].T
     return logits, np.stack(stream)
