@@ -228,6 +228,188 @@ def run_e2e(args):
         sys.exit(4)
 
 
+# ------------------------------------------------------------------------------------------ hybrid models
+BF16_PEAK_TFLOPS, F32_MFMA_PEAK_TFLOPS = 2500.0, 157.3
+# width, feed-forward, attention heads, layers: layers of the size of Qwen3-0.6B's and Qwen3-8B's
+HYBRID_SIZES = {"0.6b": (1024, 3072, 16, 16), "8b": (4096, 12288, 32, 12)}
+
+
+def hybrid_config(size):
+    """Merilorn of a published model's width: three delta-rule layers to one of latent attention, all with a
+    feed-forward; latent of 512 + 64, heads of 128."""
+    from infer_amd.config import LayerSpec, MerilornConfig
+    width, ff, heads, layers = HYBRID_SIZES[size]
+    latent = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
+              "rot": {"base": 1e6, "dims": 64, "scaling": {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+    delta = {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4, "decay_rank": 128, "gate_rank": 128}
+    specs = [LayerSpec("latent_attention", latent, ff, i) if i % 4 == 3 else LayerSpec("channel_delta", delta, ff, i)
+             for i in range(layers)]
+    return MerilornConfig(vocab_size=151936, hidden_size=width, layers=specs, embedding_scale=width ** 0.5)
+
+
+def hybrid_engine_point(size, model, batch, prompt, new):
+    """Prefill and decode throughput of the engine on ``batch`` prompts of ``prompt`` random tokens."""
+    import numpy as np
+    from infer_amd import config as C
+    from infer_amd.llm_engine import LLMEngine
+    from infer_amd.sampling_params import SamplingParams
+    width, ff, heads, layers = HYBRID_SIZES[size]
+    hf = hybrid_config(size) if model == "merilorn" else C.ModelConfig(
+        hidden_size=width, intermediate_size=ff, num_hidden_layers=layers, num_attention_heads=heads, num_key_value_heads=8)
+    blocks = batch * (-(-(prompt + new) // 256) + 1)
+    engine = LLMEngine(hf_config=hf, max_num_seqs=max(batch, 16), max_model_len=prompt + new + 1,
+                       max_num_batched_tokens=16384, num_kvcache_blocks=blocks, seed=0)
+    rng = np.random.default_rng(0)
+    params = SamplingParams(temperature=0.0, max_tokens=new, ignore_eos=True)
+    for i in range(2):                      # the first pass warms up
+        for key in engine.stats:
+            engine.stats[key] = 0
+        prompts = [[int(t) for t in rng.integers(0, hf.vocab_size, size=prompt)] for _ in range(batch)]
+        outs = engine.generate(prompts, params)
+        assert all(len(o["token_ids"]) == new for o in outs)
+    st = engine.stats
+    point = {"model": model, "layers_like": size, "layers": layers, "batch": batch, "prompt": prompt, "new_tokens": new,
+             "prefill_tokens_per_s": round(st["prefill_tokens"] / st["prefill_s"], 1),
+             "decode_tokens_per_s": round(st["decode_tokens"] / st["decode_s"], 1),
+             "decode_ms_per_step": round(1e3 * st["decode_s"] / st["decode_steps"], 3)}
+    del engine
+    torch.cuda.empty_cache()
+    return point
+
+
+def hybrid_kernels(heads=32, width=4096, ff=12288):
+    """Every kernel of the design at the sizes of an 8B model's layers, with what bounds it, beside the like kernel of
+    Qwen3 at the same sizes."""
+    from infer_amd import hybrid_ops as ho, ops, workloads
+    from infer_amd.layers import yarn_rotary_table
+    from infer_amd.step_plan import CHUNK
+    dev, bf = torch.device("cuda:0"), torch.bfloat16
+    out = {}
+
+    def rnd(*shape, dtype=bf):
+        return torch.randn(*shape, dtype=dtype, device=dev)
+
+    def hbm(name, nbytes, fn, note=""):
+        ms = gpu_time_ms_median(fn, 20, 5)
+        out[name] = {"us": round(ms * 1e3, 2), "bound": "hbm", "GBps": round(nbytes / ms / 1e6, 1),
+                     "frac": round(nbytes / ms / 1e6 / HBM_PEAK_GBS, 4), **({"note": note} if note else {})}
+
+    def mfma(name, flops, peak, fn, note=""):
+        ms = gpu_time_ms_median(fn, 20, 5)
+        out[name] = {"us": round(ms * 1e3, 2), "bound": "mfma", "TFLOPs": round(flops / ms / 1e9, 1),
+                     "frac": round(flops / ms / 1e9 / peak, 4), **({"note": note} if note else {})}
+
+    # ---- decode attention, batch 64 x ctx 4096
+    b, ctx, bs, row, rank, dim, rot, vdim = 64, 4096, 256, 576, 512, 128, 64, 128
+    nblk = b * ctx // bs
+    cache = rnd(nblk, bs, row)
+    tables = torch.randperm(nblk, device=dev).to(torch.int32).view(b, -1)
+    lens = torch.full((b,), ctx, dtype=torch.int32, device=dev)
+    for h in (16, heads, 128):
+        qx = rnd(b, h, row)
+        hbm(f"latent_attention decode, {h} heads", b * ctx * row * 2, lambda: ho.latent_attention(qx, cache, tables, lens, 0.07, rank))
+    wl = workloads.make_decode_workload("b64-ctx4096", [ctx] * b, heads, 8, seed=0, q_scale=128 ** -0.5, device=dev, device_fill=True)
+    o = torch.empty((b, heads, 128), dtype=bf, device=dev)
+    hbm("qwen3: paged decode attention", wl.decode_bytes,
+        lambda: ops.paged_attn_decode(wl.q, wl.k_cache, wl.v_cache, wl.block_table, wl.context_lens, wl.scale, o))
+    del wl
+
+    # ---- prefill attention, 8 prompts of 2048
+    n, sq = 8, 2048
+    cu = torch.arange(0, n + 1, dtype=torch.int32, device=dev) * sq
+    rows = rnd(n * sq, row)
+    q, kv, gate = rnd(n * sq, heads * (dim + rot)), rnd(n * sq, heads * (dim + vdim)), rnd(n * sq, heads)
+    at = torch.empty((n * sq, heads * vdim), dtype=bf, device=dev)
+    pairs = n * sq * (sq + 1) // 2
+    mfma("latent_prefill, 8 x 2048", 2 * heads * (dim + rot + vdim) * pairs, BF16_PEAK_TFLOPS,
+         lambda: ho.latent_prefill(q, kv[:, :heads * dim], rows[:, rank:], kv[:, heads * dim:], gate, at, cu, cu, sq, heads, dim, rot, vdim, 0.07))
+    q3, k3 = rnd(n * sq, heads, 128), rnd(n * sq, 8, 128)
+    mfma("qwen3: prefill attention, 8 x 2048", 4 * heads * 128 * pairs, BF16_PEAK_TFLOPS,
+         lambda: ops.flash_attn_varlen_func(q3, k3, k3, max_seqlen_q=sq, cu_seqlens_q=cu, max_seqlen_k=sq, cu_seqlens_k=cu))
+    seqs = torch.arange(n, dtype=torch.int32, device=dev)
+    hbm("latent_gather, 16384 rows", 2 * n * sq * row * 2, lambda: ho.latent_gather(cache, tables[:n], seqs, cu, n * sq, sq))
+    del q, kv, q3, k3
+
+    # ---- front end and per-head products
+    table = yarn_rotary_table(rot, 8192, 1e6, None, dev)
+    for t in (b, n * sq):
+        proj = rnd(t, heads * (dim + rot) + row + heads)
+        pos = torch.randint(0, 8192, (t,), device=dev)
+        slots = torch.randperm(nblk * bs, device=dev)[:t].to(torch.int32)
+        decode = t == b
+        qx = rnd(t if decode else 1, heads, row)
+        norm = torch.ones(rank, device=dev)
+        hbm(f"latent_front, {t} rows", t * 2 * (2 * heads * rot + 2 * row),
+            lambda: ho.latent_front(proj, heads, dim, rot, rot, heads * (dim + rot), rank, norm, 1e-6, table, pos, slots, cache, rank, qx, t if decode else 0))
+        qkv = rnd(t, (heads + 16) * 128)
+        qv, kk, vv = (x.view(t, -1, 128) for x in qkv.split([heads * 128, 8 * 128, 8 * 128], dim=-1))
+        kc, w128, cs = rnd(nblk, bs, 8, 128), torch.ones(128, dtype=bf, device=dev), rnd(8192, 128)
+        hbm(f"qwen3: norm + rotary + append, {t} rows", t * (2 * heads * 128 * 2 + 4 * 8 * 128 * 2),
+            lambda: ops.qk_norm_rope_store_kvcache(qv, kk, vv, pos, w128, w128, 1e-6, cs, kc, kc, slots, write_key=False))
+        del kc, qkv, proj
+    x, w = rnd(b, heads, dim), rnd(heads, rank, dim)
+    y = torch.empty((b, heads, rank), dtype=bf, device=dev)
+    hbm("head_matmul W_uk^T q, 64 rows", 2 * (x.numel() + w.numel() + y.numel()), lambda: ho.head_matmul(x, w, y, rank, dim))
+    w2 = rnd(heads, vdim, rank)
+    hbm("head_matmul W_uv c (gated), 64 rows", 2 * (x.numel() + w2.numel() + y.numel()), lambda: ho.head_matmul(y, w2, x, vdim, rank, gate=gate[:b]))
+    wn = rnd(4096, 2048)
+    xs = rnd(b, 2048)
+    hbm("qwen3: split-K GEMM 64 x 4096 x 2048 (weights of the size of the above, x4)", 2 * wn.numel(), lambda: ops.skinny_linear(xs, wn))
+    del cache
+
+    # ---- delta rule
+    s = ho.DeltaShape(heads, heads, 128, 128, 4, 1e-6)
+    slots_n = 64
+    state = torch.zeros(slots_n, heads, 128, 128, device=dev)
+    ring = torch.zeros(slots_n, 4, s.channels, dtype=bf, device=dev)
+    wts = [torch.randn(s.channels, 4, device=dev) * .5, torch.zeros(heads, device=dev), torch.full((heads * 128,), -3.0, device=dev), torch.ones(128, device=dev)]
+    proj, dec, gt = rnd(b, s.channels + heads), rnd(b, heads * 128), rnd(b, heads * 128)
+    o2 = torch.empty((b, heads * 128), dtype=bf, device=dev)
+    pos = torch.full((b,), 77, dtype=torch.int64, device=dev)
+    sl = torch.arange(b, dtype=torch.int32, device=dev)
+    hbm("delta_step, 64 sequences", 2 * state.numel() * 4 + 2 * (proj.numel() + dec.numel() + gt.numel() + 5 * s.channels // 3 * b),
+        lambda: ho.delta_step(s, proj, s.channels, dec, gt, *wts, ring, state, sl, pos, o2))
+    for n, sq in ((1, 2048), (8, 2048)):
+        t = n * sq
+        proj, dec, gt = rnd(t, s.channels + heads), rnd(t, heads * 128), rnd(t, heads * 128)
+        o3 = torch.empty((t, heads * 128), dtype=bf, device=dev)
+        per = sq // CHUNK
+        portions = torch.tensor([(i * per, per, i, 0) for i in range(n)], dtype=torch.int32, device=dev)
+        chunks = torch.tensor([(i * sq + r, CHUNK, r, 0, i, 0) for i in range(n) for r in range(0, sq, CHUNK)], dtype=torch.int32, device=dev)
+        rs = torch.tensor([(i, sq - 1 - r) for i in range(n) for r in range(sq)], dtype=torch.int32, device=dev)
+        pos = torch.arange(sq, device=dev).repeat(n)
+        # three products with the [128, 128] state and two inside the chunk, per token and head
+        mfma(f"delta_chunks, {n} x {sq}", t * heads * (6 * 128 * 128 + 4 * 16 * 128), F32_MFMA_PEAK_TFLOPS,
+             lambda: ho.delta_chunks(s, proj, s.channels, dec, gt, *wts, ring, state, portions, chunks, rs, pos, 0, o3),
+             "all three launches, against the float32 matrix peak")
+    del proj, dec, gt
+
+    # ---- residual stream and activation
+    for t in (b, 16384):
+        x32, y = rnd(t, width, dtype=torch.float32), rnd(t, width)
+        w32, wb = torch.ones(width, device=dev), torch.ones(width, dtype=bf, device=dev)
+        hbm(f"residual_norm, {t} rows", t * width * (4 + 4 + 2 + 2), lambda: ho.residual_norm(x32, 1e-6, y=y, w_post=w32, w_pre=w32))
+        res = rnd(t, width)
+        hbm(f"qwen3: rms_norm with residual, {t} rows", t * width * 8, lambda: ops.rms_norm(y, wb, 1e-6, res))
+        gu = rnd(t, 2 * ff)
+        act = torch.empty((t, ff), dtype=bf, device=dev)
+        hbm(f"gelu_tanh_and_mul, {t} rows", t * ff * 6, lambda: ho.gelu_tanh_and_mul(gu))
+        hbm(f"qwen3: silu_and_mul, {t} rows", t * ff * 6, lambda: ops.silu_and_mul(act, gu))
+    return out
+
+
+def run_hybrid(args):
+    """Merilorn beside Qwen3 at equal width, feed-forward, heads and number of layers: the engine's prefill and
+    decode throughput, then the kernels one by one."""
+    points = []
+    if not args.hybrid_kernels_only:
+        for size, batch, prompt, new in (("0.6b", 64, 1024, 64), ("8b", 64, 1024, 64), ("8b", 16, 4096, 64)):
+            for model in ("merilorn", "qwen3"):
+                points.append(hybrid_engine_point(size, model, batch, prompt, new))
+                print(points[-1], file=sys.stderr, flush=True)
+    print(json.dumps({"hybrid_engine": points, "hybrid_kernels": hybrid_kernels()}))
+
+
 # ------------------------------------------------------------------------------------------ decode curve
 def decode_point(name, wl, copies, iters, splits=0, uniform_len=None):
     """Decode op (split + merge) of one workload, timed as replays of a HIP graph that holds ``copies``
@@ -321,6 +503,9 @@ def main():
                          "a prefill-sized append (x3), the fused norm + RoPE + append (x3) and the prefill "
                          "attention (x3) of the same step")
     ap.add_argument("--decode-curve", action="store_true", help="only the decode curve, printed as JSON")
+    ap.add_argument("--hybrid", action="store_true",
+                    help="Merilorn beside Qwen3 at equal sizes: engine throughput and every kernel, printed as JSON")
+    ap.add_argument("--hybrid-kernels-only", action="store_true", help="with --hybrid: the kernels alone")
     ap.add_argument("--e2e", action="store_true",
                     help="end-to-end decode through the engine (random-init Qwen3, HIP-graph decode) instead "
                          "of the kernel benchmark")
@@ -342,6 +527,9 @@ def main():
 
     if args.e2e:
         run_e2e(args)
+        return
+    if args.hybrid:
+        run_hybrid(args)
         return
     from infer_amd import ops, workloads
     dev = torch.device("cuda:0")
