@@ -218,133 +218,257 @@ struct PortionDesc { int32_t chunk0, chunks, slot, pos0; };
 //   V   [vdim_pad / 16][256]  element (i, v):  T (beta V)
 __host__ __device__ inline int64_t record_floats(int dim_pad, int vdim_pad) { return 48 * (int64_t)dim_pad + 256 + dim_pad + 16 * (int64_t)vdim_pad; }
 
+// The convolution of four channels over tokens t0 .. t0 + 7 of a chunk, for four taps, the window in registers.
+// c: first channel, dst: LDS row of token t0, column of the channel.
 template <class T>
+__device__ __forceinline__ void conv4_silu(const DeltaArgs<T>& a, const ChunkDesc& cd, int c, int t0, float* dst, int pitch) {
+    float x[11][4], w[4][4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) load_elems<4>(a.conv + 4 * (c + e), w[e]);
+#pragma unroll
+    for (int j = 0; j < 11; ++j) {
+        const int t = t0 + j - 3, p = cd.pos0 + t;
+        // positions before the portion are in the ring; those before the sequence or behind the chunk's tokens are zero
+        const bool in = p >= 0 && t < cd.count;
+        const T* src = p >= cd.first_pos || !in ? a.proj + (int64_t)(cd.row0 + (in ? t : 0)) * a.proj_stride + c
+                                                : a.ring + ((int64_t)cd.slot * 4 + (p & 3)) * a.channels + c;
+        load_elems<4>(src, x[j]);
+        if (!in)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[j][e] = 0.f;
+    }
+#pragma unroll
+    for (int t = 0; t < 8; ++t) {
+        float y[4];
+        const bool in = t0 + t < cd.count;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            y[e] = 0.f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) y[e] += w[e][j] * x[t + j][e];
+            y[e] = in ? silu_f(y[e]) : 0.f;
+        }
+        store_elems<4>(dst + t * pitch, y);
+    }
+}
+
+// softplus in units of log2: log2(1 + e^z)
+__device__ __forceinline__ float softplus_log2(float z) {
+    const float e = __builtin_amdgcn_exp2f(-fabsf(z) * kLog2e);
+    const float l = e < 0.02f ? e * (1.f - e * (0.5f - e * (0.33333333f - 0.25f * e))) * kLog2e : __builtin_amdgcn_logf(1.f + e);
+    return fmaxf(z, 0.f) * kLog2e + l;
+}
+
+// Decay of a whole chunk, in log2 units, up to which e^{G_i - G_j} may be split into two factors.
+constexpr float kSplitRange = 48.f;
+
+// VEC: four channels at a time, four taps; otherwise any size, one element at a time.
+template <class T, bool VEC>
 __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs<T> a, const ChunkDesc* chunks, float* records) {
     extern __shared__ __attribute__((aligned(16))) float sh[];
-    const int tid = threadIdx.x, h = blockIdx.y;
+    const int tid = threadIdx.x, h = blockIdx.y, lane = tid & 63, wave = tid >> 6;
     const ChunkDesc c = chunks[blockIdx.x];
     const int dp = a.dim_pad, pk = dp + 4, pv = a.vdim_pad + 4;
-    float* qs = sh;                    // [16][pk]
-    float* ks = qs + kC * pk;
-    float* gs = ks + kC * pk;          // running log2 decay
+    float* qs = sh;                    // [16][pk] q, then e^G q
+    float* ks = qs + kC * pk;          // [16][pk] k, then e^G k
+    float* gs = ks + kC * pk;          // [16][pk] running log2 decay G, then e^{G_last - G} k
     float* vs = gs + kC * pk;          // [16][pv]
-    float* lm = vs + kC * pv;          // [16][20] beta * A below the diagonal, then T * beta
-    float* inv = lm + kC * 20;         // [2][16] 1 / length of k and q
+    float* pp = vs + kC * pv;          // [4][2][256] products of the token pairs, one part per wavefront
+    float* lt = pp + 2048;             // [16][20] column s: beta * A of the tokens behind s
+    float* tb = lt + kC * 20;          // [16][20] T * beta
+    float* gl = tb + kC * 20;          // [dp] G_last
+    float* inv = gl + dp;              // [2][16] 1 / length of k and q
     float* bs = inv + 32;              // [16] beta
     const int group = a.heads / a.kv_heads, kvh = h / group;
+    const int cq = kvh * a.dim, ck = (a.kv_heads + kvh) * a.dim, cv = 2 * a.kv_heads * a.dim + h * a.vdim;
     float* rec = records + ((int64_t)blockIdx.x * a.heads + h) * record_floats(dp, a.vdim_pad);
-    auto row_of = [&](int64_t p) { return (int64_t)c.row0 + (p - c.pos0); };
-
-    for (int i = tid; i < kC * dp; i += 256) {
-        const int t = i / dp, d = i - t * dp;
-        float q = 0.f, k = 0.f;
-        if (t < c.count && d < a.dim) {
-            q = conv_silu(a, kvh * a.dim + d, c.pos0 + t, c.first_pos, c.slot, row_of);
-            k = conv_silu(a, (a.kv_heads + kvh) * a.dim + d, c.pos0 + t, c.first_pos, c.slot, row_of);
-        }
-        qs[t * pk + d] = q;
-        ks[t * pk + d] = k;
-    }
-    for (int i = tid; i < kC * a.vdim_pad; i += 256) {
-        const int t = i / a.vdim_pad, v = i - t * a.vdim_pad;
-        vs[t * pv + v] = t < c.count && v < a.vdim
-            ? conv_silu(a, 2 * a.kv_heads * a.dim + h * a.vdim + v, c.pos0 + t, c.first_pos, c.slot, row_of) : 0.f;
-    }
     const float rate = expf(a.a_log[h]);
-    for (int d = tid; d < dp; d += 256) {
-        float sum = 0.f;
-        for (int t = 0; t < kC; ++t) {
-            if (t < c.count && d < a.dim) sum += log2_decay(a, c.row0 + t, h, d, rate);
-            gs[t * pk + d] = sum;
+
+    if constexpr (VEC) {
+        const int nd = a.dim / 4, nv = a.vdim / 4, n = 2 * nd + nv;
+        for (int i = tid; i < 2 * n; i += 256) {
+            const int half = i >= n, j = i - half * n, t0 = 8 * half;
+            if (j < nd) conv4_silu(a, c, cq + 4 * j, t0, qs + t0 * pk + 4 * j, pk);
+            else if (j < 2 * nd) conv4_silu(a, c, ck + 4 * (j - nd), t0, ks + t0 * pk + 4 * (j - nd), pk);
+            else conv4_silu(a, c, cv + 4 * (j - 2 * nd), t0, vs + t0 * pv + 4 * (j - 2 * nd), pv);
+        }
+        for (int i = tid; i < kC * nd; i += 256) {
+            const int t = i / nd, d = 4 * (i - t * nd);
+            float x[4] = {0.f, 0.f, 0.f, 0.f};
+            if (t < c.count) {
+                float dt[4];
+                load_elems<4>(a.decay + (int64_t)(c.row0 + t) * a.decay_stride + h * a.dim + d, x);
+                load_elems<4>(a.dt_bias + h * a.dim + d, dt);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[e] = -rate * softplus_log2(x[e] + dt[e]);
+            }
+            store_elems<4>(gs + t * pk + d, x);
+        }
+        for (int i = tid; i < kC * (dp - a.dim); i += 256) {
+            const int t = i / (dp - a.dim), d = a.dim + i % (dp - a.dim);
+            qs[t * pk + d] = ks[t * pk + d] = gs[t * pk + d] = 0.f;
+        }
+        for (int i = tid; i < kC * (a.vdim_pad - a.vdim); i += 256) {
+            const int t = i / (a.vdim_pad - a.vdim), v = a.vdim + i % (a.vdim_pad - a.vdim);
+            vs[t * pv + v] = 0.f;
+        }
+    } else {
+        auto row_of = [&](int64_t p) { return (int64_t)c.row0 + (p - c.pos0); };
+        for (int i = tid; i < kC * dp; i += 256) {
+            const int t = i / dp, d = i - t * dp;
+            float q = 0.f, k = 0.f, g = 0.f;
+            if (t < c.count && d < a.dim) {
+                q = conv_silu(a, cq + d, c.pos0 + t, c.first_pos, c.slot, row_of);
+                k = conv_silu(a, ck + d, c.pos0 + t, c.first_pos, c.slot, row_of);
+                g = log2_decay(a, c.row0 + t, h, d, rate);
+            }
+            qs[t * pk + d] = q;
+            ks[t * pk + d] = k;
+            gs[t * pk + d] = g;
+        }
+        for (int i = tid; i < kC * a.vdim_pad; i += 256) {
+            const int t = i / a.vdim_pad, v = i - t * a.vdim_pad;
+            vs[t * pv + v] = t < c.count && v < a.vdim ? conv_silu(a, cv + v, c.pos0 + t, c.first_pos, c.slot, row_of) : 0.f;
         }
     }
     if (tid < kC) bs[tid] = tid < c.count ? sigmoid_f((float)a.proj[(int64_t)(c.row0 + tid) * a.proj_stride + a.beta_off + h]) : 0.f;
     __syncthreads();
+
     const int i = tid >> 4, j = tid & 15;
+    int strong = 0;
+    for (int d = tid; d < dp; d += 256) {
+        float sum = 0.f;
+#pragma unroll
+        for (int t = 0; t < kC; ++t) {
+            sum += gs[t * pk + d];
+            gs[t * pk + d] = sum;
+        }
+        gl[d] = sum;
+        strong |= sum < -kSplitRange;
+    }
     {
         float sk = 0.f, sq = 0.f;
-        for (int d = j; d < dp; d += 16) { sk += ks[i * pk + d] * ks[i * pk + d]; sq += qs[i * pk + d] * qs[i * pk + d]; }
+        for (int d = 4 * j; d < dp; d += 64) {
+            const f32x4_t k = *reinterpret_cast<const f32x4_t*>(ks + i * pk + d), q = *reinterpret_cast<const f32x4_t*>(qs + i * pk + d);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { sk += k[e] * k[e]; sq += q[e] * q[e]; }
+        }
 #pragma unroll
         for (int m = 8; m >= 1; m >>= 1) { sk += __shfl_xor(sk, m, 64); sq += __shfl_xor(sq, m, 64); }
         if (j == 0) { inv[i] = rsqrtf(sk + 1e-6f); inv[16 + i] = rsqrtf(sq + 1e-6f) * a.q_scale; }
     }
-    __syncthreads();
-    {
-        // thread (i, j): both products of the token pair
-        float akk = 0.f, aqk = 0.f;
-        if (j <= i) {
-            const float *ki = ks + i * pk, *qi = qs + i * pk, *gi = gs + i * pk, *kj = ks + j * pk, *gj = gs + j * pk;
-            for (int d = 0; d < dp; d += 4) {
-                const f32x4_t k1 = *reinterpret_cast<const f32x4_t*>(ki + d), q1 = *reinterpret_cast<const f32x4_t*>(qi + d);
-                const f32x4_t g1 = *reinterpret_cast<const f32x4_t*>(gi + d), k2 = *reinterpret_cast<const f32x4_t*>(kj + d);
-                const f32x4_t g2 = *reinterpret_cast<const f32x4_t*>(gj + d);
+    strong = __syncthreads_or(strong);
+    float akk = 0.f, aqk = 0.f;                    // products of token pair (i, j), before the lengths
+    if (strong && j <= i) {
+        // some channel decays so much over the chunk that only differences of G can be exponentiated
+        const float *ki = ks + i * pk, *qi = qs + i * pk, *gi = gs + i * pk, *kj = ks + j * pk, *gj = gs + j * pk;
+        for (int d = 0; d < dp; d += 4) {
+            const f32x4_t k1 = *reinterpret_cast<const f32x4_t*>(ki + d), q1 = *reinterpret_cast<const f32x4_t*>(qi + d);
+            const f32x4_t g1 = *reinterpret_cast<const f32x4_t*>(gi + d), k2 = *reinterpret_cast<const f32x4_t*>(kj + d);
+            const f32x4_t g2 = *reinterpret_cast<const f32x4_t*>(gj + d);
 #pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    const float w = k2[e] * __builtin_amdgcn_exp2f(g1[e] - g2[e]);
-                    akk += k1[e] * w;
-                    aqk += q1[e] * w;
-                }
+            for (int e = 0; e < 4; ++e) {
+                const float w = k2[e] * __builtin_amdgcn_exp2f(g1[e] - g2[e]);
+                akk += k1[e] * w;
+                aqk += q1[e] * w;
             }
         }
-        lm[i * 20 + j] = j < i ? bs[i] * akk * inv[i] * inv[j] : 0.f;
-        rec[48 * dp + ((j >> 2) * 16 + i) * 4 + (j & 3)] = j <= i ? aqk * inv[16 + i] * inv[j] : 0.f;
+    }
+    if (strong) __syncthreads();
+    for (int x = tid; x < kC * (dp / 4); x += 256) {
+        const int t = x / (dp / 4), d = 4 * (x - t * (dp / 4));
+        f32x4_t* g = reinterpret_cast<f32x4_t*>(gs + t * pk + d);
+        f32x4_t* k = reinterpret_cast<f32x4_t*>(ks + t * pk + d);
+        f32x4_t* q = reinterpret_cast<f32x4_t*>(qs + t * pk + d);
+        const f32x4_t last = *reinterpret_cast<const f32x4_t*>(gl + d);
+        f32x4_t gv = *g, kv = *k, qv = *q;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const float up = __builtin_amdgcn_exp2f(gv[e]);
+            gv[e] = kv[e] * __builtin_amdgcn_exp2f(last[e] - gv[e]);
+            kv[e] *= up;
+            qv[e] *= up;
+        }
+        *g = gv; *k = kv; *q = qv;
     }
     __syncthreads();
-    if (tid < 64) {
-        // T = (I + L)^-1 by elimination: lane (q, m) holds rows 4 q .. 4 q + 3 of column m
-        const int q = tid >> 4, m = tid & 15;
-        float t[4];
+    const int lq = lane >> 4, lm = lane & 15;
+    if (!strong) {
+        // A_ij = sum_d (k_i e^{G_i - G_last}) (k_j e^{G_last - G_j}) on the matrix pipe, a quarter of the channels per wavefront
+        f32x4_t pk_acc = {0.f, 0.f, 0.f, 0.f}, pq_acc = pk_acc;
+        for (int t = wave; t < dp / 16; t += 4) {
+            const int d = 16 * t + 4 * lq;
+            const f32x4_t k1 = *reinterpret_cast<const f32x4_t*>(ks + lm * pk + d), q1 = *reinterpret_cast<const f32x4_t*>(qs + lm * pk + d);
+            const f32x4_t k2 = *reinterpret_cast<const f32x4_t*>(gs + lm * pk + d), last = *reinterpret_cast<const f32x4_t*>(gl + d);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) t[r] = 4 * q + r == m ? 1.f : 0.f;
-#pragma unroll
-        for (int s = 0; s < kC - 1; ++s) {
-            const float pivot = __shfl(t[s & 3], (s >> 2) * 16 + m, 64);     // T[s][m], final by now
-#pragma unroll
-            for (int r = 0; r < 4; ++r) t[r] -= lm[(4 * q + r) * 20 + s] * pivot;    // zero for rows up to s
+            for (int e = 0; e < 4; ++e) {
+                const float down = __builtin_amdgcn_exp2f(-last[e]);
+                pk_acc = __builtin_amdgcn_mfma_f32_16x16x4f32(k1[e] * down, k2[e], pk_acc, 0, 0, 0);
+                pq_acc = __builtin_amdgcn_mfma_f32_16x16x4f32(q1[e] * down, k2[e], pq_acc, 0, 0, 0);
+            }
         }
-        const float b = bs[m];
-        __builtin_amdgcn_wave_barrier();
 #pragma unroll
-        for (int r = 0; r < 4; ++r) lm[(4 * q + r) * 20 + m] = t[r] * b;
+        for (int e = 0; e < 4; ++e) {              // row 4 lq + e is token i, column lm token j
+            pp[wave * 512 + (4 * lq + e) * 16 + lm] = pk_acc[e];
+            pp[wave * 512 + 256 + (4 * lq + e) * 16 + lm] = pq_acc[e];
+        }
+        __syncthreads();
+#pragma unroll
+        for (int w = 0; w < 4; ++w) { akk += pp[w * 512 + tid]; aqk += pp[w * 512 + 256 + tid]; }
+    }
+    lt[j * 20 + i] = j < i ? bs[i] * akk * inv[i] * inv[j] : 0.f;
+    rec[48 * dp + ((j >> 2) * 16 + i) * 4 + (j & 3)] = j <= i ? aqk * inv[16 + i] * inv[j] : 0.f;
+    __syncthreads();
+    if (wave == 0) {
+        // T = (I + L)^-1 column by column: lane m holds column m, row s is final when it is used
+        float t[kC];
+#pragma unroll
+        for (int r = 0; r < kC; ++r) t[r] = r == lm ? 1.f : 0.f;
+#pragma unroll
+        for (int s = 0; s < kC - 1; ++s)
+#pragma unroll
+            for (int r4 = 0; r4 < kC; r4 += 4)
+                if (r4 + 3 > s) {
+                    const f32x4_t l = *reinterpret_cast<const f32x4_t*>(lt + s * 20 + r4);      // zero for rows up to s
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (r4 + e > s) t[r4 + e] -= l[e] * t[s];
+                }
+        if (lane < kC) {
+            const float b = bs[lm];
+#pragma unroll
+            for (int r = 0; r < kC; ++r) tb[r * 20 + lm] = t[r] * b;
+        }
+    } else {
+        const float iq = inv[16 + lm];
+        f32x4_t ik;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ik[e] = inv[4 * lq + e];
+        for (int t = wave - 1; t < dp / 16; t += 3) {
+            f32x4_t q = *reinterpret_cast<const f32x4_t*>(qs + lm * pk + 16 * t + 4 * lq), k;
+            q *= iq;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) k[e] = gs[(4 * lq + e) * pk + 16 * t + lm] * ik[e];
+            *reinterpret_cast<f32x4_t*>(rec + 16 * dp + 256 * t + 4 * lane) = q;
+            *reinterpret_cast<f32x4_t*>(rec + 32 * dp + 256 * t + 4 * lane) = k;
+        }
+        for (int d = tid - 64; d < dp; d += 192) rec[48 * dp + 256 + d] = __builtin_amdgcn_exp2f(gl[d]);
     }
     __syncthreads();
-    for (int d = tid; d < dp; d += 256) {
-        float kd[kC];
-        const float glast = gs[15 * pk + d];
-        const int dt = d >> 4, dm = d & 15;
-        float* w = rec + dt * 256 + (dm >> 2) * 64 + (dm & 3);
-        float* q = w + 16 * dp;
-        float* k = rec + 32 * dp + dt * 256 + dm * 4;
+    const f32x4_t tv = *reinterpret_cast<const f32x4_t*>(tb + lm * 20 + 4 * lq);       // T beta, row lm
+    for (int t = wave; t < dp / 16; t += 4) {      // W^T = (e^G K)^T (T beta)^T: row d, column i
+        f32x4_t w = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int t = 0; t < kC; ++t) {
-            const float gt = gs[t * pk + d];
-            const float kv = ks[t * pk + d] * inv[t];
-            kd[t] = kv * exp2f(gt);
-            q[4 * t] = qs[t * pk + d] * inv[16 + t] * exp2f(gt);
-            k[(t >> 2) * 64 + (t & 3)] = kv * exp2f(glast - gt);
-        }
-#pragma unroll
-        for (int t = 0; t < kC; ++t) {
-            float s = 0.f;
-#pragma unroll
-            for (int r = 0; r <= t; ++r) s += lm[t * 20 + r] * kd[r];
-            w[4 * t] = s;
-        }
-        rec[48 * dp + 256 + d] = exp2f(glast);
+        for (int e = 0; e < 4; ++e)
+            w = __builtin_amdgcn_mfma_f32_16x16x4f32(ks[(4 * lq + e) * pk + 16 * t + lm] * inv[4 * lq + e], tv[e], w, 0, 0, 0);
+        *reinterpret_cast<f32x4_t*>(rec + 256 * t + 4 * lane) = w;
     }
     float* uv = rec + 49 * dp + 256;
-    for (int v = tid; v < a.vdim_pad; v += 256) {
-        float x[kC];
+    for (int t = wave; t < a.vdim_pad / 16; t += 4) {
+        f32x4_t w = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int t = 0; t < kC; ++t) x[t] = vs[t * pv + v];
-        float* o = uv + (v >> 4) * 256 + (v & 15) * 4;
-#pragma unroll
-        for (int t = 0; t < kC; ++t) {
-            float s = 0.f;
-#pragma unroll
-            for (int r = 0; r <= t; ++r) s += lm[t * 20 + r] * x[r];
-            o[(t >> 2) * 64 + (t & 3)] = s;
-        }
+        for (int e = 0; e < 4; ++e) w = __builtin_amdgcn_mfma_f32_16x16x4f32(tv[e], vs[(4 * lq + e) * pv + 16 * t + lm], w, 0, 0, 0);
+        *reinterpret_cast<f32x4_t*>(uv + 256 * t + 4 * lane) = w;
     }
 }
 
@@ -443,20 +567,39 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(const PortionDesc* port
             for (int r = 0; r < 4; ++r) sp[(int64_t)(16 * t + 4 * q + r) * vdim_pad] = s[t][r];
 }
 
-// One workgroup per token row behind `row0`, one wavefront per head at a time.
-template <class T>
+// One workgroup per token row behind `row0`.  LANES lanes share a head, four values each (vdim = 4 LANES);
+// LANES = 0: any vdim, one wavefront per head.
+template <class T, int LANES>
 __global__ void __launch_bounds__(256) delta_out_kernel(DeltaArgs<T> a, const float* o, int64_t row0, const int32_t* ring_slot,
                                                         const int64_t* positions) {
     const int64_t row = row0 + blockIdx.x;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    for (int h = wave; h < a.heads; h += 4) {
-        const float* x = o + (row * a.heads + h) * a.vdim_pad;
-        float ss = 0.f;
-        for (int v = lane; v < a.vdim; v += 64) ss += x[v] * x[v];
-        const float rs = rsqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
-        const T* gr = a.gate + row * a.gate_stride + (int64_t)h * a.vdim;
-        T* out = a.out + row * a.out_stride + (int64_t)h * a.vdim;
-        for (int v = lane; v < a.vdim; v += 64) out[v] = (T)(x[v] * rs * a.norm[v] * sigmoid_f((float)gr[v]));
+    if constexpr (LANES > 0) {
+        const int v = 4 * (threadIdx.x % LANES);
+        float w[4];
+        load_elems<4>(a.norm + v, w);
+        for (int h = threadIdx.x / LANES; h < a.heads; h += 256 / LANES) {
+            float x[4], g[4];
+            load_elems<4>(o + (row * a.heads + h) * a.vdim_pad + v, x);
+            load_elems<4>(a.gate + row * a.gate_stride + (int64_t)h * a.vdim + v, g);
+            float ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+#pragma unroll
+            for (int m = LANES / 2; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, 64);
+            const float rs = rsqrtf(ss / (float)a.vdim + a.eps);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[e] *= rs * w[e] * sigmoid_f(g[e]);
+            store_elems<4>(a.out + row * a.out_stride + (int64_t)h * a.vdim + v, x);
+        }
+    } else {
+        for (int h = wave; h < a.heads; h += 4) {
+            const float* x = o + (row * a.heads + h) * a.vdim_pad;
+            float ss = 0.f;
+            for (int v = lane; v < a.vdim; v += 64) ss += x[v] * x[v];
+            const float rs = rsqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+            const T* gr = a.gate + row * a.gate_stride + (int64_t)h * a.vdim;
+            T* out = a.out + row * a.out_stride + (int64_t)h * a.vdim;
+            for (int v = lane; v < a.vdim; v += 64) out[v] = (T)(x[v] * rs * a.norm[v] * sigmoid_f((float)gr[v]));
+        }
     }
     const int slot = ring_slot[2 * row];
     if (slot < 0 || slot >= a.num_slots || ring_slot[2 * row + 1] >= a.taps) return;     // not among the portion's last inputs
@@ -530,20 +673,32 @@ template <class T>
 int launch_chunks(const DeltaArgs<T>& a, const PortionDesc* portions, int64_t num_portions, const ChunkDesc* chunks, int64_t num_chunks,
                   float* records, float* o, int64_t row0, int64_t rows, const int32_t* ring_slot, const int64_t* positions,
                   hipStream_t st) {
-    const size_t lds = (size_t)(3 * kC * (a.dim_pad + 4) + kC * (a.vdim_pad + 4) + kC * 20 + 48) * sizeof(float);
-    if (lds > 64 * 1024) {
-        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_prep_kernel<T>),
-                                                 hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    const size_t lds = (size_t)(3 * kC * (a.dim_pad + 4) + kC * (a.vdim_pad + 4) + 2048 + 2 * kC * 20 + a.dim_pad + 48) * sizeof(float);
+    // rows and channels that can be read four elements at a time
+    auto fours = [](const void* p, int64_t stride) { return ptr_aligned(p, 4 * sizeof(T)) && stride % 4 == 0; };
+    const bool rows4 = a.dim % 4 == 0 && a.vdim % 4 == 0;
+    const bool vec = rows4 && a.taps == 4 && fours(a.proj, a.proj_stride) && fours(a.ring, a.channels) && fours(a.decay, a.decay_stride) &&
+                     ptr_aligned(a.conv, 16) && ptr_aligned(a.dt_bias, 16);
+    auto prep = vec ? &delta_prep_kernel<T, true> : &delta_prep_kernel<T, false>;
+    if (lds > 60 * 1024) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(prep), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return (int)e;
     }
-    hipLaunchKernelGGL((delta_prep_kernel<T>), dim3((unsigned)num_chunks, (unsigned)a.heads), dim3(256), lds, st, a, chunks, records);
+    hipLaunchKernelGGL(prep, dim3((unsigned)num_chunks, (unsigned)a.heads), dim3(256), lds, st, a, chunks, records);
     int rc = (int)hipGetLastError();
     if (rc) return rc;
 #define GO(N) case N: rc = launch_scan<N>(portions, num_portions, chunks, records, a.state, o, a.heads, a.vdim_pad, st); break
     switch (a.dim_pad / 16) { GO(1); GO(2); GO(3); GO(4); GO(6); GO(8); GO(12); GO(16); default: return INFER_KV_EUNSUPPORTED; }
 #undef GO
     if (rc) return rc;
-    hipLaunchKernelGGL((delta_out_kernel<T>), dim3((unsigned)rows), dim3(256), 0, st, a, (const float*)o, row0, ring_slot, positions);
+    const bool out4 = rows4 && fours(a.gate, a.gate_stride) && fours(a.out, a.out_stride) && ptr_aligned(o, 16) && ptr_aligned(a.norm, 16);
+#define GO(N) hipLaunchKernelGGL((delta_out_kernel<T, N>), dim3((unsigned)rows), dim3(256), 0, st, a, (const float*)o, row0, ring_slot, positions)
+    if (out4 && a.vdim == 32) GO(8);
+    else if (out4 && a.vdim == 64) GO(16);
+    else if (out4 && a.vdim == 128) GO(32);
+    else if (out4 && a.vdim == 256) GO(64);
+    else GO(0);
+#undef GO
     return (int)hipGetLastError();
 }
 

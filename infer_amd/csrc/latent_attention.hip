@@ -312,15 +312,15 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatentAttnArgs<__
         for (int i = 0; i < NT; ++i) acc[u][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
 
-    // chunk i of this thread: 16 bytes at offset 16 (tid + 256 i) of the tile; its row and place in LDS
+    // chunk i of this thread: 16 bytes at offset 16 (tid + 256 i) of the tile; its place in LDS
     const int chunks_per_row = a.row / 8, chunks = kTile * chunks_per_row;
     u32x4_t stage[KSH];
-    int st_row[KSH], st_lds[KSH];
+    int st_lds[KSH];
 #pragma unroll
     for (int i = 0; i < KSH; ++i) {
         const int c = tid + 256 * i;
-        st_row[i] = c / chunks_per_row;
-        st_lds[i] = st_row[i] * pitch + (c - st_row[i] * chunks_per_row) * 16;
+        const int r = c / chunks_per_row;
+        st_lds[i] = r * pitch + (c - r * chunks_per_row) * 16;
     }
     const int tiles_per_block = a.block_size / kTile;
     auto fetch = [&](int t) {
@@ -328,11 +328,12 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatentAttnArgs<__
         const int blk = block_id(a, bt, col);
         const __bf16* src = a.cache + ((int64_t)blk * a.block_size + (t - col * tiles_per_block) * kTile) * a.row;
         const int rows = len - t * kTile;
+        const int have = rows < kTile ? rows * chunks_per_row : chunks;
 #pragma unroll
         for (int i = 0; i < KSH; ++i) {
             const int c = tid + 256 * i;
             stage[i] = u32x4_t{0u, 0u, 0u, 0u};                   // rows behind the last key count as zeros
-            if (c < chunks && st_row[i] < rows) stage[i] = reinterpret_cast<const u32x4_t*>(src)[c];
+            if (c < have) stage[i] = reinterpret_cast<const u32x4_t*>(src)[c];
         }
     };
     if (t0 < t1) fetch(t0);
@@ -651,6 +652,7 @@ extern "C" int infer_latent_attention(int elem, const void* qx, const void* cach
         int rc;
         if (row <= 192 && rank_pad <= 128) rc = launch_decode<3, 2>(b, n, st);
         else if (row <= 384 && rank_pad <= 256) rc = launch_decode<6, 4>(b, n, st);
+        else if (row <= 576) rc = launch_decode<9, 8>(b, n, st);
         else rc = launch_decode<10, 8>(b, n, st);
         if (rc) return rc;
         done += n;

@@ -4,7 +4,7 @@
 //
 // A wavefront owns 32 queries (two MFMA column tiles) of one head, a workgroup four wavefronts = 128
 // consecutive queries, and walks the visible keys in steps of 32 that all four share through LDS (two
-// buffers, the next step's rows travel through registers meanwhile):
+// buffers; the rows of the next two steps travel through registers meanwhile):
 //   S^T[key, query] = [k_plain | k_rot][key, :] . q^T      KS k-steps of 32
 //   O^T[v, query]  += V^T[v, key] . P^T                    VT row tiles of 16
 // Row r of the score tile t is key 8 (r / 4) + 4 t + r % 4, so that a lane's eight scores are the eight
@@ -92,50 +92,44 @@ __global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPr
     // the columns behind the real sizes stay zero in both buffers
     for (int i = tid; i < 2 * kBuf / 16; i += 256) reinterpret_cast<u32x4_t*>(lds)[i] = u32x4_t{0u, 0u, 0u, 0u};
 
-    // chunk i of this thread of the K and of the V tile: key, source, place
+    // chunk i of this thread of the K and of the V tile: key, place, and a running pointer to its source
     const int kc = qk / 8, vc = a.vdim / 8, dc = a.dim / 8;
-    int k_key[kNK], k_lds[kNK], v_key[kNV], v_lds[kNV];
-    const __bf16* k_src[kNK];
-    int64_t k_str[kNK];
-    int v_col[kNV];
+    constexpr int kN = kNK + kNV;
+    int c_key[kN], c_lds[kN], c_str[kN];                         // c_str: elements from one key to the next (checked below 2^24)
+    const __bf16* c_src[kN];
 #pragma unroll
-    for (int i = 0; i < kNK; ++i) {
-        const int c = tid + 256 * i, key = c / kc, col = c - key * kc;
-        k_key[i] = key < kStep ? key : -1;
-        k_lds[i] = key * kKPitch + col * 16;
-        const bool plain = col < dc;
-        k_src[i] = plain ? a.kp + (int64_t)h * a.dim + 8 * col : a.kr + 8 * (col - dc);
-        k_str[i] = plain ? a.kp_stride : a.kr_stride;
+    for (int i = 0; i < kN; ++i) {
+        const bool is_k = i < kNK;
+        const int c = tid + 256 * (is_k ? i : i - kNK), per = is_k ? kc : vc;
+        const int key = c / per, col = c - key * per;
+        c_key[i] = key < kStep ? key : -1;                       // -1: no such chunk; it re-reads the first value and is not stored
+        c_lds[i] = is_k ? key * kKPitch + col * 16 : kStep * kKPitch + key * kVPitch + col * 16;
+        const bool rot = is_k && col >= dc;
+        c_str[i] = key >= kStep ? 0 : (int)(!is_k ? a.v_stride : rot ? a.kr_stride : a.kp_stride);
+        const __bf16* base = !is_k ? a.v + (int64_t)h * a.vdim + 8 * col
+                             : rot ? a.kr + 8 * (col - dc) : a.kp + (int64_t)h * a.dim + 8 * col;
+        c_src[i] = (key < kStep ? base : a.v) + (int64_t)(k_beg + key) * c_str[i];
     }
+    // Two steps are under way in registers while a third is consumed from LDS: a step is shorter than the
+    // round trip to the second-level cache.
+    u32x4_t st0[kN], st1[kN];
+    auto fetch = [&](int s, u32x4_t (&st)[kN]) {
+        const int over = kStep - (sk - s * kStep);               // keys behind the last one re-read it; their weights are zero
 #pragma unroll
-    for (int i = 0; i < kNV; ++i) {
-        const int c = tid + 256 * i, key = c / vc, col = c - key * vc;
-        v_key[i] = key < kStep ? key : -1;
-        v_lds[i] = kStep * kKPitch + key * kVPitch + col * 16;
-        v_col[i] = h * a.vdim + 8 * col;
-    }
-    u32x4_t kst[kNK], vst[kNV];
-    auto fetch = [&](int s) {
-        const int last = sk - 1 - s * kStep;       // keys behind the last one re-read it; their weights are zero
-        const int64_t base = k_beg + s * kStep;
-#pragma unroll
-        for (int i = 0; i < kNK; ++i) {
-            const int r = k_key[i] < last ? k_key[i] : last;
-            if (r >= 0) kst[i] = *reinterpret_cast<const u32x4_t*>(k_src[i] + (base + r) * k_str[i]);
-        }
-#pragma unroll
-        for (int i = 0; i < kNV; ++i) {
-            const int r = v_key[i] < last ? v_key[i] : last;
-            if (r >= 0) vst[i] = *reinterpret_cast<const u32x4_t*>(a.v + (base + r) * a.v_stride + v_col[i]);
+        for (int i = 0; i < kN; ++i) {
+            const __bf16* p = c_src[i];
+            if (over > 0) {
+                const int key = c_key[i] > 0 ? c_key[i] : 0, last = kStep - 1 - over;
+                if (key > last) p -= (int64_t)(key - last) * c_str[i];
+            }
+            st[i] = *reinterpret_cast<const u32x4_t*>(p);
+            c_src[i] += (int64_t)kStep * c_str[i];
         }
     };
-    auto put = [&](unsigned char* buf) {
+    auto put = [&](unsigned char* buf, const u32x4_t (&st)[kN]) {
 #pragma unroll
-        for (int i = 0; i < kNK; ++i)
-            if (k_key[i] >= 0) *reinterpret_cast<u32x4_t*>(buf + k_lds[i]) = kst[i];
-#pragma unroll
-        for (int i = 0; i < kNV; ++i)
-            if (v_key[i] >= 0) *reinterpret_cast<u32x4_t*>(buf + v_lds[i]) = vst[i];
+        for (int i = 0; i < kN; ++i)
+            if (c_key[i] >= 0) *reinterpret_cast<u32x4_t*>(buf + c_lds[i]) = st[i];
     };
 
     f32x4_t acc[2][VT], lacc[2];
@@ -151,15 +145,16 @@ __global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPr
         for (int t = 0; t < VT; ++t) acc[u][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
 
-    fetch(0);
+    fetch(0, st0);
+    if (nsteps > 1) fetch(1, st1);
     __syncthreads();          // the zero fill
-    put(lds);
+    put(lds, st0);
     __syncthreads();
     const int k_addr = (8 * (n >> 2) + (n & 3)) * kKPitch + 16 * g;
     const int v_addr = kStep * kKPitch + (8 * g + (n >> 2)) * kVPitch + (n & 3) * 8;
-    for (int s = 0; s < nsteps; ++s) {
-        const unsigned char* buf = lds + (s & 1) * kBuf;
-        if (s + 1 < nsteps) fetch(s + 1);
+    // step s consumes buffer s % 2, requests step s + 2 into `ahead` and stores step s + 1, which is in `next`
+    auto step = [&](int s, const unsigned char* buf, unsigned char* other, u32x4_t (&ahead)[kN], u32x4_t (&next)[kN]) {
+        if (s + 2 < nsteps) fetch(s + 2, ahead);
         if (s < my_steps) {
             const int tok0 = s * kStep;
             f32x4_t sc[2][2];
@@ -214,8 +209,12 @@ __global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPr
                 for (int u = 0; u < 2; ++u) acc[u][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pb[u], acc[u][t], 0, 0, 0);
             }
         }
-        if (s + 1 < nsteps) put(lds + ((s + 1) & 1) * kBuf);
+        if (s + 1 < nsteps) put(other, next);
         __syncthreads();
+    };
+    for (int s = 0; s < nsteps; s += 2) {
+        step(s, lds, lds + kBuf, st0, st1);
+        if (s + 1 < nsteps) step(s + 1, lds + kBuf, lds, st1, st0);
     }
     if (!live) return;
 #pragma unroll
@@ -263,6 +262,7 @@ extern "C" int infer_latent_prefill(const void* q, int64_t q_stride, const void*
     if (q_stride < heads * (dim + rot) || kp_stride < heads * dim || kr_stride < rot || v_stride < heads * vdim ||
         gate_stride < heads || out_stride < heads * vdim)
         return INFER_KV_EINVAL;
+    if (kp_stride >= (1 << 24) || kr_stride >= (1 << 24) || v_stride >= (1 << 24)) return INFER_KV_EINVAL;
     if (q_stride % 8 || kp_stride % 8 || kr_stride % 8 || v_stride % 8 || out_stride % 4 || !ptr_aligned(q, 16) || !ptr_aligned(kp, 16) ||
         !ptr_aligned(kr, 16) || !ptr_aligned(v, 16) || !ptr_aligned(out, 8))
         return INFER_KV_EALIGN;
