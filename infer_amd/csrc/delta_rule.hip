@@ -219,14 +219,20 @@ struct PortionDesc { int32_t chunk0, chunks, slot, pos0; };
 __host__ __device__ inline int64_t record_floats(int dim_pad, int vdim_pad) { return 48 * (int64_t)dim_pad + 256 + dim_pad + 16 * (int64_t)vdim_pad; }
 
 // The convolution of four channels over tokens t0 .. t0 + 7 of a chunk, for four taps, the window in registers.
-// c: first channel, dst: LDS row of token t0, column of the channel.
-template <class T>
+// c: first channel, dst: LDS row of token t0, column of the channel.  INNER: all 16 tokens exist and the window of
+// the first one lies inside the portion.
+template <class T, bool INNER>
 __device__ __forceinline__ void conv4_silu(const DeltaArgs<T>& a, const ChunkDesc& cd, int c, int t0, float* dst, int pitch) {
     float x[11][4], w[4][4];
 #pragma unroll
     for (int e = 0; e < 4; ++e) load_elems<4>(a.conv + 4 * (c + e), w[e]);
+    if constexpr (INNER) {
+        const T* src = a.proj + (int64_t)(cd.row0 + t0 - 3) * a.proj_stride + c;
 #pragma unroll
-    for (int j = 0; j < 11; ++j) {
+        for (int j = 0; j < 11; ++j, src += a.proj_stride) load_elems<4>(src, x[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < (INNER ? 0 : 11); ++j) {
         const int t = t0 + j - 3, p = cd.pos0 + t;
         // positions before the portion are in the ring; those before the sequence or behind the chunk's tokens are zero
         const bool in = p >= 0 && t < cd.count;
@@ -240,7 +246,7 @@ __device__ __forceinline__ void conv4_silu(const DeltaArgs<T>& a, const ChunkDes
 #pragma unroll
     for (int t = 0; t < 8; ++t) {
         float y[4];
-        const bool in = t0 + t < cd.count;
+        const bool in = INNER || t0 + t < cd.count;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             y[e] = 0.f;
@@ -273,10 +279,10 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs<T> a, const C
     float* ks = qs + kC * pk;          // [16][pk] k, then e^G k
     float* gs = ks + kC * pk;          // [16][pk] running log2 decay G, then e^{G_last - G} k
     float* vs = gs + kC * pk;          // [16][pv]
-    float* pp = vs + kC * pv;          // [4][2][256] products of the token pairs, one part per wavefront
-    float* lt = pp + 2048;             // [16][20] column s: beta * A of the tokens behind s
-    float* tb = lt + kC * 20;          // [16][20] T * beta
-    float* gl = tb + kC * 20;          // [dp] G_last
+    float* pp = vs + kC * pv;          // [2][2][256] products of the token pairs (k k, q k), in two parts each
+    float* lt = pp + 1024;             // [16][20] column s: beta * A of the tokens behind s
+    float* tb = lt;                    // [16][20] T * beta, when those have been used
+    float* gl = lt + kC * 20;          // [dp] G_last
     float* inv = gl + dp;              // [2][16] 1 / length of k and q
     float* bs = inv + 32;              // [16] beta
     const int group = a.heads / a.kv_heads, kvh = h / group;
@@ -286,11 +292,14 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs<T> a, const C
 
     if constexpr (VEC) {
         const int nd = a.dim / 4, nv = a.vdim / 4, n = 2 * nd + nv;
+        const bool inner = c.count == kC && c.pos0 - 3 >= c.first_pos;
         for (int i = tid; i < 2 * n; i += 256) {
             const int half = i >= n, j = i - half * n, t0 = 8 * half;
-            if (j < nd) conv4_silu(a, c, cq + 4 * j, t0, qs + t0 * pk + 4 * j, pk);
-            else if (j < 2 * nd) conv4_silu(a, c, ck + 4 * (j - nd), t0, ks + t0 * pk + 4 * (j - nd), pk);
-            else conv4_silu(a, c, cv + 4 * (j - 2 * nd), t0, vs + t0 * pv + 4 * (j - 2 * nd), pv);
+            const int col = j < nd ? 4 * j : j < 2 * nd ? 4 * (j - nd) : 4 * (j - 2 * nd);
+            const int ch = col + (j < nd ? cq : j < 2 * nd ? ck : cv), pitch = j < 2 * nd ? pk : pv;
+            float* dst = (j < nd ? qs : j < 2 * nd ? ks : vs) + t0 * pitch + col;
+            if (inner) conv4_silu<T, true>(a, c, ch, t0, dst, pitch);
+            else conv4_silu<T, false>(a, c, ch, t0, dst, pitch);
         }
         for (int i = tid; i < kC * nd; i += 256) {
             const int t = i / nd, d = 4 * (i - t * nd);
@@ -394,27 +403,25 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaArgs<T> a, const C
     __syncthreads();
     const int lq = lane >> 4, lm = lane & 15;
     if (!strong) {
-        // A_ij = sum_d (k_i e^{G_i - G_last}) (k_j e^{G_last - G_j}) on the matrix pipe, a quarter of the channels per wavefront
-        f32x4_t pk_acc = {0.f, 0.f, 0.f, 0.f}, pq_acc = pk_acc;
-        for (int t = wave; t < dp / 16; t += 4) {
+        // A_ij = sum_d (k_i e^{G_i - G_last}) (k_j e^{G_last - G_j}) on the matrix pipe: wavefronts 0 and 1 take half of the
+        // channels each, 2 and 3 do the same for q
+        f32x4_t acc0 = {0.f, 0.f, 0.f, 0.f}, acc1 = acc0;
+        const float* left = (wave < 2 ? ks : qs) + lm * pk;
+        for (int t = wave & 1; t < dp / 16; t += 2) {
             const int d = 16 * t + 4 * lq;
-            const f32x4_t k1 = *reinterpret_cast<const f32x4_t*>(ks + lm * pk + d), q1 = *reinterpret_cast<const f32x4_t*>(qs + lm * pk + d);
-            const f32x4_t k2 = *reinterpret_cast<const f32x4_t*>(gs + lm * pk + d), last = *reinterpret_cast<const f32x4_t*>(gl + d);
+            const f32x4_t x1 = *reinterpret_cast<const f32x4_t*>(left + d), last = *reinterpret_cast<const f32x4_t*>(gl + d);
+            const f32x4_t k2 = *reinterpret_cast<const f32x4_t*>(gs + lm * pk + d);
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const float down = __builtin_amdgcn_exp2f(-last[e]);
-                pk_acc = __builtin_amdgcn_mfma_f32_16x16x4f32(k1[e] * down, k2[e], pk_acc, 0, 0, 0);
-                pq_acc = __builtin_amdgcn_mfma_f32_16x16x4f32(q1[e] * down, k2[e], pq_acc, 0, 0, 0);
+            for (int e = 0; e < 4; e += 2) {
+                acc0 = __builtin_amdgcn_mfma_f32_16x16x4f32(x1[e] * __builtin_amdgcn_exp2f(-last[e]), k2[e], acc0, 0, 0, 0);
+                acc1 = __builtin_amdgcn_mfma_f32_16x16x4f32(x1[e + 1] * __builtin_amdgcn_exp2f(-last[e + 1]), k2[e + 1], acc1, 0, 0, 0);
             }
         }
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {              // row 4 lq + e is token i, column lm token j
-            pp[wave * 512 + (4 * lq + e) * 16 + lm] = pk_acc[e];
-            pp[wave * 512 + 256 + (4 * lq + e) * 16 + lm] = pq_acc[e];
-        }
+        for (int e = 0; e < 4; ++e) pp[wave * 256 + (4 * lq + e) * 16 + lm] = acc0[e] + acc1[e];    // row: token i, column: token j
         __syncthreads();
-#pragma unroll
-        for (int w = 0; w < 4; ++w) { akk += pp[w * 512 + tid]; aqk += pp[w * 512 + 256 + tid]; }
+        akk = pp[tid] + pp[256 + tid];
+        aqk = pp[512 + tid] + pp[768 + tid];
     }
     lt[j * 20 + i] = j < i ? bs[i] * akk * inv[i] * inv[j] : 0.f;
     rec[48 * dp + ((j >> 2) * 16 + i) * 4 + (j & 3)] = j <= i ? aqk * inv[16 + i] * inv[j] : 0.f;
@@ -673,7 +680,7 @@ template <class T>
 int launch_chunks(const DeltaArgs<T>& a, const PortionDesc* portions, int64_t num_portions, const ChunkDesc* chunks, int64_t num_chunks,
                   float* records, float* o, int64_t row0, int64_t rows, const int32_t* ring_slot, const int64_t* positions,
                   hipStream_t st) {
-    const size_t lds = (size_t)(3 * kC * (a.dim_pad + 4) + kC * (a.vdim_pad + 4) + 2048 + 2 * kC * 20 + a.dim_pad + 48) * sizeof(float);
+    const size_t lds = (size_t)(3 * kC * (a.dim_pad + 4) + kC * (a.vdim_pad + 4) + 1024 + kC * 20 + a.dim_pad + 48) * sizeof(float);
     // rows and channels that can be read four elements at a time
     auto fours = [](const void* p, int64_t stride) { return ptr_aligned(p, 4 * sizeof(T)) && stride % 4 == 0; };
     const bool rows4 = a.dim % 4 == 0 && a.vdim % 4 == 0;

@@ -92,13 +92,14 @@ __device__ __forceinline__ float block_sum(float x, float* part) {
     return s;
 }
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+// 1 / (1 + e^-z) by the hardware's exp2 and reciprocal (one unit in the last place each)
+__device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-kLog2e * z)); }
+__device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }
 __device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 // 0.5 z (1 + tanh(u)) = z / (1 + exp(-2 u)),  u = sqrt(2 / pi) (z + 0.044715 z^3)
 __device__ __forceinline__ float gelu_tanh_f(float z) {
     const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
-    return z / (1.0f + expf(-2.0f * u));
+    return z * sigmoid_f(2.0f * u);
 }
 
 static inline bool ptr_aligned(const void* p, size_t bytes) { return (reinterpret_cast<uintptr_t>(p) & (bytes - 1)) == 0; }

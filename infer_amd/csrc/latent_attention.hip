@@ -143,6 +143,7 @@ __global__ void __launch_bounds__(256) head_matmul_mfma_kernel(HeadMatmulArgs<__
         xr[u] = a.x + (int64_t)(m < a.m ? m : a.m - 1) * a.x_row + (int64_t)h * a.x_head + 8 * g;
         acc[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
+#pragma unroll 4
     for (int k = 0; k < a.k; k += 32) {
         const bf16x8_t w = *reinterpret_cast<const bf16x8_t*>(wr + k);
         const bool in = k + 8 * g < a.k;
@@ -579,8 +580,10 @@ extern "C" int infer_head_matmul(int elem, const void* x, int64_t x_row, int64_t
                            ptr_aligned(x, 16) && ptr_aligned(w, 16) && ptr_aligned(out, 8);
         if (tiles) {
             const unsigned gx = (unsigned)((n + 63) / 64);
-            if (m <= 16) hipLaunchKernelGGL((head_matmul_mfma_kernel<1>), dim3(gx, (unsigned)heads, 1), dim3(256), 0, st, a);
-            else {
+            // few workgroups: 16 rows each instead of 64, the weights then come from the second-level cache
+            if (m <= 16 || (m + 63) / 64 * gx * heads < 512) {
+                hipLaunchKernelGGL((head_matmul_mfma_kernel<1>), dim3(gx, (unsigned)heads, (unsigned)((m + 15) / 16)), dim3(256), 0, st, a);
+            } else {
                 if ((m + 63) / 64 > 65535) return INFER_KV_EINVAL;
                 hipLaunchKernelGGL((head_matmul_mfma_kernel<4>), dim3(gx, (unsigned)heads, (unsigned)((m + 63) / 64)), dim3(256), 0, st, a);
             }
