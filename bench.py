@@ -240,7 +240,7 @@ def hybrid_config(size):
     from infer_amd.config import LayerSpec, MerilornConfig
     width, ff, heads, layers = HYBRID_SIZES[size]
     latent = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
-              "rot": {"base": 1e6, "dims": 64, "scaling": {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+              "rot": {"base": 1e5, "dims": 64, "scaling": {"factor": 2.0, "original": 32768, "fast": 16.0, "slow": 2.0}}}
     delta = {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4, "decay_rank": 128, "gate_rank": 128}
     specs = [LayerSpec("latent_attention", latent, ff, i) if i % 4 == 3 else LayerSpec("channel_delta", delta, ff, i)
              for i in range(layers)]

@@ -74,7 +74,7 @@ def test_residual_norm_of_split_k_pieces(gpu):
 
 
 @BOTH
-@pytest.mark.parametrize("d", [8, 30, 320])
+@pytest.mark.parametrize("d", [8, 30, 352])
 def test_gelu_tanh_and_mul(gpu, dtype, d):
     x = rounded(np.random.default_rng(d).standard_normal((6, 2 * d)) * 4, dtype)
     x[0, 0], x[1, 0] = 60.0, -60.0
@@ -168,7 +168,7 @@ def latent_want(q, k, rank_pad, scale):
     return p / p.sum(-1, keepdims=True) @ k[:, :rank_pad]
 
 
-SIZES = [(3, 96, 64), (6, 128, 96), (17, 192, 128), (2, 64, 32), (16, 320, 256), (40, 576, 512), (5, 160, 128), (3, 800, 768)]
+SIZES = [(3, 96, 64), (7, 160, 96), (17, 192, 128), (2, 64, 32), (16, 320, 256), (40, 576, 512), (5, 160, 128), (3, 800, 768)]
 
 
 @BOTH
@@ -191,7 +191,7 @@ def test_latent_attention_lengths_around_tiles_and_blocks(gpu, dtype, heads, row
 def test_latent_attention_one_key_stands_out(gpu, dtype, splits, at):
     """The query is aimed at one key; the last visible one and the first invisible one are told apart."""
     rng = np.random.default_rng(at)
-    heads, row, rank_pad, n = 5, 128, 96, 318
+    heads, row, rank_pad, n = 5, 160, 128, 318
     q, keys, cache, tables = latent_case(rng, [n], heads, row, rank_pad, 32, dtype)
     aim = np.broadcast_to(keys[0][at] * 2.0, (4, heads, row))
     ctx = [at + 1, max(at, 1), n, min(at + 2, n)]
@@ -224,7 +224,7 @@ def test_latent_gather(gpu):
     assert np.array_equal(host(out), np.concatenate([keys[2], keys[0]]))
 
 
-@pytest.mark.parametrize("heads,dim,rot,vdim", [(3, 16, 8, 24), (6, 32, 32, 32), (2, 96, 32, 64), (2, 64, 32, 128), (3, 128, 64, 128), (1, 192, 64, 104), (2, 24, 40, 8)])
+@pytest.mark.parametrize("heads,dim,rot,vdim", [(3, 16, 8, 24), (5, 48, 16, 40), (2, 96, 32, 64), (2, 64, 32, 128), (3, 128, 64, 128), (1, 192, 64, 104), (2, 24, 40, 8)])
 def test_latent_prefill(gpu, heads, dim, rot, vdim):
     """Portions with and without a prefix, lengths around the tiles; one query-key pair stands out."""
     rng = np.random.default_rng(dim)
@@ -320,7 +320,7 @@ class DeltaCase:
         assert (rest[:, self.s.dim:] == 0).all() and (rest[:, :, self.s.vdim:] == 0).all()
 
 
-DELTA_SIZES = [(2, 2, 64, 32, 4), (4, 2, 24, 16, 4), (3, 1, 16, 40, 3), (2, 1, 128, 128, 4), (1, 1, 100, 20, 2), (2, 2, 5, 7, 1),
+DELTA_SIZES = [(3, 3, 48, 32, 4), (4, 2, 24, 16, 4), (3, 1, 16, 40, 3), (2, 1, 128, 128, 4), (1, 1, 100, 20, 2), (2, 2, 5, 7, 1),
                (2, 1, 192, 64, 5), (1, 1, 256, 256, 4), (1, 1, 40, 300, 4)]
 
 
@@ -339,7 +339,7 @@ def test_delta_any_cut(gpu, size, cuts):
 @pytest.mark.parametrize("decay", [-9.0, 0.0, 5.0, 40.0])
 def test_delta_decay_strengths(gpu, decay):
     """From almost none to a state that is gone after one token: nothing overflows, nothing is lost."""
-    DeltaCase(2, 1, 64, 32, 4, 70, torch.float32, seed=2, decay=decay).check([64, 1, 5])
+    DeltaCase(2, 1, 48, 64, 4, 70, torch.float32, seed=2, decay=decay).check([64, 1, 5])
 
 
 def test_delta_first_token_is_still_read_far_later(gpu):
