@@ -92,6 +92,18 @@ __device__ __forceinline__ float block_sum(float x, float* part) {
     return s;
 }
 
+// maximum over the lanes l, l ^ 16, l ^ 32 and l ^ 48, on the vector pipe
+__device__ __forceinline__ float max_xor16_32(float x) {
+    const unsigned u = __builtin_bit_cast(unsigned, x);
+    const auto r = __builtin_amdgcn_permlane16_swap(u, u, false, false);
+    const unsigned a0 = r[0], a1 = r[1];
+    const float y = fmaxf(__builtin_bit_cast(float, a0), __builtin_bit_cast(float, a1));
+    const unsigned w = __builtin_bit_cast(unsigned, y);
+    const auto s = __builtin_amdgcn_permlane32_swap(w, w, false, false);
+    const unsigned b0 = s[0], b1 = s[1];
+    return fmaxf(__builtin_bit_cast(float, b0), __builtin_bit_cast(float, b1));
+}
+
 // 1 / (1 + e^-z) by the hardware's exp2 and reciprocal (one unit in the last place each)
 __device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-kLog2e * z)); }
 __device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }

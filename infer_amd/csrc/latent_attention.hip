@@ -22,11 +22,6 @@ typedef short i16x4 __attribute__((ext_vector_type(4)));
 typedef short i16x8 __attribute__((ext_vector_type(8)));
 typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
 
-__device__ __forceinline__ float max_xor16_32(float x) {
-    x = fmaxf(x, __shfl_xor(x, 16, 64));
-    return fmaxf(x, __shfl_xor(x, 32, 64));
-}
-
 // ------------------------------------------------------------------ norm, rotary, append
 template <class T>
 struct LatentFrontArgs {
@@ -186,6 +181,7 @@ struct LatentAttnArgs {
     T* out;                               // [rows][heads][rank_pad]
     float* part;                          // [rows][splits][heads][rank_pad], then [rows][splits][heads][max, sum]
     float* part_ml;
+    int rows; unsigned groups;            // MFMA kernel: query rows and head groups of the launch
 };
 
 template <class T>
@@ -270,6 +266,7 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(LatentAttnArgs<T> a) {
 // consecutive elements of row i / 4 and receives column i of the 4 x 16 block).
 constexpr int kTile = 32;
 constexpr int kSRow = kTile + 4;      // floats per score row in LDS
+constexpr float kLazy = 8.f;
 
 __host__ __device__ constexpr int tile_pitch(int row) { return 2 * row + 16; }   // bytes: odd multiple of 16 modulo 256
 
@@ -279,8 +276,13 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatentAttnArgs<__
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int g = lane >> 4, n = lane & 15;
-    const int split = blockIdx.x, row = blockIdx.z;
-    const int head0 = blockIdx.y * (16 * MT);
+    // Workgroups go to the eight dies round-robin: the head groups that read the same keys are given to one die, one
+    // behind the other, so that its second-level cache serves all but the first of them.
+    const unsigned die = blockIdx.x & 7u, turn = blockIdx.x >> 3;
+    const unsigned unit = turn / a.groups * 8u + die;
+    if (unit >= (unsigned)(a.rows * a.splits)) return;
+    const int split = (int)(unit % (unsigned)a.splits), row = (int)(unit / (unsigned)a.splits);
+    const int head0 = (int)(turn % a.groups) * (16 * MT);
     const int len = visible_keys(a, row);
     const int tiles = (len + kTile - 1) / kTile;
     const int per = (tiles + a.splits - 1) / a.splits;
@@ -313,37 +315,58 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatentAttnArgs<__
         for (int i = 0; i < NT; ++i) acc[u][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
 
-    // chunk i of this thread: 16 bytes at offset 16 (tid + 256 i) of the tile; its place in LDS
+    // chunk i of this thread: 16 bytes at offset 16 (tid + 256 i) of the tile, and its place in LDS.  Sizes below what the
+    // kernel is built for leave surplus chunks, which repeat the tile's last one (same bytes to the same place), surplus
+    // k-steps, which meet zeros in q, and surplus channel tiles, which are not stored: no branches in the loop.
     const int chunks_per_row = a.row / 8, chunks = kTile * chunks_per_row;
     u32x4_t stage[KSH];
-    int st_lds[KSH];
+    int st_src[KSH], st_lds[KSH];
 #pragma unroll
     for (int i = 0; i < KSH; ++i) {
-        const int c = tid + 256 * i;
+        const int c = tid + 256 * i < chunks ? tid + 256 * i : chunks - 1;
         const int r = c / chunks_per_row;
+        st_src[i] = 16 * c;
         st_lds[i] = r * pitch + (c - r * chunks_per_row) * 16;
     }
-    const int tiles_per_block = a.block_size / kTile;
-    auto fetch = [&](int t) {
-        const int col = t / tiles_per_block;
-        const int blk = block_id(a, bt, col);
-        const __bf16* src = a.cache + ((int64_t)blk * a.block_size + (t - col * tiles_per_block) * kTile) * a.row;
-        const int rows = len - t * kTile;
-        const int have = rows < kTile ? rows * chunks_per_row : chunks;
+    int k_off[KSH];
 #pragma unroll
-        for (int i = 0; i < KSH; ++i) {
-            const int c = tid + 256 * i;
-            stage[i] = u32x4_t{0u, 0u, 0u, 0u};                   // rows behind the last key count as zeros
-            if (c < have) stage[i] = reinterpret_cast<const u32x4_t*>(src)[c];
-        }
+    for (int j = 0; j < KSH; ++j) k_off[j] = __builtin_amdgcn_readfirstlane(2 * j + half < ksteps ? 64 * (2 * j + half) : 0);
+    // tiles are walked in order: the block changes every `tiles_per_block` tiles, and its id is looked up a block ahead
+    const int tiles_per_block = a.block_size / kTile;
+    const int64_t tile_bytes = (int64_t)2 * kTile * a.row;
+    int col = t0 / tiles_per_block, in_block = t0 - col * tiles_per_block;
+    int next_id = block_id(a, bt, col);
+    const unsigned char* src = nullptr;
+    auto open_block = [&]() {
+        src = reinterpret_cast<const unsigned char*>(a.cache) + ((int64_t)next_id * tiles_per_block + in_block) * tile_bytes;
+        ++col;
+        next_id = block_id(a, bt, col < a.table_cols ? col : a.table_cols - 1);
     };
-    if (t0 < t1) fetch(t0);
+    auto fetch = [&]() {
+        if (in_block == tiles_per_block) {
+            in_block = 0;
+            open_block();
+        }
+#pragma unroll
+        for (int i = 0; i < KSH; ++i) stage[i] = *reinterpret_cast<const u32x4_t*>(src + st_src[i]);
+        src += tile_bytes;
+        ++in_block;
+    };
+    if (t0 < t1) {
+        open_block();
+        fetch();
+    }
     for (int t = t0; t < t1; ++t) {
         __syncthreads();
+        if (len - t * kTile < kTile) {                            // rows behind the last key count as zeros
+            const int have = 16 * (len - t * kTile) * chunks_per_row;
 #pragma unroll
-        for (int i = 0; i < KSH; ++i)
-            if (tid + 256 * i < chunks) *reinterpret_cast<u32x4_t*>(lds + st_lds[i]) = stage[i];
-        if (t + 1 < t1) fetch(t + 1);
+            for (int i = 0; i < KSH; ++i)
+                if (st_src[i] >= have) stage[i] = u32x4_t{0u, 0u, 0u, 0u};
+        }
+#pragma unroll
+        for (int i = 0; i < KSH; ++i) *reinterpret_cast<u32x4_t*>(lds + st_lds[i]) = stage[i];
+        if (t + 1 < t1) fetch();
         __syncthreads();
         // ---- scores
         f32x4_t sc[MT];
@@ -352,18 +375,16 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatentAttnArgs<__
         const unsigned char* kr = lds + (16 * ktile + n) * pitch + 16 * g;
 #pragma unroll
         for (int j = 0; j < KSH; ++j) {
-            const int s = 2 * j + half;
-            if (s < ksteps) {
-                const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(kr + 64 * s);
+            const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(kr + k_off[j]);
 #pragma unroll
-                for (int u = 0; u < MT; ++u) sc[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, q[u][j], sc[u], 0, 0, 0);
-            }
+            for (int u = 0; u < MT; ++u) sc[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, q[u][j], sc[u], 0, 0, 0);
         }
 #pragma unroll
         for (int u = 0; u < MT; ++u)
             *reinterpret_cast<f32x4_t*>(sbuf + (half * MT * 16 + 16 * u + n) * kSRow + 16 * ktile + 4 * g) = sc[u];
         __syncthreads();
-        // ---- softmax over the 32 keys, in every wavefront: lane (g, n) has keys 8 g .. 8 g + 7 of head n
+        // ---- softmax over the 32 keys, in every wavefront: lane (g, n) has keys 8 g .. 8 g + 7 of head n.  The running
+        // maximum moves only when it grows by more than kLazy (log2 units); until then weights are at most 2^kLazy.
         bf16x8_t pb[MT];
         const int seen = len - t * kTile - 8 * g;       // of this lane's keys the first `seen` exist
 #pragma unroll
@@ -375,42 +396,42 @@ __global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatentAttnArgs<__
             for (int e = 0; e < 2; ++e) {
                 const f32x4_t x = *reinterpret_cast<const f32x4_t*>(s0 + 4 * e), y = *reinterpret_cast<const f32x4_t*>(s1 + 4 * e);
 #pragma unroll
-                for (int i = 0; i < 4; ++i) sv[4 * e + i] = x[i] + y[i];
+                for (int i = 0; i < 4; ++i) sv[4 * e + i] = (x[i] + y[i]) * a.scale_log2;
             }
-            float mx = -INFINITY;
+            if (len - t * kTile < kTile) {
 #pragma unroll
-            for (int i = 0; i < 8; ++i) {
-                sv[i] = i < seen ? sv[i] * a.scale_log2 : -INFINITY;
-                mx = fmaxf(mx, sv[i]);
+                for (int i = 0; i < 8; ++i) sv[i] = i < seen ? sv[i] : -INFINITY;
             }
-            const float mn = fmaxf(m[u], max_xor16_32(mx));
-            const float alpha = __builtin_amdgcn_exp2f(m[u] - mn);
-            m[u] = mn;
-            float sum = 0.f;
+            float mx = sv[0];
 #pragma unroll
-            for (int i = 0; i < 8; ++i) {
-                const float p = __builtin_amdgcn_exp2f(sv[i] - mn);
-                sum += p;
-                pb[u][i] = (__bf16)p;
-            }
-            l[u] = l[u] * alpha + sum;
-            if (__any(alpha != 1.f)) {
+            for (int i = 1; i < 8; ++i) mx = fmaxf(mx, sv[i]);
+            mx = max_xor16_32(mx);
+            const bool grow = mx > m[u] + kLazy;        // always in the first tile, whose first key exists
+            if (__any(grow)) {
+                const float alpha = grow ? __builtin_amdgcn_exp2f(m[u] - mx) : 1.f;
+                m[u] = grow ? mx : m[u];
+                l[u] *= alpha;
 #pragma unroll
                 for (int i = 0; i < NT; ++i) acc[u][i] *= alpha;
             }
+            float sum = 0.f;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                const float p = __builtin_amdgcn_exp2f(sv[i] - m[u]);
+                sum += p;
+                pb[u][i] = (__bf16)p;
+            }
+            l[u] += sum;
         }
         // ---- weighted sum of the c parts
-        const unsigned char* vr = lds + (8 * g + (n >> 2)) * pitch + (n & 3) * 8;
+        const unsigned char* vr = lds + (8 * g + (n >> 2)) * pitch + (n & 3) * 8 + 32 * wave;
 #pragma unroll
         for (int i = 0; i < NT; ++i) {
-            const int ct = wave + 4 * i;
-            if (ct < ctiles) {
-                const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 32 * ct));
-                const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 32 * ct + 4 * pitch));
-                const bf16x8_t vt = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+            const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 128 * i));
+            const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 128 * i + 4 * pitch));
+            const bf16x8_t vt = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
 #pragma unroll
-                for (int u = 0; u < MT; ++u) acc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pb[u], acc[u][i], 0, 0, 0);
-            }
+            for (int u = 0; u < MT; ++u) acc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pb[u], acc[u][i], 0, 0, 0);
         }
     }
 #pragma unroll
@@ -526,9 +547,12 @@ bool mfma_attention_fits(int64_t row, int64_t rank_pad, int64_t block_size) {
 }
 
 template <int KSH, int NT>
-int launch_decode(const LatentAttnArgs<__bf16>& a, int64_t rows, hipStream_t st) {
+int launch_decode(LatentAttnArgs<__bf16>& a, hipStream_t st) {
     const int mt = a.heads > 16 ? 2 : 1;
-    const dim3 grid((unsigned)a.splits, (unsigned)((a.heads + 16 * mt - 1) / (16 * mt)), (unsigned)rows), block(256);
+    a.groups = (unsigned)((a.heads + 16 * mt - 1) / (16 * mt));
+    const int64_t units = ((int64_t)a.rows * a.splits + 7) / 8 * 8;
+    if (units * a.groups > 0x7fffffff) return INFER_KV_EINVAL;
+    const dim3 grid((unsigned)(units * a.groups)), block(256);
     const size_t lds = (size_t)kTile * tile_pitch(a.row) + (size_t)2 * mt * 16 * kSRow * sizeof(float);
     if (mt == 2) hipLaunchKernelGGL((latent_decode_kernel<2, KSH, NT>), grid, block, lds, st, a);
     else hipLaunchKernelGGL((latent_decode_kernel<1, KSH, NT>), grid, block, lds, st, a);
@@ -630,36 +654,25 @@ extern "C" int infer_latent_attention(int elem, const void* qx, const void* cach
     const float scale_log2 = scale * kLog2e;
     if (elem == INFER_ELEM_F32) {
         LatentAttnArgs<float> a{(const float*)qx, (const float*)cache, (int)row, (int)rank_pad, block_table, bt_stride, (int)table_cols,
-                                (int)block_size, (int)num_blocks, row_seq, ctx, (int)heads, 1, scale_log2, (float*)out, nullptr, nullptr};
+                                (int)block_size, (int)num_blocks, row_seq, ctx, (int)heads, 1, scale_log2, (float*)out, nullptr, nullptr, (int)rows, 1};
         return launch_rows(a, rows, st);
     }
     if (elem != INFER_ELEM_BF16) return INFER_KV_EUNSUPPORTED;
     LatentAttnArgs<__bf16> a{(const __bf16*)qx, (const __bf16*)cache, (int)row, (int)rank_pad, block_table, bt_stride, (int)table_cols,
                              (int)block_size, (int)num_blocks, row_seq, ctx, (int)heads, (int)splits, scale_log2, (__bf16*)out,
-                             workspace, workspace ? workspace + rows * splits * heads * rank_pad : nullptr};
+                             workspace, workspace ? workspace + rows * splits * heads * rank_pad : nullptr, (int)rows, 1};
     if (!mfma_attention_fits(row, rank_pad, block_size) || !ptr_aligned(qx, 16) || !ptr_aligned(cache, 16) || !ptr_aligned(out, 8)) {
         a.splits = 1;
         return launch_rows(a, rows, st);
     }
     if (splits > 1 && (!workspace || !ptr_aligned(workspace, 16) || workspace_floats < rows * splits * heads * (rank_pad + 2)))
         return INFER_KV_EWORKSPACE;
-    int64_t done = 0;
-    while (done < rows) {           // the grid's z extent is 16 bits
-        const int64_t n = rows - done < 65535 ? rows - done : 65535;
-        LatentAttnArgs<__bf16> b = a;
-        b.qx += done * heads * row;
-        b.out += done * heads * rank_pad;
-        b.ctx += done;
-        if (b.row_seq) b.row_seq += done; else b.bt += done * bt_stride;
-        if (splits > 1) { b.part += done * splits * heads * rank_pad; b.part_ml += 2 * done * splits * heads; }
-        int rc;
-        if (row <= 192 && rank_pad <= 128) rc = launch_decode<3, 2>(b, n, st);
-        else if (row <= 384 && rank_pad <= 256) rc = launch_decode<6, 4>(b, n, st);
-        else if (row <= 576) rc = launch_decode<9, 8>(b, n, st);
-        else rc = launch_decode<10, 8>(b, n, st);
-        if (rc) return rc;
-        done += n;
-    }
+    int rc;
+    if (row <= 192 && rank_pad <= 128) rc = launch_decode<3, 2>(a, st);
+    else if (row <= 384 && rank_pad <= 256) rc = launch_decode<6, 4>(a, st);
+    else if (row <= 576) rc = launch_decode<9, 8>(a, st);
+    else rc = launch_decode<10, 8>(a, st);
+    if (rc) return rc;
     if (splits > 1) hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)rows, (unsigned)heads), dim3(128), 0, st, a);
     return (int)hipGetLastError();
 }

@@ -35,17 +35,6 @@ struct LatentPrefillArgs {
     float scale_log2;
 };
 
-__device__ __forceinline__ float max_xor16_32(float x) {
-    const unsigned u = __builtin_bit_cast(unsigned, x);
-    const auto r = __builtin_amdgcn_permlane16_swap(u, u, false, false);
-    const unsigned a0 = r[0], a1 = r[1];
-    const float y = fmaxf(__builtin_bit_cast(float, a0), __builtin_bit_cast(float, a1));
-    const unsigned w = __builtin_bit_cast(unsigned, y);
-    const auto s = __builtin_amdgcn_permlane32_swap(w, w, false, false);
-    const unsigned b0 = s[0], b1 = s[1];
-    return fmaxf(__builtin_bit_cast(float, b0), __builtin_bit_cast(float, b1));
-}
-
 template <int KS, int VT>
 __global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPrefillArgs a) {
     constexpr int kKPitch = KS * 64 + 16, kVPitch = VT * 32 + 16;              // bytes
