@@ -333,7 +333,7 @@ def hybrid_kernels(heads=32, width=4096, ff=12288):
     # ---- front end and per-head products
     table = yarn_rotary_table(rot, 8192, 1e6, None, dev)
     for t in (b, n * sq):
-        proj = rnd(t, heads * (dim + rot) + row + heads)
+        proj = rnd(t, -(-(heads * (dim + rot) + row + heads) // 64) * 64)        # rows of a PackedLinear
         pos = torch.randint(0, 8192, (t,), device=dev)
         slots = torch.randperm(nblk * bs, device=dev)[:t].to(torch.int32)
         decode = t == b

@@ -35,7 +35,31 @@ struct LatentFrontArgs {
     T* qx; int64_t qx_rows;                // rows below qx_rows: rotated q to qx[row][head][rank_pad ..], others in place
 };
 
-template <class T>
+// a rotated pair in one access where every pair is aligned to its size (EVEN)
+template <bool EVEN, class T>
+__device__ __forceinline__ void load_pair(const T* p, float& u, float& v) {
+    struct alignas(2 * sizeof(T)) Pair { T u, v; };
+    if constexpr (EVEN) {
+        const Pair x = *reinterpret_cast<const Pair*>(p);
+        u = (float)x.u;
+        v = (float)x.v;
+    } else {
+        u = (float)p[0];
+        v = (float)p[1];
+    }
+}
+template <bool EVEN, class T>
+__device__ __forceinline__ void store_pair(T* p, float u, float v) {
+    struct alignas(2 * sizeof(T)) Pair { T u, v; };
+    if constexpr (EVEN) {
+        *reinterpret_cast<Pair*>(p) = Pair{(T)u, (T)v};
+    } else {
+        p[0] = (T)u;
+        p[1] = (T)v;
+    }
+}
+
+template <class T, bool EVEN>
 __global__ void __launch_bounds__(256) latent_front_kernel(LatentFrontArgs<T> a) {
     const int64_t t = blockIdx.x;
     const int tid = threadIdx.x;
@@ -59,8 +83,7 @@ __global__ void __launch_bounds__(256) latent_front_kernel(LatentFrontArgs<T> a)
         for (int i = tid; i < (a.row - a.rank_pad) / 2; i += 256) {
             float u = 0.f, v = 0.f;
             if (2 * i < a.rot) {
-                u = (float)kv[a.rank + 2 * i];
-                v = (float)kv[a.rank + 2 * i + 1];
+                load_pair<EVEN>(kv + a.rank + 2 * i, u, v);
                 if (i < a.rot_pairs) {
                     const float c = cs[2 * i], s = cs[2 * i + 1];
                     const float u2 = u * c - v * s;
@@ -68,29 +91,30 @@ __global__ void __launch_bounds__(256) latent_front_kernel(LatentFrontArgs<T> a)
                     u = u2;
                 }
             }
-            row[a.rank_pad + 2 * i] = (T)u;
-            row[a.rank_pad + 2 * i + 1] = (T)v;
+            store_pair<EVEN>(row + a.rank_pad + 2 * i, u, v);
         }
     }
     const bool to_qx = t < a.qx_rows;
-    const int pairs = to_qx ? (a.row - a.rank_pad) / 2 : a.rot / 2;
-    for (int i = tid; i < a.heads * pairs; i += 256) {
-        const int h = i / pairs, p = i - h * pairs;
-        T* q = pr + (int64_t)h * (a.dim + a.rot) + a.dim;
-        float u = 0.f, v = 0.f;
-        if (2 * p < a.rot) {
-            u = (float)q[2 * p];
-            v = (float)q[2 * p + 1];
-            if (p < a.rot_pairs) {
-                const float c = cs[2 * p], s = cs[2 * p + 1];
-                const float u2 = u * c - v * s;
-                v = v * c + u * s;
-                u = u2;
-            }
+    const int pairs = to_qx ? (a.row - a.rank_pad) / 2 : a.rot / 2, total = a.heads * pairs;
+    T* qx = to_qx ? a.qx + t * a.heads * a.row + a.rank_pad : pr + a.dim;
+    const int qx_head = to_qx ? a.row : a.dim + a.rot;
+    // four pairs per thread at a time, all loads in front of the stores
+    for (int i0 = tid; i0 < total; i0 += 4 * 256) {
+        float u[4], v[4], c[4], s[4];
+        int h[4], p[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int i = i0 + 256 * k < total ? i0 + 256 * k : i0;
+            h[k] = i / pairs;
+            p[k] = i - h[k] * pairs;
+            u[k] = v[k] = s[k] = 0.f;
+            c[k] = 1.f;
+            if (2 * p[k] < a.rot) load_pair<EVEN>(pr + h[k] * (a.dim + a.rot) + a.dim + 2 * p[k], u[k], v[k]);
+            if (p[k] < a.rot_pairs) { c[k] = cs[2 * p[k]]; s[k] = cs[2 * p[k] + 1]; }
         }
-        T* dst = to_qx ? a.qx + (t * a.heads + h) * a.row + a.rank_pad : q;
-        dst[2 * p] = (T)u;
-        dst[2 * p + 1] = (T)v;
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+            if (i0 + 256 * k < total) store_pair<EVEN>(qx + h[k] * qx_head + 2 * p[k], u[k] * c[k] - v[k] * s[k], v[k] * c[k] + u[k] * s[k]);
     }
 }
 
@@ -526,7 +550,11 @@ bool size_in(int64_t v, int64_t lo, int64_t hi) { return v >= lo && v <= hi; }
 
 template <class T>
 int launch_front(const LatentFrontArgs<T>& a, int64_t n, hipStream_t st) {
-    hipLaunchKernelGGL((latent_front_kernel<T>), dim3((unsigned)n), dim3(256), 0, st, a);
+    const size_t pair = 2 * sizeof(T);
+    const bool even = a.dim % 2 == 0 && a.rank % 2 == 0 && a.kv_off % 2 == 0 && a.proj_stride % 2 == 0 && ptr_aligned(a.proj, pair) &&
+                      ptr_aligned(a.cache, pair) && ptr_aligned(a.qx, pair);
+    if (even) hipLaunchKernelGGL((latent_front_kernel<T, true>), dim3((unsigned)n), dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((latent_front_kernel<T, false>), dim3((unsigned)n), dim3(256), 0, st, a);
     return (int)hipGetLastError();
 }
 

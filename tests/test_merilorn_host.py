@@ -152,7 +152,7 @@ def test_every_tensor_lands_in_its_place(tmp_path):
 
 def test_packed_linear_pieces_start_aligned():
     lin = PackedLinear(4, {"q": 6, "k": 3, "v": 5, "b": 2}, torch.float32, dense=("q",))
-    assert lin.offset == {"q": 0, "k": 6, "v": 16, "b": 24} and lin.weight.shape == (32, 4)
+    assert lin.offset == {"q": 0, "k": 6, "v": 16, "b": 24} and lin.weight.shape == (64, 4)
     lin.weight_loader(lin.weight, torch.ones(5, 4), "v")
     assert float(lin.weight.sum()) == 20
     with pytest.raises(ValueError):
