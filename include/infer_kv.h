@@ -343,9 +343,24 @@ int infer_residual_norm(int elem, const int64_t* tokens, const void* embed, floa
                         int64_t partial_stride, const float* w_post, float* x, int64_t x_stride, const float* w_pre,
                         void* h, int64_t h_stride, int64_t n_rows, int64_t width, float eps, void* stream);
 
+/* The same stream with the norm behind the sum (post-norm):
+ *   x = embed[tokens[row]] * embed_scale                    if tokens,
+ *   x = z / sqrt(mean(z^2) + eps) * w_post, z = alpha * x + y
+ *                                                           if y or partial, as above,
+ *   h = x, or x / sqrt(mean(x^2) + eps) * w_last if w_last  (always written). */
+int infer_post_norm(int elem, const int64_t* tokens, const void* embed, float embed_scale, int64_t vocab,
+                    const void* y, int64_t y_stride, const float* partial, int64_t splits, int64_t split_stride,
+                    int64_t partial_stride, float alpha, const float* w_post, float* x, int64_t x_stride,
+                    const float* w_last, void* h, int64_t h_stride, int64_t n_rows, int64_t width, float eps,
+                    void* stream);
+
 /* out[r, j] = gelu_tanh(x[r, j]) * x[r, d + j]. */
 int infer_gelu_tanh_and_mul(int elem, void* out, int64_t out_stride, const void* x, int64_t x_stride,
                             int64_t n_rows, int64_t d, void* stream);
+/* out[r, j] = silu(x[r, j]) * x[r, d + j], any d and strides (infer_silu_and_mul_bf16 rounds silu(x) to bf16
+ * before the product, as the operator it replaces does; this one does not). */
+int infer_silu_and_mul(int elem, void* out, int64_t out_stride, const void* x, int64_t x_stride,
+                       int64_t n_rows, int64_t d, void* stream);
 
 /* Front end of latent attention.  A token's projection row holds q (heads x [dim | rot]) at column 0 and
  * [latent: rank | rotated key part: rot] at column kv_off.  The latent is RMS-normed (c_norm), the first
@@ -393,6 +408,66 @@ int infer_latent_prefill(const void* q, int64_t q_stride, const void* kp, int64_
                          void* out, int64_t out_stride, const int32_t* cu_q, const int32_t* cu_k, int64_t num_seqs,
                          int64_t max_seqlen_q, int64_t heads, int64_t dim, int64_t rot, int64_t vdim, float scale,
                          void* stream);
+
+/* Grouped attention with separate keys and values: heads / kv_heads consecutive query heads share a key/value head.
+ * Pages are [blocks][kv_heads][block_size][vdim_pad + dim_pad], a row holding the value, zeros, the key, zeros; both
+ * parts are padded to 32 elements.
+ *
+ * infer_grouped_front: a token's projection row holds q (heads x dim) at column 0, k (kv_heads x dim) at k_off and v
+ * (kv_heads x vdim) at v_off.  bias (per column, NULL: none) is added to all three; q and k are divided by the root
+ * mean square of the WHOLE projection and multiplied by q_norm / k_norm (NULL: no norm); the first rot_dims entries of
+ * every head turn by the token's position (interleaved pairs; table[pos] = cos, sin per pair); keys and values are
+ * stored at slots[t] (negative: skipped).  kv_heads = 0: only q, the keys are another layer's.  Rows below qx_rows get
+ * their q in qx[t][head][dim_pad], zero padded, the others in place.
+ *
+ * infer_grouped_attention: query rows against pages, as infer_latent_attention.  sink (NULL: none) is a score per head
+ * that enters the softmax denominator and is not scaled; gate (NULL: none) multiplies a head's output by
+ * sigmoid(gate[row][head]).  out[row][heads * vdim].
+ *
+ * infer_grouped_gather: as infer_latent_gather, out[.][kv_heads][row].
+ * infer_grouped_prefill: as infer_latent_prefill over dense keys and values (bf16); head h reads key head
+ * h / (heads / kv_heads), at k + that * k_head. */
+int infer_grouped_front(int elem, void* proj, int64_t proj_stride, int64_t heads, int64_t kv_heads, int64_t dim,
+                        int64_t vdim, int64_t k_off, int64_t v_off, const float* bias, const float* q_norm,
+                        const float* k_norm, float eps, const float* table, int64_t rot_dims, int64_t max_pos,
+                        const int64_t* positions, const int32_t* slots, void* cache, int64_t block_size,
+                        int64_t dim_pad, int64_t vdim_pad, int64_t num_slots, void* qx, int64_t qx_rows, int64_t n,
+                        void* stream);
+int64_t infer_grouped_attention_splits(int elem, int64_t rows, int64_t heads, int64_t kv_heads, int64_t dim_pad,
+                                       int64_t vdim_pad, int64_t block_size, int64_t max_keys);
+int infer_grouped_attention(int elem, const void* qx, const void* cache, int64_t dim_pad, int64_t vdim_pad,
+                            const int32_t* block_table, int64_t bt_stride, int64_t table_cols, int64_t block_size,
+                            int64_t num_blocks, const int32_t* row_seq, const int32_t* ctx, int64_t rows,
+                            int64_t heads, int64_t kv_heads, float scale, const float* sink, const void* gate,
+                            int64_t gate_stride, int64_t splits, void* out, int64_t out_stride, int64_t vdim,
+                            float* workspace, int64_t workspace_floats, void* stream);
+int infer_grouped_gather(const void* cache, int64_t row, int64_t kv_heads, int64_t block_size, int64_t num_blocks,
+                         const int32_t* block_table, int64_t bt_stride, int64_t table_cols, const int32_t* seqs,
+                         const int32_t* cu_k, int64_t num_seqs, int64_t max_keys, void* out, void* stream);
+int infer_grouped_prefill_supported(int64_t dim, int64_t vdim);
+int infer_grouped_prefill(const void* q, int64_t q_stride, const void* k, int64_t k_stride, int64_t k_head, const void* v,
+                          int64_t v_stride, int64_t v_head, const float* sink, const void* gate, int64_t gate_stride,
+                          void* out, int64_t out_stride, const int32_t* cu_q, const int32_t* cu_k, int64_t num_seqs,
+                          int64_t max_seqlen_q, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, float scale,
+                          void* stream);
+
+/* Linear attention with a constant decay d per head: S = d S + k v^T, o = scale * S^T q, S[dim][vdim] float32.  A
+ * token's projection row holds q, k (heads x dim), v and the gate logits (heads x vdim) at q_off, k_off, v_off and
+ * g_off.  silu: q, k and v go through silu; rot_dims > 0: the first rot_dims entries of every head of q and k turn by
+ * the token's position, entry i with entry i + rot_dims / 2 (table[pos] = cos, sin per pair).  decay[3][heads] = d
+ * rounded to float, d minus that, log2(d).  o is divided by its root mean square over the head (norm_per_head) or over
+ * all heads, multiplied by norm[heads * vdim] (NULL: ones) and by sigmoid or silu of the gate.
+ * Rows below decode_rows are single tokens with the state of slots[row] at positions[row] (a negative slot is padding:
+ * zeros come out); the others belong to spans[.][4] = first row, tokens, slot, first position, two tokens or more.
+ * state[slots][heads][rows][columns] (infer_decay_layout: [0] rows, [1] columns); a sequence at position 0 starts from
+ * zero whatever it holds. */
+int infer_decay_layout(int64_t dim, int64_t vdim, int64_t* out2);
+int infer_decay_attention(int elem, const void* proj, int64_t proj_stride, int64_t q_off, int64_t k_off, int64_t v_off,
+                          int64_t g_off, int64_t heads, int64_t dim, int64_t vdim, const float* decay, int silu,
+                          const float* table, int64_t rot_dims, int64_t max_pos, float scale, const float* norm,
+                          int norm_per_head, int gate_silu, float eps, float* state, int64_t num_slots,
+                          const int32_t* slots, const int64_t* positions, int64_t decode_rows, const int32_t* spans,
+                          int64_t num_spans, int64_t rows, void* out, int64_t out_stride, void* stream);
 
 /* Gated delta rule with a decay per key channel.  A token's projection row holds the inputs of the short
  * convolution, q and k (kv_heads x dim each) and v (heads x vdim), from column 0 and the write-strength

@@ -51,6 +51,9 @@ SIGNATURES = {
     "infer_residual_norm": (_c.c_int, [_c.c_int, _vp, _vp, _f32, _i64, _vp, _i64, _vp, _i64, _i64, _i64, _vp,
                                        _vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
     "infer_gelu_tanh_and_mul": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _i64, _i64, _i64, _vp]),
+    "infer_post_norm": (_c.c_int, [_c.c_int, _vp, _vp, _f32, _i64, _vp, _i64, _vp, _i64, _i64, _i64, _f32, _vp,
+                                   _vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
+    "infer_silu_and_mul": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _i64, _i64, _i64, _vp]),
     "infer_latent_front": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _f32, _vp,
                                       _i64, _vp, _vp, _vp, _i64, _i64, _i64, _vp, _i64, _i64, _vp]),
     "infer_head_matmul": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _i64,
@@ -62,6 +65,22 @@ SIGNATURES = {
     "infer_latent_prefill_supported": (_c.c_int, [_i64, _i64, _i64]),
     "infer_latent_prefill": (_c.c_int, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp,
                                         _vp, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp]),
+    "infer_grouped_front": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _vp, _vp, _f32,
+                                       _vp, _i64, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp, _i64, _i64,
+                                       _vp]),
+    "infer_grouped_attention_splits": (_i64, [_c.c_int, _i64, _i64, _i64, _i64, _i64, _i64, _i64]),
+    "infer_grouped_attention": (_c.c_int, [_c.c_int, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i64, _i64, _vp, _vp,
+                                           _i64, _i64, _i64, _f32, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _vp,
+                                           _i64, _vp]),
+    "infer_grouped_gather": (_c.c_int, [_vp, _i64, _i64, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _i64, _i64, _vp,
+                                        _vp]),
+    "infer_grouped_prefill_supported": (_c.c_int, [_i64, _i64]),
+    "infer_grouped_prefill": (_c.c_int, [_vp, _i64, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _i64, _vp, _i64,
+                                         _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp]),
+    "infer_decay_layout": (_c.c_int, [_i64, _i64, _vp]),
+    "infer_decay_attention": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _c.c_int,
+                                         _vp, _i64, _i64, _f32, _vp, _c.c_int, _c.c_int, _f32, _vp, _i64, _vp, _vp,
+                                         _i64, _vp, _i64, _i64, _vp, _i64, _vp]),
     "infer_delta_layout": (_c.c_int, [_i64, _i64, _vp]),
     "infer_delta_step": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp,
                                     _vp, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp, _vp, _vp, _i64, _i64,

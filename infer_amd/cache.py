@@ -40,6 +40,32 @@ class LatentPages:
         return torch.zeros(num_blocks, block_size, self.row, dtype=self.dtype, device=device)
 
 
+class GroupedPages:
+    """A row ``[value | key]`` of ``row`` elements per token and key/value head."""
+
+    def __init__(self, kv_heads: int, row: int, dtype: torch.dtype):
+        self.kv_heads, self.row, self.dtype = kv_heads, row, dtype
+
+    def block_bytes(self, block_size: int) -> int:
+        return block_size * self.kv_heads * self.row * self.dtype.itemsize
+
+    slot_bytes = 0
+
+    def allocate(self, num_blocks: int, num_slots: int, block_size: int, device):
+        return torch.zeros(num_blocks, self.kv_heads, block_size, self.row, dtype=self.dtype, device=device)
+
+
+class SharedStorage:
+    """A layer that keeps nothing of its own and reads what the earlier layer ``owner`` keeps."""
+    slot_bytes = 0
+
+    def __init__(self, owner: int):
+        self.owner = owner
+
+    def block_bytes(self, block_size: int) -> int:
+        return 0
+
+
 class StateSlots:
     """Named tensors per running sequence: ``name=(shape, dtype)``."""
 
@@ -67,4 +93,8 @@ class LayeredLayout:
         self.slot_bytes = sum(layer.slot_bytes for layer in layers)
 
     def allocate(self, num_blocks: int, num_slots: int, device) -> list:
-        return [layer.allocate(num_blocks, num_slots, self.block_size, device) for layer in self.layers]
+        storage: list = []
+        for layer in self.layers:
+            shared = isinstance(layer, SharedStorage)
+            storage.append(storage[layer.owner] if shared else layer.allocate(num_blocks, num_slots, self.block_size, device))
+        return storage

@@ -84,6 +84,16 @@ class LayerSpec:
     owner: int
 
 
+def dense_width(entry: dict, index: int) -> int | None:
+    """The width of a layer's dense feed-forward, None if it has none."""
+    mlp = entry.get("mlp")
+    if mlp is None:
+        return None
+    if mlp["kind"] != "dense":
+        raise ValueError(f"layer {index}: feed-forward kind {mlp['kind']!r} is not known")
+    return mlp["ff"]
+
+
 @dataclass
 class MerilornConfig:
     """Merilorn: ``layers`` in order, each latent attention or a gated delta rule, norms on both sides of every
@@ -113,17 +123,44 @@ class MerilornConfig:
         for i, entry in enumerate(raw["layers"]):
             owner = entry.get("weights_of", i)
             owner = i if owner is None else int(owner)
-            mixer, mlp = dict(entry["mixer"]), entry.get("mlp")
-            if mlp is not None and mlp["kind"] != "dense":
-                raise ValueError(f"layer {i}: feed-forward kind {mlp['kind']!r} is not known")
+            mixer = dict(entry["mixer"])
             if entry["type"] == "channel_delta":
                 for key, tensor in (("decay_rank", "a1"), ("gate_rank", "g1")):
                     name = f"l{owner}.mix.{tensor}"
                     if name in shapes:
                         mixer[key] = shapes[name][0]
-            layers.append(LayerSpec(entry["type"], mixer, mlp["ff"] if mlp is not None else None, owner))
+            layers.append(LayerSpec(entry["type"], mixer, dense_width(entry, i), owner))
         return cls(vocab_size=raw["vocab"], hidden_size=raw["width"], layers=layers, norm_eps=raw["norm"]["eps"],
                    embedding_scale=raw["embedding"]["scale"])
+
+
+@dataclass
+class VokelixConfig:
+    """Vokelix: ``layers`` in order, each grouped attention, lightning or retention, and a norm behind every residual sum
+    ``residual_alpha * x + sublayer(x)``.  The mixer of an attention layer with ``kv_from`` reads the keys and values of
+    that earlier layer."""
+    vocab_size: int
+    hidden_size: int
+    layers: list[LayerSpec] = field(default_factory=list)
+    norm_eps: float = 1e-6
+    residual_alpha: float = 1.0
+    max_position_embeddings: int = 1 << 20          # the design sets no bound; ``max_model_len`` does
+    torch_dtype: torch.dtype = torch.bfloat16
+
+    block_multiple = 32
+    dtypes = (torch.bfloat16, torch.float32)
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_json(cls, path: str) -> "VokelixConfig":
+        with open(path) as f:
+            raw = json.load(f)
+        layers = [LayerSpec(e["type"], dict(e["mixer"]), dense_width(e, i), i) for i, e in enumerate(raw["layers"])]
+        return cls(vocab_size=raw["vocab"], hidden_size=raw["width"], layers=layers, norm_eps=raw["norm"]["eps"],
+                   residual_alpha=raw["postln_alpha"])
 
 
 def load_model_config(directory: str):
@@ -139,7 +176,7 @@ def load_model_config(directory: str):
     raise ValueError(f"no model of this package serves {names}; known: {sorted(CONFIG_CLASSES)}")
 
 
-CONFIG_CLASSES = {"Qwen3ForCausalLM": ModelConfig, "Merilorn": MerilornConfig}
+CONFIG_CLASSES = {"Qwen3ForCausalLM": ModelConfig, "Merilorn": MerilornConfig, "Vokelix": VokelixConfig}
 
 
 @dataclass
@@ -151,7 +188,7 @@ class Config:
     gpu_memory_utilization: float = 0.9
     tensor_parallel_size: int = 1
     enforce_eager: bool = False
-    hf_config: ModelConfig | MerilornConfig | None = None
+    hf_config: ModelConfig | MerilornConfig | VokelixConfig | None = None
     eos: int = -1
     kvcache_block_size: int = 256
     num_kvcache_blocks: int = -1

@@ -1,6 +1,7 @@
-// Causal attention of long prompt portions whose keys come out of a latent: every head has its own unrotated
-// key part and value (W_uk c and W_uv c, dense rows), and one rotated key part is shared by all heads.  bf16 in,
-// float32 accumulate, output gate in the epilogue.
+// Causal attention of long prompt portions over dense keys and values, for gfx950 (MI355X).  bf16 in, float32
+// accumulate, output gate and softmax sink in the epilogue.  A key has two parts, either of which may be absent: one
+// that the heads of a group share (latent attention: W_uk c, a group of one; grouped attention: the whole key), and
+// one that all heads share (latent attention: the rotated part).
 //
 // A wavefront owns 32 queries (two MFMA column tiles) of one head, a workgroup four wavefronts = 128
 // consecutive queries, and walks the visible keys in steps of 32 that all four share through LDS (two
@@ -22,12 +23,14 @@ constexpr int kWaves = 4;
 constexpr int kQ = 32 * kWaves;         // queries per workgroup
 constexpr float kLazy = 8.f;            // log2 units a row's maximum may grow before the accumulators are rescaled
 
-struct LatentPrefillArgs {
+struct DensePrefillArgs {
     const __bf16* q; int64_t q_stride;        // [token][head * (dim + rot)]
-    const __bf16* kp; int64_t kp_stride;      // [key][head * dim]
+    const __bf16* kp; int64_t kp_stride; int kp_head;   // [key][group of heads][dim]
     const __bf16* kr; int64_t kr_stride;      // [key][rot]
-    const __bf16* v; int64_t v_stride;        // [key][head * vdim]
+    const __bf16* v; int64_t v_stride; int v_head;      // [key][group of heads][vdim]
     const __bf16* gate; int64_t gate_stride;  // [token][head]
+    const float* sink;                        // [head] or nullptr
+    int group;                                // heads that share keys and values
     __bf16* out; int64_t out_stride;          // [token][head * vdim]
     const int32_t* cu_q;                      // first token row of each sequence (rows of q, gate, out)
     const int32_t* cu_k;                      // first key row of each
@@ -36,7 +39,7 @@ struct LatentPrefillArgs {
 };
 
 template <int KS, int VT>
-__global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPrefillArgs a) {
+__global__ void __launch_bounds__(64 * kWaves, 2) dense_prefill_kernel(DensePrefillArgs a) {
     constexpr int kKPitch = KS * 64 + 16, kVPitch = VT * 32 + 16;              // bytes
     constexpr int kBuf = kStep * (kKPitch + kVPitch);
     constexpr int kNK = KS * 4 * kStep / 256, kNV = (VT * 2 * kStep + 255) / 256;    // 16-byte chunks per thread
@@ -82,6 +85,7 @@ __global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPr
     for (int i = tid; i < 2 * kBuf / 16; i += 256) reinterpret_cast<u32x4_t*>(lds)[i] = u32x4_t{0u, 0u, 0u, 0u};
 
     // chunk i of this thread of the K and of the V tile: key, place, and a running pointer to its source
+    const int hk = h / a.group;
     const int kc = qk / 8, vc = a.vdim / 8, dc = a.dim / 8;
     constexpr int kN = kNK + kNV;
     int c_key[kN], c_lds[kN], c_str[kN];                         // c_str: elements from one key to the next (checked below 2^24)
@@ -95,8 +99,8 @@ __global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPr
         c_lds[i] = is_k ? key * kKPitch + col * 16 : kStep * kKPitch + key * kVPitch + col * 16;
         const bool rot = is_k && col >= dc;
         c_str[i] = key >= kStep ? 0 : (int)(!is_k ? a.v_stride : rot ? a.kr_stride : a.kp_stride);
-        const __bf16* base = !is_k ? a.v + (int64_t)h * a.vdim + 8 * col
-                             : rot ? a.kr + 8 * (col - dc) : a.kp + (int64_t)h * a.dim + 8 * col;
+        const __bf16* base = !is_k ? a.v + (int64_t)hk * a.v_head + 8 * col
+                             : rot ? a.kr + 8 * (col - dc) : a.kp + (int64_t)hk * a.kp_head + 8 * col;
         c_src[i] = (key < kStep ? base : a.v) + (int64_t)(k_beg + key) * c_str[i];
     }
     // Two steps are under way in registers while a third is consumed from LDS: a step is shorter than the
@@ -210,7 +214,8 @@ __global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPr
     for (int u = 0; u < 2; ++u) {
         const int qi = q0 + 16 * u + n;
         if (qi >= sq) continue;
-        const float l = lacc[u][0];
+        float l = lacc[u][0];
+        if (a.sink && l > 0.f) l += __builtin_amdgcn_exp2f(a.sink[h] * kLog2e + m_neg[u]);
         const float f = (l > 0.f ? 1.f / l : 0.f) * sigmoid_f((float)a.gate[(int64_t)(q_beg + qi) * a.gate_stride + h]);
         __bf16* o = a.out + (int64_t)(q_beg + qi) * a.out_stride + (int64_t)h * a.vdim + 4 * g;
 #pragma unroll
@@ -226,46 +231,71 @@ __global__ void __launch_bounds__(64 * kWaves, 2) latent_prefill_kernel(LatentPr
 
 // (k-steps, value tiles) the kernel is built for, smallest first
 template <int KS, int VT>
-int go(const LatentPrefillArgs& a, unsigned grid, hipStream_t st) {
-    hipLaunchKernelGGL((latent_prefill_kernel<KS, VT>), dim3(grid), dim3(64 * kWaves), 0, st, a);
+int go(const DensePrefillArgs& a, unsigned grid, hipStream_t st) {
+    hipLaunchKernelGGL((dense_prefill_kernel<KS, VT>), dim3(grid), dim3(64 * kWaves), 0, st, a);
     return (int)hipGetLastError();
+}
+
+// the checks that both forms of the entry share, and the launch
+int run(DensePrefillArgs& a, int64_t num_seqs, int64_t max_seqlen_q, float scale, void* stream) {
+    if (num_seqs < 0 || max_seqlen_q < 0) return INFER_KV_EINVAL;
+    if (num_seqs == 0 || max_seqlen_q == 0) return INFER_KV_OK;
+    if (!a.q || !a.kp || !a.v || !a.gate || !a.out || !a.cu_q || !a.cu_k || !(scale > 0.f)) return INFER_KV_EINVAL;
+    const int64_t qk = a.dim + a.rot;
+    if (a.q_stride < a.heads * qk || a.gate_stride < a.heads || a.out_stride < (int64_t)a.heads * a.vdim) return INFER_KV_EINVAL;
+    if (a.kp_stride >= (1 << 24) || a.kr_stride >= (1 << 24) || a.v_stride >= (1 << 24)) return INFER_KV_EINVAL;
+    if (a.q_stride % 8 || a.kp_stride % 8 || a.kr_stride % 8 || a.v_stride % 8 || a.kp_head % 8 || a.v_head % 8 || a.out_stride % 4 ||
+        !ptr_aligned(a.q, 16) || !ptr_aligned(a.kp, 16) || !ptr_aligned(a.kr, 16) || !ptr_aligned(a.v, 16) || !ptr_aligned(a.out, 8))
+        return INFER_KV_EALIGN;
+    const int64_t qblocks = (max_seqlen_q + kQ - 1) / kQ, total = qblocks * num_seqs * a.heads;
+    if (total > 0x7fffffff) return INFER_KV_EINVAL;
+    a.nseq = (int)num_seqs;
+    a.qblocks = (int)qblocks;
+    a.scale_log2 = scale * kLog2e;
+    hipStream_t st = (hipStream_t)stream;
+    const unsigned grid = (unsigned)total;
+    if (qk <= 64 && a.vdim <= 64) return go<2, 4>(a, grid, st);
+    if (qk <= 128 && a.vdim <= 64) return go<4, 4>(a, grid, st);
+    if (qk <= 128) return go<4, 8>(a, grid, st);
+    if (qk <= 192) return go<6, 8>(a, grid, st);
+    return go<8, 8>(a, grid, st);
+}
+
+bool served(int64_t dim, int64_t rot, int64_t vdim) {
+    if (dim <= 0 || rot < 0 || vdim <= 0 || dim % 8 || rot % 8 || vdim % 8) return false;
+    return dim + rot <= 256 && vdim <= 128;
 }
 
 }  // namespace
 
 // 1 if the sizes are served by the kernel
-extern "C" int infer_latent_prefill_supported(int64_t dim, int64_t rot, int64_t vdim) {
-    if (dim <= 0 || rot <= 0 || vdim <= 0 || dim % 8 || rot % 8 || vdim % 8) return 0;
-    return dim + rot <= 256 && vdim <= 128;
-}
+extern "C" int infer_latent_prefill_supported(int64_t dim, int64_t rot, int64_t vdim) { return rot > 0 && served(dim, rot, vdim); }
+extern "C" int infer_grouped_prefill_supported(int64_t dim, int64_t vdim) { return served(dim, 0, vdim); }
 
 extern "C" int infer_latent_prefill(const void* q, int64_t q_stride, const void* kp, int64_t kp_stride, const void* kr,
                                     int64_t kr_stride, const void* v, int64_t v_stride, const void* gate, int64_t gate_stride,
                                     void* out, int64_t out_stride, const int32_t* cu_q, const int32_t* cu_k, int64_t num_seqs,
                                     int64_t max_seqlen_q, int64_t heads, int64_t dim, int64_t rot, int64_t vdim, float scale,
                                     void* stream) {
-    if (num_seqs < 0 || max_seqlen_q < 0) return INFER_KV_EINVAL;
-    if (num_seqs == 0 || max_seqlen_q == 0) return INFER_KV_OK;
-    if (!q || !kp || !kr || !v || !gate || !out || !cu_q || !cu_k || heads < 1 || heads > 4096 || !(scale > 0.f)) return INFER_KV_EINVAL;
-    if (!infer_latent_prefill_supported(dim, rot, vdim)) return INFER_KV_EUNSUPPORTED;
-    if (q_stride < heads * (dim + rot) || kp_stride < heads * dim || kr_stride < rot || v_stride < heads * vdim ||
-        gate_stride < heads || out_stride < heads * vdim)
+    if (heads < 1 || heads > 4096 || !infer_latent_prefill_supported(dim, rot, vdim)) return INFER_KV_EUNSUPPORTED;
+    if (!kr || kp_stride < heads * dim || kr_stride < rot || v_stride < heads * vdim) return INFER_KV_EINVAL;
+    DensePrefillArgs a{(const __bf16*)q, q_stride, (const __bf16*)kp, kp_stride, (int)dim, (const __bf16*)kr, kr_stride, (const __bf16*)v,
+                       v_stride, (int)vdim, (const __bf16*)gate, gate_stride, nullptr, 1, (__bf16*)out, out_stride, cu_q, cu_k, (int)heads,
+                       (int)dim, (int)rot, (int)vdim, 0, 0, 0.f};
+    return run(a, num_seqs, max_seqlen_q, scale, stream);
+}
+
+extern "C" int infer_grouped_prefill(const void* q, int64_t q_stride, const void* k, int64_t k_stride, int64_t k_head, const void* v,
+                                     int64_t v_stride, int64_t v_head, const float* sink, const void* gate, int64_t gate_stride,
+                                     void* out, int64_t out_stride, const int32_t* cu_q, const int32_t* cu_k, int64_t num_seqs,
+                                     int64_t max_seqlen_q, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, float scale,
+                                     void* stream) {
+    if (heads < 1 || heads > 4096 || !infer_grouped_prefill_supported(dim, vdim)) return INFER_KV_EUNSUPPORTED;
+    if (kv_heads < 1 || heads % kv_heads || k_head < 0 || v_head < 0 || k_stride < (kv_heads - 1) * k_head + dim ||
+        v_stride < (kv_heads - 1) * v_head + vdim)
         return INFER_KV_EINVAL;
-    if (kp_stride >= (1 << 24) || kr_stride >= (1 << 24) || v_stride >= (1 << 24)) return INFER_KV_EINVAL;
-    if (q_stride % 8 || kp_stride % 8 || kr_stride % 8 || v_stride % 8 || out_stride % 4 || !ptr_aligned(q, 16) || !ptr_aligned(kp, 16) ||
-        !ptr_aligned(kr, 16) || !ptr_aligned(v, 16) || !ptr_aligned(out, 8))
-        return INFER_KV_EALIGN;
-    const int64_t qblocks = (max_seqlen_q + kQ - 1) / kQ, total = qblocks * num_seqs * heads;
-    if (total > 0x7fffffff) return INFER_KV_EINVAL;
-    LatentPrefillArgs a{(const __bf16*)q, q_stride, (const __bf16*)kp, kp_stride, (const __bf16*)kr, kr_stride, (const __bf16*)v,
-                        v_stride, (const __bf16*)gate, gate_stride, (__bf16*)out, out_stride, cu_q, cu_k, (int)heads, (int)dim,
-                        (int)rot, (int)vdim, (int)num_seqs, (int)qblocks, scale * kLog2e};
-    hipStream_t st = (hipStream_t)stream;
-    const int64_t qk = dim + rot;
-    const unsigned grid = (unsigned)total;
-    if (qk <= 64 && vdim <= 64) return go<2, 4>(a, grid, st);
-    if (qk <= 128 && vdim <= 64) return go<4, 4>(a, grid, st);
-    if (qk <= 128) return go<4, 8>(a, grid, st);
-    if (qk <= 192) return go<6, 8>(a, grid, st);
-    return go<8, 8>(a, grid, st);
+    DensePrefillArgs a{(const __bf16*)q, q_stride, (const __bf16*)k, k_stride, (int)k_head, nullptr, 0, (const __bf16*)v, v_stride,
+                       (int)v_head, (const __bf16*)gate, gate_stride, sink, (int)(heads / kv_heads), (__bf16*)out, out_stride, cu_q, cu_k,
+                       (int)heads, (int)dim, 0, (int)vdim, 0, 0, 0.f};
+    return run(a, num_seqs, max_seqlen_q, scale, stream);
 }

@@ -8,19 +8,11 @@
 //   latent_front_kernel     RMS norm of c, interleaved rotary on the shared key part and on the queries,
 //                           append of the row to the cache
 //   head_matmul_*           per-head products with W_uk^T and W_uv, the latter with the output gate
-//   latent_rows_kernel      attention, any size and element type (one wavefront per key)
-//   latent_decode_kernel    attention on MFMA tiles, keys split over workgroups, + latent_merge_kernel
-//   latent_gather_kernel    cached rows of whole sequences as dense rows (for latent_prefill.hip)
 //
-// A query is a "row": a token, the block-table row of its sequence and the number of keys it sees.  A decode
-// step has one row per sequence; the tokens of a short prompt portion are simply several rows.
+// The attention itself is in row_attention.hip (query rows against cached rows) and dense_prefill.hip.
 #include "elem.h"
 
 namespace {
-
-typedef short i16x4 __attribute__((ext_vector_type(4)));
-typedef short i16x8 __attribute__((ext_vector_type(8)));
-typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
 
 // ------------------------------------------------------------------ norm, rotary, append
 template <class T>
@@ -192,360 +184,6 @@ __global__ void __launch_bounds__(256) head_matmul_mfma_kernel(HeadMatmulArgs<__
     }
 }
 
-// ------------------------------------------------------------------ attention over latent rows
-template <class T>
-struct LatentAttnArgs {
-    const T* qx;                          // [rows][heads][row]
-    const T* cache; int row, rank_pad;    // [blocks * block_size][row]
-    const int32_t* bt; int64_t bt_stride; int table_cols, block_size, num_blocks;
-    const int32_t* row_seq;               // block-table row of each query row; nullptr: the query row itself
-    const int32_t* ctx;                   // keys each query row sees
-    int heads, splits;
-    float scale_log2;
-    T* out;                               // [rows][heads][rank_pad]
-    float* part;                          // [rows][splits][heads][rank_pad], then [rows][splits][heads][max, sum]
-    float* part_ml;
-    int rows; unsigned groups;            // MFMA kernel: query rows and head groups of the launch
-};
-
-template <class T>
-__device__ __forceinline__ int visible_keys(const LatentAttnArgs<T>& a, int row) {
-    const int len = a.ctx[row], cap = a.table_cols * a.block_size;
-    return len < cap ? len : cap;         // a corrupt length cannot run past the table row
-}
-template <class T>
-__device__ __forceinline__ int table_row(const LatentAttnArgs<T>& a, int row) {
-    return a.row_seq ? a.row_seq[row] : row;
-}
-template <class T>
-__device__ __forceinline__ int block_id(const LatentAttnArgs<T>& a, const int32_t* bt, int col) {
-    const int b = bt[col];
-    return b < 0 ? 0 : (b >= a.num_blocks ? a.num_blocks - 1 : b);
-}
-
-// One workgroup per (query row, head); wavefront w takes keys w, w + 4, ...; lanes hold the row elements
-// lane, lane + 64, ...  NC = number of such elements a lane may hold.
-template <class T, int NC>
-__global__ void __launch_bounds__(256) latent_rows_kernel(LatentAttnArgs<T> a) {
-    __shared__ float sm[4], sl[4];
-    __shared__ float so[4][64 * NC];
-    const int row = blockIdx.x, h = blockIdx.y;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const int len = visible_keys(a, row);
-    const int32_t* bt = a.bt + (int64_t)table_row(a, row) * a.bt_stride;
-    const T* qr = a.qx + ((int64_t)row * a.heads + h) * a.row;
-    float q[NC], o[NC];
-#pragma unroll
-    for (int i = 0; i < NC; ++i) {
-        const int c = lane + 64 * i;
-        q[i] = c < a.row ? (float)qr[c] * a.scale_log2 : 0.f;
-        o[i] = 0.f;
-    }
-    float m = -INFINITY, l = 0.f;
-    for (int key = wave; key < len; key += 4) {
-        const int col = key / a.block_size;
-        const T* kr = a.cache + ((int64_t)block_id(a, bt, col) * a.block_size + (key - col * a.block_size)) * a.row;
-        float k[NC], s = 0.f;
-#pragma unroll
-        for (int i = 0; i < NC; ++i) {
-            const int c = lane + 64 * i;
-            k[i] = c < a.row ? (float)kr[c] : 0.f;
-            s += q[i] * k[i];
-        }
-        s = wave_sum(s);
-        const float mn = fmaxf(m, s);
-        const float alpha = exp2f(m - mn), p = exp2f(s - mn);
-        l = l * alpha + p;
-#pragma unroll
-        for (int i = 0; i < NC; ++i) o[i] = o[i] * alpha + p * k[i];
-        m = mn;
-    }
-    if (lane == 0) { sm[wave] = m; sl[wave] = l; }
-#pragma unroll
-    for (int i = 0; i < NC; ++i) so[wave][lane + 64 * i] = o[i];
-    __syncthreads();
-    float mt = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));
-    float w[4], lt = 0.f;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        w[i] = sm[i] == -INFINITY ? 0.f : exp2f(sm[i] - mt);
-        lt += sl[i] * w[i];
-    }
-    const float inv = lt > 0.f ? 1.f / lt : 0.f;
-    T* out = a.out + ((int64_t)row * a.heads + h) * a.rank_pad;
-    for (int c = threadIdx.x; c < a.rank_pad; c += 256) {
-        float v = 0.f;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) v += so[i][c] * w[i];
-        out[c] = (T)(v * inv);
-    }
-}
-
-// MFMA form.  A workgroup of four wavefronts serves MT x 16 heads of one query row over a run of 32-key tiles
-// (split `blockIdx.x` of the keys).  A tile is contiguous in the cache (a block holds whole tiles), is staged
-// through LDS once and serves both products:
-//   S^T[key, head] = C[key, :] . Q^T     wavefront (key tile w % 2, half w / 2 of the k-steps), sums through LDS
-//   O^T[c, head]  += C^T[c, key] . P^T   wavefront w owns the 16-channel tiles w, w + 4, ...
-// The second product reads C transposed from LDS (ds_read_b64_tr_b16: lane i of a group of 16 points at 4
-// consecutive elements of row i / 4 and receives column i of the 4 x 16 block).
-constexpr int kTile = 32;
-constexpr int kSRow = kTile + 4;      // floats per score row in LDS
-constexpr float kLazy = 8.f;
-
-__host__ __device__ constexpr int tile_pitch(int row) { return 2 * row + 16; }   // bytes: odd multiple of 16 modulo 256
-
-template <int MT, int KSH, int NT>
-__global__ void __launch_bounds__(256, 2) latent_decode_kernel(LatentAttnArgs<__bf16> a) {
-    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
-    const int tid = threadIdx.x, lane = tid & 63;
-    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int g = lane >> 4, n = lane & 15;
-    // Workgroups go to the eight dies round-robin: the head groups that read the same keys are given to one die, one
-    // behind the other, so that its second-level cache serves all but the first of them.
-    const unsigned die = blockIdx.x & 7u, turn = blockIdx.x >> 3;
-    const unsigned unit = turn / a.groups * 8u + die;
-    if (unit >= (unsigned)(a.rows * a.splits)) return;
-    const int split = (int)(unit % (unsigned)a.splits), row = (int)(unit / (unsigned)a.splits);
-    const int head0 = (int)(turn % a.groups) * (16 * MT);
-    const int len = visible_keys(a, row);
-    const int tiles = (len + kTile - 1) / kTile;
-    const int per = (tiles + a.splits - 1) / a.splits;
-    const int t0 = split * per, t1 = t0 + per < tiles ? t0 + per : tiles;
-    if (t0 >= t1 && (a.splits > 1 || len > 0)) return;     // the merge knows which splits are empty
-    const int32_t* bt = a.bt + (int64_t)table_row(a, row) * a.bt_stride;
-    const int pitch = tile_pitch(a.row), ksteps = a.row / 32, ctiles = a.rank_pad / 16;
-    float* sbuf = reinterpret_cast<float*>(lds + kTile * pitch);      // [2][MT * 16][kSRow]
-    const int half = wave >> 1, ktile = wave & 1;
-
-    bf16x8_t q[MT][KSH];
-#pragma unroll
-    for (int u = 0; u < MT; ++u) {
-        const int h = head0 + 16 * u + n;
-        const __bf16* qr = a.qx + ((int64_t)row * a.heads + (h < a.heads ? h : 0)) * a.row + 8 * g;
-#pragma unroll
-        for (int j = 0; j < KSH; ++j) {
-            const int s = 2 * j + half;
-            q[u][j] = bf16x8_t{};
-            if (s < ksteps) q[u][j] = *reinterpret_cast<const bf16x8_t*>(qr + 32 * s);
-        }
-    }
-    f32x4_t acc[MT][NT];
-    float m[MT], l[MT];
-#pragma unroll
-    for (int u = 0; u < MT; ++u) {
-        m[u] = -INFINITY;
-        l[u] = 0.f;
-#pragma unroll
-        for (int i = 0; i < NT; ++i) acc[u][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    }
-
-    // chunk i of this thread: 16 bytes at offset 16 (tid + 256 i) of the tile, and its place in LDS.  Sizes below what the
-    // kernel is built for leave surplus chunks, which repeat the tile's last one (same bytes to the same place), surplus
-    // k-steps, which meet zeros in q, and surplus channel tiles, which are not stored: no branches in the loop.
-    const int chunks_per_row = a.row / 8, chunks = kTile * chunks_per_row;
-    u32x4_t stage[KSH];
-    int st_src[KSH], st_lds[KSH];
-#pragma unroll
-    for (int i = 0; i < KSH; ++i) {
-        const int c = tid + 256 * i < chunks ? tid + 256 * i : chunks - 1;
-        const int r = c / chunks_per_row;
-        st_src[i] = 16 * c;
-        st_lds[i] = r * pitch + (c - r * chunks_per_row) * 16;
-    }
-    int k_off[KSH];
-#pragma unroll
-    for (int j = 0; j < KSH; ++j) k_off[j] = __builtin_amdgcn_readfirstlane(2 * j + half < ksteps ? 64 * (2 * j + half) : 0);
-    // tiles are walked in order: the block changes every `tiles_per_block` tiles, and its id is looked up a block ahead
-    const int tiles_per_block = a.block_size / kTile;
-    const int64_t tile_bytes = (int64_t)2 * kTile * a.row;
-    int col = t0 / tiles_per_block, in_block = t0 - col * tiles_per_block;
-    int next_id = block_id(a, bt, col);
-    const unsigned char* src = nullptr;
-    auto open_block = [&]() {
-        src = reinterpret_cast<const unsigned char*>(a.cache) + ((int64_t)next_id * tiles_per_block + in_block) * tile_bytes;
-        ++col;
-        next_id = block_id(a, bt, col < a.table_cols ? col : a.table_cols - 1);
-    };
-    auto fetch = [&]() {
-        if (in_block == tiles_per_block) {
-            in_block = 0;
-            open_block();
-        }
-#pragma unroll
-        for (int i = 0; i < KSH; ++i) stage[i] = *reinterpret_cast<const u32x4_t*>(src + st_src[i]);
-        src += tile_bytes;
-        ++in_block;
-    };
-    if (t0 < t1) {
-        open_block();
-        fetch();
-    }
-    for (int t = t0; t < t1; ++t) {
-        __syncthreads();
-        if (len - t * kTile < kTile) {                            // rows behind the last key count as zeros
-            const int have = 16 * (len - t * kTile) * chunks_per_row;
-#pragma unroll
-            for (int i = 0; i < KSH; ++i)
-                if (st_src[i] >= have) stage[i] = u32x4_t{0u, 0u, 0u, 0u};
-        }
-#pragma unroll
-        for (int i = 0; i < KSH; ++i) *reinterpret_cast<u32x4_t*>(lds + st_lds[i]) = stage[i];
-        if (t + 1 < t1) fetch();
-        __syncthreads();
-        // ---- scores
-        f32x4_t sc[MT];
-#pragma unroll
-        for (int u = 0; u < MT; ++u) sc[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-        const unsigned char* kr = lds + (16 * ktile + n) * pitch + 16 * g;
-#pragma unroll
-        for (int j = 0; j < KSH; ++j) {
-            const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(kr + k_off[j]);
-#pragma unroll
-            for (int u = 0; u < MT; ++u) sc[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, q[u][j], sc[u], 0, 0, 0);
-        }
-#pragma unroll
-        for (int u = 0; u < MT; ++u)
-            *reinterpret_cast<f32x4_t*>(sbuf + (half * MT * 16 + 16 * u + n) * kSRow + 16 * ktile + 4 * g) = sc[u];
-        __syncthreads();
-        // ---- softmax over the 32 keys, in every wavefront: lane (g, n) has keys 8 g .. 8 g + 7 of head n.  The running
-        // maximum moves only when it grows by more than kLazy (log2 units); until then weights are at most 2^kLazy.
-        bf16x8_t pb[MT];
-        const int seen = len - t * kTile - 8 * g;       // of this lane's keys the first `seen` exist
-#pragma unroll
-        for (int u = 0; u < MT; ++u) {
-            const float* s0 = sbuf + (16 * u + n) * kSRow + 8 * g;
-            const float* s1 = s0 + MT * 16 * kSRow;
-            float sv[8];
-#pragma unroll
-            for (int e = 0; e < 2; ++e) {
-                const f32x4_t x = *reinterpret_cast<const f32x4_t*>(s0 + 4 * e), y = *reinterpret_cast<const f32x4_t*>(s1 + 4 * e);
-#pragma unroll
-                for (int i = 0; i < 4; ++i) sv[4 * e + i] = (x[i] + y[i]) * a.scale_log2;
-            }
-            if (len - t * kTile < kTile) {
-#pragma unroll
-                for (int i = 0; i < 8; ++i) sv[i] = i < seen ? sv[i] : -INFINITY;
-            }
-            float mx = sv[0];
-#pragma unroll
-            for (int i = 1; i < 8; ++i) mx = fmaxf(mx, sv[i]);
-            mx = max_xor16_32(mx);
-            const bool grow = mx > m[u] + kLazy;        // always in the first tile, whose first key exists
-            if (__any(grow)) {
-                const float alpha = grow ? __builtin_amdgcn_exp2f(m[u] - mx) : 1.f;
-                m[u] = grow ? mx : m[u];
-                l[u] *= alpha;
-#pragma unroll
-                for (int i = 0; i < NT; ++i) acc[u][i] *= alpha;
-            }
-            float sum = 0.f;
-#pragma unroll
-            for (int i = 0; i < 8; ++i) {
-                const float p = __builtin_amdgcn_exp2f(sv[i] - m[u]);
-                sum += p;
-                pb[u][i] = (__bf16)p;
-            }
-            l[u] += sum;
-        }
-        // ---- weighted sum of the c parts
-        const unsigned char* vr = lds + (8 * g + (n >> 2)) * pitch + (n & 3) * 8 + 32 * wave;
-#pragma unroll
-        for (int i = 0; i < NT; ++i) {
-            const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 128 * i));
-            const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 128 * i + 4 * pitch));
-            const bf16x8_t vt = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
-#pragma unroll
-            for (int u = 0; u < MT; ++u) acc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pb[u], acc[u][i], 0, 0, 0);
-        }
-    }
-#pragma unroll
-    for (int u = 0; u < MT; ++u) {
-        const int h = head0 + 16 * u + n;
-        float sum = l[u] + __shfl_xor(l[u], 16, 64);
-        sum += __shfl_xor(sum, 32, 64);
-        if (h >= a.heads) continue;
-        if (a.splits == 1) {
-            const float inv = sum > 0.f ? 1.f / sum : 0.f;
-            __bf16* o = a.out + ((int64_t)row * a.heads + h) * a.rank_pad + 4 * g;
-#pragma unroll
-            for (int i = 0; i < NT; ++i) {
-                const int ct = wave + 4 * i;
-                if (ct < ctiles) {
-                    bf16x4_t v;
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) v[e] = (__bf16)(acc[u][i][e] * inv);
-                    *reinterpret_cast<bf16x4_t*>(o + 16 * ct) = v;
-                }
-            }
-        } else {
-            const int64_t rec = ((int64_t)row * a.splits + split) * a.heads + h;
-            float* o = a.part + rec * a.rank_pad + 4 * g;
-#pragma unroll
-            for (int i = 0; i < NT; ++i) {
-                const int ct = wave + 4 * i;
-                if (ct < ctiles) *reinterpret_cast<f32x4_t*>(o + 16 * ct) = acc[u][i];
-            }
-            if (wave == 0 && g == 0) { a.part_ml[2 * rec] = m[u]; a.part_ml[2 * rec + 1] = sum; }
-        }
-    }
-}
-
-__global__ void __launch_bounds__(128) latent_merge_kernel(LatentAttnArgs<__bf16> a) {
-    const int row = blockIdx.x, h = blockIdx.y;
-    const int tiles = (visible_keys(a, row) + kTile - 1) / kTile;
-    const int per = (tiles + a.splits - 1) / a.splits;
-    const int used = per > 0 ? (tiles + per - 1) / per : 0;
-    const int64_t rec0 = (int64_t)row * a.splits * a.heads + h;
-    float m = -INFINITY;
-    for (int s = 0; s < used; ++s) m = fmaxf(m, a.part_ml[2 * (rec0 + (int64_t)s * a.heads)]);
-    float l = 0.f;
-    for (int s = 0; s < used; ++s) {
-        const float* ml = a.part_ml + 2 * (rec0 + (int64_t)s * a.heads);
-        l += ml[1] * exp2f(ml[0] - m);
-    }
-    const float inv = l > 0.f ? 1.f / l : 0.f;
-    for (int c = threadIdx.x * 4; c < a.rank_pad; c += 512) {
-        f32x4_t o = {0.f, 0.f, 0.f, 0.f};
-        for (int s = 0; s < used; ++s) {
-            const int64_t rec = rec0 + (int64_t)s * a.heads;
-            o += *reinterpret_cast<const f32x4_t*>(a.part + rec * a.rank_pad + c) * exp2f(a.part_ml[2 * rec] - m);
-        }
-        bf16x4_t v;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = (__bf16)(o[e] * inv);
-        *reinterpret_cast<bf16x4_t*>(a.out + ((int64_t)row * a.heads + h) * a.rank_pad + c) = v;
-    }
-}
-
-// ------------------------------------------------------------------ cached rows as dense rows
-struct LatentGatherArgs {
-    const uint16_t* cache; int row; int block_size, num_blocks, table_cols;
-    const int32_t* bt; int64_t bt_stride;
-    const int32_t* seqs;       // block-table row of each sequence
-    const int32_t* cu_k;       // [sequences + 1] first dense row of each
-    uint16_t* out;             // [total][row]
-};
-
-__global__ void __launch_bounds__(256) latent_gather_kernel(LatentGatherArgs a) {
-    const int s = blockIdx.y;
-    const int k0 = a.cu_k[s];
-    int len = a.cu_k[s + 1] - k0;
-    const int cap = a.table_cols * a.block_size;
-    if (len > cap) len = cap;
-    const int32_t* bt = a.bt + (int64_t)a.seqs[s] * a.bt_stride;
-    const int chunks = a.row / 8;
-    const int first = blockIdx.x * kTile;
-    for (int i = threadIdx.x; i < kTile * chunks; i += 256) {
-        const int t = first + i / chunks, c = i % chunks;
-        if (t >= len) return;
-        const int col = t / a.block_size;
-        int b = bt[col];
-        b = b < 0 ? 0 : (b >= a.num_blocks ? a.num_blocks - 1 : b);
-        const u32x4_t v = *reinterpret_cast<const u32x4_t*>(a.cache + ((int64_t)b * a.block_size + (t - col * a.block_size)) * a.row + 8 * c);
-        *reinterpret_cast<u32x4_t*>(a.out + (int64_t)(k0 + t) * a.row + 8 * c) = v;
-    }
-}
-
 bool size_in(int64_t v, int64_t lo, int64_t hi) { return v >= lo && v <= hi; }
 
 template <class T>
@@ -555,35 +193,6 @@ int launch_front(const LatentFrontArgs<T>& a, int64_t n, hipStream_t st) {
                       ptr_aligned(a.cache, pair) && ptr_aligned(a.qx, pair);
     if (even) hipLaunchKernelGGL((latent_front_kernel<T, true>), dim3((unsigned)n), dim3(256), 0, st, a);
     else hipLaunchKernelGGL((latent_front_kernel<T, false>), dim3((unsigned)n), dim3(256), 0, st, a);
-    return (int)hipGetLastError();
-}
-
-template <class T>
-int launch_rows(const LatentAttnArgs<T>& a, int64_t rows, hipStream_t st) {
-    const dim3 grid((unsigned)rows, (unsigned)a.heads), block(256);
-    if (a.row <= 128) hipLaunchKernelGGL((latent_rows_kernel<T, 2>), grid, block, 0, st, a);
-    else if (a.row <= 256) hipLaunchKernelGGL((latent_rows_kernel<T, 4>), grid, block, 0, st, a);
-    else if (a.row <= 640) hipLaunchKernelGGL((latent_rows_kernel<T, 10>), grid, block, 0, st, a);
-    else if (a.row <= 1280) hipLaunchKernelGGL((latent_rows_kernel<T, 20>), grid, block, 0, st, a);
-    else return INFER_KV_EUNSUPPORTED;
-    return (int)hipGetLastError();
-}
-
-// sizes the MFMA attention kernel is built for
-bool mfma_attention_fits(int64_t row, int64_t rank_pad, int64_t block_size) {
-    return row <= 640 && rank_pad <= 512 && block_size % kTile == 0;
-}
-
-template <int KSH, int NT>
-int launch_decode(LatentAttnArgs<__bf16>& a, hipStream_t st) {
-    const int mt = a.heads > 16 ? 2 : 1;
-    a.groups = (unsigned)((a.heads + 16 * mt - 1) / (16 * mt));
-    const int64_t units = ((int64_t)a.rows * a.splits + 7) / 8 * 8;
-    if (units * a.groups > 0x7fffffff) return INFER_KV_EINVAL;
-    const dim3 grid((unsigned)(units * a.groups)), block(256);
-    const size_t lds = (size_t)kTile * tile_pitch(a.row) + (size_t)2 * mt * 16 * kSRow * sizeof(float);
-    if (mt == 2) hipLaunchKernelGGL((latent_decode_kernel<2, KSH, NT>), grid, block, lds, st, a);
-    else hipLaunchKernelGGL((latent_decode_kernel<1, KSH, NT>), grid, block, lds, st, a);
     return (int)hipGetLastError();
 }
 
@@ -653,70 +262,3 @@ extern "C" int infer_head_matmul(int elem, const void* x, int64_t x_row, int64_t
     return INFER_KV_EUNSUPPORTED;
 }
 
-extern "C" int64_t infer_latent_attention_splits(int elem, int64_t rows, int64_t heads, int64_t row, int64_t rank_pad,
-                                                 int64_t block_size, int64_t max_keys) {
-    if (elem != INFER_ELEM_BF16 || !mfma_attention_fits(row, rank_pad, block_size) || rows < 1 || heads < 1) return 1;
-    // two workgroups are resident per compute unit; more splits than that only add partial results
-    const int64_t groups = heads > 16 ? (heads + 31) / 32 : 1;
-    int64_t splits = (512 + rows * groups - 1) / (rows * groups);
-    const int64_t most = (max_keys + 4 * kTile - 1) / (4 * kTile);     // no split shorter than four tiles
-    if (splits > most) splits = most;
-    if (splits > 64) splits = 64;
-    return splits < 1 ? 1 : splits;
-}
-
-extern "C" int infer_latent_attention(int elem, const void* qx, const void* cache, int64_t row, int64_t rank_pad,
-                                      const int32_t* block_table, int64_t bt_stride, int64_t table_cols, int64_t block_size,
-                                      int64_t num_blocks, const int32_t* row_seq, const int32_t* ctx, int64_t rows,
-                                      int64_t heads, float scale, int64_t splits, void* out, float* workspace,
-                                      int64_t workspace_floats, void* stream) {
-    if (rows < 0 || rows > 0x7fffffff) return INFER_KV_EINVAL;
-    if (rows == 0) return INFER_KV_OK;
-    if (!qx || !cache || !block_table || !ctx || !out) return INFER_KV_EINVAL;
-    if (!size_in(heads, 1, 4096) || !size_in(row, 1, 1 << 20) || !size_in(rank_pad, 1, row) || !size_in(block_size, 1, 1 << 20) ||
-        !size_in(table_cols, 1, 1 << 24) || table_cols * block_size > 0x7fffffff || num_blocks < 1 || bt_stride < table_cols)
-        return INFER_KV_EINVAL;
-    if (row % 32 || rank_pad % 32) return INFER_KV_EALIGN;
-    if (!size_in(splits, 1, 64)) return INFER_KV_EINVAL;
-    hipStream_t st = (hipStream_t)stream;
-    const float scale_log2 = scale * kLog2e;
-    if (elem == INFER_ELEM_F32) {
-        LatentAttnArgs<float> a{(const float*)qx, (const float*)cache, (int)row, (int)rank_pad, block_table, bt_stride, (int)table_cols,
-                                (int)block_size, (int)num_blocks, row_seq, ctx, (int)heads, 1, scale_log2, (float*)out, nullptr, nullptr, (int)rows, 1};
-        return launch_rows(a, rows, st);
-    }
-    if (elem != INFER_ELEM_BF16) return INFER_KV_EUNSUPPORTED;
-    LatentAttnArgs<__bf16> a{(const __bf16*)qx, (const __bf16*)cache, (int)row, (int)rank_pad, block_table, bt_stride, (int)table_cols,
-                             (int)block_size, (int)num_blocks, row_seq, ctx, (int)heads, (int)splits, scale_log2, (__bf16*)out,
-                             workspace, workspace ? workspace + rows * splits * heads * rank_pad : nullptr, (int)rows, 1};
-    if (!mfma_attention_fits(row, rank_pad, block_size) || !ptr_aligned(qx, 16) || !ptr_aligned(cache, 16) || !ptr_aligned(out, 8)) {
-        a.splits = 1;
-        return launch_rows(a, rows, st);
-    }
-    if (splits > 1 && (!workspace || !ptr_aligned(workspace, 16) || workspace_floats < rows * splits * heads * (rank_pad + 2)))
-        return INFER_KV_EWORKSPACE;
-    int rc;
-    if (row <= 192 && rank_pad <= 128) rc = launch_decode<3, 2>(a, st);
-    else if (row <= 384 && rank_pad <= 256) rc = launch_decode<6, 4>(a, st);
-    else if (row <= 576) rc = launch_decode<9, 8>(a, st);
-    else rc = launch_decode<10, 8>(a, st);
-    if (rc) return rc;
-    if (splits > 1) hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)rows, (unsigned)heads), dim3(128), 0, st, a);
-    return (int)hipGetLastError();
-}
-
-extern "C" int infer_latent_gather(const void* cache, int64_t row, int64_t block_size, int64_t num_blocks,
-                                   const int32_t* block_table, int64_t bt_stride, int64_t table_cols, const int32_t* seqs,
-                                   const int32_t* cu_k, int64_t num_seqs, int64_t max_keys, void* out, void* stream) {
-    if (num_seqs < 0 || max_keys < 0 || num_seqs > 65535) return INFER_KV_EINVAL;
-    if (num_seqs == 0 || max_keys == 0) return INFER_KV_OK;
-    if (!cache || !block_table || !seqs || !cu_k || !out || row <= 0 || row > (1 << 20) || block_size <= 0 || num_blocks <= 0 ||
-        table_cols <= 0 || table_cols * block_size > 0x7fffffff || bt_stride < table_cols)
-        return INFER_KV_EINVAL;
-    if (row % 8 || !ptr_aligned(cache, 16) || !ptr_aligned(out, 16)) return INFER_KV_EALIGN;
-    LatentGatherArgs a{(const uint16_t*)cache, (int)row, (int)block_size, (int)num_blocks, (int)table_cols, block_table, bt_stride,
-                       seqs, cu_k, (uint16_t*)out};
-    hipLaunchKernelGGL(latent_gather_kernel, dim3((unsigned)((max_keys + kTile - 1) / kTile), (unsigned)num_seqs), dim3(256), 0,
-                       (hipStream_t)stream, a);
-    return (int)hipGetLastError();
-}

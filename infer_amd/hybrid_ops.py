@@ -1,5 +1,5 @@
-"""Python entry points of the hybrid-model kernels (latent attention, gated delta rule, float32 residual
-stream), beside ``ops``: shape and type checks on the host, then one call into ``libinfer_kv.so`` on torch's
+"""Python entry points of the hybrid-model kernels (latent and grouped attention, gated delta rule, linear attention
+with a constant decay, float32 residual stream), beside ``ops``: shape and type checks on the host, then one call into ``libinfer_kv.so`` on torch's
 current stream.  Activations are bfloat16 or float32; there is no CPU path."""
 from __future__ import annotations
 
@@ -30,11 +30,8 @@ def _f32(t: torch.Tensor, *shape) -> torch.Tensor:
 
 
 # ------------------------------------------------------------------ residual stream
-def residual_norm(x: torch.Tensor, eps: float, *, y=None, w_post=None, w_pre=None, tokens=None, embed=None,
-                  embed_scale: float = 1.0, dtype: torch.dtype = torch.bfloat16):
-    """``x`` [rows, width] float32 is updated in place: the embedding of ``tokens`` is stored, or
-    ``rms(y) * w_post`` added (``y`` may be an unreduced ``SplitKSum``).  Returns ``rms(x) * w_pre`` in ``dtype``,
-    or None without ``w_pre``."""
+def _stream_args(x, y, w_post, w_last, tokens, embed, dtype):
+    """Checks of what both forms of the residual step take; the sublayer's output as the C ABI wants it."""
     n, width = x.shape
     assert x.dtype == torch.float32
     y_stride = splits = split_stride = partial_stride = 0
@@ -49,30 +46,63 @@ def residual_norm(x: torch.Tensor, eps: float, *, y=None, w_post=None, w_pre=Non
         y_stride = _rows(y, width)
     if y is not None or partial is not None:
         _f32(w_post, width)
-    if w_pre is not None:
-        _f32(w_pre, width)
+    if w_last is not None:
+        _f32(w_last, width)
     if tokens is not None:
         assert tokens.dtype == torch.int64 and tokens.is_contiguous() and tokens.numel() == n
         assert embed.dtype == dtype and embed.is_contiguous() and embed.shape[1] == width
+    _require_gpu(x, *[t for t in (y, partial, w_post, w_last, tokens, embed) if t is not None])
+    return _ptr(y), y_stride, _ptr(partial), splits, split_stride, partial_stride
+
+
+def residual_norm(x: torch.Tensor, eps: float, *, y=None, w_post=None, w_pre=None, tokens=None, embed=None,
+                  embed_scale: float = 1.0, dtype: torch.dtype = torch.bfloat16):
+    """``x`` [rows, width] float32 is updated in place: the embedding of ``tokens`` is stored, or
+    ``rms(y) * w_post`` added (``y`` may be an unreduced ``SplitKSum``).  Returns ``rms(x) * w_pre`` in ``dtype``,
+    or None without ``w_pre``."""
+    n, width = x.shape
+    sub = _stream_args(x, y, w_post, w_pre, tokens, embed, dtype)
     out = torch.empty((n, width), dtype=dtype, device=x.device) if w_pre is not None else None
-    _require_gpu(x, *[t for t in (y, partial, w_post, w_pre, tokens, embed) if t is not None])
     rc = _lib.load().infer_residual_norm(
-        ELEM[dtype], _ptr(tokens), _ptr(embed), float(embed_scale), embed.shape[0] if embed is not None else 0,
-        _ptr(y), y_stride, _ptr(partial), splits, split_stride, partial_stride, _ptr(w_post), x.data_ptr(),
-        _rows(x, width), _ptr(w_pre), _ptr(out), width, n, width, float(eps), _stream_ptr(x))
+        ELEM[dtype], _ptr(tokens), _ptr(embed), float(embed_scale), embed.shape[0] if embed is not None else 0, *sub,
+        _ptr(w_post), x.data_ptr(), _rows(x, width), _ptr(w_pre), _ptr(out), width, n, width, float(eps), _stream_ptr(x))
     _lib.check(rc, "residual_norm")
+    return out
+
+
+def post_norm(x: torch.Tensor, eps: float, *, y=None, w_post=None, alpha: float = 1.0, w_last=None, tokens=None, embed=None,
+              embed_scale: float = 1.0, dtype: torch.dtype = torch.bfloat16) -> torch.Tensor:
+    """``x`` [rows, width] float32 is updated in place: the embedding of ``tokens``, or
+    ``rms(alpha * x + y) * w_post`` (``y`` may be an unreduced ``SplitKSum``).  Returns it in ``dtype``, with ``w_last``
+    ``rms(x) * w_last`` instead."""
+    n, width = x.shape
+    sub = _stream_args(x, y, w_post, w_last, tokens, embed, dtype)
+    out = torch.empty((n, width), dtype=dtype, device=x.device)
+    rc = _lib.load().infer_post_norm(
+        ELEM[dtype], _ptr(tokens), _ptr(embed), float(embed_scale), embed.shape[0] if embed is not None else 0, *sub,
+        float(alpha), _ptr(w_post), x.data_ptr(), _rows(x, width), _ptr(w_last), out.data_ptr(), width, n, width, float(eps),
+        _stream_ptr(x))
+    _lib.check(rc, "post_norm")
+    return out
+
+
+def _gated(entry: str, x: torch.Tensor) -> torch.Tensor:
+    d = x.shape[1] // 2
+    out = torch.empty((x.shape[0], d), dtype=x.dtype, device=x.device)
+    _require_gpu(x)
+    rc = getattr(_lib.load(), entry)(ELEM[x.dtype], out.data_ptr(), d, x.data_ptr(), _rows(x, 2 * d), x.shape[0], d, _stream_ptr(x))
+    _lib.check(rc, entry)
     return out
 
 
 def gelu_tanh_and_mul(x: torch.Tensor) -> torch.Tensor:
     """``gelu_tanh(x[:, :d]) * x[:, d:]``."""
-    d = x.shape[1] // 2
-    out = torch.empty((x.shape[0], d), dtype=x.dtype, device=x.device)
-    _require_gpu(x)
-    rc = _lib.load().infer_gelu_tanh_and_mul(ELEM[x.dtype], out.data_ptr(), d, x.data_ptr(), _rows(x, 2 * d), x.shape[0],
-                                             d, _stream_ptr(x))
-    _lib.check(rc, "gelu_tanh_and_mul")
-    return out
+    return _gated("infer_gelu_tanh_and_mul", x)
+
+
+def silu_and_mul(x: torch.Tensor) -> torch.Tensor:
+    """``silu(x[:, :d]) * x[:, d:]``."""
+    return _gated("infer_silu_and_mul", x)
 
 
 # ------------------------------------------------------------------ latent attention
@@ -181,6 +211,168 @@ def latent_prefill(q, kp, kr, v, gate, out, cu_q, cu_k, max_seqlen_q: int, heads
         v.stride(0), gate.data_ptr(), max(gate.stride(0), heads), out.data_ptr(), _rows(out, heads * vdim), cu_q.data_ptr(),
         cu_k.data_ptr(), cu_q.numel() - 1, int(max_seqlen_q), heads, dim, rot, vdim, float(scale), _stream_ptr(q))
     _lib.check(rc, "latent_prefill")
+
+
+# ------------------------------------------------------------------ grouped attention
+def grouped_front(proj, heads, kv_heads, dim, vdim, k_off, v_off, bias, q_norm, k_norm, eps, table, rot_dims, positions, slots,
+                  cache, dim_pad, vdim_pad, qx, qx_rows) -> None:
+    """Biases, norms over the whole projections, rotary positions and the append of keys and values; ``cache`` is
+    [blocks, kv_heads, block_size, vdim_pad + dim_pad], ``qx`` [>= qx_rows, heads, dim_pad].  ``kv_heads`` 0: q alone."""
+    n = proj.shape[0]
+    cols = v_off + kv_heads * vdim if kv_heads else heads * dim
+    if bias is not None:
+        assert bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() >= cols
+    if q_norm is not None:
+        _f32(q_norm, heads * dim)
+    if kv_heads and k_norm is not None:
+        _f32(k_norm, kv_heads * dim)
+    assert table.dtype == torch.float32 and table.is_contiguous() and table.shape[1:] == (rot_dims // 2, 2)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == n
+    assert slots.dtype == torch.int32 and slots.is_contiguous() and slots.numel() == n
+    assert cache.dtype == proj.dtype and cache.is_contiguous() and cache.shape[3] == dim_pad + vdim_pad
+    assert kv_heads in (0, cache.shape[1])
+    assert qx_rows == 0 or (qx.dtype == proj.dtype and qx.is_contiguous() and tuple(qx.shape[1:]) == (heads, dim_pad)
+                            and qx.shape[0] >= qx_rows)
+    _require_gpu(proj, table, positions, slots, cache)
+    rc = _lib.load().infer_grouped_front(
+        ELEM[proj.dtype], proj.data_ptr(), _rows(proj, cols), heads, kv_heads, dim, vdim, k_off, v_off, _ptr(bias), _ptr(q_norm),
+        _ptr(k_norm) if kv_heads else None, float(eps), table.data_ptr() if rot_dims else None, rot_dims, table.shape[0],
+        positions.data_ptr(), slots.data_ptr(), cache.data_ptr(), cache.shape[2], dim_pad, vdim_pad,
+        cache.shape[0] * cache.shape[2], _ptr(qx) if qx_rows else None, qx_rows, n, _stream_ptr(proj))
+    _lib.check(rc, "grouped_front")
+
+
+def grouped_attention(qx, cache, block_table, ctx, scale: float, vdim: int, out, sink=None, gate=None, row_seq=None, max_keys=None,
+                      splits: int = 0) -> None:
+    """``qx`` [rows, heads, dim_pad] against the first ``ctx[r]`` keys of the sequence in block-table row ``row_seq[r]``
+    (default ``r``); ``out`` [rows, heads * vdim].  ``sink`` [heads] float32, ``gate`` [rows, heads]."""
+    rows, heads, dim_pad = qx.shape
+    nblk, kv_heads, bs, crow = cache.shape
+    vdim_pad = crow - dim_pad
+    assert qx.is_contiguous() and cache.is_contiguous() and cache.dtype == qx.dtype == out.dtype and 0 < vdim <= vdim_pad
+    assert block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.stride(1) == 1
+    assert ctx.dtype == torch.int32 and ctx.is_contiguous() and ctx.numel() == rows and out.shape[0] == rows
+    if row_seq is None:
+        assert block_table.shape[0] >= rows
+    else:
+        assert row_seq.dtype == torch.int32 and row_seq.is_contiguous() and row_seq.numel() == rows
+    if sink is not None:
+        _f32(sink, heads)
+    if gate is not None:
+        assert gate.dtype == qx.dtype and gate.shape[0] == rows and gate.shape[1] >= heads and gate.stride(1) == 1
+    _require_gpu(qx, cache, block_table, ctx, out)
+    lib = _lib.load()
+    elem, cols = ELEM[qx.dtype], block_table.shape[1]
+    if splits <= 0:
+        splits = lib.infer_grouped_attention_splits(elem, rows, heads, kv_heads, dim_pad, vdim_pad, bs, max_keys or cols * bs)
+    need = rows * splits * heads * (vdim_pad + 2) if splits > 1 else 0
+    ws = torch.empty(need, dtype=torch.float32, device=qx.device) if need else None
+    rc = lib.infer_grouped_attention(
+        elem, qx.data_ptr(), cache.data_ptr(), dim_pad, vdim_pad, block_table.data_ptr(), max(block_table.stride(0), cols), cols, bs,
+        nblk, _ptr(row_seq), ctx.data_ptr(), rows, heads, kv_heads, float(scale), _ptr(sink), _ptr(gate),
+        max(gate.stride(0), heads) if gate is not None else 0, splits, out.data_ptr(), _rows(out, heads * vdim), vdim, _ptr(ws), need,
+        _stream_ptr(qx))
+    _lib.check(rc, "grouped_attention")
+
+
+def grouped_gather(cache, block_table, seqs, cu_k, total: int, max_keys: int) -> torch.Tensor:
+    """The cached rows of the sequences in block-table rows ``seqs`` as dense rows [total, kv_heads, row]."""
+    nblk, kv_heads, bs, row = cache.shape
+    assert cache.dtype == torch.bfloat16 and cache.is_contiguous()
+    assert block_table.dtype == torch.int32 and block_table.stride(1) == 1
+    for t in (seqs, cu_k):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    assert cu_k.numel() == seqs.numel() + 1
+    _require_gpu(cache, block_table, seqs, cu_k)
+    out = torch.empty((total, kv_heads, row), dtype=cache.dtype, device=cache.device)
+    rc = _lib.load().infer_grouped_gather(cache.data_ptr(), row, kv_heads, bs, nblk, block_table.data_ptr(),
+                                          max(block_table.stride(0), block_table.shape[1]), block_table.shape[1],
+                                          seqs.data_ptr(), cu_k.data_ptr(), seqs.numel(), max_keys, out.data_ptr(),
+                                          _stream_ptr(cache))
+    _lib.check(rc, "grouped_gather")
+    return out
+
+
+def grouped_prefill_supported(dim: int, vdim: int) -> bool:
+    """Whether the dense-key prefill kernel serves these sizes."""
+    return bool(_lib.load().infer_grouped_prefill_supported(dim, vdim))
+
+
+def grouped_prefill(q, k, v, sink, gate, out, cu_q, cu_k, max_seqlen_q: int, heads, dim, vdim, scale) -> None:
+    """Causal attention of whole portions: ``q`` [tokens, heads * dim], ``k``/``v`` [keys, kv_heads, dim / vdim] (views of dense
+    rows), ``gate`` [tokens, heads], ``out`` [tokens, heads * vdim], all bf16; ``sink`` [heads] float32 or None."""
+    for t in (q, k, v, gate, out):
+        assert t.dtype == torch.bfloat16
+    for t in (cu_q, cu_k):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    kv_heads = k.shape[1]
+    assert k.dim() == v.dim() == 3 and k.stride(2) == v.stride(2) == 1 and k.shape[:2] == v.shape[:2]
+    assert k.shape[2] >= dim and v.shape[2] >= vdim and cu_q.numel() == cu_k.numel()
+    assert q.shape[0] == gate.shape[0] == out.shape[0]
+    if sink is not None:
+        _f32(sink, heads)
+    _require_gpu(q, k, v, gate, out, cu_q, cu_k)
+    rc = _lib.load().infer_grouped_prefill(
+        q.data_ptr(), _rows(q, heads * dim), k.data_ptr(), k.stride(0), k.stride(1), v.data_ptr(), v.stride(0), v.stride(1), _ptr(sink),
+        gate.data_ptr(), max(gate.stride(0), heads), out.data_ptr(), _rows(out, heads * vdim), cu_q.data_ptr(), cu_k.data_ptr(),
+        cu_q.numel() - 1, int(max_seqlen_q), heads, kv_heads, dim, vdim, float(scale), _stream_ptr(q))
+    _lib.check(rc, "grouped_prefill")
+
+
+# ------------------------------------------------------------------ linear attention with a constant decay
+@lru_cache(maxsize=None)
+def decay_layout(dim: int, vdim: int) -> tuple[int, int]:
+    """(state rows, state columns) of a head."""
+    out = (ctypes.c_int64 * 2)()
+    _lib.check(_lib.load().infer_decay_layout(dim, vdim, ctypes.addressof(out)), "decay_layout")
+    return tuple(out)
+
+
+def decay_constants(decay, device) -> torch.Tensor:
+    """[3, heads] float32: every decay rounded to float, what that leaves out, and its base-2 logarithm."""
+    d = torch.tensor(decay, dtype=torch.float64)
+    hi = d.float()
+    return torch.stack((hi, (d - hi.double()).float(), torch.log2(d).clamp(min=-1e4).float())).contiguous().to(device)
+
+
+class DecayShape:
+    """Sizes and constants of a layer of linear attention with a constant decay per head."""
+
+    def __init__(self, heads: int, dim: int, vdim: int, eps: float, silu: bool, rot_dims: int, scale: float, norm_per_head: bool,
+                 gate_silu: bool):
+        self.heads, self.dim, self.vdim, self.eps, self.silu, self.rot_dims = heads, dim, vdim, eps, silu, rot_dims
+        self.scale, self.norm_per_head, self.gate_silu = scale, norm_per_head, gate_silu
+        self.state_rows, self.state_cols = decay_layout(dim, vdim)
+
+
+def decay_attention(s: DecayShape, proj, offsets, decay, table, norm, state, slots, positions, decode_rows: int, spans, out) -> None:
+    """``proj`` holds q, k, v and the gate logits at the columns ``offsets``.  Rows below ``decode_rows`` advance the state of
+    ``slots[r]`` by one token (negative: padding), the others belong to ``spans`` [.., 4] (first row, tokens, slot, first
+    position).  ``decay`` comes from ``decay_constants``."""
+    n = proj.shape[0]
+    q, k, v, g = offsets
+    assert proj.dtype == out.dtype and out.shape[0] == n
+    _f32(decay, 3, s.heads)
+    _f32(state, state.shape[0], s.heads, s.state_rows, s.state_cols)
+    if norm is not None:
+        _f32(norm, s.heads * s.vdim)
+    if s.rot_dims:
+        assert table.dtype == torch.float32 and table.is_contiguous() and table.shape[1:] == (s.rot_dims // 2, 2)
+    if decode_rows:
+        assert slots.dtype == torch.int32 and slots.is_contiguous() and slots.numel() >= decode_rows
+        assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() >= decode_rows
+    num_spans = 0
+    if decode_rows < n:
+        assert spans.dtype == torch.int32 and spans.is_contiguous() and spans.shape[1] == 4
+        num_spans = spans.shape[0]
+    _require_gpu(proj, decay, state, out)
+    rc = _lib.load().infer_decay_attention(
+        ELEM[proj.dtype], proj.data_ptr(), _rows(proj, max(q + s.heads * s.dim, k + s.heads * s.dim, v + s.heads * s.vdim, g + s.heads * s.vdim)),
+        q, k, v, g, s.heads, s.dim, s.vdim, decay.data_ptr(), int(s.silu), _ptr(table) if s.rot_dims else None, s.rot_dims,
+        table.shape[0] if s.rot_dims else 1, float(s.scale), _ptr(norm), int(s.norm_per_head), int(s.gate_silu), float(s.eps),
+        state.data_ptr(), state.shape[0], _ptr(slots), _ptr(positions), decode_rows, _ptr(spans) if num_spans else None, num_spans, n,
+        out.data_ptr(), _rows(out, s.heads * s.vdim), _stream_ptr(proj))
+    _lib.check(rc, "decay_attention")
 
 
 # ------------------------------------------------------------------ gated delta rule

@@ -1,11 +1,12 @@
 """Which model class serves which configuration."""
 from __future__ import annotations
 
-from .config import MerilornConfig, ModelConfig
+from .config import MerilornConfig, ModelConfig, VokelixConfig
 from .merilorn import MerilornForCausalLM
 from .qwen3 import QwenForCausalLM
+from .vokelix import VokelixForCausalLM
 
-MODELS = {ModelConfig: QwenForCausalLM, MerilornConfig: MerilornForCausalLM}
+MODELS = {ModelConfig: QwenForCausalLM, MerilornConfig: MerilornForCausalLM, VokelixConfig: VokelixForCausalLM}
 
 
 def model_class(config):

@@ -30,6 +30,8 @@ class StepPlan:
     portions: torch.Tensor | None = None
     chunks: torch.Tensor | None = None
     ring_slot: torch.Tensor | None = None
+    spans: torch.Tensor | None = None      # int32 [.., 4] first row, tokens, state slot, first position (``hybrid_ops.decay_attention``)
+    max_span: int = 0                      # tokens of the longest
     # attention: rows from dense_row on belong to long portions
     dense_row: int = 0
     dense_seqs: torch.Tensor | None = None      # int32, block-table rows
@@ -55,7 +57,7 @@ def build(portions, block_size: int, max_blocks: int, num_slots: int, num_blocks
     slots, row_seq = np.empty(rows, np.int32), np.empty(rows, np.int32)
     ring = np.empty((rows, 2), np.int32)
     tables = np.zeros((len(order), max(1, max(len(portions[i][0].block_table) for i in order))), np.int32)
-    port, chunk, dense = [], [], []
+    port, chunk, span, dense = [], [], [], []
     for s, i in enumerate(order):
         seq, n = portions[i]
         lo, r0 = seq.num_computed_tokens, int(first[s])
@@ -74,6 +76,7 @@ def build(portions, block_size: int, max_blocks: int, num_slots: int, num_blocks
         ring[r0:r0 + n, 1] = np.arange(n - 1, -1, -1)       # rows of the portion that follow
         if n > 1:
             port.append((len(chunk), -(-n // CHUNK), seq.state_slot, lo))
+            span.append((r0, n, seq.state_slot, lo))
             chunk += [(r0 + c, min(CHUNK, n - c), lo + c, lo, seq.state_slot, 0) for c in range(0, n, CHUNK)]
         if n >= DENSE_FROM:
             dense.append(s)
@@ -83,7 +86,7 @@ def build(portions, block_size: int, max_blocks: int, num_slots: int, num_blocks
              "ctx": (pos + 1).astype(np.int32), "ring": ring,
              "state": ring[:decode_rows, 0],
              "port": np.asarray(port, np.int32).reshape(-1, 4), "chunk": np.asarray(chunk, np.int32).reshape(-1, 6),
-             "dense": np.asarray(dense, np.int32)}
+             "span": np.asarray(span, np.int32).reshape(-1, 4), "dense": np.asarray(dense, np.int32)}
     ends = [portions[order[s]][0].num_computed_tokens + counts[s] for s in dense]
     parts["cu_q"] = np.concatenate(([0], np.cumsum([counts[s] for s in dense]))).astype(np.int32)
     parts["cu_k"] = np.concatenate(([0], np.cumsum(ends))).astype(np.int32)
@@ -91,6 +94,7 @@ def build(portions, block_size: int, max_blocks: int, num_slots: int, num_blocks
     plan = StepPlan(input_ids=t["ids"], positions=t["pos"], slot_mapping=t["slots"], block_tables=t["tables"],
                     row_ctx=t["ctx"], state_slots=t["state"], decode_rows=decode_rows, row_seq=t["row_seq"],
                     max_keys=int(pos.max()) + 1, portions=t["port"], chunks=t["chunk"], ring_slot=t["ring"],
+                    spans=t["span"], max_span=max((n for _, n, _, _ in span), default=0),
                     dense_row=dense_row, dense_seqs=t["dense"], dense_cu_q=t["cu_q"], dense_cu_k=t["cu_k"],
                     dense_keys=int(sum(ends)), dense_max_q=max((counts[s] for s in dense), default=0),
                     dense_max_k=max(ends, default=0))
