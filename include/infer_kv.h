@@ -460,14 +460,18 @@ int infer_grouped_prefill(const void* q, int64_t q_stride, const void* k, int64_
  * Rows below decode_rows are single tokens with the state of slots[row] at positions[row] (a negative slot is padding:
  * zeros come out); the others belong to spans[.][4] = first row, tokens, slot, first position, two tokens or more.
  * state[slots][heads][rows][columns] (infer_decay_layout: [0] rows, [1] columns); a sequence at position 0 starts from
- * zero whatever it holds. */
+ * zero whatever it holds.  max_span: tokens of the longest span (a longer one is not computed whole); the workspace
+ * holds infer_decay_workspace_floats floats. */
 int infer_decay_layout(int64_t dim, int64_t vdim, int64_t* out2);
+int64_t infer_decay_workspace_floats(int elem, int64_t heads, int64_t dim, int64_t vdim, int64_t rot_dims,
+                                     int64_t num_spans, int64_t max_span);
 int infer_decay_attention(int elem, const void* proj, int64_t proj_stride, int64_t q_off, int64_t k_off, int64_t v_off,
                           int64_t g_off, int64_t heads, int64_t dim, int64_t vdim, const float* decay, int silu,
                           const float* table, int64_t rot_dims, int64_t max_pos, float scale, const float* norm,
                           int norm_per_head, int gate_silu, float eps, float* state, int64_t num_slots,
                           const int32_t* slots, const int64_t* positions, int64_t decode_rows, const int32_t* spans,
-                          int64_t num_spans, int64_t rows, void* out, int64_t out_stride, void* stream);
+                          int64_t num_spans, int64_t max_span, int64_t rows, float* workspace,
+                          int64_t workspace_floats, void* out, int64_t out_stride, void* stream);
 
 /* Gated delta rule with a decay per key channel.  A token's projection row holds the inputs of the short
  * convolution, q and k (kv_heads x dim each) and v (heads x vdim), from column 0 and the write-strength

@@ -78,9 +78,10 @@ SIGNATURES = {
     "infer_grouped_prefill": (_c.c_int, [_vp, _i64, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _i64, _vp, _i64,
                                          _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp]),
     "infer_decay_layout": (_c.c_int, [_i64, _i64, _vp]),
+    "infer_decay_workspace_floats": (_i64, [_c.c_int, _i64, _i64, _i64, _i64, _i64, _i64]),
     "infer_decay_attention": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _c.c_int,
                                          _vp, _i64, _i64, _f32, _vp, _c.c_int, _c.c_int, _f32, _vp, _i64, _vp, _vp,
-                                         _i64, _vp, _i64, _i64, _vp, _i64, _vp]),
+                                         _i64, _vp, _i64, _i64, _i64, _vp, _i64, _vp, _i64, _vp]),
     "infer_delta_layout": (_c.c_int, [_i64, _i64, _vp]),
     "infer_delta_step": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp,
                                     _vp, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp, _vp, _vp, _i64, _i64,

@@ -5,12 +5,22 @@
 //
 //   decay_step_kernel     one token per sequence (decode): one workgroup per (sequence, head), the state passes
 //                         through registers once; with a norm per head the norm and the gate are in it too
+//   decay_chunk_kernel    prompt portions in chunks of 32 tokens on bf16 matrix instructions
+//   decay_join_kernel     carries the state over the segments that a long portion is cut into
 //   decay_scan_any_kernel prompt portions of any size and element type, token by token
 //   decay_out_kernel      norm and gate of whole rows
 //
 // A sequence at position 0 starts from a zero state whatever its slot holds, so a slot needs no clearing when another
 // sequence takes it over.  d is held as a sum of two floats: its rounding error would enter a long memory once per
 // token.
+//
+// Chunk form.  With S the state before a chunk of n tokens,
+//     o_i = c (d^{i+1} q_i^T S + sum_{j<=i} d^{i-j} (q_i k_j) v_j) ,   S' = d^n S + sum_j k_j (d^{n-1-j} v_j)^T .
+// Everything of the recurrence is held to float precision although the products run as bf16: a float is the exact sum
+// of three bf16 numbers of 8 bits each (Split), and the products of the pieces are added up in float32, without those
+// below 2^-24 of the result.  Projections, with silu behind them or not, are bf16 already: one piece.
+// A portion with few heads is cut into segments that run side by side: first every segment from a zero state, keeping
+// only its final state, then the states are joined in order, then every segment with its outputs.
 #include "elem.h"
 
 namespace {
@@ -109,6 +119,411 @@ __global__ void __launch_bounds__(kThreads) decay_scan_any_kernel(DecayArgs<T> a
                 (T)((part[c] + part[16 + c] + part[32 + c] + part[48 + c]) * a.scale);
     }
     for (int d = r; d < a.dim_pad; d += 16) sp[(int64_t)d * a.vdim_pad] = s[d * 16 + c];
+}
+
+// ------------------------------------------------------------------ chunks of 32 tokens
+typedef short i16x4 __attribute__((ext_vector_type(4)));
+typedef short i16x8 __attribute__((ext_vector_type(8)));
+typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
+typedef uint32_t u32x2_t __attribute__((ext_vector_type(2)));
+
+constexpr int kC = 32;                           // tokens per chunk
+
+struct ChunkArgs {
+    DecayArgs<__bf16> a;
+    const Span* spans;
+    int seg_len, max_seg, slabs;                 // tokens per segment (a multiple of kC), segments of the longest span
+    float* ws;                                   // [span][max_seg][heads][dim_pad][vdim_pad], if max_seg > 1
+};
+
+// x as the exact sum of three bf16 numbers: the leading 8 bits of the mantissa, the next 8, the last 8
+struct Split { uint32_t hi, mid, lo; };          // as floats, low halves zero
+__device__ __forceinline__ Split split(float x) {
+    Split s;
+    s.hi = __builtin_bit_cast(uint32_t, x) & 0xffff0000u;
+    const float r = x - __builtin_bit_cast(float, s.hi);
+    s.mid = __builtin_bit_cast(uint32_t, r) & 0xffff0000u;
+    s.lo = __builtin_bit_cast(uint32_t, r - __builtin_bit_cast(float, s.mid));
+    return s;
+}
+// the high halves of two words, `a` in front
+__device__ __forceinline__ uint32_t pack(uint32_t a, uint32_t b) { return __builtin_amdgcn_perm(b, a, 0x07060302u); }
+
+template <int N>
+__device__ __forceinline__ void split_pack(const float (&x)[N], uint32_t (&p0)[N / 2], uint32_t (&p1)[N / 2], uint32_t (&p2)[N / 2]) {
+#pragma unroll
+    for (int i = 0; i < N / 2; ++i) {
+        const Split a = split(x[2 * i]), b = split(x[2 * i + 1]);
+        p0[i] = pack(a.hi, b.hi);
+        p1[i] = pack(a.mid, b.mid);
+        p2[i] = pack(a.lo, b.lo);
+    }
+}
+__device__ __forceinline__ bf16x8_t frag(const uint32_t (&p)[4]) { return __builtin_bit_cast(bf16x8_t, u32x4_t{p[0], p[1], p[2], p[3]}); }
+
+// sum of the products of the pieces of two operands, the first in three pieces, the second in PB
+template <int PB>
+__device__ __forceinline__ f32x4_t mfma_pieces(const bf16x8_t (&x)[3], const bf16x8_t (&y)[PB], f32x4_t acc) {
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[2], y[0], acc, 0, 0, 0);
+    if constexpr (PB == 3) {
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[0], y[2], acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[1], y[1], acc, 0, 0, 0);
+    }
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[1], y[0], acc, 0, 0, 0);
+    if constexpr (PB == 3) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[0], y[1], acc, 0, 0, 0);
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[0], y[0], acc, 0, 0, 0);
+}
+
+__device__ __forceinline__ void widen(u32x4_t x, float (&y)[8]) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        y[2 * i] = __builtin_bit_cast(float, x[i] << 16);
+        y[2 * i + 1] = __builtin_bit_cast(float, x[i] & 0xffff0000u);
+    }
+}
+__device__ __forceinline__ u32x4_t silu8(u32x4_t x) {
+    float y[8];
+    widen(x, y);
+    bf16x8_t r;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) r[i] = (__bf16)silu_f(y[i]);
+    return __builtin_bit_cast(u32x4_t, r);
+}
+
+// A workgroup of four wavefronts serves one head and 64 VT columns of its state over the chunks of one segment.
+// Wavefront w owns the columns 16 VT w .. and their part of the state, DT tiles of 32 rows, as accumulators: lane (g, n)
+// holds rows 16 t + 4 g + e of column n.  That is an operand of the next product as it lies, when the rows of a
+// k-step of 32 are taken in the order 16 tau + 4 g + e.  The 32 x 32 products q_i k_j are shared out over the
+// wavefronts, weighted, and exchanged through LDS.
+// PC: pieces of q and k (3 behind a rotation, otherwise 1).  OUT = false: only the final state, from zero.
+template <int DT, int VT, int PC, bool OUT>
+__global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
+    constexpr int kRow = DT * 64 + 16, kMat = kC * kRow;         // bytes: a token of q or k, one piece of a chunk
+    constexpr int kVRow = VT * 128 + 16, kPRow = 2 * kC + 16, kPMat = kC * kPRow;
+    constexpr int NU = DT > 4 ? DT / 4 : 1;                      // units of 16 columns of q and k per thread
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
+    const DecayArgs<__bf16>& a = args.a;
+    unsigned char* kbuf = lds;                                   // [PC][kMat]
+    unsigned char* vbuf = kbuf + PC * kMat;                      // [kC][kVRow]
+    unsigned char* qbuf = vbuf + kC * kVRow;                     // [PC][kMat]
+    unsigned char* pbuf = qbuf + PC * kMat;                      // [3][kPMat]
+    const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, n = lane & 15;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int h = blockIdx.y, slab = blockIdx.x % args.slabs, seg = blockIdx.x / args.slabs;
+    const Span span = args.spans[blockIdx.z];
+    const int first = seg * args.seg_len;
+    if (span.slot < 0 || span.slot >= a.num_slots || first >= span.count) return;
+    const bool last_seg = first + args.seg_len >= span.count;
+    if (!OUT && last_seg) return;                                // nobody needs its final state yet
+    const int count = last_seg ? span.count - first : args.seg_len;
+    const int row0 = span.row0 + first, pos0 = span.pos0 + first, chunks = (count + kC - 1) / kC;
+    const int v0 = slab * 64 * VT + wave * 16 * VT;              // this wavefront's first column
+    const bool live = v0 < a.vdim_pad;
+    const float log2d = a.decay[2 * a.heads + h];
+    const int64_t state_len = (int64_t)a.dim_pad * a.vdim_pad;
+    float* from = a.state + ((int64_t)span.slot * a.heads + h) * state_len;
+    float* to = from;
+    if (args.max_seg > 1) {
+        float* ws = args.ws + (((int64_t)blockIdx.z * args.max_seg + seg) * a.heads + h) * state_len;
+        if (OUT) from = ws;
+        else to = ws;
+    }
+    const bool load = OUT && (args.max_seg > 1 || span.pos0 > 0);
+
+    f32x4_t s[2 * DT][VT];
+#pragma unroll
+    for (int t = 0; t < 2 * DT; ++t)
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+            s[t][v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+            const int col = v0 + 16 * v + n;
+            if (load && col < a.vdim_pad)
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (16 * t + 4 * g + e < a.dim_pad) s[t][v][e] = from[(int64_t)(16 * t + 4 * g + e) * a.vdim_pad + col];
+        }
+
+    // entries behind the real sizes stay zero
+    for (int i = tid; i < (2 * PC * kMat + kC * kVRow) / 16; i += 256) reinterpret_cast<u32x4_t*>(lds)[i] = u32x4_t{0u, 0u, 0u, 0u};
+
+    // unit i of this thread: token, and two blocks of 8 columns, which turn together if they are rotated
+    const int units = a.dim / 16;
+    int u_tok[NU], u_b0[NU], u_b1[NU], u_pair[NU];
+#pragma unroll
+    for (int i = 0; i < NU; ++i) {
+        const int u = tid + 256 * i, w = u % units, rotated = a.rot_pairs / 8;
+        u_tok[i] = u < kC * units ? u / units : -1;
+        u_pair[i] = PC == 3 && w < rotated ? 8 * w : -1;
+        u_b0[i] = w < rotated ? 8 * w : 2 * a.rot_pairs + 16 * (w - rotated);
+        u_b1[i] = w < rotated ? 8 * w + a.rot_pairs : u_b0[i] + 8;
+    }
+    u32x4_t qreg[NU][2], kreg[NU][2], vreg[VT];
+    f32x4_t creg[PC == 3 ? NU : 1][4];
+    auto fetch = [&](int c) {
+        const int left = count - c * kC - 1;                     // tokens behind the last one re-read it
+#pragma unroll
+        for (int i = 0; i < NU; ++i) {
+            if (u_tok[i] < 0) continue;
+            const int t = c * kC + (u_tok[i] < left ? u_tok[i] : left);
+            const __bf16* r = a.proj + (int64_t)(row0 + t) * a.proj_stride + h * a.dim;
+            kreg[i][0] = *reinterpret_cast<const u32x4_t*>(r + a.k_off + u_b0[i]);
+            kreg[i][1] = *reinterpret_cast<const u32x4_t*>(r + a.k_off + u_b1[i]);
+            if constexpr (OUT) {
+                qreg[i][0] = *reinterpret_cast<const u32x4_t*>(r + a.q_off + u_b0[i]);
+                qreg[i][1] = *reinterpret_cast<const u32x4_t*>(r + a.q_off + u_b1[i]);
+            }
+            if constexpr (PC == 3) {
+                if (u_pair[i] >= 0) {
+                    const float* cs = table_row(a, pos0 + t) + 2 * u_pair[i];
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) creg[i][e] = *reinterpret_cast<const f32x4_t*>(cs + 4 * e);
+                }
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < VT; ++i) {
+            const int x = tid + 256 * i, tok = x / (8 * VT), col = slab * 64 * VT + 8 * (x % (8 * VT));
+            const int t = c * kC + (tok < left ? tok : left);
+            if (col < a.vdim) vreg[i] = *reinterpret_cast<const u32x4_t*>(a.proj + (int64_t)(row0 + t) * a.proj_stride + a.v_off + h * a.vdim + col);
+        }
+    };
+    // one block pair of q or k to LDS
+    auto put_unit = [&](unsigned char* buf, int i, const u32x4_t (&x)[2], bool in) {
+        unsigned char* r = buf + u_tok[i] * kRow;
+        if constexpr (PC == 1) {
+            u32x4_t y0 = x[0], y1 = x[1];
+            if (a.silu) { y0 = silu8(y0); y1 = silu8(y1); }
+            if (!in) y0 = y1 = u32x4_t{0u, 0u, 0u, 0u};
+            *reinterpret_cast<u32x4_t*>(r + 2 * u_b0[i]) = y0;
+            *reinterpret_cast<u32x4_t*>(r + 2 * u_b1[i]) = y1;
+        } else {
+            float y0[8], y1[8];
+            widen(x[0], y0);
+            widen(x[1], y1);
+            if (u_pair[i] >= 0)
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    const float cv = creg[i][e / 2][2 * (e & 1)], sv = creg[i][e / 2][2 * (e & 1) + 1], u = y0[e];
+                    y0[e] = u * cv - y1[e] * sv;
+                    y1[e] = y1[e] * cv + u * sv;
+                }
+            if (!in)
+#pragma unroll
+                for (int e = 0; e < 8; ++e) y0[e] = y1[e] = 0.f;
+            uint32_t p[3][4];
+            split_pack<8>(y0, p[0], p[1], p[2]);
+#pragma unroll
+            for (int k = 0; k < 3; ++k) *reinterpret_cast<bf16x8_t*>(r + k * kMat + 2 * u_b0[i]) = frag(p[k]);
+            split_pack<8>(y1, p[0], p[1], p[2]);
+#pragma unroll
+            for (int k = 0; k < 3; ++k) *reinterpret_cast<bf16x8_t*>(r + k * kMat + 2 * u_b1[i]) = frag(p[k]);
+        }
+    };
+    auto put = [&](int c) {
+        const int left = count - c * kC;
+#pragma unroll
+        for (int i = 0; i < NU; ++i) {
+            if (u_tok[i] < 0) continue;
+            put_unit(kbuf, i, kreg[i], u_tok[i] < left);
+            if constexpr (OUT) put_unit(qbuf, i, qreg[i], u_tok[i] < left);
+        }
+#pragma unroll
+        for (int i = 0; i < VT; ++i) {
+            const int x = tid + 256 * i, tok = x / (8 * VT), c8 = x % (8 * VT);
+            if (slab * 64 * VT + 8 * c8 >= a.vdim) continue;
+            u32x4_t y = a.silu ? silu8(vreg[i]) : vreg[i];
+            if (tok >= left) y = u32x4_t{0u, 0u, 0u, 0u};
+            *reinterpret_cast<u32x4_t*>(vbuf + tok * kVRow + 16 * c8) = y;
+        }
+    };
+
+    // weights of the products: this lane's query column n of tile w / 2, keys 4 g + e of tile w % 2
+    float pw[4], qw[2], vw[8];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        const int dist = 16 * (wave >> 1) + n - (16 * (wave & 1) + 4 * g + e);
+        pw[e] = dist >= 0 ? a.scale * exp2f(dist * log2d) : 0.f;
+    }
+#pragma unroll
+    for (int t = 0; t < 2; ++t) qw[t] = a.scale * exp2f((16 * t + n + 1) * log2d);
+    auto value_weights = [&](int tokens) {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const int after = tokens - 1 - (8 * g + i);
+            vw[i] = exp2f((after > 0 ? after : 0) * log2d);      // values behind the last token are zero
+        }
+    };
+    value_weights(kC);
+    float chunk_decay = exp2f(kC * log2d);
+
+    fetch(0);
+    __syncthreads();                                             // the zero fill
+    for (int c = 0; c < chunks; ++c) {
+        put(c);
+        __syncthreads();
+        if (c + 1 < chunks) fetch(c + 1);
+        const int left = count - c * kC;
+        if (left < kC) {
+            value_weights(left);
+            chunk_decay = exp2f(left * log2d);
+        }
+        if constexpr (OUT) {
+            // ---- d^(i-j) q_i k_j: rows are keys, columns queries; the tile above the diagonal is all zeros
+            f32x4_t p = {0.f, 0.f, 0.f, 0.f};
+            if (wave != 1) {
+                const unsigned char* kr = kbuf + (16 * (wave & 1) + n) * kRow + 16 * g;
+                const unsigned char* qr = qbuf + (16 * (wave >> 1) + n) * kRow + 16 * g;
+#pragma unroll
+                for (int j = 0; j < DT; ++j) {
+                    bf16x8_t kf[PC], qf[PC];
+#pragma unroll
+                    for (int k = 0; k < PC; ++k) {
+                        kf[k] = *reinterpret_cast<const bf16x8_t*>(kr + k * kMat + 64 * j);
+                        qf[k] = *reinterpret_cast<const bf16x8_t*>(qr + k * kMat + 64 * j);
+                    }
+                    if constexpr (PC == 3) p = mfma_pieces<3>(kf, qf, p);
+                    else p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0], qf[0], p, 0, 0, 0);
+                }
+            }
+            float x[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[e] = p[e] * pw[e];
+            uint32_t p0[2], p1[2], p2[2];
+            split_pack<4>(x, p0, p1, p2);
+            unsigned char* pr = pbuf + (16 * (wave >> 1) + n) * kPRow + 2 * (16 * (wave & 1) + 4 * g);
+            *reinterpret_cast<u32x2_t*>(pr) = u32x2_t{p0[0], p0[1]};
+            *reinterpret_cast<u32x2_t*>(pr + kPMat) = u32x2_t{p1[0], p1[1]};
+            *reinterpret_cast<u32x2_t*>(pr + 2 * kPMat) = u32x2_t{p2[0], p2[1]};
+            __syncthreads();
+        }
+        if (live) {
+            bf16x8_t vf[VT];                                     // values of tokens 8 g .. + 7, column n
+            const unsigned char* vr = vbuf + (8 * g + (n >> 2)) * kVRow + (n & 3) * 8 + 32 * VT * wave;
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 32 * v));
+                const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 32 * v + 4 * kVRow));
+                vf[v] = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+            }
+            if constexpr (OUT) {
+                f32x4_t acc[VT][2];                              // rows are columns of the state, columns queries
+#pragma unroll
+                for (int v = 0; v < VT; ++v)
+#pragma unroll
+                    for (int t = 0; t < 2; ++t) acc[v][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+                // ---- q_i^T S
+#pragma unroll
+                for (int j = 0; j < DT; ++j) {
+                    bf16x8_t qf[2][PC];
+#pragma unroll
+                    for (int t = 0; t < 2; ++t)
+#pragma unroll
+                        for (int k = 0; k < PC; ++k) {
+                            const unsigned char* qr = qbuf + k * kMat + (16 * t + n) * kRow + 64 * j + 8 * g;
+                            const u32x2_t x = *reinterpret_cast<const u32x2_t*>(qr), y = *reinterpret_cast<const u32x2_t*>(qr + 32);
+                            qf[t][k] = __builtin_bit_cast(bf16x8_t, u32x4_t{x[0], x[1], y[0], y[1]});
+                        }
+#pragma unroll
+                    for (int v = 0; v < VT; ++v) {
+                        float x[8];
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) { x[e] = s[2 * j][v][e]; x[4 + e] = s[2 * j + 1][v][e]; }
+                        uint32_t p0[4], p1[4], p2[4];
+                        split_pack<8>(x, p0, p1, p2);
+                        const bf16x8_t sf[3] = {frag(p0), frag(p1), frag(p2)};
+#pragma unroll
+                        for (int t = 0; t < 2; ++t) acc[v][t] = mfma_pieces<PC>(sf, qf[t], acc[v][t]);
+                    }
+                }
+                // ---- the chunk's own tokens
+#pragma unroll
+                for (int t = 0; t < 2; ++t) {
+                    bf16x8_t pf[3];
+#pragma unroll
+                    for (int k = 0; k < 3; ++k) pf[k] = *reinterpret_cast<const bf16x8_t*>(pbuf + k * kPMat + (16 * t + n) * kPRow + 16 * g);
+#pragma unroll
+                    for (int v = 0; v < VT; ++v) {
+                        acc[v][t] *= qw[t];
+#pragma unroll
+                        for (int k = 2; k >= 0; --k) acc[v][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[v], pf[k], acc[v][t], 0, 0, 0);
+                        const int col = v0 + 16 * v + 4 * g;
+                        if (16 * t + n < left && col < a.vdim) {
+                            bf16x4_t o;
+#pragma unroll
+                            for (int e = 0; e < 4; ++e) o[e] = (__bf16)acc[v][t][e];
+                            *reinterpret_cast<bf16x4_t*>(a.o + (int64_t)(row0 + c * kC + 16 * t + n) * a.o_stride + (int64_t)h * a.vdim + col) = o;
+                        }
+                    }
+                }
+            }
+            // ---- S <- d^n S + sum_j k_j (d^(n-1-j) v_j)^T
+            bf16x8_t wf[VT][3];
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                float x[8];
+                widen(__builtin_bit_cast(u32x4_t, vf[v]), x);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) x[i] *= vw[i];
+                uint32_t p0[4], p1[4], p2[4];
+                split_pack<8>(x, p0, p1, p2);
+                wf[v][0] = frag(p0);
+                wf[v][1] = frag(p1);
+                wf[v][2] = frag(p2);
+            }
+            const unsigned char* kr = kbuf + (8 * g + (n >> 2)) * kRow + (n & 3) * 8;
+#pragma unroll
+            for (int t = 0; t < 2 * DT; ++t) {
+                bf16x8_t kf[PC];
+#pragma unroll
+                for (int k = 0; k < PC; ++k) {
+                    const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(kr + k * kMat + 32 * t));
+                    const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(kr + k * kMat + 32 * t + 4 * kRow));
+                    kf[k] = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+                }
+#pragma unroll
+                for (int v = 0; v < VT; ++v) {
+                    s[t][v] *= chunk_decay;
+                    if constexpr (PC == 3) {
+                        s[t][v] = mfma_pieces<3>(kf, wf[v], s[t][v]);
+                    } else {
+#pragma unroll
+                        for (int k = 2; k >= 0; --k) s[t][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0], wf[v][k], s[t][v], 0, 0, 0);
+                    }
+                }
+            }
+        }
+        __syncthreads();
+    }
+    if (OUT && !last_seg) return;
+#pragma unroll
+    for (int t = 0; t < 2 * DT; ++t)
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+            const int col = v0 + 16 * v + n;
+            if (col < a.vdim_pad)
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (16 * t + 4 * g + e < a.dim_pad) to[(int64_t)(16 * t + 4 * g + e) * a.vdim_pad + col] = s[t][v][e];
+        }
+}
+
+// ws[span][segment] holds what a segment adds to the state; afterwards the state before the segment
+__global__ void __launch_bounds__(kThreads) decay_join_kernel(ChunkArgs args) {
+    const DecayArgs<__bf16>& a = args.a;
+    const int h = blockIdx.y;
+    const Span span = args.spans[blockIdx.z];
+    const int64_t state_len = (int64_t)a.dim_pad * a.vdim_pad, i = ((int64_t)blockIdx.x * kThreads + threadIdx.x) * 4;
+    if (span.slot < 0 || span.slot >= a.num_slots || i >= state_len) return;
+    const float seg_decay = exp2f((float)args.seg_len * a.decay[2 * a.heads + h]);
+    f32x4_t s = {0.f, 0.f, 0.f, 0.f};
+    if (span.pos0 > 0) s = *reinterpret_cast<const f32x4_t*>(a.state + ((int64_t)span.slot * a.heads + h) * state_len + i);
+    for (int seg = 0; seg * args.seg_len < span.count; ++seg) {
+        f32x4_t* p = reinterpret_cast<f32x4_t*>(args.ws + (((int64_t)blockIdx.z * args.max_seg + seg) * a.heads + h) * state_len + i);
+        f32x4_t add = {0.f, 0.f, 0.f, 0.f};
+        if ((seg + 1) * args.seg_len < span.count) add = *p;
+        *p = s;
+        s = s * seg_decay + add;
+    }
 }
 
 // ------------------------------------------------------------------ one token per sequence
@@ -310,6 +725,63 @@ int launch_any(const DecayArgs<T>& a, const Span* spans, const int32_t* slots, c
     return (int)hipGetLastError();
 }
 
+// sizes the chunk kernel is built for
+bool chunks_fit(int elem, int64_t dim, int64_t vdim, int64_t rot_dims) {
+    return elem == INFER_ELEM_BF16 && dim % 16 == 0 && vdim % 8 == 0 && dim <= 256 && rot_dims % 16 == 0;
+}
+int tiles_of(int64_t dim_pad) { return dim_pad <= 32 ? 1 : dim_pad <= 64 ? 2 : dim_pad <= 128 ? 4 : 8; }
+int column_tiles(int64_t dim_pad, int64_t vdim_pad) { return vdim_pad <= 64 || dim_pad > 128 ? 1 : 2; }
+int slabs_of(int64_t dim_pad, int64_t vdim_pad) {
+    const int cols = 64 * column_tiles(dim_pad, vdim_pad);
+    return (int)((vdim_pad + cols - 1) / cols);
+}
+// tokens per segment: enough segments for two workgroups per compute unit, none shorter than four chunks
+int64_t segment_len(int64_t heads, int64_t slabs, int64_t num_spans, int64_t max_span) {
+    const int64_t groups = heads * slabs * num_spans;
+    int64_t n = (512 + groups - 1) / groups;
+    const int64_t most = max_span / (4 * kC);
+    if (n > most) n = most;
+    if (n <= 1) return (max_span + kC - 1) / kC * kC;
+    return ((max_span + n - 1) / n + kC - 1) / kC * kC;
+}
+
+template <int DT, int VT, int PC, bool OUT>
+int launch_chunk(const ChunkArgs& c, int64_t num_spans, hipStream_t st) {
+    const size_t lds = (size_t)kC * (2 * PC * (DT * 64 + 16) + VT * 128 + 16) + (OUT ? 3 * kC * (2 * kC + 16) : 0);
+    auto kernel = &decay_chunk_kernel<DT, VT, PC, OUT>;
+    if (lds > 64 * 1024) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return (int)e;
+    }
+    hipLaunchKernelGGL(kernel, dim3((unsigned)(c.slabs * c.max_seg), (unsigned)c.a.heads, (unsigned)num_spans), dim3(256), lds, st, c);
+    return (int)hipGetLastError();
+}
+
+template <int DT, int VT>
+int launch_chunks(const ChunkArgs& c, int64_t num_spans, hipStream_t st) {
+    const bool rot = c.a.rot_pairs > 0;
+    int rc;
+    if (c.max_seg > 1) {
+        rc = rot ? launch_chunk<DT, VT, 3, false>(c, num_spans, st) : launch_chunk<DT, VT, 1, false>(c, num_spans, st);
+        if (rc) return rc;
+        const unsigned blocks = (unsigned)(((int64_t)c.a.dim_pad * c.a.vdim_pad / 4 + kThreads - 1) / kThreads);
+        hipLaunchKernelGGL(decay_join_kernel, dim3(blocks, (unsigned)c.a.heads, (unsigned)num_spans), dim3(kThreads), 0, st, c);
+        rc = (int)hipGetLastError();
+        if (rc) return rc;
+    }
+    return rot ? launch_chunk<DT, VT, 3, true>(c, num_spans, st) : launch_chunk<DT, VT, 1, true>(c, num_spans, st);
+}
+
+int run_chunks(const ChunkArgs& c, int64_t num_spans, hipStream_t st) {
+    const int vt = column_tiles(c.a.dim_pad, c.a.vdim_pad);
+    switch (tiles_of(c.a.dim_pad)) {
+        case 1: return vt == 1 ? launch_chunks<1, 1>(c, num_spans, st) : launch_chunks<1, 2>(c, num_spans, st);
+        case 2: return vt == 1 ? launch_chunks<2, 1>(c, num_spans, st) : launch_chunks<2, 2>(c, num_spans, st);
+        case 4: return vt == 1 ? launch_chunks<4, 1>(c, num_spans, st) : launch_chunks<4, 2>(c, num_spans, st);
+        default: return launch_chunks<8, 1>(c, num_spans, st);
+    }
+}
+
 template <class T, bool FUSED>
 int launch_step(const DecayArgs<T>& a, const DecayOutArgs<T>& b, const int32_t* slots, const int64_t* positions, int64_t rows, hipStream_t st) {
     const int cgs = a.vdim_pad / 4, rgs = kThreads / cgs, np = (a.dim_pad + rgs - 1) / rgs;
@@ -339,16 +811,25 @@ extern "C" int infer_decay_layout(int64_t dim, int64_t vdim, int64_t* out2) {
     return INFER_KV_OK;
 }
 
+extern "C" int64_t infer_decay_workspace_floats(int elem, int64_t heads, int64_t dim, int64_t vdim, int64_t rot_dims, int64_t num_spans,
+                                                int64_t max_span) {
+    int64_t pad[2];
+    if (infer_decay_layout(dim, vdim, pad) || heads < 1 || num_spans < 1 || max_span < 1 || !chunks_fit(elem, dim, vdim, rot_dims)) return 0;
+    const int64_t len = segment_len(heads, slabs_of(pad[0], pad[1]), num_spans, max_span), n = (max_span + len - 1) / len;
+    return n > 1 ? num_spans * n * heads * pad[0] * pad[1] : 0;
+}
+
 extern "C" int infer_decay_attention(int elem, const void* proj, int64_t proj_stride, int64_t q_off, int64_t k_off, int64_t v_off,
                                      int64_t g_off, int64_t heads, int64_t dim, int64_t vdim, const float* decay, int silu,
                                      const float* table, int64_t rot_dims, int64_t max_pos, float scale, const float* norm,
                                      int norm_per_head, int gate_silu, float eps, float* state, int64_t num_slots,
                                      const int32_t* slots, const int64_t* positions, int64_t decode_rows, const int32_t* spans,
-                                     int64_t num_spans, int64_t rows, void* out, int64_t out_stride, void* stream) {
+                                     int64_t num_spans, int64_t max_span, int64_t rows, float* workspace, int64_t workspace_floats,
+                                     void* out, int64_t out_stride, void* stream) {
     int64_t pad[2];
     if (!size_in(rows, 0, 0x7fffffff) || !size_in(decode_rows, 0, rows) || !size_in(num_spans, 0, 65535)) return INFER_KV_EINVAL;
     if (rows == 0) return INFER_KV_OK;
-    if (!proj || !decay || !state || !out || (decode_rows > 0 && (!slots || !positions)) || (decode_rows < rows && (!spans || num_spans < 1)))
+    if (!proj || !decay || !state || !out || (decode_rows > 0 && (!slots || !positions)) || (decode_rows < rows && (!spans || num_spans < 1 || max_span < 1 || max_span > rows)))
         return INFER_KV_EINVAL;
     int rc = infer_decay_layout(dim, vdim, pad);
     if (rc) return rc;
@@ -379,7 +860,21 @@ extern "C" int infer_decay_attention(int elem, const void* proj, int64_t proj_st
             }
             if (rc) return rc;
         }
-        if (decode_rows < rows) rc = launch_any(a, (const Span*)spans, nullptr, nullptr, num_spans, st);
+        if (decode_rows < rows) {
+            bool chunked = false;
+            if constexpr (sizeof(T) == 2) {
+                chunked = chunks_fit(elem, dim, vdim, rot_dims) && (q_off | k_off | v_off | proj_stride) % 8 == 0 && ptr_aligned(proj, 16) &&
+                          out_stride % 4 == 0 && ptr_aligned(out, 8) && ptr_aligned(table, 16);
+                if (chunked) {
+                    const int slabs = slabs_of(pad[0], pad[1]);
+                    const int64_t len = segment_len(heads, slabs, num_spans, max_span), n = (max_span + len - 1) / len;
+                    if (n > 1 && (!workspace || !ptr_aligned(workspace, 16) || workspace_floats < num_spans * n * heads * pad[0] * pad[1]))
+                        return (int)INFER_KV_EWORKSPACE;
+                    rc = run_chunks(ChunkArgs{a, (const Span*)spans, (int)len, (int)n, slabs, workspace}, num_spans, st);
+                }
+            }
+            if (!chunked) rc = launch_any(a, (const Span*)spans, nullptr, nullptr, num_spans, st);
+        }
         if (rc || finished == rows) return rc;
         b.o += finished * out_stride;
         b.out += finished * out_stride;

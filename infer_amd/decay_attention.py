@@ -45,5 +45,5 @@ class DecayAttention(nn.Module):
         out = torch.empty((h.shape[0], s.heads * s.vdim), dtype=h.dtype, device=h.device)
         offset = self.in_proj.offset
         hybrid_ops.decay_attention(s, proj, [offset[name] for name in "qkvg"], self.decay, self.table, self.out_norm, cache["state"],
-                                   plan.state_slots, plan.positions, plan.decode_rows, plan.spans, out)
+                                   plan.state_slots, plan.positions, plan.decode_rows, plan.spans, plan.max_span, out)
         return self.o_proj(out, defer=True)

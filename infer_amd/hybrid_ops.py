@@ -345,10 +345,12 @@ class DecayShape:
         self.state_rows, self.state_cols = decay_layout(dim, vdim)
 
 
-def decay_attention(s: DecayShape, proj, offsets, decay, table, norm, state, slots, positions, decode_rows: int, spans, out) -> None:
+def decay_attention(s: DecayShape, proj, offsets, decay, table, norm, state, slots, positions, decode_rows: int, spans, max_span: int,
+                    out) -> None:
     """``proj`` holds q, k, v and the gate logits at the columns ``offsets``.  Rows below ``decode_rows`` advance the state of
     ``slots[r]`` by one token (negative: padding), the others belong to ``spans`` [.., 4] (first row, tokens, slot, first
-    position).  ``decay`` comes from ``decay_constants``."""
+    position).  ``max_span`` is the number of tokens of the longest.  ``decay`` comes from
+    ``decay_constants``."""
     n = proj.shape[0]
     q, k, v, g = offsets
     assert proj.dtype == out.dtype and out.shape[0] == n
@@ -361,17 +363,19 @@ def decay_attention(s: DecayShape, proj, offsets, decay, table, norm, state, slo
     if decode_rows:
         assert slots.dtype == torch.int32 and slots.is_contiguous() and slots.numel() >= decode_rows
         assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() >= decode_rows
-    num_spans = 0
+    lib, num_spans, ws, need = _lib.load(), 0, None, 0
     if decode_rows < n:
         assert spans.dtype == torch.int32 and spans.is_contiguous() and spans.shape[1] == 4
         num_spans = spans.shape[0]
+        need = lib.infer_decay_workspace_floats(ELEM[proj.dtype], s.heads, s.dim, s.vdim, s.rot_dims, num_spans, max_span)
+        ws = torch.empty(need, dtype=torch.float32, device=proj.device) if need else None
     _require_gpu(proj, decay, state, out)
-    rc = _lib.load().infer_decay_attention(
+    rc = lib.infer_decay_attention(
         ELEM[proj.dtype], proj.data_ptr(), _rows(proj, max(q + s.heads * s.dim, k + s.heads * s.dim, v + s.heads * s.vdim, g + s.heads * s.vdim)),
         q, k, v, g, s.heads, s.dim, s.vdim, decay.data_ptr(), int(s.silu), _ptr(table) if s.rot_dims else None, s.rot_dims,
         table.shape[0] if s.rot_dims else 1, float(s.scale), _ptr(norm), int(s.norm_per_head), int(s.gate_silu), float(s.eps),
-        state.data_ptr(), state.shape[0], _ptr(slots), _ptr(positions), decode_rows, _ptr(spans) if num_spans else None, num_spans, n,
-        out.data_ptr(), _rows(out, s.heads * s.vdim), _stream_ptr(proj))
+        state.data_ptr(), state.shape[0], _ptr(slots), _ptr(positions), decode_rows, _ptr(spans) if num_spans else None, num_spans, max_span, n,
+        _ptr(ws), need, out.data_ptr(), _rows(out, s.heads * s.vdim), _stream_ptr(proj))
     _lib.check(rc, "decay_attention")
 
 
