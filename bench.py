@@ -247,6 +247,23 @@ def hybrid_config(size):
     return MerilornConfig(vocab_size=151936, hidden_size=width, layers=specs, embedding_scale=width ** 0.5)
 
 
+def vokelix_config(size):
+    """Vokelix of a published model's width: two lightning layers, one of retention, one of grouped attention with 8 key
+    heads, all with a feed-forward; every second attention layer uses the keys of the one before; heads of 128."""
+    from infer_amd.config import LayerSpec, VokelixConfig
+    width, ff, heads, layers = HYBRID_SIZES[size]
+    attn = {"heads": heads, "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+            "rot": {"base": 1e6, "dims": 64, "scaling": {"factor": 4.0, "original": 8192, "fast": 16.0, "slow": 2.0}}}
+    decay = [1.0 - 2.0 ** (-4.0 - 7.0 * h / heads) for h in range(heads)]
+    linear = {"heads": heads, "dim": 128, "vdim": 128, "decay": decay}
+    kinds = {0: ("lightning", linear), 1: ("lightning", linear), 2: ("retention", {**linear, "rot": {"base": 1e4, "dims": 128}})}
+    specs = []
+    for i in range(layers):
+        kind, mixer = kinds.get(i % 4, ("attention", {**attn, "kv_from": i - 4} if i % 8 == 7 else attn))
+        specs.append(LayerSpec(kind, mixer, ff, i))
+    return VokelixConfig(vocab_size=151936, hidden_size=width, layers=specs, residual_alpha=2.0)
+
+
 def hybrid_engine_point(size, model, batch, prompt, new):
     """Prefill and decode throughput of the engine on ``batch`` prompts of ``prompt`` random tokens."""
     import numpy as np
@@ -254,8 +271,10 @@ def hybrid_engine_point(size, model, batch, prompt, new):
     from infer_amd.llm_engine import LLMEngine
     from infer_amd.sampling_params import SamplingParams
     width, ff, heads, layers = HYBRID_SIZES[size]
-    hf = hybrid_config(size) if model == "merilorn" else C.ModelConfig(
-        hidden_size=width, intermediate_size=ff, num_hidden_layers=layers, num_attention_heads=heads, num_key_value_heads=8)
+    if model == "qwen3":
+        hf = C.ModelConfig(hidden_size=width, intermediate_size=ff, num_hidden_layers=layers, num_attention_heads=heads, num_key_value_heads=8)
+    else:
+        hf = {"merilorn": hybrid_config, "vokelix": vokelix_config}[model](size)
     blocks = batch * (-(-(prompt + new) // 256) + 1)
     engine = LLMEngine(hf_config=hf, max_num_seqs=max(batch, 16), max_model_len=prompt + new + 1,
                        max_num_batched_tokens=16384, num_kvcache_blocks=blocks, seed=0)
@@ -277,16 +296,11 @@ def hybrid_engine_point(size, model, batch, prompt, new):
     return point
 
 
-def hybrid_kernels(heads=32, width=4096, ff=12288):
-    """Every kernel of the design at the sizes of an 8B model's layers, with what bounds it, beside the like kernel of
-    Qwen3 at the same sizes."""
-    from infer_amd import hybrid_ops as ho, ops, workloads
-    from infer_amd.layers import yarn_rotary_table
-    from infer_amd.step_plan import CHUNK
-    dev, bf = torch.device("cuda:0"), torch.bfloat16
+def roofline_table(dev):
+    """A dict of timed kernels, and the functions that time one against the memory bandwidth or a matrix peak."""
     out = {}
 
-    def rnd(*shape, dtype=bf):
+    def rnd(*shape, dtype=torch.bfloat16):
         return torch.randn(*shape, dtype=dtype, device=dev)
 
     def hbm(name, nbytes, fn, note=""):
@@ -298,6 +312,18 @@ def hybrid_kernels(heads=32, width=4096, ff=12288):
         ms = gpu_time_ms_median(fn, 20, 5)
         out[name] = {"us": round(ms * 1e3, 2), "bound": "mfma", "TFLOPs": round(flops / ms / 1e9, 1),
                      "frac": round(flops / ms / 1e9 / peak, 4), **({"note": note} if note else {})}
+
+    return out, rnd, hbm, mfma
+
+
+def hybrid_kernels(heads=32, width=4096, ff=12288):
+    """Every kernel of the design at the sizes of an 8B model's layers, with what bounds it, beside the like kernel of
+    Qwen3 at the same sizes."""
+    from infer_amd import hybrid_ops as ho, ops, workloads
+    from infer_amd.layers import yarn_rotary_table
+    from infer_amd.step_plan import CHUNK
+    dev, bf = torch.device("cuda:0"), torch.bfloat16
+    out, rnd, hbm, mfma = roofline_table(dev)
 
     # ---- decode attention, batch 64 x ctx 4096
     b, ctx, bs, row, rank, dim, rot, vdim = 64, 4096, 256, 576, 512, 128, 64, 128
@@ -398,16 +424,148 @@ def hybrid_kernels(heads=32, width=4096, ff=12288):
     return out
 
 
+def vokelix_kernels(heads=32, kv_heads=8, width=4096, ff=12288):
+    """Every kernel of Vokelix at the sizes of an 8B model's layers, with what bounds it, beside the like kernel of Qwen3
+    (attention, norms, activation) or Merilorn (recurrence) at the same sizes.  Buffers are larger than the caches or
+    rotated, where a kernel's bytes would fit them."""
+    from infer_amd import hybrid_ops as ho, ops, workloads
+    from infer_amd.layers import yarn_rotary_table
+    from infer_amd.step_plan import CHUNK
+    dev, bf = torch.device("cuda:0"), torch.bfloat16
+    out, rnd, hbm, mfma = roofline_table(dev)
+    d, n, sq = 128, 8, 2048
+    rows = n * sq
+
+    # ---- decode attention
+    bs = 256
+    for b, ctx in ((64, 4096), (64, 1024), (16, 4096)):
+        nblk = b * ctx // bs
+        cache = rnd(nblk, kv_heads, bs, 2 * d)
+        tables = torch.randperm(nblk, device=dev).to(torch.int32).view(b, -1)
+        lens = torch.full((b,), ctx, dtype=torch.int32, device=dev)
+        qx, gate, sink, o = rnd(b, heads, d), rnd(b, heads), torch.randn(heads, device=dev), torch.empty((b, heads * d), dtype=bf, device=dev)
+        hbm(f"grouped_attention decode, {b} x {ctx}", b * ctx * kv_heads * 2 * d * 2,
+            lambda: ho.grouped_attention(qx, cache, tables, lens, 0.09, d, o, sink, gate))
+        wl = workloads.make_decode_workload("point", [ctx] * b, heads, kv_heads, seed=0, q_scale=d ** -0.5, device=dev, device_fill=True)
+        o3 = torch.empty((b, heads, d), dtype=bf, device=dev)
+        hbm(f"qwen3: paged decode attention, {b} x {ctx}", wl.decode_bytes,
+            lambda: ops.paged_attn_decode(wl.q, wl.k_cache, wl.v_cache, wl.block_table, wl.context_lens, wl.scale, o3))
+        del wl, cache
+
+    # ---- prefill attention
+    cu = torch.arange(0, n + 1, dtype=torch.int32, device=dev) * sq
+    nblk = rows // bs
+    cache = rnd(nblk, kv_heads, bs, 2 * d)
+    tables = torch.randperm(nblk, device=dev).to(torch.int32).view(n, -1)
+    seqs = torch.arange(n, dtype=torch.int32, device=dev)
+    hbm(f"grouped_gather, {rows} rows", 2 * cache.numel() * 2, lambda: ho.grouped_gather(cache, tables, seqs, cu, rows, sq))
+    kv = ho.grouped_gather(cache, tables, seqs, cu, rows, sq)
+    proj, at, sink = rnd(rows, (heads + 2 * kv_heads) * d + 64), torch.empty((rows, heads * d), dtype=bf, device=dev), torch.randn(heads, device=dev)
+    pairs = n * sq * (sq + 1) // 2
+    mfma("grouped_prefill, 8 x 2048", 4 * heads * d * pairs, BF16_PEAK_TFLOPS,
+         lambda: ho.grouped_prefill(proj, kv[:, :, d:], kv[:, :, :d], sink, proj[:, -heads:], at, cu, cu, sq, heads, d, d, 0.09))
+    q3, k3 = rnd(rows, heads, d), rnd(rows, kv_heads, d)
+    mfma("qwen3: prefill attention, 8 x 2048", 4 * heads * d * pairs, BF16_PEAK_TFLOPS,
+         lambda: ops.flash_attn_varlen_func(q3, k3, k3, max_seqlen_q=sq, cu_seqlens_q=cu, max_seqlen_k=sq, cu_seqlens_k=cu))
+    del q3, k3, kv
+
+    # ---- front end
+    table = yarn_rotary_table(64, 8192, 1e6, None, dev)
+    for t in (64, rows):
+        pos = torch.randint(0, 8192, (t,), device=dev)
+        slots = torch.randperm(nblk * bs, device=dev)[:t].to(torch.int32)
+        x = proj[:t]
+        bias, qn, kn = (torch.randn(c, device=dev) for c in (proj.shape[1], heads * d, kv_heads * d))
+        qx = rnd(t if t == 64 else 1, heads, d)
+        moved = t * 2 * (2 * heads + 4 * kv_heads) * d
+        hbm(f"grouped_front, {t} rows", moved, lambda: ho.grouped_front(
+            x, heads, kv_heads, d, d, heads * d, (heads + kv_heads) * d, bias, qn, kn, 1e-6, table, 64, pos, slots, cache, d, d, qx, t if t == 64 else 0))
+        qkv = rnd(t, (heads + 2 * kv_heads) * d)
+        qv, kk, vv = (y.view(t, -1, d) for y in qkv.split([heads * d, kv_heads * d, kv_heads * d], dim=-1))
+        kc, w128, cs = rnd(nblk, bs, kv_heads, d), torch.ones(d, dtype=bf, device=dev), rnd(8192, d)
+        hbm(f"qwen3: norm + rotary + append, {t} rows", moved,
+            lambda: ops.qk_norm_rope_store_kvcache(qv, kk, vv, pos, w128, w128, 1e-6, cs, kc, kc, slots, write_key=False))
+        del kc, qkv
+    del proj, at, cache
+
+    # ---- linear attention
+    state = torch.zeros(64, heads, d, d, device=dev)
+    hd = heads * d
+    decay = ho.decay_constants([1.0 - 2.0 ** (-4.0 - 7.0 * h / heads) for h in range(heads)], dev)
+    table = yarn_rotary_table(d, 8192, 1e4, None, dev)
+    kinds = {"lightning": (ho.DecayShape(heads, d, d, 1e-6, True, 0, 1.0, False, False), None, torch.ones(hd, device=dev)),
+             "retention": (ho.DecayShape(heads, d, d, 1e-6, False, d, d ** -0.5, True, True), table, None)}
+    sl, pos = torch.arange(64, dtype=torch.int32, device=dev), torch.full((64,), 77, dtype=torch.int64, device=dev)
+    off = [0, hd, 2 * hd, 3 * hd]
+    x, o2 = rnd(64, 4 * hd), torch.empty((64, hd), dtype=bf, device=dev)
+    for kind, (s, tab, norm) in kinds.items():
+        hbm(f"decay_attention ({kind}), one token x 64", 2 * state.numel() * 4 + 5 * 64 * hd * 2,
+            lambda: ho.decay_attention(s, x, off, decay, tab, norm, state, sl, pos, 64, None, 0, o2))
+    for m, length in ((1, 2048), (8, 2048), (1, 16384)):
+        t = m * length
+        x, o2 = rnd(t, 4 * hd), torch.empty((t, hd), dtype=bf, device=dev)
+        spans = torch.tensor([(i * length, length, i, 0) for i in range(m)], dtype=torch.int32, device=dev)
+        for kind, (s, tab, norm) in kinds.items():
+            tab = yarn_rotary_table(d, 16384, 1e4, None, dev) if tab is not None else None
+            hbm(f"decay_attention ({kind}), {m} x {length}", 5 * t * hd * 2,
+                lambda: ho.decay_attention(s, x, off, decay, tab, norm, state, None, None, 0, spans, length, o2), "all launches; q, k, v, gate, result")
+    del x
+    s = ho.DeltaShape(heads, heads, d, d, 4, 1e-6)
+    ring = torch.zeros(64, 4, s.channels, dtype=bf, device=dev)
+    wts = [torch.randn(s.channels, 4, device=dev) * .5, torch.zeros(heads, device=dev), torch.full((hd,), -3.0, device=dev), torch.ones(d, device=dev)]
+    x, dec, gt = rnd(64, s.channels + heads), rnd(64, hd), rnd(64, hd)
+    o2 = torch.empty((64, hd), dtype=bf, device=dev)
+    hbm("merilorn: delta_step, one token x 64", 2 * state.numel() * 4 + 2 * (x.numel() + 3 * dec.numel() + 5 * s.channels // 3 * 64),
+        lambda: ho.delta_step(s, x, s.channels, dec, gt, *wts, ring, state, sl, pos, o2))
+    for m in (1, 8):
+        t = m * sq
+        x, dec, gt, o2 = rnd(t, s.channels + heads), rnd(t, hd), rnd(t, hd), torch.empty((t, hd), dtype=bf, device=dev)
+        per = sq // CHUNK
+        portions = torch.tensor([(i * per, per, i, 0) for i in range(m)], dtype=torch.int32, device=dev)
+        chunks = torch.tensor([(i * sq + r, CHUNK, r, 0, i, 0) for i in range(m) for r in range(0, sq, CHUNK)], dtype=torch.int32, device=dev)
+        rs = torch.tensor([(i, sq - 1 - r) for i in range(m) for r in range(sq)], dtype=torch.int32, device=dev)
+        pos = torch.arange(sq, device=dev).repeat(m)
+        mfma(f"merilorn: delta_chunks, {m} x {sq}", t * heads * (6 * d * d + 4 * 16 * d), F32_MFMA_PEAK_TFLOPS,
+             lambda: ho.delta_chunks(s, x, s.channels, dec, gt, *wts, ring, state, portions, chunks, rs, pos, 0, o2))
+        us = out[f"merilorn: delta_chunks, {m} x {sq}"]["us"]
+        out[f"merilorn: delta_chunks, {m} x {sq}"]["note"] = "frac: of the float32 matrix peak; of the memory bandwidth: %.3f" % (
+            6 * t * hd * 2 / us / 1e3 / HBM_PEAK_GBS)
+    del x, dec, gt
+
+    # ---- residual stream and activation
+    for t in (64, rows):
+        x32, y, w32, wb = rnd(t, width, dtype=torch.float32), rnd(t, width), torch.ones(width, device=dev), torch.ones(width, dtype=bf, device=dev)
+        hbm(f"post_norm, {t} rows", t * width * 12, lambda: ho.post_norm(x32, 1e-6, y=y, w_post=w32, alpha=2.0))
+        hbm(f"merilorn: residual_norm, {t} rows", t * width * 12, lambda: ho.residual_norm(x32, 1e-6, y=y, w_post=w32, w_pre=w32))
+        res = rnd(t, width)
+        hbm(f"qwen3: rms_norm with residual, {t} rows", t * width * 8, lambda: ops.rms_norm(y, wb, 1e-6, res))
+        gu = rnd(t, 2 * ff)
+        act = torch.empty((t, ff), dtype=bf, device=dev)
+        hbm(f"silu_and_mul, {t} rows", t * ff * 6, lambda: ho.silu_and_mul(gu))
+        hbm(f"qwen3: silu_and_mul, {t} rows", t * ff * 6, lambda: ops.silu_and_mul(act, gu))
+    return out
+
+
+def engine_points(models):
+    points = []
+    for size, batch, prompt, new in (("0.6b", 64, 1024, 64), ("8b", 64, 1024, 64), ("8b", 16, 4096, 64)):
+        for model in models:
+            points.append(hybrid_engine_point(size, model, batch, prompt, new))
+            print(points[-1], file=sys.stderr, flush=True)
+    return points
+
+
 def run_hybrid(args):
     """Merilorn beside Qwen3 at equal width, feed-forward, heads and number of layers: the engine's prefill and
     decode throughput, then the kernels one by one."""
-    points = []
-    if not args.hybrid_kernels_only:
-        for size, batch, prompt, new in (("0.6b", 64, 1024, 64), ("8b", 64, 1024, 64), ("8b", 16, 4096, 64)):
-            for model in ("merilorn", "qwen3"):
-                points.append(hybrid_engine_point(size, model, batch, prompt, new))
-                print(points[-1], file=sys.stderr, flush=True)
+    points = [] if args.hybrid_kernels_only else engine_points(("merilorn", "qwen3"))
     print(json.dumps({"hybrid_engine": points, "hybrid_kernels": hybrid_kernels()}))
+
+
+def run_vokelix(args):
+    """Vokelix beside Qwen3 and Merilorn, as ``run_hybrid``."""
+    points = [] if args.hybrid_kernels_only else engine_points(("vokelix", "qwen3", "merilorn"))
+    print(json.dumps({"vokelix_engine": points, "vokelix_kernels": vokelix_kernels()}))
 
 
 # ------------------------------------------------------------------------------------------ decode curve
@@ -505,7 +663,9 @@ def main():
     ap.add_argument("--decode-curve", action="store_true", help="only the decode curve, printed as JSON")
     ap.add_argument("--hybrid", action="store_true",
                     help="Merilorn beside Qwen3 at equal sizes: engine throughput and every kernel, printed as JSON")
-    ap.add_argument("--hybrid-kernels-only", action="store_true", help="with --hybrid: the kernels alone")
+    ap.add_argument("--vokelix", action="store_true",
+                    help="Vokelix beside Qwen3 and Merilorn at equal sizes: engine throughput and every kernel, printed as JSON")
+    ap.add_argument("--hybrid-kernels-only", action="store_true", help="with --hybrid or --vokelix: the kernels alone")
     ap.add_argument("--e2e", action="store_true",
                     help="end-to-end decode through the engine (random-init Qwen3, HIP-graph decode) instead "
                          "of the kernel benchmark")
@@ -528,8 +688,8 @@ def main():
     if args.e2e:
         run_e2e(args)
         return
-    if args.hybrid:
-        run_hybrid(args)
+    if args.hybrid or args.vokelix:
+        (run_vokelix if args.vokelix else run_hybrid)(args)
         return
     from infer_amd import ops, workloads
     dev = torch.device("cuda:0")
