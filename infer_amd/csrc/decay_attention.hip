@@ -16,11 +16,14 @@
 //
 // Chunk form.  With S the state before a chunk of n tokens,
 //     o_i = c (d^{i+1} q_i^T S + sum_{j<=i} d^{i-j} (q_i k_j) v_j) ,   S' = d^n S + sum_j k_j (d^{n-1-j} v_j)^T .
-// Everything of the recurrence is held to float precision although the products run as bf16: a float is the exact sum
-// of three bf16 numbers of 8 bits each (Split), and the products of the pieces are added up in float32, without those
-// below 2^-24 of the result.  Projections, with silu behind them or not, are bf16 already: one piece.
+// What enters the state is held to float precision although the products run as bf16: a float is the exact sum of
+// three bf16 numbers of 8 bits each, and the products of the pieces are added up in float32, without those below 2^-24
+// of the result.  The products of the output, which leave the recurrence and are rounded to bf16 behind it, take two
+// pieces (2^-17).  Projections, with silu behind them or not, are bf16 already: one piece.
 // A portion with few heads is cut into segments that run side by side: first every segment from a zero state, keeping
 // only its final state, then the states are joined in order, then every segment with its outputs.
+#include <type_traits>
+
 #include "elem.h"
 
 namespace {
@@ -131,47 +134,57 @@ constexpr int kC = 32;                           // tokens per chunk
 
 struct ChunkArgs {
     DecayArgs<__bf16> a;
+    DecayOutArgs<__bf16> b;
+    bool finish;                                 // norm (per head) and gate here; a.o is not written
     const Span* spans;
     int seg_len, max_seg, slabs;                 // tokens per segment (a multiple of kC), segments of the longest span
     float* ws;                                   // [span][max_seg][heads][dim_pad][vdim_pad], if max_seg > 1
 };
 
-// x as the exact sum of three bf16 numbers: the leading 8 bits of the mantissa, the next 8, the last 8
-struct Split { uint32_t hi, mid, lo; };          // as floats, low halves zero
-__device__ __forceinline__ Split split(float x) {
-    Split s;
-    s.hi = __builtin_bit_cast(uint32_t, x) & 0xffff0000u;
-    const float r = x - __builtin_bit_cast(float, s.hi);
-    s.mid = __builtin_bit_cast(uint32_t, r) & 0xffff0000u;
-    s.lo = __builtin_bit_cast(uint32_t, r - __builtin_bit_cast(float, s.mid));
-    return s;
+__device__ __forceinline__ float head(float x) { return __builtin_bit_cast(float, __builtin_bit_cast(uint32_t, x) & 0xffff0000u); }
+// the leading halves of two floats, `a` in front
+__device__ __forceinline__ uint32_t pack(float a, float b) {
+    return __builtin_amdgcn_perm(__builtin_bit_cast(uint32_t, b), __builtin_bit_cast(uint32_t, a), 0x07060302u);
 }
-// the high halves of two words, `a` in front
-__device__ __forceinline__ uint32_t pack(uint32_t a, uint32_t b) { return __builtin_amdgcn_perm(b, a, 0x07060302u); }
-
-template <int N>
-__device__ __forceinline__ void split_pack(const float (&x)[N], uint32_t (&p0)[N / 2], uint32_t (&p1)[N / 2], uint32_t (&p2)[N / 2]) {
+__device__ __forceinline__ uint32_t round_pack(float a, float b) {
+    typedef __bf16 bf16x2_t __attribute__((ext_vector_type(2)));
+    const bf16x2_t r = {(__bf16)a, (__bf16)b};
+    return __builtin_bit_cast(uint32_t, r);
+}
+// N floats as the sum of P bf16 numbers each: the leading 8 bits of the mantissa, the next 8, the last 8 (P = 3: exact;
+// P = 2: the second piece rounded)
+template <int P, int N>
+__device__ __forceinline__ void split(const float (&x)[N], uint32_t (&p)[P][N / 2]) {
 #pragma unroll
     for (int i = 0; i < N / 2; ++i) {
-        const Split a = split(x[2 * i]), b = split(x[2 * i + 1]);
-        p0[i] = pack(a.hi, b.hi);
-        p1[i] = pack(a.mid, b.mid);
-        p2[i] = pack(a.lo, b.lo);
+        const float a = x[2 * i], b = x[2 * i + 1], ra = a - head(a), rb = b - head(b);
+        p[0][i] = pack(a, b);
+        if constexpr (P == 2) {
+            p[1][i] = round_pack(ra, rb);
+        } else {
+            p[1][i] = pack(ra, rb);
+            p[2][i] = pack(ra - head(ra), rb - head(rb));
+        }
     }
 }
 __device__ __forceinline__ bf16x8_t frag(const uint32_t (&p)[4]) { return __builtin_bit_cast(bf16x8_t, u32x4_t{p[0], p[1], p[2], p[3]}); }
+template <int P>
+__device__ __forceinline__ void split_frags(const float (&x)[8], bf16x8_t (&f)[P]) {
+    uint32_t p[P][4];
+    split<P, 8>(x, p);
+#pragma unroll
+    for (int k = 0; k < P; ++k) f[k] = frag(p[k]);
+}
 
-// sum of the products of the pieces of two operands, the first in three pieces, the second in PB
-template <int PB>
-__device__ __forceinline__ f32x4_t mfma_pieces(const bf16x8_t (&x)[3], const bf16x8_t (&y)[PB], f32x4_t acc) {
-    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[2], y[0], acc, 0, 0, 0);
-    if constexpr (PB == 3) {
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[0], y[2], acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[1], y[1], acc, 0, 0, 0);
-    }
-    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[1], y[0], acc, 0, 0, 0);
-    if constexpr (PB == 3) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[0], y[1], acc, 0, 0, 0);
-    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[0], y[0], acc, 0, 0, 0);
+// sum of the products of pieces i of x and j of y with i + j < MOST, the small ones first
+template <int MOST, int PX, int PY>
+__device__ __forceinline__ f32x4_t mfma_pieces(const bf16x8_t (&x)[PX], const bf16x8_t (&y)[PY], f32x4_t acc) {
+#pragma unroll
+    for (int k = MOST - 1; k >= 0; --k)
+#pragma unroll
+        for (int i = 0; i <= k; ++i)
+            if (i < PX && k - i < PY) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x[i], y[k - i], acc, 0, 0, 0);
+    return acc;
 }
 
 __device__ __forceinline__ void widen(u32x4_t x, float (&y)[8]) {
@@ -194,19 +207,22 @@ __device__ __forceinline__ u32x4_t silu8(u32x4_t x) {
 // Wavefront w owns the columns 16 VT w .. and their part of the state, DT tiles of 32 rows, as accumulators: lane (g, n)
 // holds rows 16 t + 4 g + e of column n.  That is an operand of the next product as it lies, when the rows of a
 // k-step of 32 are taken in the order 16 tau + 4 g + e.  The 32 x 32 products q_i k_j are shared out over the
-// wavefronts, weighted, and exchanged through LDS.
-// PC: pieces of q and k (3 behind a rotation, otherwise 1).  OUT = false: only the final state, from zero.
+// wavefronts, weighted, and exchanged through LDS while the products with the state run.
+// PC: pieces of k (3 behind a rotation, otherwise 1; q then has 2).  OUT = false: only the final state, from zero.
 template <int DT, int VT, int PC, bool OUT>
 __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
     constexpr int kRow = DT * 64 + 16, kMat = kC * kRow;         // bytes: a token of q or k, one piece of a chunk
-    constexpr int kVRow = VT * 128 + 16, kPRow = 2 * kC + 16, kPMat = kC * kPRow;
+    constexpr int kSlab = 64 * VT;
+    constexpr int PQ = PC == 3 ? 2 : 1;                          // pieces of q
+    constexpr int kVRow = 2 * kSlab + 16, kPRow = 2 * kC + 16, kPMat = kC * kPRow;
     constexpr int NU = DT > 4 ? DT / 4 : 1;                      // units of 16 columns of q and k per thread
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
     const DecayArgs<__bf16>& a = args.a;
     unsigned char* kbuf = lds;                                   // [PC][kMat]
     unsigned char* vbuf = kbuf + PC * kMat;                      // [kC][kVRow]
-    unsigned char* qbuf = vbuf + kC * kVRow;                     // [PC][kMat]
-    unsigned char* pbuf = qbuf + PC * kMat;                      // [3][kPMat]
+    unsigned char* qbuf = vbuf + kC * kVRow;                     // [PQ][kMat]
+    unsigned char* pbuf = qbuf + PQ * kMat;                      // [2][kPMat]
+    float* squares = reinterpret_cast<float*>(pbuf + 2 * kPMat); // [4][kC]
     const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, n = lane & 15;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int h = blockIdx.y, slab = blockIdx.x % args.slabs, seg = blockIdx.x / args.slabs;
@@ -217,7 +233,7 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
     if (!OUT && last_seg) return;                                // nobody needs its final state yet
     const int count = last_seg ? span.count - first : args.seg_len;
     const int row0 = span.row0 + first, pos0 = span.pos0 + first, chunks = (count + kC - 1) / kC;
-    const int v0 = slab * 64 * VT + wave * 16 * VT;              // this wavefront's first column
+    const int v0 = slab * kSlab + wave * 16 * VT;                // this wavefront's first column
     const bool live = v0 < a.vdim_pad;
     const float log2d = a.decay[2 * a.heads + h];
     const int64_t state_len = (int64_t)a.dim_pad * a.vdim_pad;
@@ -244,53 +260,69 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
         }
 
     // entries behind the real sizes stay zero
-    for (int i = tid; i < (2 * PC * kMat + kC * kVRow) / 16; i += 256) reinterpret_cast<u32x4_t*>(lds)[i] = u32x4_t{0u, 0u, 0u, 0u};
+    for (int i = tid; i < ((PC + (OUT ? PQ : 0)) * kMat + kC * kVRow) / 16; i += 256) reinterpret_cast<u32x4_t*>(lds)[i] = u32x4_t{0u, 0u, 0u, 0u};
 
     // unit i of this thread: token, and two blocks of 8 columns, which turn together if they are rotated
-    const int units = a.dim / 16;
+    // (token -1: there is no such unit; its loads repeat another one and are not stored)
+    const int half = PC == 3 ? a.rot_pairs : a.dim / 2, units = a.dim / 16;
     int u_tok[NU], u_b0[NU], u_b1[NU], u_pair[NU];
+    const __bf16* u_src[NU];
+    const float* u_cs[NU];
 #pragma unroll
     for (int i = 0; i < NU; ++i) {
-        const int u = tid + 256 * i, w = u % units, rotated = a.rot_pairs / 8;
+        const int u = tid + 256 * i, w = u % units, rotated = half / 8;
         u_tok[i] = u < kC * units ? u / units : -1;
         u_pair[i] = PC == 3 && w < rotated ? 8 * w : -1;
-        u_b0[i] = w < rotated ? 8 * w : 2 * a.rot_pairs + 16 * (w - rotated);
-        u_b1[i] = w < rotated ? 8 * w + a.rot_pairs : u_b0[i] + 8;
+        u_b0[i] = w < rotated ? 8 * w : 2 * half + 16 * (w - rotated);
+        u_b1[i] = w < rotated ? 8 * w + half : u_b0[i] + 8;
+        u_src[i] = a.proj + (int64_t)(row0 + (u_tok[i] > 0 ? u_tok[i] : 0)) * a.proj_stride + h * a.dim;
+        u_cs[i] = a.table + 2 * (u_pair[i] > 0 ? u_pair[i] : 0);
     }
-    u32x4_t qreg[NU][2], kreg[NU][2], vreg[VT];
+    int v_tok[VT], v_col[VT];
+    const __bf16* v_src[VT];
+#pragma unroll
+    for (int i = 0; i < VT; ++i) {
+        const int x = tid + 256 * i;
+        v_tok[i] = x / (kSlab / 8);
+        v_col[i] = slab * kSlab + 8 * (x % (kSlab / 8));
+        v_src[i] = a.proj + (int64_t)(row0 + v_tok[i]) * a.proj_stride + a.v_off + h * a.vdim + (v_col[i] < a.vdim ? v_col[i] : 0);
+    }
+    const int64_t step = kC * a.proj_stride;
+    u32x4_t kreg[NU][2], qreg[NU][2], vreg[VT];
     f32x4_t creg[PC == 3 ? NU : 1][4];
+    // requests chunk c, the one behind the last request; no branches, so that nothing waits for a request before its use
     auto fetch = [&](int c) {
-        const int left = count - c * kC - 1;                     // tokens behind the last one re-read it
+        const int last = count - c * kC - 1;                     // tokens behind the last one re-read it
 #pragma unroll
         for (int i = 0; i < NU; ++i) {
-            if (u_tok[i] < 0) continue;
-            const int t = c * kC + (u_tok[i] < left ? u_tok[i] : left);
-            const __bf16* r = a.proj + (int64_t)(row0 + t) * a.proj_stride + h * a.dim;
+            const int over = u_tok[i] > last ? (u_tok[i] > 0 ? u_tok[i] : 0) - last : 0;
+            const __bf16* r = u_src[i] - over * a.proj_stride;
             kreg[i][0] = *reinterpret_cast<const u32x4_t*>(r + a.k_off + u_b0[i]);
             kreg[i][1] = *reinterpret_cast<const u32x4_t*>(r + a.k_off + u_b1[i]);
             if constexpr (OUT) {
                 qreg[i][0] = *reinterpret_cast<const u32x4_t*>(r + a.q_off + u_b0[i]);
                 qreg[i][1] = *reinterpret_cast<const u32x4_t*>(r + a.q_off + u_b1[i]);
             }
+            u_src[i] += step;
             if constexpr (PC == 3) {
-                if (u_pair[i] >= 0) {
-                    const float* cs = table_row(a, pos0 + t) + 2 * u_pair[i];
+                int64_t pos = pos0 + c * kC + u_tok[i];
+                pos = pos < 0 ? 0 : (pos >= a.max_pos ? a.max_pos - 1 : pos);
+                const float* cs = u_cs[i] + pos * (2 * a.rot_pairs);
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) creg[i][e] = *reinterpret_cast<const f32x4_t*>(cs + 4 * e);
-                }
+                for (int e = 0; e < 4; ++e) creg[i][e] = *reinterpret_cast<const f32x4_t*>(cs + 4 * e);
             }
         }
 #pragma unroll
         for (int i = 0; i < VT; ++i) {
-            const int x = tid + 256 * i, tok = x / (8 * VT), col = slab * 64 * VT + 8 * (x % (8 * VT));
-            const int t = c * kC + (tok < left ? tok : left);
-            if (col < a.vdim) vreg[i] = *reinterpret_cast<const u32x4_t*>(a.proj + (int64_t)(row0 + t) * a.proj_stride + a.v_off + h * a.vdim + col);
+            const int over = v_tok[i] > last ? v_tok[i] - last : 0;
+            vreg[i] = *reinterpret_cast<const u32x4_t*>(v_src[i] - over * a.proj_stride);
+            v_src[i] += step;
         }
     };
-    // one block pair of q or k to LDS
-    auto put_unit = [&](unsigned char* buf, int i, const u32x4_t (&x)[2], bool in) {
-        unsigned char* r = buf + u_tok[i] * kRow;
-        if constexpr (PC == 1) {
+    // the two blocks of a unit to LDS, in PB pieces
+    auto put_unit = [&](auto pieces, unsigned char* r, int i, const u32x4_t (&x)[2], bool in) {
+        constexpr int PB = decltype(pieces)::value;
+        if constexpr (PB == 1) {
             u32x4_t y0 = x[0], y1 = x[1];
             if (a.silu) { y0 = silu8(y0); y1 = silu8(y1); }
             if (!in) y0 = y1 = u32x4_t{0u, 0u, 0u, 0u};
@@ -310,13 +342,13 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
             if (!in)
 #pragma unroll
                 for (int e = 0; e < 8; ++e) y0[e] = y1[e] = 0.f;
-            uint32_t p[3][4];
-            split_pack<8>(y0, p[0], p[1], p[2]);
+            bf16x8_t f[PB];
+            split_frags<PB>(y0, f);
 #pragma unroll
-            for (int k = 0; k < 3; ++k) *reinterpret_cast<bf16x8_t*>(r + k * kMat + 2 * u_b0[i]) = frag(p[k]);
-            split_pack<8>(y1, p[0], p[1], p[2]);
+            for (int k = 0; k < PB; ++k) *reinterpret_cast<bf16x8_t*>(r + k * kMat + 2 * u_b0[i]) = f[k];
+            split_frags<PB>(y1, f);
 #pragma unroll
-            for (int k = 0; k < 3; ++k) *reinterpret_cast<bf16x8_t*>(r + k * kMat + 2 * u_b1[i]) = frag(p[k]);
+            for (int k = 0; k < PB; ++k) *reinterpret_cast<bf16x8_t*>(r + k * kMat + 2 * u_b1[i]) = f[k];
         }
     };
     auto put = [&](int c) {
@@ -324,16 +356,15 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
 #pragma unroll
         for (int i = 0; i < NU; ++i) {
             if (u_tok[i] < 0) continue;
-            put_unit(kbuf, i, kreg[i], u_tok[i] < left);
-            if constexpr (OUT) put_unit(qbuf, i, qreg[i], u_tok[i] < left);
+            put_unit(std::integral_constant<int, PC>{}, kbuf + u_tok[i] * kRow, i, kreg[i], u_tok[i] < left);
+            if constexpr (OUT) put_unit(std::integral_constant<int, PQ>{}, qbuf + u_tok[i] * kRow, i, qreg[i], u_tok[i] < left);
         }
 #pragma unroll
         for (int i = 0; i < VT; ++i) {
-            const int x = tid + 256 * i, tok = x / (8 * VT), c8 = x % (8 * VT);
-            if (slab * 64 * VT + 8 * c8 >= a.vdim) continue;
+            if (v_col[i] >= a.vdim) continue;
             u32x4_t y = a.silu ? silu8(vreg[i]) : vreg[i];
-            if (tok >= left) y = u32x4_t{0u, 0u, 0u, 0u};
-            *reinterpret_cast<u32x4_t*>(vbuf + tok * kVRow + 16 * c8) = y;
+            if (v_tok[i] >= left) y = u32x4_t{0u, 0u, 0u, 0u};
+            *reinterpret_cast<u32x4_t*>(vbuf + v_tok[i] * kVRow + 2 * (v_col[i] - slab * kSlab)) = y;
         }
     };
 
@@ -356,44 +387,93 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
     value_weights(kC);
     float chunk_decay = exp2f(kC * log2d);
 
+#pragma unroll
+    for (int t = 0; t < 2 * DT; ++t)
+#pragma unroll
+        for (int v = 0; v < VT; ++v)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {                        // the state has arrived: nothing in the loop waits for it
+                float x = s[t][v][e];
+                asm volatile("" : "+v"(x));
+                s[t][v][e] = x;
+            }
     fetch(0);
     __syncthreads();                                             // the zero fill
     for (int c = 0; c < chunks; ++c) {
         put(c);
         __syncthreads();
-        if (c + 1 < chunks) fetch(c + 1);
         const int left = count - c * kC;
+        fetch(c + 1);
         if (left < kC) {
             value_weights(left);
             chunk_decay = exp2f(left * log2d);
         }
+        u32x2_t gate[VT][2];                                     // of this chunk's results, for when they are there
+        f32x4_t acc[VT][2];                                      // rows are columns of the state, columns queries
         if constexpr (OUT) {
             // ---- d^(i-j) q_i k_j: rows are keys, columns queries; the tile above the diagonal is all zeros
-            f32x4_t p = {0.f, 0.f, 0.f, 0.f};
-            if (wave != 1) {
-                const unsigned char* kr = kbuf + (16 * (wave & 1) + n) * kRow + 16 * g;
-                const unsigned char* qr = qbuf + (16 * (wave >> 1) + n) * kRow + 16 * g;
+            {
+                f32x4_t p = {0.f, 0.f, 0.f, 0.f};
+                if (wave != 1) {
+                    const unsigned char* kr = kbuf + (16 * (wave & 1) + n) * kRow + 16 * g;
+                    const unsigned char* qr = qbuf + (16 * (wave >> 1) + n) * kRow + 16 * g;
+#pragma unroll
+                    for (int j = 0; j < DT; ++j) {
+                        bf16x8_t kf[PQ], qf[PQ];
+#pragma unroll
+                        for (int k = 0; k < PQ; ++k) {
+                            kf[k] = *reinterpret_cast<const bf16x8_t*>(kr + k * kMat + 64 * j);
+                            qf[k] = *reinterpret_cast<const bf16x8_t*>(qr + k * kMat + 64 * j);
+                        }
+                        p = mfma_pieces<2>(kf, qf, p);
+                    }
+                }
+                float x[4];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[e] = p[e] * pw[e];
+                uint32_t pp[2][2];
+                split<2, 4>(x, pp);
+                unsigned char* pr = pbuf + (16 * (wave >> 1) + n) * kPRow + 2 * (16 * (wave & 1) + 4 * g);
+#pragma unroll
+                for (int k = 0; k < 2; ++k) *reinterpret_cast<u32x2_t*>(pr + k * kPMat) = u32x2_t{pp[k][0], pp[k][1]};
+            }
+            // ---- q_i^T S
+#pragma unroll
+            for (int v = 0; v < VT; ++v)
+#pragma unroll
+                for (int t = 0; t < 2; ++t) acc[v][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+            if (live)
 #pragma unroll
                 for (int j = 0; j < DT; ++j) {
-                    bf16x8_t kf[PC], qf[PC];
+                    bf16x8_t qf[2][PQ];
 #pragma unroll
-                    for (int k = 0; k < PC; ++k) {
-                        kf[k] = *reinterpret_cast<const bf16x8_t*>(kr + k * kMat + 64 * j);
-                        qf[k] = *reinterpret_cast<const bf16x8_t*>(qr + k * kMat + 64 * j);
+                    for (int t = 0; t < 2; ++t)
+#pragma unroll
+                        for (int k = 0; k < PQ; ++k) {
+                            const unsigned char* qr = qbuf + k * kMat + (16 * t + n) * kRow + 64 * j + 8 * g;
+                            const u32x2_t x = *reinterpret_cast<const u32x2_t*>(qr), y = *reinterpret_cast<const u32x2_t*>(qr + 32);
+                            qf[t][k] = __builtin_bit_cast(bf16x8_t, u32x4_t{x[0], x[1], y[0], y[1]});
+                        }
+#pragma unroll
+                    for (int v = 0; v < VT; ++v) {
+                        float x[8];
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) { x[e] = s[2 * j][v][e]; x[4 + e] = s[2 * j + 1][v][e]; }
+                        bf16x8_t sf[2];
+                        split_frags<2>(x, sf);
+#pragma unroll
+                        for (int t = 0; t < 2; ++t) acc[v][t] = mfma_pieces<2>(sf, qf[t], acc[v][t]);
                     }
-                    if constexpr (PC == 3) p = mfma_pieces<3>(kf, qf, p);
-                    else p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0], qf[0], p, 0, 0, 0);
                 }
-            }
-            float x[4];
+            if (args.finish)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) x[e] = p[e] * pw[e];
-            uint32_t p0[2], p1[2], p2[2];
-            split_pack<4>(x, p0, p1, p2);
-            unsigned char* pr = pbuf + (16 * (wave >> 1) + n) * kPRow + 2 * (16 * (wave & 1) + 4 * g);
-            *reinterpret_cast<u32x2_t*>(pr) = u32x2_t{p0[0], p0[1]};
-            *reinterpret_cast<u32x2_t*>(pr + kPMat) = u32x2_t{p1[0], p1[1]};
-            *reinterpret_cast<u32x2_t*>(pr + 2 * kPMat) = u32x2_t{p2[0], p2[1]};
+                for (int v = 0; v < VT; ++v)
+#pragma unroll
+                    for (int t = 0; t < 2; ++t) {
+                        const int tok = 16 * t + n < left ? 16 * t + n : left - 1, col = v0 + 16 * v + 4 * g;
+                        gate[v][t] = *reinterpret_cast<const u32x2_t*>(args.b.gate + (int64_t)(row0 + c * kC + tok) * args.b.gate_stride +
+                                                                       (int64_t)h * a.vdim + (col < a.vdim ? col : 0));
+                    }
             __syncthreads();
         }
         if (live) {
@@ -406,53 +486,25 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
                 vf[v] = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
             }
             if constexpr (OUT) {
-                f32x4_t acc[VT][2];                              // rows are columns of the state, columns queries
-#pragma unroll
-                for (int v = 0; v < VT; ++v)
-#pragma unroll
-                    for (int t = 0; t < 2; ++t) acc[v][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-                // ---- q_i^T S
-#pragma unroll
-                for (int j = 0; j < DT; ++j) {
-                    bf16x8_t qf[2][PC];
-#pragma unroll
-                    for (int t = 0; t < 2; ++t)
-#pragma unroll
-                        for (int k = 0; k < PC; ++k) {
-                            const unsigned char* qr = qbuf + k * kMat + (16 * t + n) * kRow + 64 * j + 8 * g;
-                            const u32x2_t x = *reinterpret_cast<const u32x2_t*>(qr), y = *reinterpret_cast<const u32x2_t*>(qr + 32);
-                            qf[t][k] = __builtin_bit_cast(bf16x8_t, u32x4_t{x[0], x[1], y[0], y[1]});
-                        }
-#pragma unroll
-                    for (int v = 0; v < VT; ++v) {
-                        float x[8];
-#pragma unroll
-                        for (int e = 0; e < 4; ++e) { x[e] = s[2 * j][v][e]; x[4 + e] = s[2 * j + 1][v][e]; }
-                        uint32_t p0[4], p1[4], p2[4];
-                        split_pack<8>(x, p0, p1, p2);
-                        const bf16x8_t sf[3] = {frag(p0), frag(p1), frag(p2)};
-#pragma unroll
-                        for (int t = 0; t < 2; ++t) acc[v][t] = mfma_pieces<PC>(sf, qf[t], acc[v][t]);
-                    }
-                }
                 // ---- the chunk's own tokens
 #pragma unroll
                 for (int t = 0; t < 2; ++t) {
-                    bf16x8_t pf[3];
+                    bf16x8_t pf[2];
 #pragma unroll
-                    for (int k = 0; k < 3; ++k) pf[k] = *reinterpret_cast<const bf16x8_t*>(pbuf + k * kPMat + (16 * t + n) * kPRow + 16 * g);
+                    for (int k = 0; k < 2; ++k) pf[k] = *reinterpret_cast<const bf16x8_t*>(pbuf + k * kPMat + (16 * t + n) * kPRow + 16 * g);
+                    float ss = 0.f;
 #pragma unroll
                     for (int v = 0; v < VT; ++v) {
                         acc[v][t] *= qw[t];
 #pragma unroll
-                        for (int k = 2; k >= 0; --k) acc[v][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[v], pf[k], acc[v][t], 0, 0, 0);
-                        const int col = v0 + 16 * v + 4 * g;
-                        if (16 * t + n < left && col < a.vdim) {
-                            bf16x4_t o;
+                        for (int k = 1; k >= 0; --k) acc[v][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[v], pf[k], acc[v][t], 0, 0, 0);
 #pragma unroll
-                            for (int e = 0; e < 4; ++e) o[e] = (__bf16)acc[v][t][e];
-                            *reinterpret_cast<bf16x4_t*>(a.o + (int64_t)(row0 + c * kC + 16 * t + n) * a.o_stride + (int64_t)h * a.vdim + col) = o;
-                        }
+                        for (int e = 0; e < 4; ++e) ss += acc[v][t][e] * acc[v][t][e];       // columns that pad the size are zero
+                    }
+                    if (args.finish) {
+                        ss += __shfl_xor(ss, 16, 64);
+                        ss += __shfl_xor(ss, 32, 64);
+                        if (g == 0) squares[wave * kC + 16 * t + n] = ss;
                     }
                 }
             }
@@ -464,11 +516,7 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
                 widen(__builtin_bit_cast(u32x4_t, vf[v]), x);
 #pragma unroll
                 for (int i = 0; i < 8; ++i) x[i] *= vw[i];
-                uint32_t p0[4], p1[4], p2[4];
-                split_pack<8>(x, p0, p1, p2);
-                wf[v][0] = frag(p0);
-                wf[v][1] = frag(p1);
-                wf[v][2] = frag(p2);
+                split_frags<3>(x, wf[v]);
             }
             const unsigned char* kr = kbuf + (8 * g + (n >> 2)) * kRow + (n & 3) * 8;
 #pragma unroll
@@ -483,16 +531,48 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
 #pragma unroll
                 for (int v = 0; v < VT; ++v) {
                     s[t][v] *= chunk_decay;
-                    if constexpr (PC == 3) {
-                        s[t][v] = mfma_pieces<3>(kf, wf[v], s[t][v]);
-                    } else {
-#pragma unroll
-                        for (int k = 2; k >= 0; --k) s[t][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0], wf[v][k], s[t][v], 0, 0, 0);
-                    }
+                    s[t][v] = mfma_pieces<3>(kf, wf[v], s[t][v]);
                 }
             }
+        } else if (OUT && args.finish && lane < kC) {
+            squares[wave * kC + lane] = 0.f;
         }
         __syncthreads();
+        if constexpr (OUT) {
+            // ---- results, with the norm over the head and the gate if nobody else does them
+            if (live)
+#pragma unroll
+                for (int t = 0; t < 2; ++t) {
+                    if (16 * t + n >= left) continue;
+                    const int64_t row = row0 + c * kC + 16 * t + n;
+                    float rs = 1.f;
+                    if (args.finish) {
+                        float ss = 0.f;
+#pragma unroll
+                        for (int w = 0; w < 4; ++w) ss += squares[w * kC + 16 * t + n];
+                        rs = rsqrtf(ss / (float)a.vdim + args.b.eps);
+                    }
+#pragma unroll
+                    for (int v = 0; v < VT; ++v) {
+                        const int col = v0 + 16 * v + 4 * g;
+                        if (col >= a.vdim) continue;
+                        float x[4];
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) x[e] = acc[v][t][e];
+                        __bf16* o = a.o + row * a.o_stride + (int64_t)h * a.vdim + col;
+                        if (args.finish) {
+                            const bf16x4_t z = __builtin_bit_cast(bf16x4_t, gate[v][t]);
+#pragma unroll
+                            for (int e = 0; e < 4; ++e) x[e] *= rs * gate_of(args.b, (float)z[e]);
+                            if (args.b.norm)
+#pragma unroll
+                                for (int e = 0; e < 4; ++e) x[e] *= args.b.norm[h * a.vdim + col + e];
+                            o = args.b.out + row * args.b.out_stride + (int64_t)h * a.vdim + col;
+                        }
+                        store_elems<4>(o, x);
+                    }
+                }
+        }
     }
     if (OUT && !last_seg) return;
 #pragma unroll
@@ -730,7 +810,7 @@ bool chunks_fit(int elem, int64_t dim, int64_t vdim, int64_t rot_dims) {
     return elem == INFER_ELEM_BF16 && dim % 16 == 0 && vdim % 8 == 0 && dim <= 256 && rot_dims % 16 == 0;
 }
 int tiles_of(int64_t dim_pad) { return dim_pad <= 32 ? 1 : dim_pad <= 64 ? 2 : dim_pad <= 128 ? 4 : 8; }
-int column_tiles(int64_t dim_pad, int64_t vdim_pad) { return vdim_pad <= 64 || dim_pad > 128 ? 1 : 2; }
+int column_tiles(int64_t dim_pad, int64_t vdim_pad) { return vdim_pad <= 64 || dim_pad > 128 ? 1 : 2; }    // per wavefront
 int slabs_of(int64_t dim_pad, int64_t vdim_pad) {
     const int cols = 64 * column_tiles(dim_pad, vdim_pad);
     return (int)((vdim_pad + cols - 1) / cols);
@@ -747,7 +827,7 @@ int64_t segment_len(int64_t heads, int64_t slabs, int64_t num_spans, int64_t max
 
 template <int DT, int VT, int PC, bool OUT>
 int launch_chunk(const ChunkArgs& c, int64_t num_spans, hipStream_t st) {
-    const size_t lds = (size_t)kC * (2 * PC * (DT * 64 + 16) + VT * 128 + 16) + (OUT ? 3 * kC * (2 * kC + 16) : 0);
+    const size_t lds = (size_t)kC * ((OUT ? PC == 3 ? 5 : 2 : PC) * (DT * 64 + 16) + 128 * VT + 16) + (OUT ? kC * (2 * (2 * kC + 16) + 16) : 0);
     auto kernel = &decay_chunk_kernel<DT, VT, PC, OUT>;
     if (lds > 64 * 1024) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -870,7 +950,10 @@ extern "C" int infer_decay_attention(int elem, const void* proj, int64_t proj_st
                     const int64_t len = segment_len(heads, slabs, num_spans, max_span), n = (max_span + len - 1) / len;
                     if (n > 1 && (!workspace || !ptr_aligned(workspace, 16) || workspace_floats < num_spans * n * heads * pad[0] * pad[1]))
                         return (int)INFER_KV_EWORKSPACE;
-                    rc = run_chunks(ChunkArgs{a, (const Span*)spans, (int)len, (int)n, slabs, workspace}, num_spans, st);
+                    // a workgroup that has the whole head norms it, too
+                    const bool finish = norm_per_head && slabs == 1 && finished == decode_rows && ptr_aligned(proj, 8) && g_off % 4 == 0;
+                    rc = run_chunks(ChunkArgs{a, b, finish, (const Span*)spans, (int)len, (int)n, slabs, workspace}, num_spans, st);
+                    if (finish) finished = rows;
                 }
             }
             if (!chunked) rc = launch_any(a, (const Span*)spans, nullptr, nullptr, num_spans, st);

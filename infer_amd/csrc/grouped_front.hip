@@ -73,58 +73,86 @@ __device__ __forceinline__ void fill_padding(const GroupedFrontArgs<T>& a, T* ro
         for (int i = threadIdx.x; i < a.heads * pad; i += 256) qx[i / pad * a.dim_pad + a.dim + i % pad] = (T)0.f;
 }
 
-// NCH: chunks of four columns of q and k per thread; everything is a multiple of four
-template <class T, int NCH>
+// NCH: chunks of eight columns of q, k and v per thread; everything is a multiple of eight.  SAME: 2048 columns, the
+// distance between a thread's chunks, are whole heads, so that all its chunks of q and k start with the same pair.
+template <class T, int NCH, bool SAME>
 __global__ void __launch_bounds__(256) grouped_front_kernel(GroupedFrontArgs<T> a) {
     __shared__ float part[2][4];
     const int64_t t = blockIdx.x;
     const int tid = threadIdx.x;
     T* pr = a.proj + t * a.proj_stride;
+    T* row = cache_row(a, a.slots[t]);
     int64_t pos = a.positions[t];
     pos = pos < 0 ? 0 : (pos >= a.max_pos ? a.max_pos - 1 : pos);
     const float* cs = a.table + pos * (2 * a.rot_pairs);
-    T* row = cache_row(a, a.slots[t]);
     const int64_t head_rows = (int64_t)a.block_size * (a.dim_pad + a.vdim_pad);
-    const int nq = a.heads * a.dim / 4, nk = row ? a.kv_heads * a.dim / 4 : 0, nv = row ? a.kv_heads * a.vdim / 4 : 0;
-    float x[NCH][4], sq = 0.f, sk = 0.f;
+    const int nq = a.heads * a.dim / 8, nk = row ? a.kv_heads * a.dim / 8 : 0, total = nq + nk + (row ? a.kv_heads * a.vdim / 8 : 0);
+    // cosine and sine of four pairs from p on
+    auto turn_of = [&](int p, float (&turn)[8]) {
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            turn[2 * k] = 1.f;
+            turn[2 * k + 1] = 0.f;
+            if (p + k < a.rot_pairs) {
+                const float2 v = *reinterpret_cast<const float2*>(cs + 2 * (p + k));
+                turn[2 * k] = v.x;
+                turn[2 * k + 1] = v.y;
+            }
+        }
+    };
+    float x[NCH][8], turn[8], sq = 0.f, sk = 0.f;
 #pragma unroll
     for (int j = 0; j < NCH; ++j) {
         const int i = tid + 256 * j;
-        if (i < nq + nk) {
-            const bool is_q = i < nq;
-            load_biased(a, pr, is_q ? 4 * i : a.k_off + 4 * (i - nq), x[j]);
-            const float s = x[j][0] * x[j][0] + x[j][1] * x[j][1] + x[j][2] * x[j][2] + x[j][3] * x[j][3];
-            sq += is_q ? s : 0.f;
-            sk += is_q ? 0.f : s;
-        }
+        if (i < total) load_biased(a, pr, i < nq ? 8 * i : i < nq + nk ? a.k_off + 8 * (i - nq) : a.v_off + 8 * (i - nq - nk), x[j]);
+    }
+    if constexpr (SAME) turn_of(8 * tid % a.dim / 2, turn);
+#pragma unroll
+    for (int j = 0; j < NCH; ++j) {
+        const int i = tid + 256 * j;
+        float s = 0.f;
+        if (i < nq + nk)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) s += x[j][e] * x[j][e];
+        sq += i < nq ? s : 0.f;
+        sk += i < nq ? 0.f : s;
     }
     block_sum2(sq, sk, part);
-    const float rq = rsqrtf(sq / (float)(a.heads * a.dim) + a.eps), rk = rsqrtf(sk / (float)(4 * (nk > 0 ? nk : 1)) + a.eps);
+    const float rq = rsqrtf(sq / (float)(8 * nq) + a.eps), rk = rsqrtf(sk / (float)(8 * (nk > 0 ? nk : 1)) + a.eps);
     T* qx = t < a.qx_rows ? a.qx + t * a.heads * a.dim_pad : nullptr;
 #pragma unroll
     for (int j = 0; j < NCH; ++j) {
         const int i = tid + 256 * j;
+        if (i >= total) continue;
+        T* to;
         if (i < nq + nk) {
             const bool is_q = i < nq;
-            const int col = 4 * (is_q ? i : i - nq), h = col / a.dim, d = col - h * a.dim;
+            const int col = 8 * (is_q ? i : i - nq);
             const float* norm = is_q ? a.q_norm : a.k_norm;
             if (norm) {
-                float w[4];
-                load_elems<4>(norm + col, w);
+                float w[8];
+                load_elems<8>(norm + col, w);
 #pragma unroll
-                for (int e = 0; e < 4; ++e) x[j][e] *= (is_q ? rq : rk) * w[e];
+                for (int e = 0; e < 8; ++e) x[j][e] *= (is_q ? rq : rk) * w[e];
             }
-            rotate_pair(a, cs, d / 2, x[j][0], x[j][1]);
-            rotate_pair(a, cs, d / 2 + 1, x[j][2], x[j][3]);
-            T* to = !is_q ? row + h * head_rows + a.vdim_pad + d : qx ? qx + h * a.dim_pad + d : pr + col;
-            store_elems<4>(to, x[j]);
+            if constexpr (!SAME) turn_of(col % a.dim / 2, turn);
+#pragma unroll
+            for (int e = 0; e < 8; e += 2) {
+                const float u = x[j][e], v = x[j][e + 1];
+                x[j][e] = u * turn[e] - v * turn[e + 1];
+                x[j][e + 1] = v * turn[e] + u * turn[e + 1];
+            }
+            if (is_q && !qx) {
+                to = pr + col;
+            } else {
+                const int h = col / a.dim, d = col - h * a.dim;
+                to = is_q ? qx + h * a.dim_pad + d : row + h * head_rows + a.vdim_pad + d;
+            }
+        } else {
+            const int col = 8 * (i - nq - nk), h = col / a.vdim;
+            to = row + h * head_rows + (col - h * a.vdim);
         }
-    }
-    for (int i = tid; i < nv; i += 256) {
-        const int h = 4 * i / a.vdim, d = 4 * i - h * a.vdim;
-        float v[4];
-        load_biased(a, pr, a.v_off + 4 * i, v);
-        store_elems<4>(row + h * head_rows + d, v);
+        store_elems<8>(to, x[j]);
     }
     fill_padding(a, row, head_rows, qx);
 }
@@ -181,17 +209,20 @@ __global__ void __launch_bounds__(256) grouped_front_any_kernel(GroupedFrontArgs
 
 template <class T>
 int launch(const GroupedFrontArgs<T>& a, int64_t n, hipStream_t st) {
-    const size_t four = 4 * sizeof(T);
-    const bool vec = a.dim % 4 == 0 && a.vdim % 4 == 0 && a.k_off % 4 == 0 && a.v_off % 4 == 0 && a.proj_stride % 4 == 0 &&
-                     ptr_aligned(a.proj, four) && ptr_aligned(a.cache, four) && ptr_aligned(a.qx, four) && ptr_aligned(a.bias, 16) &&
-                     ptr_aligned(a.q_norm, 16) && ptr_aligned(a.k_norm, 16);
-    const int chunks = ((a.heads + a.kv_heads) * a.dim / 4 + 255) / 256;
+    const bool vec = a.dim % 8 == 0 && a.vdim % 8 == 0 && a.k_off % 8 == 0 && a.v_off % 8 == 0 && a.proj_stride % 8 == 0 &&
+                     ptr_aligned(a.proj, 16) && ptr_aligned(a.cache, 16) && ptr_aligned(a.qx, 16) && ptr_aligned(a.bias, 16) &&
+                     ptr_aligned(a.q_norm, 16) && ptr_aligned(a.k_norm, 16) && ptr_aligned(a.table, 8);
+    const int chunks = ((a.heads + a.kv_heads) * a.dim / 8 + a.kv_heads * a.vdim / 8 + 255) / 256;
     const dim3 grid((unsigned)n), block(256);
-#define GO(N) hipLaunchKernelGGL((grouped_front_kernel<T, N>), grid, block, 0, st, a)
+#define GO(N) \
+    do { \
+        if (2048 % a.dim == 0) hipLaunchKernelGGL((grouped_front_kernel<T, N, true>), grid, block, 0, st, a); \
+        else hipLaunchKernelGGL((grouped_front_kernel<T, N, false>), grid, block, 0, st, a); \
+    } while (0)
     if (vec && chunks <= 1) GO(1);
     else if (vec && chunks <= 2) GO(2);
-    else if (vec && chunks <= 5) GO(5);
-    else if (vec && chunks <= 10) GO(10);
+    else if (vec && chunks <= 3) GO(3);
+    else if (vec && chunks <= 6) GO(6);
     else hipLaunchKernelGGL((grouped_front_any_kernel<T>), grid, block, 0, st, a);
 #undef GO
     return (int)hipGetLastError();
