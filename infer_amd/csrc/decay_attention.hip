@@ -295,7 +295,7 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
         const int last = count - c * kC - 1;                     // tokens behind the last one re-read it
 #pragma unroll
         for (int i = 0; i < NU; ++i) {
-            const int over = u_tok[i] > last ? (u_tok[i] > 0 ? u_tok[i] : 0) - last : 0;
+            const int tok = u_tok[i] > 0 ? u_tok[i] : 0, over = tok > last ? tok - last : 0;
             const __bf16* r = u_src[i] - over * a.proj_stride;
             kreg[i][0] = *reinterpret_cast<const u32x4_t*>(r + a.k_off + u_b0[i]);
             kreg[i][1] = *reinterpret_cast<const u32x4_t*>(r + a.k_off + u_b1[i]);
@@ -305,7 +305,7 @@ __global__ void __launch_bounds__(256, 2) decay_chunk_kernel(ChunkArgs args) {
             }
             u_src[i] += step;
             if constexpr (PC == 3) {
-                int64_t pos = pos0 + c * kC + u_tok[i];
+                int64_t pos = pos0 + c * kC + tok;
                 pos = pos < 0 ? 0 : (pos >= a.max_pos ? a.max_pos - 1 : pos);
                 const float* cs = u_cs[i] + pos * (2 * a.rot_pairs);
 #pragma unroll

@@ -182,3 +182,23 @@ def test_spans_cover_the_rows_behind_the_decoded_tokens():
     assert plan.spans.tolist() == [[first[2], 2, 2, 17], [first[3], 33, 3, 33], [first[1], 70, 1, 0]]
     alone, _ = build(portions[:1], bs, 4, 4, 16, "cpu")
     assert alone.spans.shape == (0, 4) and alone.max_span == 0
+
+
+def requested_rows(count, dim):
+    """The rows of a span of ``count`` tokens that the chunk kernel of constant-decay attention requests for q and k: its
+    index arithmetic, for every thread and every chunk, the request behind the last chunk included."""
+    per_thread, units = max(1, dim // 128 if dim <= 128 else 2), dim // 16
+    u = np.arange(256)[:, None] + 256 * np.arange(per_thread)
+    tok = np.where(u < 32 * units, u // units, 0)
+    rows = []
+    for c in range(-(-count // 32) + 1):
+        last = count - c * 32 - 1
+        rows.append(tok + 32 * c - np.maximum(tok - last, 0))
+    return np.concatenate(rows)
+
+
+@pytest.mark.parametrize("dim", [16, 32, 48, 64, 80, 96, 112, 128, 192, 256])
+def test_requests_of_the_chunk_kernel_stay_inside_the_span(dim):
+    for count in (2, 3, 31, 32, 33, 63, 64, 65, 96, 100, 128, 512):
+        rows = requested_rows(count, dim)
+        assert rows.min() == 0 and rows.max() == count - 1
