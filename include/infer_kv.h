@@ -361,6 +361,9 @@ int infer_gelu_tanh_and_mul(int elem, void* out, int64_t out_stride, const void*
  * before the product, as the operator it replaces does; this one does not). */
 int infer_silu_and_mul(int elem, void* out, int64_t out_stride, const void* x, int64_t x_stride,
                        int64_t n_rows, int64_t d, void* stream);
+/* out[r][c] = g sigmoid(1.702 g) (u + 1) with g = min(x[r][c], limit), u = clamp(x[r][d + c], -limit, limit). */
+int infer_clamped_gate_and_mul(int elem, void* out, int64_t out_stride, const void* x, int64_t x_stride, int64_t n_rows,
+                               int64_t d, float limit, void* stream);
 
 /* Front end of latent attention.  A token's projection row holds q (heads x [dim | rot]) at column 0 and
  * [latent: rank | rotated key part: rot] at column kv_off.  The latent is RMS-normed (c_norm), the first
@@ -450,6 +453,98 @@ int infer_grouped_prefill(const void* q, int64_t q_stride, const void* k, int64_
                           void* out, int64_t out_stride, const int32_t* cu_q, const int32_t* cu_k, int64_t num_seqs,
                           int64_t max_seqlen_q, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, float scale,
                           void* stream);
+
+/* Pre-norm decoders with a learned scale behind every sublayer.
+ *
+ * infer_pre_norm, per row of the float32 stream x:  x <- x + y * scale [+ first] [+ step];  h <- rms(x) * w.
+ * y is the sum of: the tensor y or the `splits` unreduced pieces of a split-K product; and for k < top, weights[row][k] times
+ * row places[row][k] of `experts` (-1: the row itself of h_in).  scale, first and step may be NULL (1, 0, 0); first is
+ * [row][width].  With `tokens` the sum is the embedding instead: embed[token] plus, with `bigram`, row
+ * (prev * mul_prev + token * mul_cur) mod buckets of it (prev < 0: row `buckets`); first is then written (before step).
+ * infer_softcap: out = cap * tanh(x / cap), float32 [rows][cols]. */
+int infer_pre_norm(int elem, const int64_t* tokens, const void* embed, int64_t vocab, const int64_t* prev,
+                   const void* bigram, int64_t buckets, int64_t mul_prev, int64_t mul_cur, const void* y,
+                   int64_t y_stride, const float* partial, int64_t splits, int64_t split_stride,
+                   int64_t partial_stride, const void* experts, const int32_t* places, const float* weights,
+                   int64_t top, int64_t num_places, const void* h_in, int64_t h_in_stride, const float* scale,
+                   float* first, const float* step, float* x, int64_t x_stride, const float* w, void* h,
+                   int64_t h_stride, int64_t n_rows, int64_t width, float eps, void* stream);
+int infer_softcap(int elem, const void* x, int64_t x_stride, float* out, int64_t n_rows, int64_t cols, float cap,
+                  void* stream);
+
+/* Masked attention: pages [blocks][kv_heads][block_size][vdim_pad + key_pad], a row holding the value, zeros, the keys of
+ * all maps one behind the other, zeros; both parts are padded to 32 elements.  maps = 2: a head has two queries and two keys
+ * (head by head, map by map in the projections) beside one value.
+ *
+ * infer_head_front: projections q, k, v of a token at columns q_off, k_off, v_off; biases per column (NULL: none); RMS norm
+ * per head (and map) with a weight [dim] (NULL: no norm); entry i < rot_dims / 2 turns with entry i + rot_dims / 2 by the token's
+ * position; keys and values are stored at slots[t] (negative: skipped).  Rows below qx_rows get their q in
+ * qx[t][head][map][key_pad] (zero where the other map's key stands), the others in place.
+ *
+ * infer_masked_attention: query rows against pages, as infer_grouped_attention.  mask_kind 0: all keys in front; 1: those of the
+ * same chunk of mask_size tokens, counted from the sequence's start; 2: the last mask_size, itself among them.  biased: a score
+ * loses 2^(-8 (h + 1) / heads) per token of distance.  The result is multiplied by out_scale.  maps = 2: the result is
+ * rms(o1 - lambda o2) (eps) * out_scale, and the workspace always holds rows * splits * heads * 2 * (vdim_pad + 2) floats;
+ * neither sink nor bias then.  Splits as infer_grouped_attention_splits for heads * maps heads and key_pad.
+ * infer_masked_gather: as infer_grouped_gather, without the keys in front of what the first query of a portion sees.
+ * infer_masked_prefill: as infer_grouped_prefill, gate optional; q [tokens][head][map][dim], k [keys][kv_head][map][dim]. */
+int infer_head_front(int elem, void* proj, int64_t proj_stride, int64_t heads, int64_t kv_heads, int64_t maps,
+                     int64_t dim, int64_t vdim, int64_t q_off, int64_t k_off, int64_t v_off, const float* bias,
+                     const float* q_norm, const float* k_norm, float eps, const float* table, int64_t rot_dims,
+                     int64_t max_pos, const int64_t* positions, const int32_t* slots, void* cache,
+                     int64_t block_size, int64_t key_pad, int64_t vdim_pad, int64_t num_slots, void* qx,
+                     int64_t qx_rows, int64_t n, void* stream);
+int infer_masked_attention(int elem, const void* qx, const void* cache, int64_t key_pad, int64_t vdim_pad,
+                           const int32_t* block_table, int64_t bt_stride, int64_t table_cols, int64_t block_size,
+                           int64_t num_blocks, const int32_t* row_seq, const int32_t* ctx, int64_t rows,
+                           int64_t heads, int64_t kv_heads, int64_t maps, float scale, int mask_kind,
+                           int64_t mask_size, int biased, const float* sink, const void* gate, int64_t gate_stride,
+                           float out_scale, float lambda, float eps, int64_t splits, void* out, int64_t out_stride,
+                           int64_t vdim, float* workspace, int64_t workspace_floats, void* stream);
+int infer_masked_gather(const void* cache, int64_t row, int64_t kv_heads, int64_t block_size, int64_t num_blocks,
+                        const int32_t* block_table, int64_t bt_stride, int64_t table_cols, const int32_t* seqs,
+                        const int32_t* cu_q, const int32_t* cu_k, int64_t num_seqs, int64_t max_keys, int mask_kind,
+                        int64_t mask_size, void* out, void* stream);
+int infer_masked_prefill_supported(int64_t maps, int64_t dim, int64_t vdim);
+int infer_masked_prefill(const void* q, int64_t q_stride, const void* k, int64_t k_stride, int64_t k_head,
+                         const void* v, int64_t v_stride, int64_t v_head, const float* sink, const void* gate,
+                         int64_t gate_stride, void* out, int64_t out_stride, const int32_t* cu_q,
+                         const int32_t* cu_k, int64_t num_seqs, int64_t max_seqlen_q, int64_t heads,
+                         int64_t kv_heads, int64_t maps, int64_t dim, int64_t vdim, float scale, int mask_kind,
+                         int64_t mask_size, int biased, float out_scale, float lambda, float eps, void* stream);
+
+/* Selective state space: S <- e^{a dt} S + dt B x^T, y = S^T C + D x per head, dt = softplus(. + dt_bias), a = -e^{a_log}; x, B and C
+ * behind a causal convolution per channel and silu, heads / groups consecutive heads share B and C; behind it
+ * rms(y silu(z)) * norm over norm_parts equal parts of a row.  A projection row holds z [heads * vdim] at z_off, x, B
+ * [groups * state_n] and C one behind the other at x_off, dt [heads] at dt_off.  conv [channels][taps], the last column for the
+ * current token.  ring [slots][taps][channels] (position mod taps), state [slots][heads][state_n][vdim] float32.
+ * Rows below decode_rows advance slots[r] by one token (negative: padding); the others belong to spans (first row, tokens,
+ * slot, first position; max_span is the longest) and ring_slot[row] = (slot, rows of the span that follow).  xbc holds
+ * (n - decode_rows) * channels elements, y n * heads * vdim. */
+int64_t infer_state_space_workspace_floats(int elem, int64_t heads, int64_t vdim, int64_t state_n, int64_t num_spans,
+                                           int64_t max_span);
+int infer_state_space(int elem, const void* proj, int64_t proj_stride, int64_t z_off, int64_t x_off, int64_t dt_off,
+                      int64_t heads, int64_t vdim, int64_t state_n, int64_t groups, int64_t taps, const float* conv,
+                      const float* conv_bias, const float* dt_bias, const float* a_log, const float* d,
+                      const float* norm, int64_t norm_parts, float eps, void* ring, float* state, int64_t num_slots,
+                      const int32_t* slots, const int64_t* positions, int64_t decode_rows, const int32_t* spans,
+                      int64_t num_spans, int64_t max_span, const int32_t* ring_slot, int64_t n, void* xbc, void* y,
+                      float* workspace, int64_t workspace_floats, void* out, int64_t out_stride, void* stream);
+
+/* Mixture of experts.  Router logits in float32, softmax over all experts + identity entries, choice scores = softmax +
+ * correction (NULL: 0); of `groups` equal groups of neighbours the `keep` with the largest choice scores are open, of their
+ * entries the `top` largest are chosen, with the softmax value times scale as weight.  Chosen experts (not identities) get a
+ * row ("place") each: act = silu(gate) * up, out[place] = down act.  gate_up [experts][2 ff][width], down
+ * [experts][width][ff_pad] (zero behind ff), act [places][ff_pad].  counts [experts] is zero before and after.  weights and places
+ * (-1: identity) are [n][top]; ids, ranks, row_token, row_expert n * top, offsets experts + 1, tiles 2 * max_tiles integers.
+ * infer_moe_layout: out = {places, tiles, rows per tile} for n tokens. */
+int infer_moe_layout(int elem, int64_t n, int64_t width, int64_t ff_pad, int64_t experts, int64_t top, int64_t* out);
+int infer_moe(int elem, const void* h, int64_t h_stride, const void* router, const float* correction, int64_t n,
+              int64_t width, int64_t experts, int64_t identity, int64_t top, int64_t groups, int64_t keep,
+              float scale, const void* gate_up, const void* down, int64_t ff, int64_t ff_pad, int32_t* counts,
+              int32_t* ids, float* weights, int32_t* ranks, int32_t* places, int32_t* row_token, int32_t* row_expert,
+              int32_t* offsets, int32_t* tiles, int64_t max_tiles, void* act, void* out, int64_t max_places,
+              void* stream);
 
 /* Linear attention with a constant decay d per head: S = d S + k v^T, o = scale * S^T q, S[dim][vdim] float32.  A
  * token's projection row holds q, k (heads x dim), v and the gate logits (heads x vdim) at q_off, k_off, v_off and

@@ -54,6 +54,7 @@ SIGNATURES = {
     "infer_post_norm": (_c.c_int, [_c.c_int, _vp, _vp, _f32, _i64, _vp, _i64, _vp, _i64, _i64, _i64, _f32, _vp,
                                    _vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
     "infer_silu_and_mul": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _i64, _i64, _i64, _vp]),
+    "infer_clamped_gate_and_mul": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _i64, _i64, _i64, _f32, _vp]),
     "infer_latent_front": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _f32, _vp,
                                       _i64, _vp, _vp, _vp, _i64, _i64, _i64, _vp, _i64, _i64, _vp]),
     "infer_head_matmul": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _i64,
@@ -77,6 +78,29 @@ SIGNATURES = {
     "infer_grouped_prefill_supported": (_c.c_int, [_i64, _i64]),
     "infer_grouped_prefill": (_c.c_int, [_vp, _i64, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _i64, _vp, _i64,
                                          _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp]),
+    "infer_pre_norm": (_c.c_int, [_c.c_int, _vp, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _vp, _i64, _vp, _i64, _i64,
+                                  _i64, _vp, _vp, _vp, _i64, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _vp, _vp,
+                                  _i64, _i64, _i64, _f32, _vp]),
+    "infer_softcap": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _i64, _i64, _f32, _vp]),
+    "infer_head_front": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _vp,
+                                    _vp, _f32, _vp, _i64, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp, _i64,
+                                    _i64, _vp]),
+    "infer_masked_attention": (_c.c_int, [_c.c_int, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i64, _i64, _vp, _vp,
+                                          _i64, _i64, _i64, _i64, _f32, _c.c_int, _i64, _c.c_int, _vp, _vp, _i64,
+                                          _f32, _f32, _f32, _i64, _vp, _i64, _i64, _vp, _i64, _vp]),
+    "infer_masked_gather": (_c.c_int, [_vp, _i64, _i64, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _vp, _i64, _i64,
+                                       _c.c_int, _i64, _vp, _vp]),
+    "infer_masked_prefill_supported": (_c.c_int, [_i64, _i64, _i64]),
+    "infer_masked_prefill": (_c.c_int, [_vp, _i64, _vp, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _i64, _vp, _i64, _vp,
+                                        _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _c.c_int, _i64,
+                                        _c.c_int, _f32, _f32, _f32, _vp]),
+    "infer_state_space_workspace_floats": (_i64, [_c.c_int, _i64, _i64, _i64, _i64, _i64]),
+    "infer_state_space": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _vp,
+                                     _vp, _vp, _vp, _vp, _i64, _f32, _vp, _vp, _i64, _vp, _vp, _i64, _vp, _i64, _i64,
+                                     _vp, _i64, _vp, _vp, _vp, _i64, _vp, _i64, _vp]),
+    "infer_moe_layout": (_c.c_int, [_c.c_int, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "infer_moe": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp, _vp,
+                             _i64, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _i64, _vp]),
     "infer_decay_layout": (_c.c_int, [_i64, _i64, _vp]),
     "infer_decay_workspace_floats": (_i64, [_c.c_int, _i64, _i64, _i64, _i64, _i64, _i64]),
     "infer_decay_attention": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _c.c_int,

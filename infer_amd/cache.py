@@ -84,6 +84,20 @@ class StateSlots:
                 for name, (shape, dtype) in self.tensors.items()}
 
 
+class StorageGroup:
+    """What several parts of one layer keep, by name."""
+
+    def __init__(self, parts: dict):
+        self.parts = parts
+        self.slot_bytes = sum(p.slot_bytes for p in parts.values())
+
+    def block_bytes(self, block_size: int) -> int:
+        return sum(p.block_bytes(block_size) for p in self.parts.values())
+
+    def allocate(self, num_blocks: int, num_slots: int, block_size: int, device):
+        return {name: p.allocate(num_blocks, num_slots, block_size, device) for name, p in self.parts.items()}
+
+
 class LayeredLayout:
     """One storage description per layer; ``allocate`` returns one storage per layer."""
 

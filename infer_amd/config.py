@@ -77,11 +77,12 @@ def checkpoint_shapes(directory: str) -> dict[str, tuple[int, ...]]:
 class LayerSpec:
     """One layer of a model whose layers differ: the kind of its mixer, the mixer's sizes and constants, the
     width of its feed-forward (None: it has none) and the layer whose weights it uses (its own index unless
-    weights are shared)."""
+    weights are shared).  ``mlp`` is the whole description of a feed-forward that is more than a width."""
     kind: str
     mixer: dict
     ff: int | None
     owner: int
+    mlp: dict | None = None
 
 
 def dense_width(entry: dict, index: int) -> int | None:
@@ -163,6 +164,62 @@ class VokelixConfig:
                    residual_alpha=raw["postln_alpha"])
 
 
+@dataclass
+class LayerLoop:
+    """Layers ``start`` .. ``stop - 1`` run ``times`` times in a row with the same weights."""
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass
+class DogetarConfig:
+    """Dogetar: ``layers`` in order, each masked attention or masked attention beside a state space, with a dense feed-forward, a
+    mixture of experts or none; ``loop`` repeats some of them.  ``bigram`` (``mul_prev``, ``mul_cur``, ``buckets``) adds a second
+    embedding."""
+    vocab_size: int
+    hidden_size: int
+    layers: list[LayerSpec] = field(default_factory=list)
+    norm_eps: float = 1e-6
+    bigram: dict | None = None
+    loop: LayerLoop | None = None
+    logit_softcap: float | None = None
+    max_position_embeddings: int = 1 << 20          # the design sets no bound; ``max_model_len`` does
+    torch_dtype: torch.dtype = torch.bfloat16
+
+    block_multiple = 32
+    dtypes = (torch.bfloat16, torch.float32)
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    def runs(self) -> list[tuple[int, int | None]]:
+        """(layer, number of the pass or None) in the order of execution."""
+        n = len(self.layers)
+        if self.loop is None:
+            return [(i, None) for i in range(n)]
+        a, b = self.loop.start, self.loop.stop
+        if not (0 <= a < b <= n and self.loop.times >= 1):
+            raise ValueError(f"layers {a} .. {b - 1} of {n} cannot run {self.loop.times} times")
+        return [(i, None) for i in range(a)] + [(i, t) for t in range(self.loop.times) for i in range(a, b)] + [(i, None) for i in range(b, n)]
+
+    @classmethod
+    def from_json(cls, path: str) -> "DogetarConfig":
+        with open(path) as f:
+            raw = json.load(f)
+        layers = []
+        for i, e in enumerate(raw["layers"]):
+            mlp = e.get("mlp")
+            if mlp is not None and mlp["kind"] not in ("dense", "moe"):
+                raise ValueError(f"layer {i}: feed-forward kind {mlp['kind']!r} is not known")
+            layers.append(LayerSpec(e["type"], dict(e["mixer"]), mlp["ff"] if mlp is not None and mlp["kind"] == "dense" else None, i, mlp))
+        loop = raw.get("loop")
+        return cls(vocab_size=raw["vocab"], hidden_size=raw["width"], layers=layers, norm_eps=raw["norm"]["eps"],
+                   bigram=(raw.get("embedding") or {}).get("bigram"),
+                   loop=LayerLoop(loop["start"], loop["stop"], loop["times"]) if loop else None, logit_softcap=raw.get("logit_softcap"))
+
+
 def load_model_config(directory: str):
     """The configuration of the model in a directory, of the class its ``config.json`` names (``architecture``, or the
     ``architectures`` list of the transformers layout; without either it is read as Qwen3)."""
@@ -176,7 +233,8 @@ def load_model_config(directory: str):
     raise ValueError(f"no model of this package serves {names}; known: {sorted(CONFIG_CLASSES)}")
 
 
-CONFIG_CLASSES = {"Qwen3ForCausalLM": ModelConfig, "Merilorn": MerilornConfig, "Vokelix": VokelixConfig}
+CONFIG_CLASSES = {"Qwen3ForCausalLM": ModelConfig, "Merilorn": MerilornConfig, "Vokelix": VokelixConfig,
+                  "Dogetar": DogetarConfig}
 
 
 @dataclass
@@ -188,7 +246,7 @@ class Config:
     gpu_memory_utilization: float = 0.9
     tensor_parallel_size: int = 1
     enforce_eager: bool = False
-    hf_config: ModelConfig | MerilornConfig | VokelixConfig | None = None
+    hf_config: ModelConfig | MerilornConfig | VokelixConfig | DogetarConfig | None = None
     eos: int = -1
     kvcache_block_size: int = 256
     num_kvcache_blocks: int = -1

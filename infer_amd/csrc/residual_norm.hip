@@ -8,7 +8,7 @@
 //                          split-K GEMM (skinny_gemm.hip).
 //                          POST: the norm behind the residual sum instead,
 //                          x <- rms(alpha * x + y) * w_post ;  h <- x, or rms(x) * w_pre behind the last sublayer
-//   gated_act_kernel       h <- act(g) * u with act = gelu_tanh or silu
+//   gated_act_kernel       h <- act(g) * u with act = gelu_tanh or silu, or a clamped gate
 //
 // HBM / latency bound: a row is read once, held in registers between the reductions and written once.
 #include "elem.h"
@@ -172,9 +172,16 @@ struct GatedActArgs {
     const T* x; int64_t x_stride;
     int d;
     int64_t total;      // rows * d / VEC
+    float limit;        // kClamped
 };
 
-enum class Act { kGeluTanh, kSilu };
+enum class Act { kGeluTanh, kSilu, kClamped };
+
+// min(g, limit) sigmoid(1.702 min(g, limit)) (clamp(u, -limit, limit) + 1)
+__device__ __forceinline__ float clamped_gate_f(float g, float u, float limit) {
+    g = fminf(g, limit);
+    return g * sigmoid_f(1.702f * g) * (fminf(fmaxf(u, -limit), limit) + 1.f);
+}
 
 template <class T, int VEC, Act ACT>
 __global__ void __launch_bounds__(256) gated_act_kernel(GatedActArgs<T> a) {
@@ -187,31 +194,35 @@ __global__ void __launch_bounds__(256) gated_act_kernel(GatedActArgs<T> a) {
     load_elems<VEC>(a.x + row * a.x_stride + c, g);
     load_elems<VEC>(a.x + row * a.x_stride + a.d + c, u);
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) g[e] = (ACT == Act::kSilu ? silu_f(g[e]) : gelu_tanh_f(g[e])) * u[e];
+    for (int e = 0; e < VEC; ++e) {
+        if constexpr (ACT == Act::kClamped) g[e] = clamped_gate_f(g[e], u[e], a.limit);
+        else g[e] = (ACT == Act::kSilu ? silu_f(g[e]) : gelu_tanh_f(g[e])) * u[e];
+    }
     store_elems<VEC>(a.out + row * a.out_stride + c, g);
 }
 
 template <class T, Act ACT>
 int launch_gated_act(void* out, int64_t out_stride, const void* x, int64_t x_stride, int64_t rows, int64_t d,
-                     hipStream_t stream) {
+                     float limit, hipStream_t stream) {
     const size_t bytes = 8 * sizeof(T) < 16 ? 8 * sizeof(T) : 16;
     const bool vec = d % 8 == 0 && out_stride % 8 == 0 && x_stride % 8 == 0 && ptr_aligned(out, bytes) && ptr_aligned(x, bytes);
     const int64_t total = rows * (vec ? d / 8 : d);
     const int64_t blocks = (total + 255) / 256;
     if (blocks > 0x7fffffff) return INFER_KV_EINVAL;
-    GatedActArgs<T> a{(T*)out, out_stride, (const T*)x, x_stride, (int)d, total};
+    GatedActArgs<T> a{(T*)out, out_stride, (const T*)x, x_stride, (int)d, total, limit};
     if (vec) hipLaunchKernelGGL((gated_act_kernel<T, 8, ACT>), dim3((unsigned)blocks), dim3(256), 0, stream, a);
     else hipLaunchKernelGGL((gated_act_kernel<T, 1, ACT>), dim3((unsigned)blocks), dim3(256), 0, stream, a);
     return (int)hipGetLastError();
 }
 
 template <Act ACT>
-int gated_act(int elem, void* out, int64_t out_stride, const void* x, int64_t x_stride, int64_t n_rows, int64_t d, void* stream) {
+int gated_act(int elem, void* out, int64_t out_stride, const void* x, int64_t x_stride, int64_t n_rows, int64_t d, void* stream,
+              float limit = 0.f) {
     if (n_rows < 0 || d <= 0 || d > (1 << 24)) return INFER_KV_EINVAL;
     if (n_rows == 0) return INFER_KV_OK;
     if (!out || !x || out_stride < d || x_stride < 2 * d) return INFER_KV_EINVAL;
-    if (elem == INFER_ELEM_BF16) return launch_gated_act<__bf16, ACT>(out, out_stride, x, x_stride, n_rows, d, (hipStream_t)stream);
-    if (elem == INFER_ELEM_F32) return launch_gated_act<float, ACT>(out, out_stride, x, x_stride, n_rows, d, (hipStream_t)stream);
+    if (elem == INFER_ELEM_BF16) return launch_gated_act<__bf16, ACT>(out, out_stride, x, x_stride, n_rows, d, limit, (hipStream_t)stream);
+    if (elem == INFER_ELEM_F32) return launch_gated_act<float, ACT>(out, out_stride, x, x_stride, n_rows, d, limit, (hipStream_t)stream);
     return INFER_KV_EUNSUPPORTED;
 }
 
@@ -270,4 +281,9 @@ extern "C" int infer_gelu_tanh_and_mul(int elem, void* out, int64_t out_stride, 
 extern "C" int infer_silu_and_mul(int elem, void* out, int64_t out_stride, const void* x, int64_t x_stride,
                                   int64_t n_rows, int64_t d, void* stream) {
     return gated_act<Act::kSilu>(elem, out, out_stride, x, x_stride, n_rows, d, stream);
+}
+
+extern "C" int infer_clamped_gate_and_mul(int elem, void* out, int64_t out_stride, const void* x, int64_t x_stride,
+                                          int64_t n_rows, int64_t d, float limit, void* stream) {
+    return gated_act<Act::kClamped>(elem, out, out_stride, x, x_stride, n_rows, d, stream, limit);
 }

@@ -9,8 +9,14 @@
 //   row_attention_tile_kernel    MFMA tiles, keys split over workgroups, + row_attention_merge_kernel
 //   row_gather_kernel            cached rows of whole sequences as dense rows (for dense_prefill.hip)
 //
-// The softmax may have a sink (a learned score per head with neither key nor value), the output a gate per head.
+// The softmax may have a sink (a learned score per head with neither key nor value), the scores a bias that grows with the
+// distance, the output a gate per head.  A query may see only the keys of its chunk or of a window (masks.h).
+//
+// A head may have two maps: two attentions over the same values whose difference is the output.  Each map is a query head
+// of its own here (its query is zero where the other map's key stands in the row), their sums stay unreduced, and
+//   row_attention_merge2_kernel  takes the difference, norms it and applies the gate.
 #include "elem.h"
+#include "masks.h"
 
 namespace {
 
@@ -35,6 +41,10 @@ struct RowAttnArgs {
     float* part;                          // [rows][splits][heads][val_len], then [rows][splits][heads][max, sum]
     float* part_ml;
     int rows; unsigned groups;            // MFMA kernel: query rows and head groups of the launch
+    KeyMask mask;                         // which of the keys in front of it a query sees
+    bool biased;                          // scores lose distance_slope(head) per token of distance
+    float out_scale;                      // of the output
+    bool keep_parts;                      // two maps: sums are left in part, part_ml
 };
 
 template <class T>
@@ -57,7 +67,7 @@ __device__ __forceinline__ int block_id(const RowAttnArgs<T>& a, const int32_t* 
 template <class T>
 __device__ __forceinline__ float out_factor(const RowAttnArgs<T>& a, int row, int h, float m, float sum) {
     if (a.sink && sum > 0.f) sum += exp2f(a.sink[h] * kLog2e - m);
-    const float inv = sum > 0.f ? 1.f / sum : 0.f;
+    const float inv = sum > 0.f ? a.out_scale / sum : 0.f;
     return a.gate ? inv * sigmoid_f((float)a.gate[(int64_t)row * a.gate_row + h]) : inv;
 }
 template <class T>
@@ -98,7 +108,8 @@ __global__ void __launch_bounds__(256) row_attention_any_kernel(RowAttnArgs<T> a
         o[i] = 0.f;
     }
     float m = -INFINITY, l = 0.f;
-    for (int key = wave; key < len; key += 4) {
+    const float slope = a.biased ? distance_slope(h, a.heads) * kLog2e : 0.f;
+    for (int key = a.mask.first(len - 1) + wave; key < len; key += 4) {
         const int col = key / a.block_size;
         const T* kr = a.cache + (((int64_t)block_id(a, bt, col) * a.kv_heads + kvh) * a.block_size + (key - col * a.block_size)) * a.row;
         float k[NC], s = 0.f;
@@ -108,7 +119,7 @@ __global__ void __launch_bounds__(256) row_attention_any_kernel(RowAttnArgs<T> a
             k[i] = c < a.row ? (float)kr[c] : 0.f;
             s += q[i] * k[i];
         }
-        s = wave_sum(s);
+        s = wave_sum(s) - slope * (float)(len - 1 - key);
         const float mn = fmaxf(m, s);
         const float alpha = exp2f(m - mn), p = exp2f(s - mn);
         l = l * alpha + p;
@@ -127,13 +138,19 @@ __global__ void __launch_bounds__(256) row_attention_any_kernel(RowAttnArgs<T> a
         w[i] = sm[i] == -INFINITY ? 0.f : exp2f(sm[i] - mt);
         lt += sl[i] * w[i];
     }
-    const float f = out_factor(a, row, h, mt, lt);
-    T* out = out_row(a, row, h);
-    for (int c = threadIdx.x; c < a.out_n; c += 256) {
+    const int64_t rec = (int64_t)row * a.heads + h;
+    const float f = a.keep_parts ? 1.f : out_factor(a, row, h, mt, lt);
+    T* out = a.keep_parts ? nullptr : out_row(a, row, h);
+    for (int c = threadIdx.x; c < (a.keep_parts ? a.val_len : a.out_n); c += 256) {
         float v = 0.f;
 #pragma unroll
         for (int i = 0; i < 4; ++i) v += so[i][c] * w[i];
-        out[c] = (T)(v * f);
+        if (a.keep_parts) a.part[rec * a.val_len + c] = v;
+        else out[c] = (T)(v * f);
+    }
+    if (a.keep_parts && threadIdx.x == 0) {
+        a.part_ml[2 * rec] = mt;
+        a.part_ml[2 * rec + 1] = lt;
     }
 }
 
@@ -166,9 +183,9 @@ __global__ void __launch_bounds__(256, 2) row_attention_tile_kernel(RowAttnArgs<
     const int kvh = (int)(turn % a.groups) / per_kv;
     const int head0 = kvh * shared + ((int)(turn % a.groups) - kvh * per_kv) * (16 * MT), head_end = (kvh + 1) * shared;
     const int len = visible_keys(a, row);
-    const int tiles = (len + kTile - 1) / kTile;
-    const int per = (tiles + a.splits - 1) / a.splits;
-    const int t0 = split * per, t1 = t0 + per < tiles ? t0 + per : tiles;
+    const int lo = a.mask.first(len - 1), tiles = (len + kTile - 1) / kTile, tile0 = lo / kTile;
+    const int per = (tiles - tile0 + a.splits - 1) / a.splits;
+    const int t0 = tile0 + split * per, t1 = t0 + per < tiles ? t0 + per : tiles;
     if (t0 >= t1 && (a.splits > 1 || len > 0)) return;     // the merge knows which splits are empty
     const int32_t* bt = a.bt + (int64_t)table_row(a, row) * a.bt_stride;
     const int pitch = tile_pitch(a.row), ksteps = a.key_len / 32, ctiles = a.val_len / 16;
@@ -188,11 +205,12 @@ __global__ void __launch_bounds__(256, 2) row_attention_tile_kernel(RowAttnArgs<
         }
     }
     f32x4_t acc[MT][NT];
-    float m[MT], l[MT];
+    float m[MT], l[MT], slope[MT];
 #pragma unroll
     for (int u = 0; u < MT; ++u) {
         m[u] = -INFINITY;
         l[u] = 0.f;
+        slope[u] = a.biased ? distance_slope(head0 + 16 * u + n, a.heads) * kLog2e : 0.f;
 #pragma unroll
         for (int i = 0; i < NT; ++i) acc[u][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
@@ -269,6 +287,7 @@ __global__ void __launch_bounds__(256, 2) row_attention_tile_kernel(RowAttnArgs<
         // maximum moves only when it grows by more than kLazy (log2 units); until then weights are at most 2^kLazy.
         bf16x8_t pb[MT];
         const int seen = len - t * kTile - 8 * g;       // of this lane's keys the first `seen` exist
+        const int hidden = lo - t * kTile - 8 * g;      // and the first `hidden` lie in front of what the query sees
 #pragma unroll
         for (int u = 0; u < MT; ++u) {
             const float* s0 = sbuf + (16 * u + n) * kSRow + 8 * g;
@@ -280,15 +299,19 @@ __global__ void __launch_bounds__(256, 2) row_attention_tile_kernel(RowAttnArgs<
 #pragma unroll
                 for (int i = 0; i < 4; ++i) sv[4 * e + i] = (x[i] + y[i]) * a.scale_log2;
             }
-            if (len - t * kTile < kTile) {
+            if (a.biased) {
 #pragma unroll
-                for (int i = 0; i < 8; ++i) sv[i] = i < seen ? sv[i] : -INFINITY;
+                for (int i = 0; i < 8; ++i) sv[i] += slope[u] * (float)(i + 1 - seen);
+            }
+            if (len - t * kTile < kTile || t == tile0) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) sv[i] = i < seen && i >= hidden ? sv[i] : -INFINITY;
             }
             float mx = sv[0];
 #pragma unroll
             for (int i = 1; i < 8; ++i) mx = fmaxf(mx, sv[i]);
             mx = max_xor16_32(mx);
-            const bool grow = mx > m[u] + kLazy;        // always in the first tile, whose first key exists
+            const bool grow = mx > m[u] + kLazy;        // always in the first tile, which has a key that is seen
             if (__any(grow)) {
                 const float alpha = grow ? __builtin_amdgcn_exp2f(m[u] - mx) : 1.f;
                 m[u] = grow ? mx : m[u];
@@ -322,7 +345,7 @@ __global__ void __launch_bounds__(256, 2) row_attention_tile_kernel(RowAttnArgs<
         float sum = l[u] + __shfl_xor(l[u], 16, 64);
         sum += __shfl_xor(sum, 32, 64);
         if (h >= head_end) continue;
-        if (a.splits == 1) {
+        if (a.splits == 1 && !a.keep_parts) {
             const float f = out_factor(a, row, h, m[u], sum);
             __bf16* o = out_row(a, row, h);
 #pragma unroll
@@ -343,11 +366,55 @@ __global__ void __launch_bounds__(256, 2) row_attention_tile_kernel(RowAttnArgs<
     }
 }
 
+// splits of a query row that have keys
+template <class T>
+__device__ __forceinline__ int used_splits(const RowAttnArgs<T>& a, int row) {
+    const int len = visible_keys(a, row), tiles = (len + kTile - 1) / kTile - a.mask.first(len - 1) / kTile;
+    const int per = (tiles + a.splits - 1) / a.splits;
+    return per > 0 ? (tiles + per - 1) / per : 0;
+}
+
+// Two maps: out = rms(o1 - lambda o2) * gain, with the gate.  One wavefront per (query row, head).
+struct TwoMaps { float lambda, gain, eps; };
+template <class T, int NC>
+__global__ void __launch_bounds__(64) row_attention_merge2_kernel(RowAttnArgs<T> a, TwoMaps d) {
+    const int row = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+    const int used = used_splits(a, row);
+    float o[NC];
+#pragma unroll
+    for (int i = 0; i < NC; ++i) o[i] = 0.f;
+#pragma unroll
+    for (int map = 0; map < 2; ++map) {
+        const int64_t rec0 = (int64_t)row * a.splits * a.heads + 2 * h + map;
+        float m = -INFINITY, l = 0.f;
+        for (int s = 0; s < used; ++s) m = fmaxf(m, a.part_ml[2 * (rec0 + (int64_t)s * a.heads)]);
+        for (int s = 0; s < used; ++s) {
+            const float* ml = a.part_ml + 2 * (rec0 + (int64_t)s * a.heads);
+            l += ml[1] * exp2f(ml[0] - m);
+        }
+        const float f = l > 0.f ? (map ? -d.lambda : 1.f) / l : 0.f;
+        for (int s = 0; s < used; ++s) {
+            const int64_t rec = rec0 + (int64_t)s * a.heads;
+            const float w = f * exp2f(a.part_ml[2 * rec] - m);
+#pragma unroll
+            for (int i = 0; i < NC; ++i)
+                if (lane + 64 * i < a.out_n) o[i] += w * a.part[rec * a.val_len + lane + 64 * i];
+        }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NC; ++i) ss += o[i] * o[i];
+    float f = rsqrtf(wave_sum(ss) / (float)a.out_n + d.eps) * d.gain;
+    if (a.gate) f *= sigmoid_f((float)a.gate[(int64_t)row * a.gate_row + h]);
+    T* out = out_row(a, row, h);
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+        if (lane + 64 * i < a.out_n) out[lane + 64 * i] = (T)(o[i] * f);
+}
+
 __global__ void __launch_bounds__(128) row_attention_merge_kernel(RowAttnArgs<__bf16> a) {
     const int row = blockIdx.x, h = blockIdx.y;
-    const int tiles = (visible_keys(a, row) + kTile - 1) / kTile;
-    const int per = (tiles + a.splits - 1) / a.splits;
-    const int used = per > 0 ? (tiles + per - 1) / per : 0;
+    const int used = used_splits(a, row);
     const int64_t rec0 = (int64_t)row * a.splits * a.heads + h;
     float m = -INFINITY;
     for (int s = 0; s < used; ++s) m = fmaxf(m, a.part_ml[2 * (rec0 + (int64_t)s * a.heads)]);
@@ -375,6 +442,8 @@ struct RowGatherArgs {
     const int32_t* seqs;       // block-table row of each sequence
     const int32_t* cu_k;       // [sequences + 1] first dense row of each
     uint16_t* out;             // [total][kv_heads][row]
+    const int32_t* cu_q;       // [sequences + 1] or nullptr: rows that no query of these portions sees are left out
+    KeyMask mask;
 };
 
 __global__ void __launch_bounds__(256) row_gather_kernel(RowGatherArgs a) {
@@ -386,6 +455,7 @@ __global__ void __launch_bounds__(256) row_gather_kernel(RowGatherArgs a) {
     const int32_t* bt = a.bt + (int64_t)a.seqs[s] * a.bt_stride;
     const int row_chunks = a.row / 8, chunks = a.kv_heads * row_chunks;
     const int first = blockIdx.x * kTile;
+    if (a.cu_q && first + kTile <= a.mask.first(len - (a.cu_q[s + 1] - a.cu_q[s])) / kTile * kTile) return;
     for (int i = threadIdx.x; i < kTile * chunks; i += 256) {
         const int t = first + i / chunks, c = i % chunks;
         if (t >= len) return;
@@ -448,15 +518,12 @@ int run_rows(RowAttnArgs<T>& a, float* workspace, int64_t workspace_floats, hipS
     if (a.rows == 0) return INFER_KV_OK;
     if (!a.qx || !a.cache || !a.bt || !a.ctx || !a.out) return INFER_KV_EINVAL;
     if (!size_in(a.splits, 1, 64)) return INFER_KV_EINVAL;
-    if constexpr (sizeof(T) == 4) {
-        return launch_any(a, a.rows, st);
-    } else {
-        if (!tiles_fit(a.row, a.val_len, a.block_size) || !ptr_aligned(a.qx, 16) || !ptr_aligned(a.cache, 16)) {
-            a.splits = 1;
-            return launch_any(a, a.rows, st);
-        }
-        const int64_t records = (int64_t)a.rows * a.splits * a.heads;
-        if (a.splits > 1) {
+    const bool tiled = sizeof(T) == 2 && tiles_fit(a.row, a.val_len, a.block_size) && ptr_aligned(a.qx, 16) && ptr_aligned(a.cache, 16);
+    if (!tiled) a.splits = 1;
+    const int64_t records = (int64_t)a.rows * a.splits * a.heads;
+    if constexpr (sizeof(T) == 2) {
+        if (!tiled) goto any;
+        if (a.splits > 1 || a.keep_parts) {
             if (!workspace || !ptr_aligned(workspace, 16) || workspace_floats < records * (a.val_len + 2)) return INFER_KV_EWORKSPACE;
             a.part = workspace;
             a.part_ml = workspace + records * a.val_len;
@@ -472,14 +539,37 @@ int run_rows(RowAttnArgs<T>& a, float* workspace, int64_t workspace_floats, hipS
         else if (a.key_len <= 256 && a.val_len <= 256) rc = launch_tiles<4, 4, 8>(a, st);
         else rc = launch_tiles<10, 8, 10>(a, st);
         if (rc) return rc;
-        if (a.splits > 1) hipLaunchKernelGGL(row_attention_merge_kernel, dim3((unsigned)a.rows, (unsigned)a.heads), dim3(128), 0, st, a);
+        if (a.splits > 1 && !a.keep_parts) hipLaunchKernelGGL(row_attention_merge_kernel, dim3((unsigned)a.rows, (unsigned)a.heads), dim3(128), 0, st, a);
         return (int)hipGetLastError();
     }
+any:
+    if (a.keep_parts) {
+        if (!workspace || !ptr_aligned(workspace, 16) || workspace_floats < records * (a.val_len + 2)) return INFER_KV_EWORKSPACE;
+        a.part = workspace;
+        a.part_ml = workspace + records * a.val_len;
+    }
+    return launch_any(a, a.rows, st);
+}
+
+// both maps' sums, then their difference; `a` has the maps as query heads
+template <class T>
+int run_two_maps(RowAttnArgs<T>& a, TwoMaps d, float* workspace, int64_t workspace_floats, hipStream_t st) {
+    a.keep_parts = true;
+    if (a.rows == 0) return INFER_KV_OK;
+    if (a.out_n > 1024) return INFER_KV_EUNSUPPORTED;
+    const int rc = run_rows(a, workspace, workspace_floats, st);
+    if (rc) return rc;
+    const dim3 grid((unsigned)a.rows, (unsigned)(a.heads / 2)), block(64);
+    if (a.out_n <= 64) hipLaunchKernelGGL((row_attention_merge2_kernel<T, 1>), grid, block, 0, st, a, d);
+    else if (a.out_n <= 128) hipLaunchKernelGGL((row_attention_merge2_kernel<T, 2>), grid, block, 0, st, a, d);
+    else if (a.out_n <= 256) hipLaunchKernelGGL((row_attention_merge2_kernel<T, 4>), grid, block, 0, st, a, d);
+    else hipLaunchKernelGGL((row_attention_merge2_kernel<T, 16>), grid, block, 0, st, a, d);
+    return (int)hipGetLastError();
 }
 
 int row_gather(const void* cache, int64_t row, int64_t kv_heads, int64_t block_size, int64_t num_blocks, const int32_t* block_table,
                int64_t bt_stride, int64_t table_cols, const int32_t* seqs, const int32_t* cu_k, int64_t num_seqs, int64_t max_keys,
-               void* out, void* stream) {
+               void* out, void* stream, const int32_t* cu_q = nullptr, KeyMask mask = KeyMask{}) {
     if (num_seqs < 0 || max_keys < 0 || num_seqs > 65535) return INFER_KV_EINVAL;
     if (num_seqs == 0 || max_keys == 0) return INFER_KV_OK;
     if (!cache || !block_table || !seqs || !cu_k || !out || row <= 0 || row > (1 << 20) || kv_heads < 1 || kv_heads > 4096 ||
@@ -487,7 +577,7 @@ int row_gather(const void* cache, int64_t row, int64_t kv_heads, int64_t block_s
         return INFER_KV_EINVAL;
     if (row % 8 || !ptr_aligned(cache, 16) || !ptr_aligned(out, 16)) return INFER_KV_EALIGN;
     RowGatherArgs a{(const uint16_t*)cache, (int)row, (int)kv_heads, (int)block_size, (int)num_blocks, (int)table_cols, block_table,
-                    bt_stride, seqs, cu_k, (uint16_t*)out};
+                    bt_stride, seqs, cu_k, (uint16_t*)out, cu_q, mask};
     hipLaunchKernelGGL(row_gather_kernel, dim3((unsigned)((max_keys + kTile - 1) / kTile), (unsigned)num_seqs), dim3(256), 0,
                        (hipStream_t)stream, a);
     return (int)hipGetLastError();
@@ -514,7 +604,8 @@ extern "C" int infer_latent_attention(int elem, const void* qx, const void* cach
         using T = decltype(zero);
         RowAttnArgs<T> a{(const T*)qx, (const T*)cache, (int)row, (int)rank_pad, 0, (int)row, block_table, bt_stride, (int)table_cols,
                          (int)block_size, (int)num_blocks, row_seq, ctx, (int)heads, 1, (int)splits, scale * kLog2e, nullptr, nullptr, 0,
-                         (T*)out, heads * rank_pad, (int)rank_pad, (int)rank_pad, ptr_aligned(out, 8), nullptr, nullptr, (int)rows, 1};
+                         (T*)out, heads * rank_pad, (int)rank_pad, (int)rank_pad, ptr_aligned(out, 8), nullptr, nullptr, (int)rows, 1,
+                         KeyMask{}, false, 1.f, false};
         return run_rows(a, workspace, workspace_floats, (hipStream_t)stream);
     };
     if (elem == INFER_ELEM_BF16) return go(__bf16(0.f));
@@ -550,7 +641,8 @@ extern "C" int infer_grouped_attention(int elem, const void* qx, const void* cac
         RowAttnArgs<T> a{(const T*)qx, (const T*)cache, (int)(dim_pad + vdim_pad), (int)vdim_pad, (int)vdim_pad, (int)dim_pad, block_table,
                          bt_stride, (int)table_cols, (int)block_size, (int)num_blocks, row_seq, ctx, (int)heads, (int)kv_heads,
                          (int)splits, scale * kLog2e, sink, (const T*)gate, gate_stride, (T*)out, out_stride, (int)vdim, (int)vdim,
-                         ptr_aligned(out, 4 * sizeof(T)) && out_stride % 4 == 0 && vdim % 4 == 0, nullptr, nullptr, (int)rows, 1};
+                         ptr_aligned(out, 4 * sizeof(T)) && out_stride % 4 == 0 && vdim % 4 == 0, nullptr, nullptr, (int)rows, 1,
+                         KeyMask{}, false, 1.f, false};
         return run_rows(a, workspace, workspace_floats, (hipStream_t)stream);
     };
     if (elem == INFER_ELEM_BF16) return go(__bf16(0.f));
@@ -563,4 +655,42 @@ extern "C" int infer_grouped_gather(const void* cache, int64_t row, int64_t kv_h
                                     const int32_t* cu_k, int64_t num_seqs, int64_t max_keys, void* out, void* stream) {
     return row_gather(cache, row, kv_heads, block_size, num_blocks, block_table, bt_stride, table_cols, seqs, cu_k, num_seqs, max_keys,
                       out, stream);
+}
+
+extern "C" int infer_masked_attention(int elem, const void* qx, const void* cache, int64_t key_pad, int64_t vdim_pad,
+                                      const int32_t* block_table, int64_t bt_stride, int64_t table_cols, int64_t block_size,
+                                      int64_t num_blocks, const int32_t* row_seq, const int32_t* ctx, int64_t rows, int64_t heads,
+                                      int64_t kv_heads, int64_t maps, float scale, int mask_kind, int64_t mask_size, int biased,
+                                      const float* sink, const void* gate, int64_t gate_stride, float out_scale, float lambda,
+                                      float eps, int64_t splits, void* out, int64_t out_stride, int64_t vdim, float* workspace,
+                                      int64_t workspace_floats, void* stream) {
+    if (!size_in(rows, 0, 0x7fffffff) || !size_in(kv_heads, 1, 4096) || !size_in(heads, 1, 4096) || heads % kv_heads ||
+        !size_in(maps, 1, 2) || !size_in(key_pad, 1, 1 << 16) || !size_in(vdim_pad, 1, 1 << 16) || !size_in(vdim, 1, vdim_pad) ||
+        !size_in(block_size, 1, 1 << 20) || !size_in(table_cols, 1, 1 << 24) || table_cols * block_size > 0x7fffffff ||
+        num_blocks < 1 || bt_stride < table_cols || out_stride < heads * vdim || (gate && gate_stride < heads) ||
+        (maps == 2 && (sink || biased)) || !mask_valid(mask_kind, mask_size))
+        return INFER_KV_EINVAL;
+    if (key_pad % 32 || vdim_pad % 32) return INFER_KV_EALIGN;
+    auto go = [&](auto zero) {
+        using T = decltype(zero);
+        RowAttnArgs<T> a{(const T*)qx, (const T*)cache, (int)(key_pad + vdim_pad), (int)vdim_pad, (int)vdim_pad, (int)key_pad, block_table,
+                         bt_stride, (int)table_cols, (int)block_size, (int)num_blocks, row_seq, ctx, (int)(heads * maps), (int)kv_heads,
+                         (int)splits, scale * kLog2e, sink, (const T*)gate, gate_stride, (T*)out, out_stride, (int)vdim, (int)vdim,
+                         ptr_aligned(out, 4 * sizeof(T)) && out_stride % 4 == 0 && vdim % 4 == 0, nullptr, nullptr, (int)rows, 1,
+                         KeyMask{mask_kind, (int)mask_size}, biased != 0, out_scale, false};
+        if (maps == 2) return run_two_maps(a, TwoMaps{lambda, out_scale, eps}, workspace, workspace_floats, (hipStream_t)stream);
+        return run_rows(a, workspace, workspace_floats, (hipStream_t)stream);
+    };
+    if (elem == INFER_ELEM_BF16) return go(__bf16(0.f));
+    if (elem == INFER_ELEM_F32) return go(0.f);
+    return INFER_KV_EUNSUPPORTED;
+}
+
+extern "C" int infer_masked_gather(const void* cache, int64_t row, int64_t kv_heads, int64_t block_size, int64_t num_blocks,
+                                   const int32_t* block_table, int64_t bt_stride, int64_t table_cols, const int32_t* seqs,
+                                   const int32_t* cu_q, const int32_t* cu_k, int64_t num_seqs, int64_t max_keys, int mask_kind,
+                                   int64_t mask_size, void* out, void* stream) {
+    if (!cu_q || !mask_valid(mask_kind, mask_size)) return INFER_KV_EINVAL;
+    return row_gather(cache, row, kv_heads, block_size, num_blocks, block_table, bt_stride, table_cols, seqs, cu_k, num_seqs, max_keys,
+                      out, stream, cu_q, KeyMask{mask_kind, (int)mask_size});
 }

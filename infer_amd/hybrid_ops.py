@@ -1,9 +1,10 @@
-"""Python entry points of the hybrid-model kernels (latent and grouped attention, gated delta rule, linear attention
-with a constant decay, float32 residual stream), beside ``ops``: shape and type checks on the host, then one call into ``libinfer_kv.so`` on torch's
-current stream.  Activations are bfloat16 or float32; there is no CPU path."""
+"""Python entry points of the hybrid-model kernels (latent, grouped and masked attention, gated delta rule, linear attention
+with a constant decay, selective state space, mixture of experts, float32 residual stream), beside ``ops``: shape and type
+checks on the host, then one call into ``libinfer_kv.so`` on torch's current stream.  Activations are bfloat16 or float32; there is no CPU path."""
 from __future__ import annotations
 
 import ctypes
+from dataclasses import dataclass
 from functools import lru_cache
 
 import torch
@@ -86,11 +87,72 @@ def post_norm(x: torch.Tensor, eps: float, *, y=None, w_post=None, alpha: float 
     return out
 
 
-def _gated(entry: str, x: torch.Tensor) -> torch.Tensor:
+@dataclass
+class ExpertSum:
+    """The output of a mixture of experts, not summed yet: for every token, ``weights`` times the rows ``places`` of ``rows`` (-1:
+    the token's own row of ``h``), and ``shared`` (a tensor, a ``SplitKSum`` or None)."""
+    rows: torch.Tensor
+    places: torch.Tensor
+    weights: torch.Tensor
+    h: torch.Tensor
+    shared: object = None
+
+
+def pre_norm(x: torch.Tensor, w: torch.Tensor, eps: float, *, y=None, scale=None, first=None, step=None, tokens=None, embed=None,
+             prev=None, bigram=None, multipliers=(0, 0), dtype: torch.dtype = torch.bfloat16) -> torch.Tensor:
+    """``x`` [rows, width] float32 is updated in place: ``x + y * scale`` (``y`` a tensor, a ``SplitKSum`` or an ``ExpertSum``), plus
+    ``first`` and ``step``; with ``tokens`` their embedding instead, plus the row of ``bigram`` that ``prev`` and the token
+    address through ``multipliers``, which is written to ``first``, plus ``step``.  Returns ``rms(x) * w``."""
+    n, width = x.shape
+    _f32(w, width)
+    experts = y if isinstance(y, ExpertSum) else None
+    if experts is not None:
+        y = experts.shared
+        assert experts.rows.dtype == experts.h.dtype == dtype and experts.rows.is_contiguous() and experts.rows.shape[1] == width
+        assert experts.places.dtype == torch.int32 and experts.places.is_contiguous() and experts.places.shape[0] == n
+        _f32(experts.weights, *experts.places.shape)
+        assert tuple(experts.h.shape) == (n, width)
+    sub = _stream_args(x, y, scale if scale is not None else w, None, tokens, embed, dtype)
+    for vector in (scale, step):
+        if vector is not None:
+            _f32(vector, width)
+    if first is not None:
+        _f32(first, n, width)
+    buckets = 0
+    if bigram is not None:
+        assert bigram.dtype == dtype and bigram.is_contiguous() and bigram.shape[1] == width
+        assert prev.dtype == torch.int64 and prev.is_contiguous() and prev.numel() == n
+        buckets = bigram.shape[0] - 1
+    _require_gpu(x, w, *[t for t in (scale, first, step, prev, bigram) if t is not None])
+    out = torch.empty((n, width), dtype=dtype, device=x.device)
+    e = experts
+    rc = _lib.load().infer_pre_norm(
+        ELEM[dtype], _ptr(tokens), _ptr(embed), embed.shape[0] if embed is not None else 0, _ptr(prev), _ptr(bigram), buckets,
+        multipliers[0], multipliers[1], *sub, *((e.rows.data_ptr(), e.places.data_ptr(), e.weights.data_ptr(), e.places.shape[1],
+                                                 e.rows.shape[0], e.h.data_ptr(), _rows(e.h, width)) if e is not None
+                                                else (None, None, None, 0, 0, None, 0)),
+        _ptr(scale), _ptr(first), _ptr(step), x.data_ptr(), _rows(x, width), w.data_ptr(), out.data_ptr(), width, n, width, float(eps),
+        _stream_ptr(x))
+    _lib.check(rc, "pre_norm")
+    return out
+
+
+def softcap(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """``cap * tanh(x / cap)`` in float32."""
+    n, cols = x.shape
+    out = torch.empty((n, cols), dtype=torch.float32, device=x.device)
+    _require_gpu(x)
+    _lib.check(_lib.load().infer_softcap(ELEM[x.dtype], x.data_ptr(), _rows(x, cols), out.data_ptr(), n, cols, float(cap), _stream_ptr(x)),
+               "softcap")
+    return out
+
+
+def _gated(entry: str, x: torch.Tensor, *constants: float) -> torch.Tensor:
     d = x.shape[1] // 2
     out = torch.empty((x.shape[0], d), dtype=x.dtype, device=x.device)
     _require_gpu(x)
-    rc = getattr(_lib.load(), entry)(ELEM[x.dtype], out.data_ptr(), d, x.data_ptr(), _rows(x, 2 * d), x.shape[0], d, _stream_ptr(x))
+    rc = getattr(_lib.load(), entry)(ELEM[x.dtype], out.data_ptr(), d, x.data_ptr(), _rows(x, 2 * d), x.shape[0], d, *constants,
+                                       _stream_ptr(x))
     _lib.check(rc, entry)
     return out
 
@@ -103,6 +165,11 @@ def gelu_tanh_and_mul(x: torch.Tensor) -> torch.Tensor:
 def silu_and_mul(x: torch.Tensor) -> torch.Tensor:
     """``silu(x[:, :d]) * x[:, d:]``."""
     return _gated("infer_silu_and_mul", x)
+
+
+def clamped_gate_and_mul(x: torch.Tensor, limit: float) -> torch.Tensor:
+    """``g * sigmoid(1.702 g) * (u + 1)`` with ``g = min(x[:, :d], limit)`` and ``u = clamp(x[:, d:], -limit, limit)``."""
+    return _gated("infer_clamped_gate_and_mul", x, float(limit))
 
 
 # ------------------------------------------------------------------ latent attention
@@ -317,6 +384,257 @@ def grouped_prefill(q, k, v, sink, gate, out, cu_q, cu_k, max_seqlen_q: int, hea
         gate.data_ptr(), max(gate.stride(0), heads), out.data_ptr(), _rows(out, heads * vdim), cu_q.data_ptr(), cu_k.data_ptr(),
         cu_q.numel() - 1, int(max_seqlen_q), heads, kv_heads, dim, vdim, float(scale), _stream_ptr(q))
     _lib.check(rc, "grouped_prefill")
+
+
+# ------------------------------------------------------------------ masked attention
+MASKS = {None: 0, "chunk": 1, "window": 2}
+
+
+@dataclass(frozen=True)
+class MaskedShape:
+    """Sizes and constants of masked attention.  ``maps`` 2: the difference of two attentions over the same values
+    (``lam``, and ``out_scale`` behind its norm); otherwise ``out_scale`` multiplies the output."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    maps: int = 1
+    mask: str | None = None
+    mask_size: int = 1
+    distance_bias: bool = False
+    out_scale: float = 1.0
+    lam: float = 0.0
+    eps: float = 0.0
+    rot_dims: int = 0
+
+    @property
+    def key_pad(self) -> int:
+        return -(-self.maps * self.dim // 32) * 32
+
+    @property
+    def vdim_pad(self) -> int:
+        return -(-self.vdim // 32) * 32
+
+
+def head_front(s: MaskedShape, proj, offsets, bias, q_norm, k_norm, table, positions, slots, cache, qx, qx_rows: int) -> None:
+    """Biases, norms per head, rotary positions and the append of keys and values; ``cache`` is
+    [blocks, kv_heads, block_size, vdim_pad + key_pad], ``qx`` [>= qx_rows, heads * maps, key_pad]."""
+    n = proj.shape[0]
+    cols = max(offsets[0] + s.heads * s.maps * s.dim, offsets[1] + s.kv_heads * s.maps * s.dim, offsets[2] + s.kv_heads * s.vdim)
+    if bias is not None:
+        assert bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() >= cols
+    for norm in (q_norm, k_norm):
+        if norm is not None:
+            _f32(norm, s.dim)
+    if s.rot_dims:
+        assert table.dtype == torch.float32 and table.is_contiguous() and table.shape[1:] == (s.rot_dims // 2, 2)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == n
+    assert slots.dtype == torch.int32 and slots.is_contiguous() and slots.numel() == n
+    assert cache.dtype == proj.dtype and cache.is_contiguous() and cache.shape[1] == s.kv_heads and cache.shape[3] == s.key_pad + s.vdim_pad
+    assert qx_rows == 0 or (qx.dtype == proj.dtype and qx.is_contiguous() and tuple(qx.shape[1:]) == (s.heads * s.maps, s.key_pad)
+                            and qx.shape[0] >= qx_rows)
+    _require_gpu(proj, positions, slots, cache)
+    rc = _lib.load().infer_head_front(
+        ELEM[proj.dtype], proj.data_ptr(), _rows(proj, cols), s.heads, s.kv_heads, s.maps, s.dim, s.vdim, *offsets, _ptr(bias),
+        _ptr(q_norm), _ptr(k_norm), float(s.eps), _ptr(table) if s.rot_dims else None, s.rot_dims, table.shape[0] if s.rot_dims else 1,
+        positions.data_ptr(), slots.data_ptr(), cache.data_ptr(), cache.shape[2], s.key_pad, s.vdim_pad,
+        cache.shape[0] * cache.shape[2], _ptr(qx) if qx_rows else None, qx_rows, n, _stream_ptr(proj))
+    _lib.check(rc, "head_front")
+
+
+def _optional_heads(sink, gate, s: MaskedShape, rows: int, dtype) -> tuple:
+    if sink is not None:
+        _f32(sink, s.heads)
+    if gate is not None:
+        assert gate.dtype == dtype and gate.shape[0] == rows and gate.shape[1] >= s.heads and gate.stride(1) == 1
+    return _ptr(sink), _ptr(gate), max(gate.stride(0), s.heads) if gate is not None else 0
+
+
+def masked_attention(s: MaskedShape, qx, cache, block_table, ctx, out, sink=None, gate=None, row_seq=None, max_keys=None,
+                     splits: int = 0) -> None:
+    """``qx`` [rows, heads * maps, key_pad] against what the mask shows of the first ``ctx[r]`` keys of the sequence in block-table
+    row ``row_seq[r]`` (default ``r``); ``out`` [rows, heads * vdim].  ``sink`` [heads] float32, ``gate`` [rows, heads]."""
+    rows, heads = qx.shape[:2]
+    nblk, kv_heads, bs, crow = cache.shape
+    assert qx.is_contiguous() and cache.is_contiguous() and cache.dtype == qx.dtype == out.dtype
+    assert heads == s.heads * s.maps and qx.shape[2] == s.key_pad and kv_heads == s.kv_heads and crow == s.key_pad + s.vdim_pad
+    assert block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.stride(1) == 1
+    assert ctx.dtype == torch.int32 and ctx.is_contiguous() and ctx.numel() == rows and out.shape[0] == rows
+    if row_seq is None:
+        assert block_table.shape[0] >= rows
+    else:
+        assert row_seq.dtype == torch.int32 and row_seq.is_contiguous() and row_seq.numel() == rows
+    extra = _optional_heads(sink, gate, s, rows, qx.dtype)
+    _require_gpu(qx, cache, block_table, ctx, out)
+    lib = _lib.load()
+    elem, cols = ELEM[qx.dtype], block_table.shape[1]
+    if splits <= 0:
+        keys = max_keys or cols * bs
+        if s.mask is not None:
+            keys = min(keys, s.mask_size + 31)           # whole tiles of keys are read
+        splits = lib.infer_grouped_attention_splits(elem, rows, heads, kv_heads, s.key_pad, s.vdim_pad, bs, keys)
+    need = rows * splits * heads * (s.vdim_pad + 2) if splits > 1 or s.maps == 2 else 0
+    ws = torch.empty(need, dtype=torch.float32, device=qx.device) if need else None
+    rc = lib.infer_masked_attention(
+        elem, qx.data_ptr(), cache.data_ptr(), s.key_pad, s.vdim_pad, block_table.data_ptr(), max(block_table.stride(0), cols), cols, bs,
+        nblk, _ptr(row_seq), ctx.data_ptr(), rows, s.heads, s.kv_heads, s.maps, float(s.scale), MASKS[s.mask], s.mask_size,
+        int(s.distance_bias), *extra, float(s.out_scale), float(s.lam), float(s.eps), splits, out.data_ptr(),
+        _rows(out, s.heads * s.vdim), s.vdim, _ptr(ws), need, _stream_ptr(qx))
+    _lib.check(rc, "masked_attention")
+
+
+def masked_gather(s: MaskedShape, cache, block_table, seqs, cu_q, cu_k, total: int, max_keys: int) -> torch.Tensor:
+    """The cached rows of the sequences in block-table rows ``seqs`` as dense rows [total, kv_heads, row]; rows in front of what the
+    first query of a portion sees are left out."""
+    nblk, kv_heads, bs, row = cache.shape
+    assert cache.dtype == torch.bfloat16 and cache.is_contiguous()
+    assert block_table.dtype == torch.int32 and block_table.stride(1) == 1
+    for t in (seqs, cu_q, cu_k):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    assert cu_q.numel() == cu_k.numel() == seqs.numel() + 1
+    _require_gpu(cache, block_table, seqs, cu_q, cu_k)
+    out = torch.empty((total, kv_heads, row), dtype=cache.dtype, device=cache.device)
+    rc = _lib.load().infer_masked_gather(cache.data_ptr(), row, kv_heads, bs, nblk, block_table.data_ptr(),
+                                         max(block_table.stride(0), block_table.shape[1]), block_table.shape[1], seqs.data_ptr(),
+                                         cu_q.data_ptr(), cu_k.data_ptr(), seqs.numel(), max_keys, MASKS[s.mask], s.mask_size,
+                                         out.data_ptr(), _stream_ptr(cache))
+    _lib.check(rc, "masked_gather")
+    return out
+
+
+def masked_prefill_supported(s: MaskedShape) -> bool:
+    """Whether the dense-key prefill kernel serves these sizes."""
+    return bool(_lib.load().infer_masked_prefill_supported(s.maps, s.dim, s.vdim))
+
+
+def masked_prefill(s: MaskedShape, q, rows, out, cu_q, cu_k, max_seqlen_q: int, sink=None, gate=None) -> None:
+    """Whole portions: ``q`` [tokens, heads * maps * dim], ``rows`` [keys, kv_heads, row] dense rows, ``gate`` [tokens, heads], ``out``
+    [tokens, heads * vdim], all bf16; ``sink`` [heads] float32."""
+    for t in (q, rows, out):
+        assert t.dtype == torch.bfloat16
+    for t in (cu_q, cu_k):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    assert rows.is_contiguous() and rows.shape[1:] == (s.kv_heads, s.key_pad + s.vdim_pad) and cu_q.numel() == cu_k.numel()
+    assert q.shape[0] == out.shape[0]
+    k = rows[:, :, s.vdim_pad:]
+    extra = _optional_heads(sink, gate, s, q.shape[0], q.dtype)
+    _require_gpu(q, rows, out, cu_q, cu_k)
+    rc = _lib.load().infer_masked_prefill(
+        q.data_ptr(), _rows(q, s.heads * s.maps * s.dim), k.data_ptr(), k.stride(0), k.stride(1), rows.data_ptr(), rows.stride(0),
+        rows.stride(1), *extra, out.data_ptr(), _rows(out, s.heads * s.vdim), cu_q.data_ptr(), cu_k.data_ptr(), cu_q.numel() - 1,
+        int(max_seqlen_q), s.heads, s.kv_heads, s.maps, s.dim, s.vdim, float(s.scale), MASKS[s.mask], s.mask_size, int(s.distance_bias),
+        float(s.out_scale), float(s.lam), float(s.eps), _stream_ptr(q))
+    _lib.check(rc, "masked_prefill")
+
+
+# ------------------------------------------------------------------ selective state space
+@dataclass(frozen=True)
+class StateSpaceShape:
+    """Sizes and constants of a state-space layer; ``groups`` of heads share B and C, the norm has ``norm_parts`` parts."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    taps: int
+    norm_parts: int
+    eps: float
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def channels(self) -> int:
+        return self.inner + 2 * self.groups * self.state
+
+
+def state_space(s: StateSpaceShape, proj, offsets, conv, conv_bias, dt_bias, a_log, d, norm, ring, state, slots, positions,
+                decode_rows: int, spans, max_span: int, ring_slot, out) -> None:
+    """``proj`` holds z, [x | B | C] and dt at the columns ``offsets``.  Rows below ``decode_rows`` advance the state of
+    ``slots[r]`` by one token (negative: padding), the others belong to ``spans`` [.., 4] (first row, tokens, slot, first
+    position); ``ring_slot`` [rows, 2] is a row's slot and the rows of its span that follow."""
+    n = proj.shape[0]
+    z, x, dt = offsets
+    assert proj.dtype == out.dtype == ring.dtype and out.shape[0] == n
+    _f32(conv, s.channels, s.taps)
+    _f32(conv_bias, s.channels)
+    for vector in (dt_bias, a_log, d):
+        _f32(vector, s.heads)
+    _f32(norm, s.inner)
+    _f32(state, state.shape[0], s.heads, s.state, s.vdim)
+    assert ring.is_contiguous() and tuple(ring.shape) == (state.shape[0], s.taps, s.channels)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == n
+    if decode_rows:
+        assert slots.dtype == torch.int32 and slots.is_contiguous() and slots.numel() >= decode_rows
+    lib, elem = _lib.load(), ELEM[proj.dtype]
+    num_spans, need, ws, xbc = 0, 0, None, None
+    if decode_rows < n:
+        assert spans.dtype == torch.int32 and spans.is_contiguous() and spans.shape[1] == 4
+        assert ring_slot.dtype == torch.int32 and ring_slot.is_contiguous() and tuple(ring_slot.shape) == (n, 2)
+        num_spans = spans.shape[0]
+        need = lib.infer_state_space_workspace_floats(elem, s.heads, s.vdim, s.state, num_spans, max_span)
+        ws = torch.empty(need, dtype=torch.float32, device=proj.device) if need else None
+        xbc = torch.empty((n - decode_rows, s.channels), dtype=proj.dtype, device=proj.device)
+    y = torch.empty((n, s.inner), dtype=proj.dtype, device=proj.device)
+    _require_gpu(proj, conv, ring, state, out)
+    rc = lib.infer_state_space(
+        elem, proj.data_ptr(), _rows(proj, max(z + s.inner, x + s.channels, dt + s.heads)), z, x, dt, s.heads, s.vdim, s.state, s.groups,
+        s.taps, conv.data_ptr(), conv_bias.data_ptr(), dt_bias.data_ptr(), a_log.data_ptr(), d.data_ptr(), norm.data_ptr(), s.norm_parts,
+        float(s.eps), ring.data_ptr(), state.data_ptr(), state.shape[0], _ptr(slots) if decode_rows else None, positions.data_ptr(),
+        decode_rows, _ptr(spans) if num_spans else None, num_spans, max_span, _ptr(ring_slot) if num_spans else None, n, _ptr(xbc),
+        y.data_ptr(), _ptr(ws), need, out.data_ptr(), _rows(out, s.inner), _stream_ptr(proj))
+    _lib.check(rc, "state_space")
+
+
+# ------------------------------------------------------------------ mixture of experts
+@dataclass(frozen=True)
+class MoeShape:
+    """Sizes and constants of a router and its experts; ``identity`` entries behind the experts give the input itself.  Of ``groups``
+    equal groups of entries the best ``keep`` are open to choice."""
+    width: int
+    ff: int
+    experts: int
+    top: int
+    identity: int = 0
+    groups: int = 1
+    keep: int = 1
+    scale: float = 1.0
+
+    @property
+    def ff_pad(self) -> int:
+        return -(-self.ff // 8) * 8
+
+
+def moe(s: MoeShape, h, router, correction, gate_up, down, counts) -> ExpertSum:
+    """``h`` [tokens, width]; ``router`` [experts + identity, width], ``correction`` (float32) of the choice; ``gate_up``
+    [experts, 2 * ff, width], ``down`` [experts, width, ff_pad] (zeros behind ff); ``counts`` [experts] int32 zeros."""
+    n = h.shape[0]
+    assert h.dtype == router.dtype == gate_up.dtype == down.dtype
+    assert router.is_contiguous() and tuple(router.shape) == (s.experts + s.identity, s.width)
+    assert gate_up.is_contiguous() and tuple(gate_up.shape) == (s.experts, 2 * s.ff, s.width)
+    assert down.is_contiguous() and tuple(down.shape) == (s.experts, s.width, s.ff_pad)
+    assert counts.dtype == torch.int32 and counts.is_contiguous() and counts.numel() == s.experts
+    if correction is not None:
+        _f32(correction, s.experts + s.identity)
+    _require_gpu(h, router, gate_up, down, counts)
+    lib, elem = _lib.load(), ELEM[h.dtype]
+    layout = (ctypes.c_int64 * 3)()
+    _lib.check(lib.infer_moe_layout(elem, n, s.width, s.ff_pad, s.experts, s.top, ctypes.addressof(layout)), "moe_layout")
+    places_n, tiles_n, _ = layout
+    ints = torch.empty(5 * places_n + 2 * tiles_n + s.experts + 1, dtype=torch.int32, device=h.device)
+    ids, ranks, places, row_token, row_expert = (ints[i * places_n:(i + 1) * places_n] for i in range(5))
+    tiles, offsets = ints[5 * places_n:5 * places_n + 2 * tiles_n], ints[5 * places_n + 2 * tiles_n:]
+    weights = torch.empty((n, s.top), dtype=torch.float32, device=h.device)
+    act = torch.empty((places_n, s.ff_pad), dtype=h.dtype, device=h.device)
+    rows = torch.empty((places_n, s.width), dtype=h.dtype, device=h.device)
+    rc = lib.infer_moe(
+        elem, h.data_ptr(), _rows(h, s.width), router.data_ptr(), _ptr(correction), n, s.width, s.experts, s.identity, s.top, s.groups,
+        s.keep, float(s.scale), gate_up.data_ptr(), down.data_ptr(), s.ff, s.ff_pad, counts.data_ptr(), ids.data_ptr(),
+        weights.data_ptr(), ranks.data_ptr(), places.data_ptr(), row_token.data_ptr(), row_expert.data_ptr(), offsets.data_ptr(),
+        tiles.data_ptr(), tiles_n, act.data_ptr(), rows.data_ptr(), places_n, _stream_ptr(h))
+    _lib.check(rc, "moe")
+    return ExpertSum(rows, places.view(n, s.top), weights, h)
 
 
 # ------------------------------------------------------------------ linear attention with a constant decay

@@ -112,21 +112,22 @@ class ModelRunner:
 
     def _alloc_step_buffers(self):
         """Static buffers of a decode step.  The staging buffer is one int32 array
-        ``[input_ids | seq_lens | state_slots | block_table]`` that exists twice, pinned on the host and on the device."""
+        ``[input_ids | seq_lens | state_slots | previous_ids | block_table]`` that exists twice, pinned on the host and on the device."""
         config = self.config
         self.max_bs = min(config.max_num_seqs, 512)
         self.max_num_blocks = (config.max_model_len + self.block_size - 1) // self.block_size
         n, m = self.max_bs, self.max_num_blocks
-        self.stage_host = torch.zeros(n * (3 + m), dtype=torch.int32, pin_memory=True)
-        self.stage_dev = torch.zeros(n * (3 + m), dtype=torch.int32, device=self.device)
+        self.stage_host = torch.zeros(n * (4 + m), dtype=torch.int32, pin_memory=True)
+        self.stage_dev = torch.zeros(n * (4 + m), dtype=torch.int32, device=self.device)
         host = self.stage_host.numpy()
-        self.h_input_ids, self.h_seq_lens, self.h_state_slots = host[:n], host[n:2 * n], host[2 * n:3 * n]
-        self.h_block_tables = host[3 * n:].reshape(n, m)
+        self.h_input_ids, self.h_seq_lens, self.h_state_slots, self.h_prev_ids = host[:4 * n].reshape(4, n)
+        self.h_block_tables = host[4 * n:].reshape(n, m)
         self._staged = torch.cuda.Event()       # the last copy of the staging buffer has left the host
         self._staged_tables = [None] * n        # what each host row of the block table currently holds
-        self.d_input_ids, self.d_seq_lens = self.stage_dev[:n], self.stage_dev[n:2 * n]
-        self.d_state_slots = self.stage_dev[2 * n:3 * n]
-        self.d_block_tables = self.stage_dev[3 * n:].view(n, m)
+        per_row = self.stage_dev[:4 * n].view(4, n)
+        self.d_input_ids, self.d_seq_lens, self.d_state_slots = per_row[:3]
+        self.d_token_pairs = per_row[::3]       # a row's token and the one in front of it
+        self.d_block_tables = self.stage_dev[4 * n:].view(n, m)
         self.d_positions = torch.zeros(n, dtype=torch.int64, device=self.device)
         self.d_slot_mapping = torch.full((n,), -1, dtype=torch.int32, device=self.device)
         self.d_context_lens = torch.zeros(n, dtype=torch.int32, device=self.device)
@@ -157,6 +158,8 @@ class ModelRunner:
                 raise RuntimeError("a sequence's state slot lies outside the pool")
             self.h_state_slots[:bs] = slots
             self.h_state_slots[bs:run_bs] = -1
+            self.h_prev_ids[:bs] = [seq.token_ids[seq.num_computed_tokens - 1] if seq.num_computed_tokens else -1 for seq in seqs]
+            self.h_prev_ids[bs:run_bs] = -1
         else:
             ids[:bs] = [seq.last_token for seq in seqs]
             lens[:bs] = [len(seq) for seq in seqs]
@@ -186,9 +189,9 @@ class ModelRunner:
                             slot_mapping, context_lens)
         input_ids, plan = self.d_input_ids[:run_bs], None
         if self.mixed:
-            input_ids = input_ids.long()
+            input_ids, prev_ids = self.d_token_pairs[:, :run_bs].long()
             plan = step_plan.StepPlan(input_ids, positions, slot_mapping, block_tables, row_ctx=context_lens,
-                                      state_slots=self.d_state_slots[:run_bs], decode_rows=run_bs, dense_row=run_bs)
+                                      state_slots=self.d_state_slots[:run_bs], prev_ids=prev_ids, decode_rows=run_bs, dense_row=run_bs)
         set_context(False, slot_mapping=slot_mapping, context_lens=context_lens, block_tables=block_tables, step=plan)
         return self.model(input_ids, positions)
 
@@ -266,6 +269,7 @@ class ModelRunner:
         self.h_seq_lens[:] = 0
         self.h_input_ids[:] = 0
         self.h_state_slots[:] = -1
+        self.h_prev_ids[:] = -1
         self.stage_dev.copy_(self.stage_host)
         for bs in reversed(self.graph_bs):
             graph = torch.cuda.CUDAGraph()

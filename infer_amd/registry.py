@@ -1,12 +1,14 @@
 """Which model class serves which configuration."""
 from __future__ import annotations
 
-from .config import MerilornConfig, ModelConfig, VokelixConfig
+from .config import DogetarConfig, MerilornConfig, ModelConfig, VokelixConfig
+from .dogetar import DogetarForCausalLM
 from .merilorn import MerilornForCausalLM
 from .qwen3 import QwenForCausalLM
 from .vokelix import VokelixForCausalLM
 
-MODELS = {ModelConfig: QwenForCausalLM, MerilornConfig: MerilornForCausalLM, VokelixConfig: VokelixForCausalLM}
+MODELS = {ModelConfig: QwenForCausalLM, MerilornConfig: MerilornForCausalLM, VokelixConfig: VokelixForCausalLM,
+          DogetarConfig: DogetarForCausalLM}
 
 
 def model_class(config):

@@ -23,6 +23,7 @@ class StepPlan:
     block_tables: torch.Tensor             # int32 [sequences, columns]
     row_ctx: torch.Tensor                  # int32 [rows] keys each row sees
     state_slots: torch.Tensor              # int32 [decode_rows]
+    prev_ids: torch.Tensor                 # int64 [rows] the token in front of each in its sequence, -1: none
     decode_rows: int                       # rows that are the only one of their portion
     row_seq: torch.Tensor | None = None    # int32 [rows] block-table row of each row; None: the row itself
     max_keys: int | None = None            # largest row_ctx, where the host knows it
@@ -53,7 +54,7 @@ def build(portions, block_size: int, max_blocks: int, num_slots: int, num_blocks
     counts = [portions[i][1] for i in order]
     first = np.concatenate(([0], np.cumsum(counts)))
     rows = int(first[-1])
-    ids, pos = np.empty(rows, np.int64), np.empty(rows, np.int64)
+    ids, pos, prev = (np.empty(rows, np.int64) for _ in range(3))
     slots, row_seq = np.empty(rows, np.int32), np.empty(rows, np.int32)
     ring = np.empty((rows, 2), np.int32)
     tables = np.zeros((len(order), max(1, max(len(portions[i][0].block_table) for i in order))), np.int32)
@@ -70,6 +71,8 @@ def build(portions, block_size: int, max_blocks: int, num_slots: int, num_blocks
         p = np.arange(lo, lo + n)
         ids[r0:r0 + n] = seq.token_ids[lo:lo + n]
         pos[r0:r0 + n] = p
+        prev[r0] = seq.token_ids[lo - 1] if lo else -1
+        prev[r0 + 1:r0 + n] = ids[r0:r0 + n - 1]
         slots[r0:r0 + n] = table[p // block_size] * block_size + p % block_size
         row_seq[r0:r0 + n] = s
         ring[r0:r0 + n, 0] = seq.state_slot
@@ -82,7 +85,7 @@ def build(portions, block_size: int, max_blocks: int, num_slots: int, num_blocks
             dense.append(s)
     decode_rows = sum(1 for n in counts if n == 1)
     dense_row = int(first[dense[0]]) if dense else rows
-    parts = {"ids": ids, "pos": pos, "slots": slots, "tables": tables, "row_seq": row_seq,
+    parts = {"ids": ids, "pos": pos, "prev": prev, "slots": slots, "tables": tables, "row_seq": row_seq,
              "ctx": (pos + 1).astype(np.int32), "ring": ring,
              "state": ring[:decode_rows, 0],
              "port": np.asarray(port, np.int32).reshape(-1, 4), "chunk": np.asarray(chunk, np.int32).reshape(-1, 6),
@@ -92,7 +95,7 @@ def build(portions, block_size: int, max_blocks: int, num_slots: int, num_blocks
     parts["cu_k"] = np.concatenate(([0], np.cumsum(ends))).astype(np.int32)
     t = _upload(parts, device)
     plan = StepPlan(input_ids=t["ids"], positions=t["pos"], slot_mapping=t["slots"], block_tables=t["tables"],
-                    row_ctx=t["ctx"], state_slots=t["state"], decode_rows=decode_rows, row_seq=t["row_seq"],
+                    row_ctx=t["ctx"], state_slots=t["state"], prev_ids=t["prev"], decode_rows=decode_rows, row_seq=t["row_seq"],
                     max_keys=int(pos.max()) + 1, portions=t["port"], chunks=t["chunk"], ring_slot=t["ring"],
                     spans=t["span"], max_span=max((n for _, n, _, _ in span), default=0),
                     dense_row=dense_row, dense_seqs=t["dense"], dense_cu_q=t["cu_q"], dense_cu_k=t["cu_k"],
