@@ -290,11 +290,11 @@ class Ssm:
     def inputs(self, n):
         return rounded(self.rng.standard_normal((n, self.cols)), self.dtype)
 
-    def want(self, x):
-        """Outputs, final states and step sizes of one whole sequence."""
+    def want(self, x, cast=lambda a: a):
+        """Outputs and final states of one whole sequence; ``cast`` is applied behind the convolution and to what the norm gets."""
         s = self.s
         z, xbc, dt = (x[:, a:b] for a, b in ((self.off[0], self.off[1]), (self.off[1], self.off[2]), (self.off[2], self.off[2] + s.heads)))
-        xbc = silu(ref.causal_conv(xbc, self.conv, self.conv_b))
+        xbc = cast(silu(ref.causal_conv(xbc, self.conv, self.conv_b)))
         dt = ref.softplus(dt + self.dt_bias)
         n, y, states = len(x), np.zeros((len(x), s.heads, s.vdim)), []
         b = xbc[:, s.inner:s.inner + s.groups * s.state].reshape(n, s.groups, s.state)
@@ -303,7 +303,7 @@ class Ssm:
             g = h // (s.heads // s.groups)
             y[:, h], st = ref.state_space_scan(xbc[:, h * s.vdim:(h + 1) * s.vdim], b[:, g], c[:, g], dt[:, h], -np.exp(self.a_log[h]), self.d[h])
             states.append(st)
-        return ref.gated_part_norm(y.reshape(n, -1), z, s.norm_parts, self.norm, s.eps), np.stack(states)
+        return ref.gated_part_norm(cast(y.reshape(n, -1)), z, s.norm_parts, self.norm, s.eps), np.stack(states)
 
     def run(self, portions):
         """``portions``: (slot, first position, rows), decoded tokens first.  One step; the outputs in that order."""
@@ -369,16 +369,18 @@ def test_state_space_segments_of_a_long_portion(gpu, shape):
 @BOTH
 @pytest.mark.parametrize("a_log,dt", [((4.0, 9.0), 3.0), ((-20.0, -12.0), 1.0), ((-1.0, 0.0), 12.0)])
 def test_state_space_extreme_decays(gpu, dtype, a_log, dt):
-    """Total loss from token to token, none at all, and step sizes from 0 to 20 side by side."""
+    """Total loss from token to token, none at all, and step sizes from 0 to 20 side by side.  Large steps enlarge what
+    rounding does to small products of B and C, so the limit is a multiple of that."""
     m = Ssm(np.random.default_rng(7), SSM[0], dtype, a_log=a_log, dt=dt)
     x = m.inputs(97)
     want, states = m.want(x)
+    alone = np.abs(m.want(x, lambda a: rounded(a, torch.bfloat16))[0] - want).max() / np.abs(want).max()
     for slot, cuts in enumerate(([97], [1] * 97, [40, 57])):
         lo, got = 0, []
         for c in cuts:
             got += m.run([(slot, lo, x[lo:lo + c])])
             lo += c
-        close(torch.tensor(np.concatenate(got)), want, tol(dtype, 2e-5, 2e-2))
+        close(torch.tensor(np.concatenate(got)), want, tol(dtype, 2e-5, max(2e-2, 2 * alone)))
         close(m.state[slot], states, tol(dtype, 2e-5, 1e-2))
 
 
