@@ -264,6 +264,28 @@ def vokelix_config(size):
     return VokelixConfig(vocab_size=151936, hidden_size=width, layers=specs, residual_alpha=2.0)
 
 
+def dogetar_config(size):
+    """Dogetar of a published model's width: eight layers of which four run twice.  Every fourth has biased attention beside a state
+    space and a dense feed-forward; the others attention of two maps in chunks or windowed attention, and a mixture whose chosen experts and
+    shared expert together are as wide as the feed-forward."""
+    from infer_amd.config import DogetarConfig, LayerLoop, LayerSpec
+    width, ff, heads, runs = HYBRID_SIZES[size]
+    rot = {"base": 5e5, "dims": 64}
+    attn = {"kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+    two_maps = {**attn, "heads": heads, "dim": 64, "diff": 0.5, "scale": 0.125, "mask": {"size": 2048}, "rot": rot}
+    window = {**attn, "heads": heads, "mask": {"size": 1024}, "rot": {**rot, "scaling": {"factor": 4.0, "original": 8192, "low": 1.0, "high": 4.0}}}
+    parallel = {"left": {**attn, "heads": heads // 2, "mask": {"size": 2048}}, "left_scale": 1.0, "right_scale": 1.0,
+                "right": {"heads": heads * 2, "vdim": 64, "state": 128, "groups": 2, "conv": 4, "norm_groups": 2}}
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "shared": {"ff": ff // 4},
+           "router": {"experts": 14, "identity": 2, "top": 3, "scale": 2.0, "groups": {"count": 4, "keep": 2}}}
+    kinds = [("parallel", parallel, dense), ("attention", two_maps, moe), ("attention_2", window, moe), ("attention", two_maps, moe)]
+    layers = runs * 2 // 3
+    specs = [LayerSpec(kind, mixer, ff if mlp is dense else None, i, mlp) for i in range(layers) for kind, mixer, mlp in (kinds[i % 4],)]
+    return DogetarConfig(vocab_size=151936, hidden_size=width, layers=specs, bigram={"buckets": 65521, "mul_prev": 131, "mul_cur": 17},
+                         loop=LayerLoop(2, 2 + runs - layers, 2), logit_softcap=30.0)
+
+
 def hybrid_engine_point(size, model, batch, prompt, new):
     """Prefill and decode throughput of the engine on ``batch`` prompts of ``prompt`` random tokens."""
     import numpy as np
@@ -274,7 +296,7 @@ def hybrid_engine_point(size, model, batch, prompt, new):
     if model == "qwen3":
         hf = C.ModelConfig(hidden_size=width, intermediate_size=ff, num_hidden_layers=layers, num_attention_heads=heads, num_key_value_heads=8)
     else:
-        hf = {"merilorn": hybrid_config, "vokelix": vokelix_config}[model](size)
+        hf = {"merilorn": hybrid_config, "vokelix": vokelix_config, "dogetar": dogetar_config}[model](size)
     blocks = batch * (-(-(prompt + new) // 256) + 1)
     engine = LLMEngine(hf_config=hf, max_num_seqs=max(batch, 16), max_model_len=prompt + new + 1,
                        max_num_batched_tokens=16384, num_kvcache_blocks=blocks, seed=0)
@@ -546,6 +568,150 @@ def vokelix_kernels(heads=32, kv_heads=8, width=4096, ff=12288):
     return out
 
 
+def dogetar_kernels(heads=32, kv_heads=8, width=4096, ff=12288):
+    """Every kernel of Dogetar at the sizes of an 8B model's layers, with what bounds it, beside the like kernel of Qwen3 (attention, norms,
+    products) or Vokelix (recurrence, residual, activation) at the same sizes."""
+    from infer_amd import hybrid_ops as ho, ops, workloads
+    from infer_amd.layers import banded_rotary_table
+    dev, bf = torch.device("cuda:0"), torch.bfloat16
+    out, rnd, hbm, mfma = roofline_table(dev)
+    d, n, sq, bs = 128, 8, 2048, 256
+    rows = n * sq
+
+    def shape(maps=1, mask="window", size=1 << 20, bias=False):
+        return ho.MaskedShape(heads, kv_heads, d // maps, d, 0.09, maps=maps, mask=mask, mask_size=size, distance_bias=bias, lam=0.4, eps=1e-6,
+                              rot_dims=64)
+
+    # ---- decode attention: b sequences of which every query sees `seen` keys
+    gate, sink = rnd(64, heads), torch.randn(heads, device=dev)
+    for b, seen in ((64, 4096), (64, 1024), (16, 4096)):
+        nblk = b * 4096 // bs
+        cache = rnd(nblk, kv_heads, bs, 2 * d)
+        tables = torch.randperm(nblk, device=dev).to(torch.int32).view(b, -1)
+        lens, o = torch.full((b,), 4096, dtype=torch.int32, device=dev), torch.empty((b, heads * d), dtype=bf, device=dev)
+        for name, s, extra in (("window", shape(size=seen), (None, None)), ("chunk, bias, sink", shape(1, "chunk", seen, True), (sink, None)),
+                               ("chunk, two maps, gate", shape(2, "chunk", seen), (None, gate[:b]))):
+            qx = rnd(b, heads * s.maps, s.key_pad)
+            hbm(f"masked_attention decode ({name}), {b} x {seen}", b * seen * kv_heads * 2 * d * 2,
+                lambda: ho.masked_attention(s, qx, cache, tables, lens, o, *extra, max_keys=4096))
+        wl = workloads.make_decode_workload("point", [seen] * b, heads, kv_heads, seed=0, q_scale=d ** -0.5, device=dev, device_fill=True)
+        o3 = torch.empty((b, heads, d), dtype=bf, device=dev)
+        hbm(f"qwen3: paged decode attention, {b} x {seen}", wl.decode_bytes,
+            lambda: ops.paged_attn_decode(wl.q, wl.k_cache, wl.v_cache, wl.block_table, wl.context_lens, wl.scale, o3))
+        del wl, cache
+
+    # ---- prefill attention
+    cu = torch.arange(0, n + 1, dtype=torch.int32, device=dev) * sq
+    nblk = rows // bs
+    cache = rnd(nblk, kv_heads, bs, 2 * d)
+    tables = torch.randperm(nblk, device=dev).to(torch.int32).view(n, -1)
+    seqs = torch.arange(n, dtype=torch.int32, device=dev)
+    hbm(f"masked_gather, {rows} rows", 2 * cache.numel() * 2, lambda: ho.masked_gather(shape(), cache, tables, seqs, cu, cu, rows, sq))
+    kv = ho.masked_gather(shape(), cache, tables, seqs, cu, cu, rows, sq)
+    proj, at = rnd(rows, (heads + 2 * kv_heads) * d + 64), torch.empty((rows, heads * d), dtype=bf, device=dev)
+    triangle, half = sq * (sq + 1) // 2, sq // 2
+    for name, s, pairs, extra in (("window", shape(), triangle, (None, None)), ("chunk, bias, sink", shape(1, "chunk", sq, True), triangle, (sink, None)),
+                                  ("chunk, two maps, gate", shape(2, "chunk", sq), triangle, (None, proj[:, -heads:])),
+                                  ("window of 1024", shape(size=half), triangle - half * (half + 1) // 2, (None, None)),
+                                  ("chunks of 1024, two maps", shape(2, "chunk", half), half * (half + 1), (None, None))):
+        # two maps: two products of half as many entries with the keys, two with the values
+        mfma(f"masked_prefill ({name}), 8 x 2048", 2 * heads * d * (1 + s.maps) * n * pairs, BF16_PEAK_TFLOPS,
+             lambda: ho.masked_prefill(s, proj, kv, at, cu, cu, sq, *extra))
+    q3, k3 = rnd(rows, heads, d), rnd(rows, kv_heads, d)
+    mfma("qwen3: prefill attention, 8 x 2048", 4 * heads * d * n * triangle, BF16_PEAK_TFLOPS,
+         lambda: ops.flash_attn_varlen_func(q3, k3, k3, max_seqlen_q=sq, cu_seqlens_q=cu, max_seqlen_k=sq, cu_seqlens_k=cu))
+    zero = torch.zeros(rows, heads, dtype=bf, device=dev)
+    mfma("vokelix: grouped_prefill, 8 x 2048", 4 * heads * d * n * triangle, BF16_PEAK_TFLOPS,
+         lambda: ho.grouped_prefill(proj, kv[:, :, d:], kv[:, :, :d], sink, zero, at, cu, cu, sq, heads, d, d, 0.09))
+    del q3, k3, kv, zero
+
+    # ---- front end
+    table = banded_rotary_table(64, 8192, 1e6, None, dev)
+    for t in (64, rows):
+        pos, slots = torch.randint(0, 8192, (t,), device=dev), torch.randperm(nblk * bs, device=dev)[:t].to(torch.int32)
+        x, bias = proj[:t], torch.randn(proj.shape[1], device=dev)
+        moved = t * 2 * (2 * heads + 4 * kv_heads) * d
+        for name, s, extra in (("bias, norm", shape(), (bias, torch.ones(d, device=dev), torch.ones(d, device=dev))),
+                               ("two maps", shape(2), (None, None, None))):
+            split = t if t == 64 else 0
+            qx = rnd(max(split, 1), heads * s.maps, s.key_pad)
+            hbm(f"head_front ({name}), {t} rows", moved + split * 2 * heads * d * (s.maps - 1),
+                lambda: ho.head_front(s, x, [0, heads * d, (heads + kv_heads) * d], *extra, table, pos, slots, cache, qx, split))
+        qkv = rnd(t, (heads + 2 * kv_heads) * d)
+        qv, kk, vv = (y.view(t, -1, d) for y in qkv.split([heads * d, kv_heads * d, kv_heads * d], dim=-1))
+        kc, w128, cs = rnd(nblk, bs, kv_heads, d), torch.ones(d, dtype=bf, device=dev), rnd(8192, d)
+        hbm(f"qwen3: norm + rotary + append, {t} rows", moved,
+            lambda: ops.qk_norm_rope_store_kvcache(qv, kk, vv, pos, w128, w128, 1e-6, cs, kc, kc, slots, write_key=False))
+        del kc, qkv
+    del proj, at, cache
+
+    # ---- recurrence
+    s = ho.StateSpaceShape(2 * heads, 64, 128, 2, 4, 2, 1e-6)
+    hd, cols = s.inner, 2 * s.inner + 2 * s.groups * s.state + 2 * heads
+    cols = -(-cols // 64) * 64
+    state, ring = torch.zeros(64, s.heads, s.state, s.vdim, device=dev), torch.zeros(64, 4, s.channels, dtype=bf, device=dev)
+    wts = [torch.randn(s.channels, 4, device=dev) * .5, torch.zeros(s.channels, device=dev), torch.zeros(s.heads, device=dev),
+           torch.zeros(s.heads, device=dev), torch.ones(s.heads, device=dev), torch.ones(hd, device=dev)]
+    off, sl, pos = (0, hd, hd + s.channels), torch.arange(64, dtype=torch.int32, device=dev), torch.full((64,), 77, dtype=torch.int64, device=dev)
+    x, o2 = rnd(64, cols), torch.empty((64, hd), dtype=bf, device=dev)
+    hbm("state_space, one token x 64", 2 * state.numel() * 4 + 64 * 2 * (2 * hd + 4 * s.channels),
+        lambda: ho.state_space(s, x, off, *wts, ring, state, sl, pos, 64, None, 0, None, o2))
+    dec = ho.DecayShape(heads, d, d, 1e-6, True, 0, 1.0, False, False)
+    decay = ho.decay_constants([1.0 - 2.0 ** (-4.0 - 7.0 * h / heads) for h in range(heads)], dev)
+    dstate, dnorm, doff = torch.zeros(64, heads, d, d, device=dev), torch.ones(heads * d, device=dev), [i * heads * d for i in range(4)]
+    x4 = rnd(64, 4 * heads * d)
+    hbm("vokelix: decay_attention (lightning), one token x 64", 2 * dstate.numel() * 4 + 5 * 64 * heads * d * 2,
+        lambda: ho.decay_attention(dec, x4, doff, decay, None, dnorm, dstate, sl, pos, 64, None, 0, o2))
+    for m, length in ((1, 2048), (8, 2048), (1, 16384)):
+        t = m * length
+        x, o2, x4 = rnd(t, cols), torch.empty((t, hd), dtype=bf, device=dev), rnd(t, 4 * heads * d)
+        spans = torch.tensor([(i * length, length, i, 0) for i in range(m)], dtype=torch.int32, device=dev)
+        rs = torch.stack((torch.arange(m, device=dev).repeat_interleave(length), torch.arange(length - 1, -1, -1, device=dev).repeat(m)), 1).to(torch.int32)
+        pos = torch.arange(length, device=dev).repeat(m)
+        hbm(f"state_space, {m} x {length}", t * 2 * (2 * hd + s.channels + s.heads),
+            lambda: ho.state_space(s, x, off, *wts, ring, state, None, pos, 0, spans, length, rs, o2), "all launches; z, x, B, C, dt, result")
+        hbm(f"vokelix: decay_attention (lightning), {m} x {length}", 5 * t * heads * d * 2,
+            lambda: ho.decay_attention(dec, x4, doff, decay, None, dnorm, dstate, None, None, 0, spans, length, o2), "all launches; q, k, v, gate, result")
+    del x, x4, state, dstate
+
+    # ---- mixture of experts, and products of the same numbers as dense ones
+    experts, top, eff = 16, 4, ff // 4
+    ms = ho.MoeShape(width, eff, experts, top, 0, 4, 2, 1.0)
+    wr, wu, wd = rnd(experts, width), rnd(experts, 2 * eff, width), rnd(experts, width, eff)
+    counts, corr = torch.zeros(experts, dtype=torch.int32, device=dev), torch.zeros(experts, device=dev)
+    du, dd = rnd(2 * eff * top, width), rnd(width, eff * top)
+    for t in (16, 64, rows):
+        h = rnd(t, width) * 0.05
+        if t < rows:
+            weights = 3 * eff * width * 2
+            r = ho.moe(ms, h, wr, corr, wu, wd, counts)
+            used = int((torch.bincount((wr.float() @ h.float().T).topk(top, 0).indices.flatten(), minlength=experts) > 0).sum())
+            places = r.rows.shape[0]
+            hbm(f"moe, {t} rows", weights * experts + places * 2 * (2 * width + 2 * eff), lambda: ho.moe(ms, h, wr, corr, wu, wd, counts),
+                f"all launches: routing, sort, two products; weights of all experts ({used} of {experts} chosen without groups)")
+            act = rnd(t, eff * top)
+            hbm(f"qwen3: two dense products of as many columns per row, {t} rows", weights * top, lambda: (ops.linear(h, du), ops.linear(act, dd)))
+        else:
+            mfma(f"moe, {t} rows", 2 * t * top * 3 * eff * width, BF16_PEAK_TFLOPS, lambda: ho.moe(ms, h, wr, corr, wu, wd, counts),
+                 "all launches: routing, sort, two products")
+            act = rnd(t, eff * top)
+            mfma(f"qwen3: two dense products of as many columns per row, {t} rows", 2 * t * top * 3 * eff * width, BF16_PEAK_TFLOPS,
+                 lambda: (torch.nn.functional.linear(h, du), torch.nn.functional.linear(act, dd)), "vendor GEMM")
+        r = ho.moe(ms, h, wr, corr, wu, wd, counts)
+        x32, w32, y = rnd(t, width, dtype=torch.float32), torch.ones(width, device=dev), rnd(t, width)
+        hbm(f"pre_norm, {t} rows", t * width * 12, lambda: ho.pre_norm(x32, w32, 1e-6, y=y, scale=w32))
+        r.shared = y
+        hbm(f"pre_norm with {top} experts, {t} rows", t * width * (12 + 2 * top), lambda: ho.pre_norm(x32, w32, 1e-6, y=r, scale=w32))
+        hbm(f"vokelix: post_norm, {t} rows", t * width * 12, lambda: ho.post_norm(x32, 1e-6, y=y, w_post=w32, alpha=1.0))
+        gu = rnd(t, 2 * ff)
+        hbm(f"clamped_gate_and_mul, {t} rows", t * ff * 6, lambda: ho.clamped_gate_and_mul(gu, 7.0))
+        hbm(f"vokelix: silu_and_mul, {t} rows", t * ff * 6, lambda: ho.silu_and_mul(gu))
+        del r, gu, act
+    logits = rnd(64, 151936)
+    hbm("softcap, 64 rows of 151936", logits.numel() * 6, lambda: ho.softcap(logits, 30.0))
+    return out
+
+
 def engine_points(models):
     points = []
     for size, batch, prompt, new in (("0.6b", 64, 1024, 64), ("8b", 64, 1024, 64), ("8b", 16, 4096, 64)):
@@ -566,6 +732,12 @@ def run_vokelix(args):
     """Vokelix beside Qwen3 and Merilorn, as ``run_hybrid``."""
     points = [] if args.hybrid_kernels_only else engine_points(("vokelix", "qwen3", "merilorn"))
     print(json.dumps({"vokelix_engine": points, "vokelix_kernels": vokelix_kernels()}))
+
+
+def run_dogetar(args):
+    """Dogetar beside Qwen3 and Vokelix, as ``run_hybrid``."""
+    points = [] if args.hybrid_kernels_only else engine_points(("dogetar", "qwen3", "vokelix"))
+    print(json.dumps({"dogetar_engine": points, "dogetar_kernels": dogetar_kernels()}))
 
 
 # ------------------------------------------------------------------------------------------ decode curve
@@ -665,7 +837,9 @@ def main():
                     help="Merilorn beside Qwen3 at equal sizes: engine throughput and every kernel, printed as JSON")
     ap.add_argument("--vokelix", action="store_true",
                     help="Vokelix beside Qwen3 and Merilorn at equal sizes: engine throughput and every kernel, printed as JSON")
-    ap.add_argument("--hybrid-kernels-only", action="store_true", help="with --hybrid or --vokelix: the kernels alone")
+    ap.add_argument("--dogetar", action="store_true",
+                    help="Dogetar beside Qwen3 and Vokelix at equal sizes: engine throughput and every kernel, printed as JSON")
+    ap.add_argument("--hybrid-kernels-only", action="store_true", help="with --hybrid, --vokelix or --dogetar: the kernels alone")
     ap.add_argument("--e2e", action="store_true",
                     help="end-to-end decode through the engine (random-init Qwen3, HIP-graph decode) instead "
                          "of the kernel benchmark")
@@ -688,8 +862,8 @@ def main():
     if args.e2e:
         run_e2e(args)
         return
-    if args.hybrid or args.vokelix:
-        (run_vokelix if args.vokelix else run_hybrid)(args)
+    if args.hybrid or args.vokelix or args.dogetar:
+        (run_dogetar if args.dogetar else run_vokelix if args.vokelix else run_hybrid)(args)
         return
     from infer_amd import ops, workloads
     dev = torch.device("cuda:0")
