@@ -3,7 +3,8 @@
 //   moe_logits_kernel / moe_route_*   router logits in float32, softmax, the choice of experts inside the best groups, weights, and
 //                                     every choice's rank among the choices of its expert
 //   moe_scatter_kernel    rows sorted by expert: place of every choice, token and expert of every place, row tiles
-//   moe_tile_kernel       products of large row tiles: 128 rows x 128 columns per workgroup, through LDS
+//   moe_block_kernel      products of many rows per expert: 256 rows x 256 columns per workgroup, straight from memory to LDS
+//   moe_tile_kernel       products of large row tiles: 128 rows x 128 columns per workgroup, through registers to LDS
 //   moe_row_kernel        products of 16-row tiles (decode): the weights stream past the rows, k split over wavefronts
 //   moe_any_kernel        any size and element type
 //
@@ -106,34 +107,35 @@ __device__ __forceinline__ void choose(const RouteArgs<T>& a, const float* z, in
 // behind the choices of a workgroup's tokens: their ranks among all choices of their experts
 template <class T>
 __device__ __forceinline__ void finish_ranks(const RouteArgs<T>& a, int64_t token0, int tokens, int* hist, const int* ranks) {
+    const int threads = blockDim.x;
     __syncthreads();
-    for (int e = threadIdx.x; e < a.experts; e += kThreads) {
+    for (int e = threadIdx.x; e < a.experts; e += threads) {
         const int c = hist[e];
         hist[e] = c ? atomicAdd(&a.counts[e], c) : 0;
     }
     __syncthreads();
-    for (int i = threadIdx.x; i < tokens * a.top; i += kThreads) {
+    for (int i = threadIdx.x; i < tokens * a.top; i += threads) {
         const int64_t at = token0 * a.top + i;
         const int id = a.ids[at];
         a.ranks[at] = id < a.experts ? hist[id] + ranks[i] : 0;
     }
 }
 
-// ET tiles of 16 experts, 32 tokens per workgroup; wavefront w takes the k-steps w, w + 4, ...
-constexpr int kRouteTokens = 32;
-template <int ET>
-__global__ void __launch_bounds__(kThreads) moe_route_tile_kernel(RouteArgs<__bf16> a) {
-    constexpr int kRow = 16 * ET + 1;
-    __shared__ float z[kRouteTokens * kRow];
-    __shared__ int hist[kMaxExperts], ranks[kRouteTokens * 64];
+// ET tiles of 16 experts, U tiles of 16 tokens per workgroup; wavefront w of W takes the k-steps w, w + W, ...  Few tokens: one tile
+// and many wavefronts, so that the chain of requests is short; many tokens: two tiles, so that the router is read half as often.
+template <int ET, int U, int W>
+__global__ void __launch_bounds__(64 * W) moe_route_tile_kernel(RouteArgs<__bf16> a) {
+    constexpr int kRow = 16 * ET + 1, kAhead = U + ET <= 3 ? 8 : U + ET <= 6 ? 4 : 2;
+    __shared__ float z[16 * U * kRow];
+    __shared__ int hist[kMaxExperts], ranks[16 * U * 64];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, n = lane & 15;
-    const int64_t token0 = (int64_t)blockIdx.x * kRouteTokens;
-    for (int e = tid; e < a.experts; e += kThreads) hist[e] = 0;
-    f32x4_t acc[2][ET];
-    const __bf16* hr[2];
+    const int64_t token0 = (int64_t)blockIdx.x * (16 * U);
+    for (int e = tid; e < a.experts; e += 64 * W) hist[e] = 0;
+    f32x4_t acc[U][ET];
+    const __bf16* hr[U];
     const __bf16* rr[ET];
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
+    for (int u = 0; u < U; ++u) {
         const int64_t t = token0 + 16 * u + n;
         hr[u] = a.h + (t < a.n ? t : a.n - 1) * a.h_stride + 8 * g;
 #pragma unroll
@@ -141,22 +143,22 @@ __global__ void __launch_bounds__(kThreads) moe_route_tile_kernel(RouteArgs<__bf
     }
 #pragma unroll
     for (int i = 0; i < ET; ++i) rr[i] = a.router + (int64_t)(16 * i + n < a.all ? 16 * i + n : a.all - 1) * a.width + 8 * g;
-#pragma unroll 2
-    for (int k = 32 * wave; k < a.width; k += 128) {
-        bf16x8_t x[2];
+#pragma unroll kAhead
+    for (int k = 32 * wave; k < a.width; k += 32 * W) {
+        bf16x8_t x[U];
 #pragma unroll
-        for (int u = 0; u < 2; ++u) x[u] = *reinterpret_cast<const bf16x8_t*>(hr[u] + k);
+        for (int u = 0; u < U; ++u) x[u] = *reinterpret_cast<const bf16x8_t*>(hr[u] + k);
 #pragma unroll
         for (int i = 0; i < ET; ++i) {
             const bf16x8_t w = *reinterpret_cast<const bf16x8_t*>(rr[i] + k);
 #pragma unroll
-            for (int u = 0; u < 2; ++u) acc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, x[u], acc[u][i], 0, 0, 0);
+            for (int u = 0; u < U; ++u) acc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, x[u], acc[u][i], 0, 0, 0);
         }
     }
-    for (int w = 0; w < 4; ++w) {
+    for (int w = 0; w < W; ++w) {
         if (wave == w)
 #pragma unroll
-            for (int u = 0; u < 2; ++u)
+            for (int u = 0; u < U; ++u)
 #pragma unroll
                 for (int i = 0; i < ET; ++i)
 #pragma unroll
@@ -166,9 +168,15 @@ __global__ void __launch_bounds__(kThreads) moe_route_tile_kernel(RouteArgs<__bf
                     }
         __syncthreads();
     }
-    const int tokens = token0 + kRouteTokens < a.n ? kRouteTokens : (int)(a.n - token0);
-    for (int t = wave; t < tokens; t += 4) choose<(ET + 3) / 4>(a, z + t * kRow, token0 + t, hist, ranks + t * a.top);
+    const int tokens = token0 + 16 * U < a.n ? 16 * U : (int)(a.n - token0);
+    for (int t = wave; t < tokens; t += W) choose<(ET + 3) / 4>(a, z + t * kRow, token0 + t, hist, ranks + t * a.top);
     finish_ranks(a, token0, tokens, hist, ranks);
+}
+
+template <int ET>
+void launch_route(const RouteArgs<__bf16>& a, hipStream_t st) {
+    if (a.n <= 2048) hipLaunchKernelGGL((moe_route_tile_kernel<ET, 1, 16>), dim3((unsigned)((a.n + 15) / 16)), dim3(1024), 0, st, a);
+    else hipLaunchKernelGGL((moe_route_tile_kernel<ET, 2, 4>), dim3((unsigned)((a.n + 31) / 32)), dim3(256), 0, st, a);
 }
 
 // any size: one token per wavefront, four per workgroup
@@ -394,6 +402,111 @@ __global__ void __launch_bounds__(kThreads, 2) moe_tile_kernel(GemmArgs<__bf16> 
     }
 }
 
+// A workgroup of eight wavefronts: 256 rows of one expert x 256 rows of W (GATED: 128 gate rows and the same 128 up rows), k in steps
+// of 64 (a multiple of which k is) through two LDS buffers that are filled from memory without passing through registers: the
+// requests of the next step travel while this one is consumed.  Wavefront (wm, wn) has 128 rows x 64 rows of W as 8 x 4 tiles.
+// A row of a buffer is eight units of 16 bytes, unit c at place c ^ (row % 8), so that reads of a column meet all banks.
+constexpr int kBlockRows = 256, kBlockThreads = 512;
+// (tiles, column blocks) that one die works on at a time: as many as it has compute units, and as square as column blocks of 256 allow
+constexpr int kPatchTiles = 4, kPatchCols = 8, kPatch = kPatchTiles * kPatchCols;
+template <bool GATED>
+__global__ void __launch_bounds__(kBlockThreads, 2) moe_block_kernel(GemmArgs<__bf16> a) {
+    constexpr int kMat = kBlockRows * 128, kBuf = 2 * kMat;      // bytes
+    __shared__ __attribute__((aligned(1024))) unsigned char lds[2 * kBuf];
+    if (a.zero && blockIdx.x == 0)
+        for (int i = threadIdx.x; i < a.num_zero; i += kBlockThreads) a.zero[i] = 0;
+    const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, n = lane & 15;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    // workgroups go to the eight dies round-robin, and so do the patches
+    const unsigned seq = blockIdx.x >> 3, patch = seq / kPatch * 8u + (blockIdx.x & 7u), in_patch = seq % kPatch;
+    const unsigned across = (unsigned)(a.col_blocks + kPatchCols - 1) / kPatchCols;
+    const int tile = (int)(patch / across * kPatchTiles + in_patch % kPatchTiles);
+    const int cb = (int)(patch % across * kPatchCols + in_patch / kPatchTiles);
+    if (tile >= a.max_tiles || cb >= a.col_blocks) return;
+    const int expert = a.tiles[2 * tile];
+    if (expert < 0 || expert >= a.experts) return;
+    const int first = a.offsets[expert] + a.tiles[2 * tile + 1], end = a.offsets[expert + 1];
+    const int rows = end - first < kBlockRows ? end - first : kBlockRows;
+    const int c0 = cb * (GATED ? 128 : 256);
+    // load i of a wavefront fills rows 8 (4 wave + i) .. + 7: lane l place l % 8 of row l / 8
+    uint32_t x_off[4], w_off[4], to[4];                          // bytes (checked on the host to fit)
+    const uint32_t base = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) void*)lds;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int r = 8 * (4 * wave + i) + (lane >> 3), unit = (lane & 7) ^ (lane >> 3);
+        const int xr = first + (r < rows ? r : rows - 1);
+        x_off[i] = 2u * ((uint32_t)(a.row_token ? a.row_token[xr] : xr) * (uint32_t)a.x_stride + 8u * unit);
+        int col = GATED ? c0 + 32 * (r >> 6) + (r & 31) : c0 + r;
+        col = col < a.cols ? col : a.cols - 1;
+        w_off[i] = 2u * ((uint32_t)(GATED && (r & 32) ? a.up_row + col : col) * (uint32_t)a.w_stride + 8u * unit);
+        to[i] = __builtin_amdgcn_readfirstlane(base + (uint32_t)(1024 * (4 * wave + i)));
+    }
+    const __bf16* xs = a.x;
+    const __bf16* ws = a.w + (int64_t)expert * a.w_expert;
+    // Inline assembly, since the compiler would put a wait for all requests in front of every read of LDS.  Nothing else here uses M0.
+    auto request = [&](uint32_t off, const __bf16* from, uint32_t at) {
+        __asm__ volatile("s_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, %1" :: "v"(off), "s"(from), "s"(at) : "memory", "m0");
+    };
+    auto fetch = [&](int s, uint32_t buf) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            request(x_off[i], xs + 64 * s, to[i] + buf);
+            request(w_off[i], ws + 64 * s, to[i] + buf + kMat);
+        }
+    };
+    const int wm = wave & 1, wn = wave >> 1;
+    const bool live = 128 * wm < rows;
+    f32x4_t acc[4][8];                                           // [tile of W][tile of rows]
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[i][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const int steps = a.k / 64;
+    fetch(0, 0);
+    const int unit0 = n * 128 + 16 * (g ^ (n & 7));
+    for (int s = 0; s < steps; ++s) {
+        // this wavefront's requests have landed; behind the barrier everybody's have, and nobody reads the other buffer any more
+        __builtin_amdgcn_s_waitcnt(0x0F70);
+        __syncthreads();
+        if (s + 1 < steps) fetch(s + 1, (uint32_t)((s + 1) & 1) * kBuf);
+        if (!live) continue;
+        const unsigned char* xb = lds + (s & 1) * kBuf + 128 * 128 * wm;
+        const unsigned char* wb = lds + (s & 1) * kBuf + kMat + 64 * 128 * wn;
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+            const int at = unit0 ^ (64 * k);
+            bf16x8_t xf[8], wf[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) wf[i] = *reinterpret_cast<const bf16x8_t*>(wb + at + 2048 * i);
+#pragma unroll
+            for (int j = 0; j < 8; ++j) xf[j] = *reinterpret_cast<const bf16x8_t*>(xb + at + 2048 * j);
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], xf[j], acc[i][j], 0, 0, 0);
+        }
+    }
+    // lane (g, n): row n of a row tile, columns 4 g + e
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+        const int r = 128 * wm + 16 * j + n;
+        if (r >= rows) continue;
+        __bf16* o = a.out + (int64_t)(first + r) * a.out_stride;
+#pragma unroll
+        for (int i = 0; i < (GATED ? 2 : 4); ++i) {
+            const int c = c0 + (GATED ? 32 : 64) * wn + 16 * i + 4 * g;
+            bf16x4_t v;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                float x = acc[i][j][e];
+                if constexpr (GATED) x = silu_f(x) * acc[i + 2][j][e];
+                v[e] = (__bf16)(c + e < a.cols ? x : 0.f);
+            }
+            if (c + 4 <= a.out_cols) *reinterpret_cast<bf16x4_t*>(o + c) = v;       // out_cols is a multiple of eight
+        }
+    }
+}
+
 // A workgroup: 16 rows of one expert x 32 rows of W (GATED: 16 gate and 16 up); wavefront w takes the k-steps w, w + 4, ...
 constexpr int kSmallRows = 16;
 template <bool GATED>
@@ -487,6 +600,15 @@ int gemm(GemmArgs<T>& a, bool gated, int tile_rows, int64_t max_places, hipStrea
     const dim3 block(kThreads);
     int64_t grid;
     if constexpr (sizeof(T) == 2) {
+        if (tile_rows == kBlockRows) {
+            a.col_blocks = (a.out_cols + (gated ? 127 : 255)) / (gated ? 128 : 256);
+            const int64_t patches = (int64_t)((a.max_tiles + kPatchTiles - 1) / kPatchTiles) * ((a.col_blocks + kPatchCols - 1) / kPatchCols);
+            grid = (patches + 7) / 8 * 8 * kPatch;
+            if (grid > 0x7fffffff) return INFER_KV_EINVAL;
+            if (gated) hipLaunchKernelGGL((moe_block_kernel<true>), dim3((unsigned)grid), dim3(kBlockThreads), 0, st, a);
+            else hipLaunchKernelGGL((moe_block_kernel<false>), dim3((unsigned)grid), dim3(kBlockThreads), 0, st, a);
+            return (int)hipGetLastError();
+        }
         if (tile_rows == kBigRows || tile_rows == kSmallRows) {
             const int per = tile_rows == kBigRows ? (gated ? 64 : 128) : (gated ? 16 : 32);
             a.col_blocks = (a.out_cols + per - 1) / per;
@@ -513,7 +635,11 @@ int gemm(GemmArgs<T>& a, bool gated, int tile_rows, int64_t max_places, hipStrea
 // rows per tile: 0 where only the any-size kernels serve
 int rows_per_tile(int elem, int64_t n, int64_t width, int64_t ff_pad, int64_t experts, int64_t top) {
     if (elem != INFER_ELEM_BF16 || width % 8 || ff_pad % 8) return 0;
-    return n * top <= 24 * experts ? kSmallRows : kBigRows;
+    if (n * top <= 24 * experts) return kSmallRows;
+    // large blocks pay when most of them are full; their offsets are 32 bits
+    const int64_t far = 1ll << 31;
+    const bool fits = width % 64 == 0 && ff_pad % 64 == 0 && n * width < far && n * top * ff_pad < far && 2 * ff_pad * width < far;
+    return fits && n * top >= 512 * experts ? kBlockRows : kBigRows;
 }
 
 }  // namespace
@@ -554,16 +680,16 @@ extern "C" int infer_moe(int elem, const void* h, int64_t h_stride, const void* 
         bool routed = false;
         if constexpr (sizeof(T) == 2) {
             if (aligned && width % 32 == 0 && all <= 256 && ptr_aligned(router, 16)) {
-                const dim3 grid((unsigned)((n + kRouteTokens - 1) / kRouteTokens)), block(kThreads);
-                if (all <= 16) hipLaunchKernelGGL((moe_route_tile_kernel<1>), grid, block, 0, st, r);
-                else if (all <= 64) hipLaunchKernelGGL((moe_route_tile_kernel<4>), grid, block, 0, st, r);
-                else if (all <= 128) hipLaunchKernelGGL((moe_route_tile_kernel<8>), grid, block, 0, st, r);
-                else hipLaunchKernelGGL((moe_route_tile_kernel<16>), grid, block, 0, st, r);
+                if (all <= 16) launch_route<1>(r, st);
+                else if (all <= 64) launch_route<4>(r, st);
+                else if (all <= 128) launch_route<8>(r, st);
+                else launch_route<16>(r, st);
                 routed = true;
             }
         }
         if (!routed) hipLaunchKernelGGL((moe_route_any_kernel<T>), dim3((unsigned)((n + 3) / 4)), dim3(kThreads), 0, st, r);
         const int tile_rows = aligned ? (int)layout[2] : 0;
+        if (tile_rows == kBlockRows && n * h_stride >= (1ll << 31)) return INFER_KV_EUNSUPPORTED;
         const int64_t choices = n * top;
         const ScatterArgs s{ids, ranks, counts, (int)experts, (int)top, tile_rows ? tile_rows : kBigRows, (int)max_tiles, choices, places, row_token,
                             row_expert, offsets, tiles};

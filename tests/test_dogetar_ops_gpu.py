@@ -443,6 +443,39 @@ def test_moe(gpu, dtype, width, ff, experts, top, identity, groups, keep, n):
     assert np.array_equal(places < 0, chosen >= experts)
 
 
+@pytest.mark.parametrize("width,ff,experts,top", [(128, 64, 2, 1), (192, 320, 3, 2), (64, 100, 4, 1)])
+def test_moe_of_many_rows_per_expert(gpu, width, ff, experts, top):
+    """Rows enough for the largest blocks, unequal numbers of them, blocks that are nearly empty; both products and every row's place.
+    The last case pads the inner width to no multiple of the large blocks' step."""
+    rng, n, bf = np.random.default_rng(ff), 2500, torch.bfloat16
+    s = ho.MoeShape(width, ff, experts, top, 0, 1, 1, 1.5)
+    router, correction = rounded(rng.standard_normal((experts, width)) * 2 * width ** -0.5, bf), np.linspace(-0.15, 0.2, experts)
+    gate, up = rounded(rng.standard_normal((2, experts, ff, width)) * width ** -0.5, bf)
+    down = rounded(rng.standard_normal((experts, width, ff)) * ff ** -0.5, bf)
+    pool = rounded(rng.standard_normal((4 * n, width)), bf)
+    p = np.exp(pool @ router.T)
+    choice = np.sort(p / p.sum(-1, keepdims=True) + correction, -1)
+    h = pool[choice[:, -top] - choice[:, -top - 1] > 2e-3][:n]
+    assert len(h) == n
+    w = {"router": router, "correction": correction}
+    for e in range(experts):
+        w[f"e{e}.gate"], w[f"e{e}.up"], w[f"e{e}.down"] = gate[e], up[e], down[e]
+    want = ref.mixture(h, {"router": {"experts": experts, "top": top, "scale": 1.5}}, w.get)
+    padded = np.zeros((experts, width, s.ff_pad))
+    padded[..., :ff] = down
+    counts = torch.zeros(experts, dtype=torch.int32, device=gpu)
+    weights = dev(router, bf), dev(correction), dev(np.concatenate([gate, up], 1), bf), dev(padded, bf), counts
+    r = ho.moe(s, dev(h, bf), *weights)
+    x = torch.zeros((n, width), device=gpu)
+    ho.pre_norm(x, torch.ones(width, device=gpu), 1e-6, y=r)
+    close(x, want, 2e-2)
+    assert not counts.any()
+    few = ho.moe(s, dev(h[:70], bf), *weights)                 # other kernels: a token's result does not depend on the batch
+    y = torch.zeros((70, width), device=gpu)
+    ho.pre_norm(y, torch.ones(width, device=gpu), 1e-6, y=few)
+    close(y, host(x[:70]), 1e-2)
+
+
 def test_moe_when_all_tokens_want_the_same_expert(gpu):
     rng, n, width, experts = np.random.default_rng(0), 700, 64, 6
     s = ho.MoeShape(width, 32, experts, 1, 0, 1, 1, 1.0)
