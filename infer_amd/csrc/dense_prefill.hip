@@ -165,9 +165,14 @@ __global__ void __launch_bounds__(64 * kWaves, 2) dense_prefill_kernel(DensePref
             const int tok0 = s * kStep;
             f32x4_t sc[2][2];
 #pragma unroll
-            for (int u = 0; u < 2; ++u)
+            for (int u = 0; u < 2; ++u) {
+                // the accumulators start at the bias of the distance
+                const float from = MAPS == 1 && a.biased ? slope * (float)(tok0 + 8 * g - limit[u]) : 0.f;
 #pragma unroll
-                for (int t = 0; t < 2; ++t) sc[u][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+                for (int t = 0; t < 2; ++t)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) sc[u][t][e] = MAPS == 1 ? from + slope * (float)(4 * t + e) : 0.f;
+            }
 #pragma unroll
             for (int j = 0; j < KS; ++j)
 #pragma unroll
@@ -187,11 +192,6 @@ __global__ void __launch_bounds__(64 * kWaves, 2) dense_prefill_kernel(DensePref
                 for (int t = 0; t < 2; ++t)
 #pragma unroll
                     for (int e = 0; e < 4; ++e) sv[4 * t + e] = sc[u][t][e];
-                if (a.biased) {
-                    const int rel = limit[u] - tok0 - 8 * g;
-#pragma unroll
-                    for (int i = 0; i < 8; ++i) sv[i] += slope * (float)(i - rel);
-                }
                 if (tok0 + kStep - 1 > q0 + kTileQ * u + shift) {      // the earliest query of the tile does not see all of it
                     const int rel = limit[u] - tok0 - 8 * g;
 #pragma unroll

@@ -31,6 +31,7 @@ typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
 constexpr int kThreads = 256;
 constexpr int kC = 32;          // tokens per chunk
 constexpr int kSlab = 64;       // state columns per workgroup of the chunk kernel
+constexpr int kAhead = kThreads / 64;   // chunks whose step sizes are computed together, one per wavefront
 
 struct Span { int32_t row0, count, slot, pos0; };       // consecutive tokens of one sequence
 
@@ -167,22 +168,33 @@ __global__ void __launch_bounds__(kThreads) ssm_conv_kernel(SsmArgs<T> a, const 
             for (int e = 0; e < VEC; ++e) w[k][e] = a.conv[(int64_t)(c + e) * TAPS + k];
 #pragma unroll
         for (int k = 0; k + 1 < TAPS; ++k) input(i0 + k - (TAPS - 1), x[k]);
+        // inputs are requested in batches: the compiler moves no load in front of a store
+        struct alignas(sizeof(T) * VEC < 16 ? sizeof(T) * VEC : 16) Raw { T e[VEC]; };
+        constexpr int kBatch = 8;
 #pragma unroll
-        for (int i = 0; i < kConvTokens; ++i) {
-            load_elems<VEC>(in + (int64_t)(i0 + (i < end ? i : end - 1)) * a.proj_stride, x[TAPS - 1]);
-            float v[VEC];
+        for (int b = 0; b < kConvTokens; b += kBatch) {
+            if (b >= end) break;
+            Raw raw[kBatch];
 #pragma unroll
-            for (int e = 0; e < VEC; ++e) {
-                v[e] = bias[e];
+            for (int i = 0; i < kBatch; ++i)
+                raw[i] = *reinterpret_cast<const Raw*>(in + (int64_t)(i0 + (b + i < end ? b + i : end - 1)) * a.proj_stride);
 #pragma unroll
-                for (int k = 0; k < TAPS; ++k) v[e] += w[k][e] * x[k][e];
-                v[e] = silu_f(v[e]);
+            for (int i = 0; i < kBatch; ++i) {
+                float v[VEC];
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) {
+                    x[TAPS - 1][e] = (float)raw[i].e[e];
+                    v[e] = bias[e];
+#pragma unroll
+                    for (int k = 0; k < TAPS; ++k) v[e] += w[k][e] * x[k][e];
+                    v[e] = silu_f(v[e]);
+                }
+                if (b + i < end) store_elems<VEC>(o + (int64_t)(b + i) * a.xbc_stride, v);
+#pragma unroll
+                for (int k = 0; k + 1 < TAPS; ++k)
+#pragma unroll
+                    for (int e = 0; e < VEC; ++e) x[k][e] = x[k + 1][e];
             }
-            if (i < end) store_elems<VEC>(o + (int64_t)i * a.xbc_stride, v);
-#pragma unroll
-            for (int k = 0; k + 1 < TAPS; ++k)
-#pragma unroll
-                for (int e = 0; e < VEC; ++e) x[k][e] = x[k + 1][e];
         }
     } else {
         for (int i = 0; i < end; ++i) {
@@ -271,7 +283,7 @@ __global__ void __launch_bounds__(kThreads, 2) ssm_chunk_kernel(ChunkArgs args) 
     constexpr int NU = NS > 2 ? NS / 2 : 1;                      // 16-byte units of B (and of C) per thread
     __shared__ __attribute__((aligned(16))) unsigned char bbuf[kC * kRow], cbuf[OUT ? kC * kRow : 16], xbuf[kC * kXRow];
     __shared__ __attribute__((aligned(16))) unsigned char mbuf[OUT ? 2 * kC * kMRow : 16];
-    __shared__ __attribute__((aligned(16))) float sum[kC], step[kC], weight[kC];
+    __shared__ __attribute__((aligned(16))) float sums[kAhead][kC], steps[kAhead][kC], weights[kAhead][kC];
     const SsmArgs<__bf16>& a = args.a;
     const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, n = lane & 15;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -336,25 +348,32 @@ __global__ void __launch_bounds__(kThreads, 2) ssm_chunk_kernel(ChunkArgs args) 
             if constexpr (OUT) creg[i] = *reinterpret_cast<const u32x4_t*>(c_src + r + u_col[i]);
         }
         xreg = *reinterpret_cast<const u32x4_t*>(x_src + tok(x_tok) * a.xbc_stride);
-        dtreg = dt_src[(int64_t)tok(lane & 31) * a.proj_stride];
+    };
+    auto fetch_dt = [&](int c) {
+        const int t = c * kC + (lane & 31);
+        dtreg = dt_src[(int64_t)(t < count ? t : count - 1) * a.proj_stride];
     };
     const float a2 = -expf(a.a_log[h]) * kLog2e, bias = a.dt_bias[h], dh = a.d[h];
     float total = 0.f;                                           // log2 of the segment's decay
     fetch(0);
+    fetch_dt(wave);
     for (int c = 0; c < chunks; ++c) {
         __syncthreads();
-        const float dt = c * kC + (lane & 31) < count ? softplus_f((float)dtreg + bias) : 0.f;
-        float G = fmaxf(a2 * dt, -160.f);                        // nothing is left beyond, and sums stay precise
+        if (c % kAhead == 0) {                                   // this wavefront's chunk is c + wave
+            const float dt = (c + wave) * kC + (lane & 31) < count ? softplus_f((float)dtreg + bias) : 0.f;
+            float G = fmaxf(a2 * dt, -160.f);                    // nothing is left beyond, and sums stay precise
 #pragma unroll
-        for (int m = 1; m < kC; m <<= 1) {
-            const float up = __shfl_up(G, m, 32);
-            G += (lane & 31) >= m ? up : 0.f;
-        }
-        const float G_end = __shfl(G, kC - 1, 64);
-        if (tid < kC) {
-            sum[tid] = G;
-            step[tid] = dt;
-            weight[tid] = __builtin_amdgcn_exp2f(G_end - G) * dt;
+            for (int m = 1; m < kC; m <<= 1) {
+                const float up = __shfl_up(G, m, 32);
+                G += (lane & 31) >= m ? up : 0.f;
+            }
+            const float end = __shfl(G, kC - 1, 64);
+            if (lane < kC) {
+                sums[wave][lane] = G;
+                steps[wave][lane] = dt;
+                weights[wave][lane] = __builtin_amdgcn_exp2f(end - G) * dt;
+            }
+            fetch_dt(c + kAhead + wave);
         }
 #pragma unroll
         for (int i = 0; i < NU; ++i)
@@ -365,6 +384,10 @@ __global__ void __launch_bounds__(kThreads, 2) ssm_chunk_kernel(ChunkArgs args) 
         if (x_in) *reinterpret_cast<u32x4_t*>(xbuf + x_tok * kXRow + 2 * x_col) = xreg;
         if (c + 1 < chunks) fetch(c + 1);
         __syncthreads();
+        const float* sum = sums[c % kAhead];
+        const float* step = steps[c % kAhead];
+        const float* weight = weights[c % kAhead];
+        const float G_end = sum[kC - 1];
         // x of this wavefront's columns: lane (g, n) has tokens 8 g .. 8 g + 7 of column n
         const unsigned char* xr = xbuf + (8 * g + (n >> 2)) * kXRow + (n & 3) * 8 + 32 * wave;
         const i16x4 xlo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)xr);
@@ -560,7 +583,7 @@ bool chunked(int elem, int64_t vdim, int64_t state_n) { return elem == INFER_ELE
 // segments that portions are cut into, so that enough workgroups run: tokens per segment and their largest number
 void segments(int64_t heads, int64_t slabs, int64_t num_spans, int64_t max_span, int64_t& seg_len, int64_t& max_seg) {
     const int64_t units = heads * slabs * num_spans, chunks = (max_span + kC - 1) / kC;
-    int64_t want = units > 0 ? (512 + units - 1) / units : 1;
+    int64_t want = units > 0 && units < 512 ? (768 + units - 1) / units : 1;       // three workgroups per compute unit
     if (want > chunks / 4) want = chunks / 4;              // no segment shorter than four chunks
     if (want < 1) want = 1;
     const int64_t per = (chunks + want - 1) / want;
