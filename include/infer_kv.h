@@ -461,7 +461,7 @@ int infer_grouped_prefill(const void* q, int64_t q_stride, const void* k, int64_
  * row places[row][k] of `experts` (-1: the row itself of h_in).  scale, first and step may be NULL (1, 0, 0); first is
  * [row][width].  With `tokens` the sum is the embedding instead: embed[token] plus, with `bigram`, row
  * (prev * mul_prev + token * mul_cur) mod buckets of it (prev < 0: row `buckets`); first is then written (before step).
- * infer_softcap: out = cap * tanh(x / cap), float32 [rows][cols]. */
+ * infer_softcap: out = cap * tanh(scale * x / cap), float32 [rows][cols]. */
 int infer_pre_norm(int elem, const int64_t* tokens, const void* embed, int64_t vocab, const int64_t* prev,
                    const void* bigram, int64_t buckets, int64_t mul_prev, int64_t mul_cur, const void* y,
                    int64_t y_stride, const float* partial, int64_t splits, int64_t split_stride,
@@ -470,7 +470,7 @@ int infer_pre_norm(int elem, const int64_t* tokens, const void* embed, int64_t v
                    float* first, const float* step, float* x, int64_t x_stride, const float* w, void* h,
                    int64_t h_stride, int64_t n_rows, int64_t width, float eps, void* stream);
 int infer_softcap(int elem, const void* x, int64_t x_stride, float* out, int64_t n_rows, int64_t cols, float cap,
-                  void* stream);
+                  float scale, void* stream);
 
 /* Masked attention: pages [blocks][kv_heads][block_size][vdim_pad + key_pad], a row holding the value, zeros, the keys of
  * all maps one behind the other, zeros; both parts are padded to 32 elements.  maps = 2: a head has two queries and two keys
@@ -512,6 +512,52 @@ int infer_masked_prefill(const void* q, int64_t q_stride, const void* k, int64_t
                          const int32_t* cu_k, int64_t num_seqs, int64_t max_seqlen_q, int64_t heads,
                          int64_t kv_heads, int64_t maps, int64_t dim, int64_t vdim, float scale, int mask_kind,
                          int64_t mask_size, int biased, float out_scale, float lambda, float eps, void* stream);
+
+/* Float32 residual stream of a pre-norm decoder whose norm is a squashing function, norm(x) = tanh(alpha x) * w + b.  infer_tanh_norm:
+ * x <- x + y + bias (y a tensor or split-K pieces as in infer_residual_norm, bias [width] or NULL), h <- norm(x).  With `tokens`
+ * x <- the norm (in_alpha, in_w, in_b) of embed[token] * embed_scale instead.
+ * infer_xielu: out = act(x + bias), act(z) = p z^2 + z / 2 for z > 0, q (e^z - 1 - z) + z / 2 otherwise. */
+int infer_tanh_norm(int elem, const int64_t* tokens, const void* embed, int64_t vocab, float embed_scale, float in_alpha,
+                    const float* in_w, const float* in_b, const void* y, int64_t y_stride, const float* partial,
+                    int64_t splits, int64_t split_stride, int64_t partial_stride, const float* bias, float* x,
+                    int64_t x_stride, float alpha, const float* w, const float* b, void* h, int64_t h_stride,
+                    int64_t n_rows, int64_t width, void* stream);
+int infer_xielu(int elem, const void* x, int64_t x_stride, const float* bias, float p, float q, void* out,
+                int64_t out_stride, int64_t n_rows, int64_t cols, void* stream);
+
+/* Talking-heads attention: softmax weights (one added to every denominator) of all heads are mixed by talk [heads][heads] before they
+ * meet the values, w'_h = sum_g talk[h][g] w_g.  Pages: keys [blocks][kv_heads][block_size][key_pad], values
+ * [blocks][kv_heads][block_size][vdim_pad], both padded with zeros to 32 elements.
+ *
+ * infer_unit_head_front: as infer_head_front for these pages; q, k and (norm_values) v of every head are divided by their root mean
+ * square (eps), q is multiplied by 1 + temp_coef ln(floor((position + 1) / temp_every) + 1) (temp_every 0: by one).
+ * infer_talking_attention: query rows qx [rows][heads][key_pad] against the first ctx[r] keys of the sequence in block-table row
+ * row_seq[r] (NULL: r); ctx is at most max_keys.  out [rows][heads * vdim], multiplied by out_scale.  Between its kernels the scores
+ * are in the workspace (infer_talking_attention_workspace_floats).
+ * infer_talking_prefill: whole portions, bf16 (infer_talking_prefill_supported): q [tokens][head][dim], rows cu_q[s] .. cu_q[s + 1] are
+ * the last tokens of the sequence in block-table row seqs[s], which has cu_k[s + 1] - cu_k[s] keys; workspace of heads * tokens floats. */
+int infer_unit_head_front(int elem, void* proj, int64_t proj_stride, int64_t heads, int64_t kv_heads, int64_t dim,
+                          int64_t vdim, int64_t q_off, int64_t k_off, int64_t v_off, float eps, int norm_values,
+                          float temp_coef, double temp_every, const int64_t* positions, const int32_t* slots, void* keys,
+                          void* values, int64_t block_size, int64_t key_pad, int64_t vdim_pad, int64_t num_slots,
+                          void* qx, int64_t qx_rows, int64_t n, void* stream);
+int64_t infer_talking_attention_splits(int elem, int64_t rows, int64_t heads, int64_t kv_heads, int64_t key_pad,
+                                       int64_t vdim_pad, int64_t block_size, int64_t max_keys);
+int64_t infer_talking_attention_workspace_floats(int64_t rows, int64_t heads, int64_t vdim_pad, int64_t splits,
+                                                 int64_t max_keys);
+int infer_talking_attention(int elem, const void* qx, const void* keys, const void* values, int64_t key_pad,
+                            int64_t vdim_pad, const int32_t* block_table, int64_t bt_stride, int64_t table_cols,
+                            int64_t block_size, int64_t num_blocks, const int32_t* row_seq, const int32_t* ctx,
+                            int64_t rows, int64_t heads, int64_t kv_heads, float scale, const void* talk, float out_scale,
+                            int64_t splits, int64_t max_keys, void* out, int64_t out_stride, int64_t vdim,
+                            float* workspace, int64_t workspace_floats, void* stream);
+int infer_talking_prefill_supported(int64_t heads, int64_t dim, int64_t vdim, int64_t block_size);
+int infer_talking_prefill(const void* q, int64_t q_stride, const void* keys, const void* values, int64_t key_pad,
+                          int64_t vdim_pad, const int32_t* block_table, int64_t bt_stride, int64_t table_cols,
+                          int64_t block_size, int64_t num_blocks, const int32_t* seqs, const int32_t* cu_q,
+                          const int32_t* cu_k, int64_t num_seqs, int64_t tokens, int64_t max_seqlen_q, int64_t heads,
+                          int64_t kv_heads, int64_t dim, int64_t vdim, float scale, const void* talk, float out_scale,
+                          void* out, int64_t out_stride, float* workspace, int64_t workspace_floats, void* stream);
 
 /* Selective state space: S <- e^{a dt} S + dt B x^T, y = S^T C + D x per head, dt = softplus(. + dt_bias), a = -e^{a_log}; x, B and C
  * behind a causal convolution per channel and silu, heads / groups consecutive heads share B and C; behind it

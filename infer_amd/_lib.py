@@ -81,7 +81,19 @@ SIGNATURES = {
     "infer_pre_norm": (_c.c_int, [_c.c_int, _vp, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _vp, _i64, _vp, _i64, _i64,
                                   _i64, _vp, _vp, _vp, _i64, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _vp, _vp,
                                   _i64, _i64, _i64, _f32, _vp]),
-    "infer_softcap": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _i64, _i64, _f32, _vp]),
+    "infer_softcap": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _i64, _i64, _f32, _f32, _vp]),
+    "infer_tanh_norm": (_c.c_int, [_c.c_int, _vp, _vp, _i64, _f32, _f32, _vp, _vp, _vp, _i64, _vp, _i64, _i64, _i64, _vp, _vp,
+                                   _i64, _f32, _vp, _vp, _vp, _i64, _i64, _i64, _vp]),
+    "infer_xielu": (_c.c_int, [_c.c_int, _vp, _i64, _vp, _f32, _f32, _vp, _i64, _i64, _i64, _vp]),
+    "infer_unit_head_front": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _f32, _c.c_int, _f32,
+                                         _c.c_double, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp, _i64, _i64, _vp]),
+    "infer_talking_attention_splits": (_i64, [_c.c_int, _i64, _i64, _i64, _i64, _i64, _i64, _i64]),
+    "infer_talking_attention_workspace_floats": (_i64, [_i64, _i64, _i64, _i64, _i64]),
+    "infer_talking_attention": (_c.c_int, [_c.c_int, _vp, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i64, _i64, _vp, _vp, _i64,
+                                           _i64, _i64, _f32, _vp, _f32, _i64, _i64, _vp, _i64, _i64, _vp, _i64, _vp]),
+    "infer_talking_prefill_supported": (_c.c_int, [_i64, _i64, _i64, _i64]),
+    "infer_talking_prefill": (_c.c_int, [_vp, _i64, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _i64,
+                                         _i64, _i64, _i64, _i64, _i64, _f32, _vp, _f32, _vp, _i64, _vp, _i64, _vp]),
     "infer_head_front": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _vp,
                                     _vp, _f32, _vp, _i64, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp, _i64,
                                     _i64, _vp]),

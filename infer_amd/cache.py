@@ -55,6 +55,22 @@ class GroupedPages:
         return torch.zeros(num_blocks, self.kv_heads, block_size, self.row, dtype=self.dtype, device=device)
 
 
+class SplitPages:
+    """A key of ``key_row`` and a value of ``value_row`` elements per token and key/value head, in pages of their own: for kernels that
+    read the one without the other."""
+
+    def __init__(self, kv_heads: int, key_row: int, value_row: int, dtype: torch.dtype):
+        self.kv_heads, self.rows, self.dtype = kv_heads, {"keys": key_row, "values": value_row}, dtype
+
+    def block_bytes(self, block_size: int) -> int:
+        return block_size * self.kv_heads * sum(self.rows.values()) * self.dtype.itemsize
+
+    slot_bytes = 0
+
+    def allocate(self, num_blocks: int, num_slots: int, block_size: int, device):
+        return {name: torch.zeros(num_blocks, self.kv_heads, block_size, row, dtype=self.dtype, device=device) for name, row in self.rows.items()}
+
+
 class SharedStorage:
     """A layer that keeps nothing of its own and reads what the earlier layer ``owner`` keeps."""
     slot_bytes = 0

@@ -220,6 +220,35 @@ class DogetarConfig:
                    loop=LayerLoop(loop["start"], loop["stop"], loop["times"]) if loop else None, logit_softcap=raw.get("logit_softcap"))
 
 
+@dataclass
+class TuluraxConfig:
+    """Tulurax: ``layers`` in order, each talking-heads attention beside retention, with a dense feed-forward or none."""
+    vocab_size: int
+    hidden_size: int
+    layers: list[LayerSpec] = field(default_factory=list)
+    norm_eps: float = 1e-6
+    embedding_scale: float = 1.0
+    logit_scale: float = 1.0
+    logit_softcap: float | None = None
+    max_position_embeddings: int = 1 << 20          # the design sets no bound; ``max_model_len`` does
+    torch_dtype: torch.dtype = torch.bfloat16
+
+    block_multiple = 32
+    dtypes = (torch.bfloat16, torch.float32)
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_json(cls, path: str) -> "TuluraxConfig":
+        with open(path) as f:
+            raw = json.load(f)
+        layers = [LayerSpec(e["type"], dict(e["mixer"]), dense_width(e, i), i) for i, e in enumerate(raw["layers"])]
+        return cls(vocab_size=raw["vocab"], hidden_size=raw["width"], layers=layers, norm_eps=raw["norm"]["eps"],
+                   embedding_scale=raw["embedding"]["scale"], logit_scale=raw["logit_scale"], logit_softcap=raw.get("logit_softcap"))
+
+
 def load_model_config(directory: str):
     """The configuration of the model in a directory, of the class its ``config.json`` names (``architecture``, or the
     ``architectures`` list of the transformers layout; without either it is read as Qwen3)."""
@@ -234,7 +263,7 @@ def load_model_config(directory: str):
 
 
 CONFIG_CLASSES = {"Qwen3ForCausalLM": ModelConfig, "Merilorn": MerilornConfig, "Vokelix": VokelixConfig,
-                  "Dogetar": DogetarConfig}
+                  "Dogetar": DogetarConfig, "Tulurax": TuluraxConfig}
 
 
 @dataclass
@@ -246,7 +275,7 @@ class Config:
     gpu_memory_utilization: float = 0.9
     tensor_parallel_size: int = 1
     enforce_eager: bool = False
-    hf_config: ModelConfig | MerilornConfig | VokelixConfig | DogetarConfig | None = None
+    hf_config: ModelConfig | MerilornConfig | VokelixConfig | DogetarConfig | TuluraxConfig | None = None
     eos: int = -1
     kvcache_block_size: int = 256
     num_kvcache_blocks: int = -1

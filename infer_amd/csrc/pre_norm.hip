@@ -5,7 +5,7 @@
 //                     product, and/or the weighted sum of what a token's experts gave (moe.hip).  The sum can be the
 //                     embedding lookup instead, with a second table that is addressed by a token and its predecessor.
 //                     `first` (the embedding) and `step` (a vector) enter where a repeated run of layers starts.
-//   softcap_kernel    logits <- cap * tanh(logits / cap)
+//   softcap_kernel    logits <- cap * tanh(scale * logits / cap)
 //
 // HBM / latency bound: a row is read once, held in registers and written once.
 #include "elem.h"
@@ -150,10 +150,10 @@ int launch_pre_norm(const PreNormArgs<T>& a, int64_t rows, hipStream_t stream) {
 }
 
 template <class T>
-__global__ void __launch_bounds__(256) softcap_kernel(const T* x, int64_t x_stride, float* out, int64_t cols, float cap, float inv) {
+__global__ void __launch_bounds__(256) softcap_kernel(const T* x, int64_t x_stride, float* out, int64_t cols, float cap, float factor) {
     const int64_t row = blockIdx.y;
     for (int64_t c = (int64_t)blockIdx.x * 256 + threadIdx.x; c < cols; c += (int64_t)gridDim.x * 256)
-        out[row * cols + c] = cap * tanhf((float)x[row * x_stride + c] * inv);
+        out[row * cols + c] = cap * tanhf((float)x[row * x_stride + c] * factor);
 }
 
 }  // namespace
@@ -191,16 +191,16 @@ extern "C" int infer_pre_norm(int elem, const int64_t* tokens, const void* embed
 }
 
 extern "C" int infer_softcap(int elem, const void* x, int64_t x_stride, float* out, int64_t n_rows, int64_t cols, float cap,
-                             void* stream) {
+                             float scale, void* stream) {
     if (n_rows < 0 || cols <= 0 || !(cap > 0.f) || n_rows > 65535) return INFER_KV_EINVAL;
     if (n_rows == 0) return INFER_KV_OK;
     if (!x || !out || x_stride < cols) return INFER_KV_EINVAL;
     const int64_t blocks = (cols + 1023) / 1024;
     const dim3 grid((unsigned)(blocks < 4096 ? blocks : 4096), (unsigned)n_rows), block(256);
     if (elem == INFER_ELEM_BF16)
-        hipLaunchKernelGGL((softcap_kernel<__bf16>), grid, block, 0, (hipStream_t)stream, (const __bf16*)x, x_stride, out, cols, cap, 1.f / cap);
+        hipLaunchKernelGGL((softcap_kernel<__bf16>), grid, block, 0, (hipStream_t)stream, (const __bf16*)x, x_stride, out, cols, cap, scale / cap);
     else if (elem == INFER_ELEM_F32)
-        hipLaunchKernelGGL((softcap_kernel<float>), grid, block, 0, (hipStream_t)stream, (const float*)x, x_stride, out, cols, cap, 1.f / cap);
+        hipLaunchKernelGGL((softcap_kernel<float>), grid, block, 0, (hipStream_t)stream, (const float*)x, x_stride, out, cols, cap, scale / cap);
     else
         return INFER_KV_EUNSUPPORTED;
     return (int)hipGetLastError();

@@ -1,5 +1,5 @@
-"""Python entry points of the hybrid-model kernels (latent, grouped and masked attention, gated delta rule, linear attention
-with a constant decay, selective state space, mixture of experts, float32 residual stream), beside ``ops``: shape and type
+"""Python entry points of the hybrid-model kernels (latent, grouped, masked and talking-heads attention, gated delta rule, linear
+attention with a constant decay, selective state space, mixture of experts, float32 residual stream), beside ``ops``: shape and type
 checks on the host, then one call into ``libinfer_kv.so`` on torch's current stream.  Activations are bfloat16 or float32; there is no CPU path."""
 from __future__ import annotations
 
@@ -137,13 +137,52 @@ def pre_norm(x: torch.Tensor, w: torch.Tensor, eps: float, *, y=None, scale=None
     return out
 
 
-def softcap(x: torch.Tensor, cap: float) -> torch.Tensor:
-    """``cap * tanh(x / cap)`` in float32."""
+def softcap(x: torch.Tensor, cap: float, scale: float = 1.0) -> torch.Tensor:
+    """``cap * tanh(scale * x / cap)`` in float32."""
     n, cols = x.shape
     out = torch.empty((n, cols), dtype=torch.float32, device=x.device)
     _require_gpu(x)
-    _lib.check(_lib.load().infer_softcap(ELEM[x.dtype], x.data_ptr(), _rows(x, cols), out.data_ptr(), n, cols, float(cap), _stream_ptr(x)),
-               "softcap")
+    _lib.check(_lib.load().infer_softcap(ELEM[x.dtype], x.data_ptr(), _rows(x, cols), out.data_ptr(), n, cols, float(cap), float(scale),
+                                         _stream_ptr(x)), "softcap")
+    return out
+
+
+@dataclass(frozen=True)
+class TanhNorm:
+    """``tanh(alpha * x) * weight + bias``: a norm without statistics."""
+    alpha: float
+    weight: torch.Tensor
+    bias: torch.Tensor
+
+
+def tanh_norm(x: torch.Tensor, norm: TanhNorm, *, y=None, bias=None, tokens=None, embed=None, embed_scale: float = 1.0,
+              embed_norm: TanhNorm | None = None, dtype: torch.dtype = torch.bfloat16) -> torch.Tensor:
+    """``x`` [rows, width] float32 is updated in place: ``x + y + bias`` (``y`` a tensor or a ``SplitKSum``), or with ``tokens`` the
+    ``embed_norm`` of their scaled embedding.  Returns its ``norm``."""
+    n, width = x.shape
+    sub = _stream_args(x, y, norm.weight, norm.weight, tokens, embed, dtype)
+    vectors = [norm.weight, norm.bias] + ([embed_norm.weight, embed_norm.bias] if tokens is not None else []) + ([bias] if bias is not None else [])
+    for v in vectors:
+        _f32(v, width)
+    _require_gpu(x, *vectors)
+    out = torch.empty((n, width), dtype=dtype, device=x.device)
+    first = embed_norm if tokens is not None else TanhNorm(1.0, None, None)
+    rc = _lib.load().infer_tanh_norm(
+        ELEM[dtype], _ptr(tokens), _ptr(embed), embed.shape[0] if embed is not None else 0, float(embed_scale), float(first.alpha),
+        _ptr(first.weight), _ptr(first.bias), *sub, _ptr(bias), x.data_ptr(), _rows(x, width), float(norm.alpha), norm.weight.data_ptr(),
+        norm.bias.data_ptr(), out.data_ptr(), width, n, width, _stream_ptr(x))
+    _lib.check(rc, "tanh_norm")
+    return out
+
+
+def xielu(x: torch.Tensor, bias: torch.Tensor, p: float, q: float) -> torch.Tensor:
+    """Of ``z = x + bias``: ``p z^2 + z / 2`` where it is positive, ``q (e^z - 1 - z) + z / 2`` elsewhere."""
+    n, cols = x.shape
+    _f32(bias, cols)
+    out = torch.empty((n, cols), dtype=x.dtype, device=x.device)
+    _require_gpu(x, bias)
+    _lib.check(_lib.load().infer_xielu(ELEM[x.dtype], x.data_ptr(), _rows(x, cols), bias.data_ptr(), float(p), float(q), out.data_ptr(),
+                                       cols, n, cols, _stream_ptr(x)), "xielu")
     return out
 
 
@@ -526,6 +565,117 @@ def masked_prefill(s: MaskedShape, q, rows, out, cu_q, cu_k, max_seqlen_q: int, 
         int(max_seqlen_q), s.heads, s.kv_heads, s.maps, s.dim, s.vdim, float(s.scale), MASKS[s.mask], s.mask_size, int(s.distance_bias),
         float(s.out_scale), float(s.lam), float(s.eps), _stream_ptr(q))
     _lib.check(rc, "masked_prefill")
+
+
+# ------------------------------------------------------------------ talking-heads attention
+@dataclass(frozen=True)
+class TalkShape:
+    """Sizes and constants of attention whose heads mix their weights.  ``temp_every`` 0: no temperature of the queries."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    eps: float
+    norm_values: bool = True
+    temp_coef: float = 0.0
+    temp_every: float = 0.0
+    out_scale: float = 1.0
+
+    @property
+    def key_pad(self) -> int:
+        return -(-self.dim // 32) * 32
+
+    @property
+    def vdim_pad(self) -> int:
+        return -(-self.vdim // 32) * 32
+
+
+def _talk_pages(s: TalkShape, keys, values, dtype):
+    """(blocks, block size) of checked pages."""
+    assert keys.dtype == values.dtype == dtype and keys.is_contiguous() and values.is_contiguous() and keys.shape[:3] == values.shape[:3]
+    assert keys.shape[1] == s.kv_heads and keys.shape[3] == s.key_pad and values.shape[3] == s.vdim_pad
+    return keys.shape[0], keys.shape[2]
+
+
+def unit_head_front(s: TalkShape, proj, offsets, positions, slots, keys, values, qx, qx_rows: int) -> None:
+    """Norms per head, the temperature of the queries and the append of keys [blocks, kv_heads, block_size, key_pad] and values
+    [blocks, kv_heads, block_size, vdim_pad]; ``qx`` [>= qx_rows, heads, key_pad]."""
+    n = proj.shape[0]
+    blocks, bs = _talk_pages(s, keys, values, proj.dtype)
+    cols = max(offsets[0] + s.heads * s.dim, offsets[1] + s.kv_heads * s.dim, offsets[2] + s.kv_heads * s.vdim)
+    assert positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == n
+    assert slots.dtype == torch.int32 and slots.is_contiguous() and slots.numel() == n
+    assert qx_rows == 0 or (qx.dtype == proj.dtype and qx.is_contiguous() and tuple(qx.shape[1:]) == (s.heads, s.key_pad)
+                            and qx.shape[0] >= qx_rows)
+    _require_gpu(proj, positions, slots, keys, values)
+    rc = _lib.load().infer_unit_head_front(
+        ELEM[proj.dtype], proj.data_ptr(), _rows(proj, cols), s.heads, s.kv_heads, s.dim, s.vdim, *offsets, float(s.eps), int(s.norm_values),
+        float(s.temp_coef), float(s.temp_every), positions.data_ptr(), slots.data_ptr(), keys.data_ptr(), values.data_ptr(), bs, s.key_pad,
+        s.vdim_pad, blocks * bs, _ptr(qx) if qx_rows else None, qx_rows, n, _stream_ptr(proj))
+    _lib.check(rc, "unit_head_front")
+
+
+TALK_SCORES = 1 << 28          # scores that one call may keep at a time (1 GiB of float32)
+
+
+def talking_attention(s: TalkShape, qx, keys, values, talk, block_table, ctx, out, row_seq=None, max_keys=None, splits: int = 0) -> None:
+    """``qx`` [rows, heads, key_pad] against the first ``ctx[r]`` keys of the sequence in block-table row ``row_seq[r]`` (default
+    ``r``); ``talk`` [heads, heads]; ``out`` [rows, heads * vdim].  ``max_keys`` bounds ``ctx`` (default: what a block-table row can
+    address).  Many rows with many keys run in turns, so that their scores fit a workspace."""
+    rows = qx.shape[0]
+    blocks, bs = _talk_pages(s, keys, values, qx.dtype)
+    assert qx.is_contiguous() and tuple(qx.shape[1:]) == (s.heads, s.key_pad) and out.dtype == qx.dtype and out.shape[0] == rows
+    assert talk.dtype == qx.dtype and talk.is_contiguous() and tuple(talk.shape) == (s.heads, s.heads)
+    assert block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.stride(1) == 1
+    assert ctx.dtype == torch.int32 and ctx.is_contiguous() and ctx.numel() == rows
+    if row_seq is None:
+        assert block_table.shape[0] >= rows
+    else:
+        assert row_seq.dtype == torch.int32 and row_seq.is_contiguous() and row_seq.numel() == rows
+    _require_gpu(qx, keys, values, talk, block_table, ctx, out)
+    lib, elem, cols = _lib.load(), ELEM[qx.dtype], block_table.shape[1]
+    max_keys = min(max_keys or cols * bs, cols * bs)
+    turn = max(1, min(rows, TALK_SCORES // (s.heads * max_keys)))
+    forced = splits
+    for lo in range(0, rows, turn):
+        n = min(turn, rows - lo)
+        splits = forced or lib.infer_talking_attention_splits(elem, n, s.heads, s.kv_heads, s.key_pad, s.vdim_pad, bs, max_keys)
+        need = lib.infer_talking_attention_workspace_floats(n, s.heads, s.vdim_pad, splits, max_keys)
+        ws = torch.empty(need, dtype=torch.float32, device=qx.device)
+        table = block_table[lo:] if row_seq is None else block_table
+        rc = lib.infer_talking_attention(
+            elem, qx[lo:].data_ptr(), keys.data_ptr(), values.data_ptr(), s.key_pad, s.vdim_pad, table.data_ptr(), max(block_table.stride(0), cols),
+            cols, bs, blocks, None if row_seq is None else row_seq[lo:].data_ptr(), ctx[lo:].data_ptr(), n, s.heads, s.kv_heads, float(s.scale),
+            talk.data_ptr(), float(s.out_scale), splits, max_keys, out[lo:].data_ptr(), _rows(out, s.heads * s.vdim), s.vdim, ws.data_ptr(), need,
+            _stream_ptr(qx))
+        _lib.check(rc, "talking_attention")
+
+
+def talking_prefill_supported(s: TalkShape, block_size: int) -> bool:
+    """Whether the kernels for whole portions serve these sizes."""
+    return bool(_lib.load().infer_talking_prefill_supported(s.heads, s.dim, s.vdim, block_size))
+
+
+def talking_prefill(s: TalkShape, q, keys, values, talk, block_table, seqs, cu_q, cu_k, max_seqlen_q: int, out) -> None:
+    """Whole portions: ``q`` [tokens, heads * dim] (behind ``unit_head_front``) are the last tokens of the sequences in block-table rows
+    ``seqs``, whose numbers of keys ``cu_k`` sums up; ``out`` [tokens, heads * vdim], all bf16."""
+    blocks, bs = _talk_pages(s, keys, values, torch.bfloat16)
+    assert q.dtype == out.dtype == talk.dtype == torch.bfloat16 and q.shape[0] == out.shape[0]
+    assert talk.is_contiguous() and tuple(talk.shape) == (s.heads, s.heads)
+    assert block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.stride(1) == 1
+    for t in (seqs, cu_q, cu_k):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    assert cu_q.numel() == cu_k.numel() == seqs.numel() + 1
+    _require_gpu(q, keys, values, talk, block_table, seqs, cu_q, cu_k, out)
+    tokens, cols = q.shape[0], block_table.shape[1]
+    ws = torch.empty(s.heads * tokens, dtype=torch.float32, device=q.device)
+    rc = _lib.load().infer_talking_prefill(
+        q.data_ptr(), _rows(q, s.heads * s.dim), keys.data_ptr(), values.data_ptr(), s.key_pad, s.vdim_pad, block_table.data_ptr(),
+        max(block_table.stride(0), cols), cols, bs, blocks, seqs.data_ptr(), cu_q.data_ptr(), cu_k.data_ptr(), seqs.numel(), tokens,
+        int(max_seqlen_q), s.heads, s.kv_heads, s.dim, s.vdim, float(s.scale), talk.data_ptr(), float(s.out_scale), out.data_ptr(),
+        _rows(out, s.heads * s.vdim), ws.data_ptr(), ws.numel(), _stream_ptr(q))
+    _lib.check(rc, "talking_prefill")
 
 
 # ------------------------------------------------------------------ selective state space
