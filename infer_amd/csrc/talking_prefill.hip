@@ -1,8 +1,480 @@
+// Attention whose heads mix their softmax weights (talking_attention.hip), for long prompt portions, for gfx950 (MI355X).  bf16 in, float32
+// accumulate, keys and values straight from their pages.
+//
+//     w_h(i, j) = e^{s_h(i, j)} / (1 + sum_j' e^{s_h(i, j')}) ,   o_h(i) = c sum_j (sum_g T[h][g] w_g(i, j)) v_j
+//
+// A running rescale does not commute with the mixture, so denominators come first, and the scores are computed twice instead of passing
+// through memory:
+//   talk_lse_kernel   log2 of every (head, query)'s denominator.  A wavefront owns 64 queries of a head and reads keys straight into operands.
+//   talk_mix_kernel   a workgroup of eight wavefronts owns 16 QT queries and ALL heads, UH heads per wavefront, and walks the keys in
+//                     steps of 32:
+//       S^T[key, query] = K[key, :] . q^T           per wavefront its heads; weights e^{S - lse} go to LDS as two bf16 pieces each
+//                                                   (2^-17), one record [head][piece] per (query, key)
+//       P'^T[key, h]    = W^T[key, g] . T^T[g, h]    per wavefront 2 QT queries, the pieces side by side along k; to LDS as bf16
+//       O^T[v, query]  += V^T[v, key] . P'^T[key, query]      per wavefront its heads; values transposed by a buffer of its own in LDS
+//                     Nothing is rescaled: what is added up is final.
+// Row r of tile x of the first two products is key 8 (r / 4) + 4 x + r % 4, so that a lane's eight results are eight consecutive keys.
 #include "elem.h"
-extern "C" int infer_talking_prefill_supported(int64_t, int64_t, int64_t, int64_t) { return 0; }
+#include "pieces.h"
+
+namespace {
+
+typedef short i16x4 __attribute__((ext_vector_type(4)));
+typedef short i16x8 __attribute__((ext_vector_type(8)));
+typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
+typedef uint32_t u32x2_t __attribute__((ext_vector_type(2)));
+
+constexpr int kStep = 32;
+constexpr int kLseWaves = 4, kLseQ = 64;  // queries per wavefront
+constexpr int kMixWaves = 8;
+constexpr float kLow = -1e30f;            // a maximum before any key was seen; finite, since hidden scores are -inf
+constexpr float kLazy = 8.f;              // log2 units by which a sum's terms may exceed one before it is rescaled
+
+struct TalkPrefillArgs {
+    const __bf16* q; int64_t q_stride;    // [token][head * dim]
+    const __bf16* keys; const __bf16* values;                 // [blocks][kv_heads][block_size][key_pad], .. [vdim_pad]
+    int key_pad, vdim_pad;
+    const int32_t* bt; int64_t bt_stride; int table_cols, block_size, num_blocks;
+    const int32_t* seqs; const int32_t* cu_q; const int32_t* cu_k;
+    int heads, kv_heads, dim, vdim, nseq, qblocks;
+    float scale_log2;
+    const __bf16* talk;                   // [heads][heads]
+    float out_scale;
+    __bf16* out; int64_t out_stride;      // [token][head * vdim]
+    float* lse; int64_t tokens;           // [heads][tokens]
+};
+
+// The tiles of 32 keys of a sequence, one behind the other; a tile lies in one block, whose id is looked up one block ahead.
+struct PageWalk {
+    const int32_t* bt;
+    int tiles_per_block, col, in_block, id, next_id;
+    __device__ __forceinline__ int lookup(const TalkPrefillArgs& a, int c) const {
+        const int b = bt[c < a.table_cols ? c : a.table_cols - 1];
+        return b < 0 ? 0 : (b >= a.num_blocks ? a.num_blocks - 1 : b);
+    }
+    __device__ __forceinline__ PageWalk(const TalkPrefillArgs& a, int seq) {
+        bt = a.bt + (int64_t)a.seqs[seq] * a.bt_stride;
+        tiles_per_block = a.block_size / kStep;
+        col = in_block = 0;
+        id = lookup(a, 0);
+        next_id = lookup(a, 1);
+    }
+    // the tile's number among the tiles of all blocks of one head (of kv_heads), for key/value head 0; then moves on
+    __device__ __forceinline__ int64_t next(const TalkPrefillArgs& a) {
+        const int64_t at = (int64_t)id * a.kv_heads * tiles_per_block + in_block;
+        if (++in_block == tiles_per_block) {
+            in_block = 0;
+            ++col;
+            id = next_id;
+            next_id = lookup(a, col + 1);
+        }
+        return at;
+    }
+};
+
+// Workgroups go to the eight dies round-robin; die k works through the k-th contiguous eighth of the units.
+__device__ __forceinline__ unsigned unit_of(unsigned id, unsigned total) {
+    const unsigned die = id & 7u, per_die = total >> 3, extra = total & 7u;
+    return die * per_die + (die < extra ? die : extra) + (id >> 3);
+}
+
+template <int KS>
+__global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefillArgs a) {
+    constexpr int U = kLseQ / 16;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, n = lane & 15;
+    const unsigned wg = unit_of(blockIdx.x, gridDim.x);
+    const int qblk = a.qblocks - 1 - (int)(wg % a.qblocks);      // late blocks see the most keys: first
+    const int b = (int)((wg / a.qblocks) % a.nseq), h = (int)(wg / ((unsigned)a.qblocks * a.nseq));
+    const int q_beg = a.cu_q[b], sq = a.cu_q[b + 1] - q_beg, sk = a.cu_k[b + 1] - a.cu_k[b], shift = sk - sq;
+    const int q0 = (qblk * kLseWaves + wave) * kLseQ;
+    if (q0 >= sq) return;
+    const int last_q = q0 + kLseQ < sq ? q0 + kLseQ - 1 : sq - 1, steps = (last_q + shift) / kStep + 1;
+    bf16x8_t q[U][KS];
+    float m[U], l[U];
+    int limit[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+        const int qi = q0 + 16 * u + n < sq ? q0 + 16 * u + n : sq - 1;
+        limit[u] = qi + shift;
+        m[u] = kLow;
+        l[u] = 0.f;
+        const __bf16* qp = a.q + (int64_t)(q_beg + qi) * a.q_stride + (int64_t)h * a.dim + 8 * g;
+#pragma unroll
+        for (int j = 0; j < KS; ++j) {
+            q[u][j] = bf16x8_t{};
+            if (32 * j + 8 * g < a.dim) q[u][j] = *reinterpret_cast<const bf16x8_t*>(qp + 32 * j);
+        }
+    }
+    int k_off[2][KS];                                 // k-steps behind the size repeat the first one, which meets zeros
+#pragma unroll
+    for (int x = 0; x < 2; ++x)
+#pragma unroll
+        for (int j = 0; j < KS; ++j) k_off[x][j] = (8 * (n >> 2) + 4 * x + (n & 3)) * a.key_pad + (32 * j < a.key_pad ? 32 * j : 0) + 8 * g;
+    const int64_t head_at = (int64_t)(h / (a.heads / a.kv_heads)) * a.block_size * a.key_pad;
+    PageWalk walk(a, b);
+    bf16x8_t kf[2][KS];
+    auto fetch = [&]() {
+        const __bf16* src = a.keys + walk.next(a) * kStep * a.key_pad + head_at;
+#pragma unroll
+        for (int x = 0; x < 2; ++x)
+#pragma unroll
+            for (int j = 0; j < KS; ++j) kf[x][j] = *reinterpret_cast<const bf16x8_t*>(src + k_off[x][j]);
+    };
+    fetch();
+    for (int s = 0; s < steps; ++s) {
+        f32x4_t sc[U][2];
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+            for (int x = 0; x < 2; ++x) sc[u][x] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j = 0; j < KS; ++j)
+#pragma unroll
+            for (int x = 0; x < 2; ++x)
+#pragma unroll
+                for (int u = 0; u < U; ++u) sc[u][x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[x][j], q[u][j], sc[u][x], 0, 0, 0);
+        if (s + 1 < steps) fetch();
+        const int tok0 = s * kStep;
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            float sv[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) sv[i] = sc[u][i >> 2][i & 3];
+            if (tok0 + kStep - 1 > q0 + 16 * u + shift) {        // the earliest query of the tile does not see all of it
+                const int rel = limit[u] - tok0 - 8 * g;
+#pragma unroll
+                for (int i = 0; i < 8; ++i)
+                    if (i > rel) sv[i] = -INFINITY;
+            }
+            float mx = sv[0];
+#pragma unroll
+            for (int i = 1; i < 8; ++i) mx = fmaxf(mx, sv[i]);
+            mx *= a.scale_log2;
+            const bool grow = mx > m[u] + kLazy;
+            if (__any(grow)) {
+                l[u] *= grow ? __builtin_amdgcn_exp2f(m[u] - mx) : 1.f;
+                m[u] = grow ? mx : m[u];
+            }
+            float sum = 0.f;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) sum += __builtin_amdgcn_exp2f(__builtin_fmaf(sv[i], a.scale_log2, -m[u]));
+            l[u] += sum;
+        }
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+#pragma unroll
+        for (int x = 16; x <= 32; x *= 2) {
+            const float m2 = __shfl_xor(m[u], x, 64), l2 = __shfl_xor(l[u], x, 64), top = fmaxf(m[u], m2);
+            l[u] = l[u] * exp2f(m[u] - top) + l2 * exp2f(m2 - top);
+            m[u] = top;
+        }
+        const float top = fmaxf(m[u], 0.f);
+        if (g == 0 && q0 + 16 * u + n < sq)
+            a.lse[(int64_t)h * a.tokens + q_beg + q0 + 16 * u + n] = top + log2f(l[u] * exp2f(m[u] - top) + exp2f(-top));
+    }
+}
+
+// byte addresses of LDS records that lanes reach with a stride of 128 and more
+__device__ __forceinline__ int spread(int addr) { return addr ^ (((addr >> 7) & 7) << 4); }
+
+template <int KS, int VT, int UH, int QT, bool SHARE>
+__global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefillArgs a) {
+    constexpr int HP = kMixWaves * UH, Q = 16 * QT;              // head slots, queries
+    constexpr int kRec = 4 * HP;                                 // bytes of a record: every head's weight in two pieces
+    constexpr int KP = UH == 4 ? 2 : 1, RT = UH == 4 ? 2 : 1;    // k-steps and head tiles of the mixture
+    constexpr int kVRow = 32 * VT, kVBuf = kStep * kVRow;        // bytes of a value; units of 32 bytes are permuted by row
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
+    unsigned char* wbuf = lds;                                   // [Q][32 keys][kRec]
+    unsigned char* pbuf = wbuf + Q * kStep * kRec;               // [Q][HP][32 keys] bf16
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, n = lane & 15;
+    unsigned char* vbuf = pbuf + Q * HP * 2 * kStep + wave * kVBuf;
+    const unsigned wg = a.nseq >= 8 ? unit_of(blockIdx.x, gridDim.x) : blockIdx.x;
+    const int qblk = a.qblocks - 1 - (int)(wg % a.qblocks), b = (int)(wg / a.qblocks);
+    const int q_beg = a.cu_q[b], sq = a.cu_q[b + 1] - q_beg, sk = a.cu_k[b + 1] - a.cu_k[b], shift = sk - sq;
+    const int q0 = qblk * Q;
+    if (q0 >= sq) return;
+    const int last_q = q0 + Q < sq ? q0 + Q - 1 : sq - 1, steps = (last_q + shift) / kStep + 1;
+    const int group = a.heads / a.kv_heads;
+    const bool live = wave * UH < a.heads;                       // slots of wavefronts without heads stay zero
+
+    bf16x8_t q[UH][QT][KS];
+    float lse[UH][QT];
+    int limit[QT], hd[UH];
+    int64_t k_head[UH], v_head[UH];
+#pragma unroll
+    for (int u = 0; u < UH; ++u) {
+        hd[u] = wave * UH + u < a.heads ? wave * UH + u : a.heads - 1;       // a surplus slot repeats the last head and meets zeros in T
+        k_head[u] = (int64_t)(hd[u] / group) * a.block_size * a.key_pad;
+        v_head[u] = (int64_t)(hd[u] / group) * a.block_size * a.vdim_pad;
+#pragma unroll
+        for (int t = 0; t < QT; ++t) {
+            const int qi = q0 + 16 * t + n < sq ? q0 + 16 * t + n : sq - 1;
+            limit[t] = qi + shift;
+            lse[u][t] = a.lse[(int64_t)hd[u] * a.tokens + q_beg + qi];
+            const __bf16* qp = a.q + (int64_t)(q_beg + qi) * a.q_stride + (int64_t)hd[u] * a.dim + 8 * g;
+#pragma unroll
+            for (int j = 0; j < KS; ++j) {
+                q[u][t][j] = bf16x8_t{};
+                if (32 * j + 8 * g < a.dim) q[u][t][j] = *reinterpret_cast<const bf16x8_t*>(qp + 32 * j);
+            }
+        }
+    }
+    // T^T: entry i of lane (g, n) is column (head) 16 s + 4 g + i / 2 of row (head) 16 r + n, once for either piece
+    bf16x8_t talk[KP][RT];
+#pragma unroll
+    for (int s = 0; s < KP; ++s)
+#pragma unroll
+        for (int r = 0; r < RT; ++r)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                const int from = 16 * s + 4 * g + i / 2, to = 16 * r + n;
+                talk[s][r][i] = from < HP && from < a.heads && to < a.heads ? a.talk[(int64_t)to * a.heads + from] : (__bf16)0.f;
+            }
+    for (int i = tid; i < Q * kStep * kRec / 16; i += 64 * kMixWaves) reinterpret_cast<u32x4_t*>(wbuf)[i] = u32x4_t{0u, 0u, 0u, 0u};
+
+    const int k_row = (8 * (n >> 2) + (n & 3)) * a.key_pad + 8 * g;
+    int k_step[KS];
+#pragma unroll
+    for (int j = 0; j < KS; ++j) k_step[j] = 32 * j < a.key_pad ? 32 * j : 0;            // surplus steps meet zeros in q
+    // chunk i of this lane: 16 bytes of a value row; surplus ones repeat the tile's last
+    const int per_row = a.vdim_pad / 8, chunks = kStep * per_row;
+    int c_row[VT], c_col[VT];
+#pragma unroll
+    for (int i = 0; i < VT; ++i) {
+        const int c = lane + 64 * i < chunks ? lane + 64 * i : chunks - 1;
+        c_row[i] = c / per_row;
+        c_col[i] = c - c_row[i] * per_row;
+    }
+    auto v_place = [&](int row, int byte) { return row * kVRow + (byte ^ ((row & (VT - 1)) * 32)); };
+
+    f32x4_t acc[UH][QT][VT];
+#pragma unroll
+    for (int u = 0; u < UH; ++u)
+#pragma unroll
+        for (int t = 0; t < QT; ++t)
+#pragma unroll
+            for (int v = 0; v < VT; ++v) acc[u][t][v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+
+    PageWalk walk(a, b);
+    bf16x8_t kf[2][KS];
+    u32x4_t vreg[VT];
+    auto fetch_k = [&](int64_t tile, int u) {
+        const __bf16* src = a.keys + tile * kStep * a.key_pad + k_head[u] + k_row;
+#pragma unroll
+        for (int x = 0; x < 2; ++x)
+#pragma unroll
+            for (int j = 0; j < KS; ++j) kf[x][j] = *reinterpret_cast<const bf16x8_t*>(src + 4 * x * a.key_pad + k_step[j]);
+    };
+    auto fetch_v = [&](int64_t tile, int u, int last) {          // values behind the last one repeat it; their weights are zero
+        const __bf16* src = a.values + tile * kStep * a.vdim_pad + v_head[u];
+#pragma unroll
+        for (int i = 0; i < VT; ++i) vreg[i] = *reinterpret_cast<const u32x4_t*>(src + (c_row[i] < last ? c_row[i] : last) * a.vdim_pad + 8 * c_col[i]);
+    };
+    int64_t tile = walk.next(a);
+    fetch_k(tile, 0);
+    __syncthreads();                                             // the zero fill
+    for (int s = 0; s < steps; ++s) {
+        const int tok0 = s * kStep, last = sk - 1 - tok0;
+        const int64_t here = tile;
+        if (s + 1 < steps) tile = walk.next(a);
+        if (live) {
+            // ---- scores and weights
+            f32x4_t sc[UH][QT][2];
+#pragma unroll
+            for (int u = 0; u < UH; ++u) {
+#pragma unroll
+                for (int t = 0; t < QT; ++t)
+#pragma unroll
+                    for (int x = 0; x < 2; ++x) sc[u][t][x] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+                if (!SHARE && u > 0) fetch_k(here, u);
+#pragma unroll
+                for (int j = 0; j < KS; ++j)
+#pragma unroll
+                    for (int x = 0; x < 2; ++x)
+#pragma unroll
+                        for (int t = 0; t < QT; ++t) sc[u][t][x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[x][j], q[u][t][j], sc[u][t][x], 0, 0, 0);
+            }
+            fetch_v(here, 0, last);
+            fetch_k(tile, 0);                                    // of the next step; the last one's repeats its own
+#pragma unroll
+            for (int t = 0; t < QT; ++t) {
+                uint32_t w[UH][8];
+#pragma unroll
+                for (int u = 0; u < UH; ++u) {
+                    float p[8];
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) p[i] = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[u][t][i >> 2][i & 3], a.scale_log2, -lse[u][t]));
+                    if (tok0 + kStep - 1 > q0 + 16 * t + shift) {
+                        const int rel = limit[t] - tok0 - 8 * g;
+#pragma unroll
+                        for (int i = 0; i < 8; ++i)
+                            if (i > rel) p[i] = 0.f;
+                    }
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) w[u][i] = round_pack(head(p[i]), p[i] - head(p[i]));
+                }
+#pragma unroll
+                for (int i = 0; i < 8; ++i) {
+                    unsigned char* to = wbuf + spread(((16 * t + n) * kStep + 8 * g + i) * kRec + wave * UH * 4);
+                    if constexpr (UH == 4) *reinterpret_cast<u32x4_t*>(to) = u32x4_t{w[0][i], w[1][i], w[2][i], w[3][i]};
+                    else if constexpr (UH == 2) *reinterpret_cast<u32x2_t*>(to) = u32x2_t{w[0][i], w[1][i]};
+                    else *reinterpret_cast<uint32_t*>(to) = w[0][i];
+                }
+            }
+        }
+        __syncthreads();
+        // ---- the mixture, for queries 2 QT wave and on
+#pragma unroll
+        for (int k = 0; k < 2 * QT; ++k) {
+            const int qi = 2 * QT * wave + k;
+            f32x4_t mixed[RT][2];
+#pragma unroll
+            for (int x = 0; x < 2; ++x) {
+#pragma unroll
+                for (int r = 0; r < RT; ++r) mixed[r][x] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+                const int rec = (qi * kStep + 8 * (n >> 2) + 4 * x + (n & 3)) * kRec;
+#pragma unroll
+                for (int y = 0; y < KP; ++y) {
+                    const bf16x8_t wf = *reinterpret_cast<const bf16x8_t*>(wbuf + spread(rec + 64 * y + 16 * (UH == 1 ? g & 1 : g)));
+#pragma unroll
+                    for (int r = 0; r < RT; ++r) mixed[r][x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, talk[y][r], mixed[r][x], 0, 0, 0);
+                }
+            }
+#pragma unroll
+            for (int r = 0; r < RT; ++r) {
+                bf16x8_t p;
+#pragma unroll
+                for (int i = 0; i < 8; ++i) p[i] = (__bf16)mixed[r][i >> 2][i & 3];
+                const int to = 16 * r + n;
+                if (HP >= 16 || to < HP) *reinterpret_cast<bf16x8_t*>(pbuf + (qi * HP + (to ^ (qi & (HP - 1)))) * 64 + 16 * g) = p;
+            }
+        }
+        __syncthreads();
+        // ---- weighted sum of the values
+        if (live) {
+#pragma unroll
+            for (int u = 0; u < UH; ++u) {
+                if (!SHARE || u == 0) {
+#pragma unroll
+                    for (int i = 0; i < VT; ++i) *reinterpret_cast<u32x4_t*>(vbuf + v_place(c_row[i], 16 * c_col[i])) = vreg[i];
+                    // a wavefront's own LDS operations happen in order; the compiler has to keep them so
+                    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+                    __builtin_amdgcn_wave_barrier();
+                    if (!SHARE && u + 1 < UH) fetch_v(here, u + 1, last);
+                }
+                bf16x8_t pb[SHARE ? UH : 1][QT];
+                if (!SHARE || u == 0)
+#pragma unroll
+                    for (int w = 0; w < (SHARE ? UH : 1); ++w)
+#pragma unroll
+                        for (int t = 0; t < QT; ++t) {
+                            const int qi = 16 * t + n, slot = wave * UH + (SHARE ? w : u);
+                            pb[w][t] = *reinterpret_cast<const bf16x8_t*>(pbuf + (qi * HP + (slot ^ (qi & (HP - 1)))) * 64 + 16 * g);
+                        }
+                if (SHARE && u > 0) continue;
+#pragma unroll
+                for (int v = 0; v < VT; ++v) {
+                    const int row = 8 * g + (n >> 2), at = 32 * v + (n & 3) * 8;
+                    const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vbuf + v_place(row, at)));
+                    const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vbuf + v_place(row + 4, at)));
+                    const bf16x8_t vt = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+#pragma unroll
+                    for (int w = 0; w < (SHARE ? UH : 1); ++w)
+#pragma unroll
+                        for (int t = 0; t < QT; ++t) {
+                            f32x4_t& o = acc[SHARE ? w : u][t][v];
+                            o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pb[w][t], o, 0, 0, 0);
+                        }
+                }
+                __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+                __builtin_amdgcn_wave_barrier();
+            }
+        }
+    }
+    if (!live) return;
+#pragma unroll
+    for (int u = 0; u < UH; ++u) {
+        if (wave * UH + u >= a.heads) continue;
+#pragma unroll
+        for (int t = 0; t < QT; ++t) {
+            const int qi = q0 + 16 * t + n;
+            if (qi >= sq) continue;
+            __bf16* o = a.out + (int64_t)(q_beg + qi) * a.out_stride + (int64_t)hd[u] * a.vdim + 4 * g;
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                if (16 * v + 4 * g >= a.vdim) continue;
+                bf16x4_t x;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[e] = (__bf16)(acc[u][t][v][e] * a.out_scale);
+                *reinterpret_cast<bf16x4_t*>(o + 16 * v) = x;
+            }
+        }
+    }
+}
+
+template <int KS>
+int launch_lse(TalkPrefillArgs a, int64_t max_seqlen_q, hipStream_t st) {
+    const int64_t per = kLseQ * kLseWaves, qblocks = (max_seqlen_q + per - 1) / per, total = qblocks * a.nseq * a.heads;
+    if (total > 0x7fffffff) return INFER_KV_EINVAL;
+    a.qblocks = (int)qblocks;
+    hipLaunchKernelGGL((talk_lse_kernel<KS>), dim3((unsigned)total), dim3(64 * kLseWaves), 0, st, a);
+    return (int)hipGetLastError();
+}
+
+template <int KS, int VT, int UH, int QT, bool SHARE>
+int launch_mix(TalkPrefillArgs a, int64_t max_seqlen_q, hipStream_t st) {
+    const int64_t qblocks = (max_seqlen_q + 16 * QT - 1) / (16 * QT), total = qblocks * a.nseq;
+    if (total > 0x7fffffff) return INFER_KV_EINVAL;
+    a.qblocks = (int)qblocks;
+    auto kernel = &talk_mix_kernel<KS, VT, UH, QT, SHARE>;
+    constexpr size_t lds = (size_t)16 * QT * kStep * kMixWaves * UH * (4 + 2) + (size_t)kMixWaves * kStep * 32 * VT;
+    static_assert(lds <= 160 * 1024, "LDS of a compute unit");
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return (int)e;
+    hipLaunchKernelGGL(kernel, dim3((unsigned)total), dim3(64 * kMixWaves), lds, st, a);
+    return (int)hipGetLastError();
+}
+
+template <int KS, int VT>
+int launch(const TalkPrefillArgs& a, int64_t max_seqlen_q, hipStream_t st) {
+    const int rc = launch_lse<KS>(a, max_seqlen_q, st);
+    if (rc) return rc;
+    const int group = a.heads / a.kv_heads;
+    if (a.heads <= 8) return launch_mix<KS, VT, 1, 2, true>(a, max_seqlen_q, st);
+    if (a.heads <= 16) return group % 2 == 0 ? launch_mix<KS, VT, 2, 1, true>(a, max_seqlen_q, st) : launch_mix<KS, VT, 2, 1, false>(a, max_seqlen_q, st);
+    return group % 4 == 0 ? launch_mix<KS, VT, 4, 1, true>(a, max_seqlen_q, st) : launch_mix<KS, VT, 4, 1, false>(a, max_seqlen_q, st);
+}
+
+}  // namespace
+
+// 1 if the sizes are served
+extern "C" int infer_talking_prefill_supported(int64_t heads, int64_t dim, int64_t vdim, int64_t block_size) {
+    return heads >= 1 && heads <= 32 && dim >= 8 && dim <= 128 && dim % 8 == 0 && vdim >= 8 && vdim <= 128 && vdim % 8 == 0 && block_size >= kStep &&
+           block_size % kStep == 0;
+}
+
 extern "C" int infer_talking_prefill(const void* q, int64_t q_stride, const void* keys, const void* values, int64_t key_pad,
-                          int64_t vdim_pad, const int32_t* block_table, int64_t bt_stride, int64_t table_cols,
-                          int64_t block_size, int64_t num_blocks, const int32_t* seqs, const int32_t* cu_q,
-                          const int32_t* cu_k, int64_t num_seqs, int64_t tokens, int64_t max_seqlen_q, int64_t heads,
-                          int64_t kv_heads, int64_t dim, int64_t vdim, float scale, const void* talk, float out_scale,
-                          void* out, int64_t out_stride, float* workspace, int64_t workspace_floats, void* stream) { return -1; }
+                                     int64_t vdim_pad, const int32_t* block_table, int64_t bt_stride, int64_t table_cols,
+                                     int64_t block_size, int64_t num_blocks, const int32_t* seqs, const int32_t* cu_q,
+                                     const int32_t* cu_k, int64_t num_seqs, int64_t tokens, int64_t max_seqlen_q, int64_t heads,
+                                     int64_t kv_heads, int64_t dim, int64_t vdim, float scale, const void* talk, float out_scale,
+                                     void* out, int64_t out_stride, float* workspace, int64_t workspace_floats, void* stream) {
+    if (!infer_talking_prefill_supported(heads, dim, vdim, block_size)) return INFER_KV_EUNSUPPORTED;
+    if (num_seqs < 0 || max_seqlen_q < 0 || tokens < 0 || num_seqs > 0x7fffffff || max_seqlen_q > 0x7fffffff || max_seqlen_q > tokens) return INFER_KV_EINVAL;
+    if (num_seqs == 0 || max_seqlen_q == 0) return INFER_KV_OK;
+    if (!q || !keys || !values || !block_table || !seqs || !cu_q || !cu_k || !talk || !out || kv_heads < 1 || heads % kv_heads ||
+        q_stride < heads * dim || out_stride < heads * vdim || key_pad != (dim + 31) / 32 * 32 || vdim_pad != (vdim + 31) / 32 * 32 ||
+        block_size > (1 << 20) || table_cols < 1 || table_cols * block_size > 0x7fffffff || bt_stride < table_cols || num_blocks < 1 ||
+        num_blocks > 0x7fffffff || !(scale > 0.f))
+        return INFER_KV_EINVAL;
+    if (q_stride % 8 || out_stride % 4 || !ptr_aligned(q, 16) || !ptr_aligned(keys, 16) || !ptr_aligned(values, 16) || !ptr_aligned(out, 8))
+        return INFER_KV_EALIGN;
+    if (!workspace || workspace_floats < heads * tokens) return INFER_KV_EWORKSPACE;
+    const TalkPrefillArgs a{(const __bf16*)q, q_stride, (const __bf16*)keys, (const __bf16*)values, (int)key_pad, (int)vdim_pad, block_table,
+                            bt_stride, (int)table_cols, (int)block_size, (int)num_blocks, seqs, cu_q, cu_k, (int)heads, (int)kv_heads, (int)dim,
+                            (int)vdim, (int)num_seqs, 0, scale * kLog2e, (const __bf16*)talk, out_scale, (__bf16*)out, out_stride, workspace, tokens};
+    hipStream_t st = (hipStream_t)stream;
+    if (dim <= 64) return vdim <= 64 ? launch<2, 4>(a, max_seqlen_q, st) : launch<2, 8>(a, max_seqlen_q, st);
+    return vdim <= 64 ? launch<4, 4>(a, max_seqlen_q, st) : launch<4, 8>(a, max_seqlen_q, st);
+}
