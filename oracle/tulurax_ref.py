@@ -48,16 +48,16 @@ def apply_weights(weights, v):
     return np.stack([weights[h] @ v[:, h // group] for h in range(heads)], axis=1)
 
 
-def talking_attention(h, m, w, eps):
+def talking_attention(h, m, w, eps, cast=lambda a: a):
     t, heads, kv = len(h), m["heads"], m["kv_heads"]
-    q = rms_norm((h @ w("q").T).reshape(t, heads, m["dim"]), 1.0, eps)
-    k = rms_norm((h @ w("k").T).reshape(t, kv, m["dim"]), 1.0, eps)
-    v = rms_norm((h @ w("v").T).reshape(t, kv, m["vdim"]), 1.0, eps)
+    q = rms_norm(cast(h @ w("q").T).reshape(t, heads, m["dim"]), 1.0, eps)
+    k = cast(rms_norm(cast(h @ w("k").T).reshape(t, kv, m["dim"]), 1.0, eps))
+    v = cast(rms_norm(cast(h @ w("v").T).reshape(t, kv, m["vdim"]), 1.0, eps))
     temp = m.get("q_temp")
     if temp:
         q = q * query_temperature(np.arange(t), temp["coef"], temp["every"])[:, None, None]
-    o = apply_weights(mix_heads(sink_weights(q, k, m["scale"]), w("talk")), v)
-    return o.reshape(t, -1) @ w("o").T
+    o = apply_weights(mix_heads(sink_weights(cast(q), k, m["scale"]), w("talk")), v)
+    return cast(o.reshape(t, -1)) @ w("o").T
 
 
 # ------------------------------------------------------------------ retention
@@ -71,13 +71,13 @@ def retention_scan(q, k, v, decay, state=None):
     return out, s
 
 
-def retention(h, m, w, eps):
+def retention(h, m, w, eps, cast=lambda a: a):
     t, heads, dim, vdim = len(h), m["heads"], m["dim"], m["vdim"]
-    q = (h @ w("q").T).reshape(t, heads, dim)
-    k = (h @ w("k").T).reshape(t, heads, dim) * dim ** -0.5
-    v = (h @ w("v").T).reshape(t, heads, vdim)
+    q = cast(h @ w("q").T).reshape(t, heads, dim)
+    k = cast(h @ w("k").T).reshape(t, heads, dim) * dim ** -0.5
+    v = cast(h @ w("v").T).reshape(t, heads, vdim)
     o = np.stack([retention_scan(q[:, i], k[:, i], v[:, i], m["decay"][i])[0] for i in range(heads)], axis=1)
-    return (rms_norm(o, 1.0, eps).reshape(t, -1) * silu(h @ w("g").T)) @ w("o").T
+    return cast(rms_norm(o, 1.0, eps).reshape(t, -1) * silu(cast(h @ w("g").T))) @ w("o").T
 
 
 # ------------------------------------------------------------------ feed-forward
@@ -86,14 +86,14 @@ def xielu(z, p, q):
     return np.where(z > 0, softplus(p) * z * z, (0.5 + softplus(q)) * (np.expm1(low) - low)) + 0.5 * z
 
 
-def plain_mlp(h, w):
-    return xielu(h @ w("up").T + w("up.b"), *w("act")) @ w("down").T + w("down.b")
+def plain_mlp(h, w, cast=lambda a: a):
+    return cast(xielu(cast(h @ w("up").T) + w("up.b"), *w("act"))) @ w("down").T + w("down.b")
 
 
 # ------------------------------------------------------------------ the model
 def forward(config, weights, tokens, cast=lambda a: a):
     """Logits [tokens, vocab] and the residual stream after every layer [layers, tokens, width].  ``cast`` is applied to what goes
-    into and comes out of every sublayer: with a rounding function it shows what rounding alone does."""
+    into and comes out of every product: with a rounding function it shows what rounding alone does."""
     eps = config["norm"]["eps"]
 
     def norm(x, name):
@@ -104,10 +104,10 @@ def forward(config, weights, tokens, cast=lambda a: a):
     for i, layer in enumerate(config["layers"]):
         name, m = f"l{i}.", layer["mixer"]
         h = cast(norm(x, name + "norm1"))
-        x = x + cast(m["left_scale"] * talking_attention(h, m["left"], lambda key: weights[name + "mix.left." + key], eps)
-                     + m["right_scale"] * retention(h, m["right"], lambda key: weights[name + "mix.right." + key], eps))
+        x = x + cast(m["left_scale"] * talking_attention(h, m["left"], lambda key: weights[name + "mix.left." + key], eps, cast)
+                     + m["right_scale"] * retention(h, m["right"], lambda key: weights[name + "mix.right." + key], eps, cast))
         if layer["mlp"] is not None:
-            x = x + cast(plain_mlp(cast(norm(x, name + "norm2")), lambda key: weights[name + "mlp." + key]))
+            x = x + cast(plain_mlp(cast(norm(x, name + "norm2")), lambda key: weights[name + "mlp." + key], cast))
         stream.append(x)
     logits = cast(norm(x, "final.norm")) @ weights["head"].T * config.get("logit_scale", 1.0)
     cap = config.get("logit_softcap")
