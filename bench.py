@@ -286,6 +286,19 @@ def dogetar_config(size):
                          loop=LayerLoop(2, 2 + runs - layers, 2), logit_softcap=30.0)
 
 
+def tulurax_config(size):
+    """Tulurax of a published model's width: half of the heads talking (8 key heads), half retention, all of 128; a feed-forward without a
+    gate in every layer, so half again as wide to have as many weights as one with a gate."""
+    from infer_amd.config import LayerSpec, TuluraxConfig
+    width, ff, heads, layers = HYBRID_SIZES[size]
+    half = heads // 2
+    mixer = {"left": {"heads": half, "kv_heads": min(half, 8), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "q_temp": {"coef": 0.1, "every": 8192}},
+             "left_scale": 0.7, "right_scale": 0.7,
+             "right": {"heads": half, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-4.0 - 7.0 * h / half) for h in range(half)]}}
+    return TuluraxConfig(vocab_size=151936, hidden_size=width, layers=[LayerSpec("parallel", mixer, ff * 3 // 2, i) for i in range(layers)],
+                         embedding_scale=1.0, logit_scale=1.0, logit_softcap=30.0)
+
+
 def hybrid_engine_point(size, model, batch, prompt, new):
     """Prefill and decode throughput of the engine on ``batch`` prompts of ``prompt`` random tokens."""
     import numpy as np
@@ -296,7 +309,8 @@ def hybrid_engine_point(size, model, batch, prompt, new):
     if model == "qwen3":
         hf = C.ModelConfig(hidden_size=width, intermediate_size=ff, num_hidden_layers=layers, num_attention_heads=heads, num_key_value_heads=8)
     else:
-        hf = {"merilorn": hybrid_config, "vokelix": vokelix_config, "dogetar": dogetar_config}[model](size)
+        hf = {"merilorn": hybrid_config, "vokelix": vokelix_config, "dogetar": dogetar_config,
+              "tulurax": tulurax_config}[model](size)
     blocks = batch * (-(-(prompt + new) // 256) + 1)
     engine = LLMEngine(hf_config=hf, max_num_seqs=max(batch, 16), max_model_len=prompt + new + 1,
                        max_num_batched_tokens=16384, num_kvcache_blocks=blocks, seed=0)
@@ -712,6 +726,117 @@ def dogetar_kernels(heads=32, kv_heads=8, width=4096, ff=12288):
     return out
 
 
+def tulurax_kernels(width=4096, ff=18432):
+    """Every kernel of Tulurax at the sizes of an 8B model's layers, with what bounds it, beside the like kernel of Vokelix (attention,
+    recurrence, residual, activation) or Qwen3 (attention) at the same sizes."""
+    from infer_amd import hybrid_ops as ho, ops, workloads
+    from infer_amd.layers import yarn_rotary_table
+    dev, bf = torch.device("cuda:0"), torch.bfloat16
+    out, rnd, hbm, mfma = roofline_table(dev)
+    d, n, sq, bs, kv_heads = 128, 8, 2048, 256, 8
+    rows = n * sq
+
+    # ---- decode attention
+    for heads in (16, 32):
+        s = ho.TalkShape(heads, kv_heads, d, d, 0.09, 1e-6)
+        talk, sink = rnd(heads, heads), torch.randn(heads, device=dev)
+        for b, seen in ((64, 4096), (64, 1024), (16, 4096)):
+            nblk = b * seen // bs
+            keys, values = rnd(nblk, kv_heads, bs, d), rnd(nblk, kv_heads, bs, d)
+            tables = torch.randperm(nblk, device=dev).to(torch.int32).view(b, -1)
+            lens, o, qx = torch.full((b,), seen, dtype=torch.int32, device=dev), torch.empty((b, heads * d), dtype=bf, device=dev), rnd(b, heads, d)
+            moved = b * seen * kv_heads * 2 * d * 2
+            hbm(f"talking_attention decode, {heads} heads, {b} x {seen}", moved,
+                lambda: ho.talking_attention(s, qx, keys, values, talk, tables, lens, o), "all launches; keys and values")
+            cache = torch.cat((values, keys), -1)
+            hbm(f"vokelix: grouped_attention decode, {heads} heads, {b} x {seen}", moved,
+                lambda: ho.grouped_attention(qx, cache, tables, lens, 0.09, d, o, sink, qx[:, :, 0].contiguous()))
+            del cache, keys, values
+            wl = workloads.make_decode_workload("point", [seen] * b, heads, kv_heads, seed=0, q_scale=d ** -0.5, device=dev, device_fill=True)
+            o3 = torch.empty((b, heads, d), dtype=bf, device=dev)
+            hbm(f"qwen3: paged decode attention, {heads} heads, {b} x {seen}", wl.decode_bytes,
+                lambda: ops.paged_attn_decode(wl.q, wl.k_cache, wl.v_cache, wl.block_table, wl.context_lens, wl.scale, o3))
+            del wl
+
+    # ---- prefill attention
+    triangle = sq * (sq + 1) // 2
+    nblk = rows // bs
+    for m, length in ((8, 2048), (1, 16384), (1, 2048)):
+        t, blocks = m * length, m * length // bs
+        cu = torch.arange(0, m + 1, dtype=torch.int32, device=dev) * length
+        tables = torch.randperm(blocks, device=dev).to(torch.int32).view(m, -1)
+        seqs, pairs = torch.arange(m, dtype=torch.int32, device=dev), m * length * (length + 1) // 2
+        for heads, kv in ((16, 8), (16, 16), (32, 8)) if m == 8 else ((16, 8),):
+            s = ho.TalkShape(heads, kv, d, d, 0.09, 1e-6)
+            talk, q, at = rnd(heads, heads), rnd(t, heads * d), torch.empty((t, heads * d), dtype=bf, device=dev)
+            keys, values = rnd(blocks, kv, bs, d), rnd(blocks, kv, bs, d)
+            mfma(f"talking_prefill, {heads} heads of {kv} keys, {m} x {length}", (4 * heads * d + 2 * heads * heads) * pairs, BF16_PEAK_TFLOPS,
+                 lambda: ho.talking_prefill(s, q, keys, values, talk, tables, seqs, cu, cu, length, at),
+                 "both launches; each product counted once")
+            dense = torch.cat((values, keys), -1).transpose(1, 2).reshape(-1, kv, 2 * d).contiguous()
+            zero, sink = torch.zeros(t, heads, dtype=bf, device=dev), torch.zeros(heads, device=dev)
+            mfma(f"vokelix: grouped_prefill, {heads} heads of {kv} keys, {m} x {length}", 4 * heads * d * pairs, BF16_PEAK_TFLOPS,
+                 lambda: ho.grouped_prefill(q, dense[:, :, d:], dense[:, :, :d], sink, zero, at, cu, cu, length, heads, d, d, 0.09))
+            del dense, zero
+            if heads > kv:
+                q3, k3 = q.view(t, heads, d), rnd(t, kv, d)
+                mfma(f"qwen3: prefill attention, {heads} heads of {kv} keys, {m} x {length}", 4 * heads * d * pairs, BF16_PEAK_TFLOPS,
+                     lambda: ops.flash_attn_varlen_func(q3, k3, k3, max_seqlen_q=length, cu_seqlens_q=cu, max_seqlen_k=length, cu_seqlens_k=cu))
+                del q3, k3
+            del q, at, keys, values
+
+    # ---- front end
+    heads = 16
+    s = ho.TalkShape(heads, kv_heads, d, d, 0.09, 1e-6, True, 0.1, 8192)
+    keys, values, cache = rnd(nblk, kv_heads, bs, d), rnd(nblk, kv_heads, bs, d), rnd(nblk, kv_heads, bs, 2 * d)
+    table, ones = yarn_rotary_table(64, 8192, 1e6, None, dev), torch.ones(heads * d, device=dev)
+    for t in (64, rows):
+        pos, slots = torch.randint(0, 8192, (t,), device=dev), torch.randperm(nblk * bs, device=dev)[:t].to(torch.int32)
+        x, split = rnd(t, (heads + 2 * kv_heads) * d), t if t == 64 else 0
+        qx, moved = rnd(max(split, 1), heads, d), t * 2 * (2 * heads + 4 * kv_heads) * d
+        hbm(f"unit_head_front, {t} rows", moved,
+            lambda: ho.unit_head_front(s, x, [0, heads * d, (heads + kv_heads) * d], pos, slots, keys, values, qx, split))
+        hbm(f"vokelix: grouped_front, {t} rows", moved,
+            lambda: ho.grouped_front(x, heads, kv_heads, d, d, heads * d, (heads + kv_heads) * d, torch.zeros(x.shape[1], device=dev), ones, ones[:kv_heads * d].contiguous(),
+                                     1e-6, table, 64, pos, slots, cache, d, d, qx, split))
+    del keys, values, cache
+
+    # ---- retention, without and with rotation
+    decay = ho.decay_constants([1.0 - 2.0 ** (-4.0 - 7.0 * h / heads) for h in range(heads)], dev)
+    plain, turned = (ho.DecayShape(heads, d, d, 1e-6, False, rot, d ** -0.5, True, True) for rot in (0, d))
+    wide = yarn_rotary_table(d, 16384, 1e4, None, dev)
+    state, gain, off = torch.zeros(64, heads, d, d, device=dev), torch.full((heads * d,), 0.7, device=dev), [i * heads * d for i in range(4)]
+    sl, pos = torch.arange(64, dtype=torch.int32, device=dev), torch.full((64,), 77, dtype=torch.int64, device=dev)
+    x, o2 = rnd(64, 4 * heads * d), torch.empty((64, heads * d), dtype=bf, device=dev)
+    for name, shape, tab, norm in (("", plain, None, gain), ("vokelix: ", turned, wide, None)):
+        hbm(f"{name}decay_attention (retention), one token x 64", 2 * state.numel() * 4 + 5 * 64 * heads * d * 2,
+            lambda: ho.decay_attention(shape, x, off, decay, tab, norm, state, sl, pos, 64, None, 0, o2))
+    for m, length in ((1, 2048), (8, 2048), (1, 16384)):
+        t = m * length
+        x, o2 = rnd(t, 4 * heads * d), torch.empty((t, heads * d), dtype=bf, device=dev)
+        spans = torch.tensor([(i * length, length, i, 0) for i in range(m)], dtype=torch.int32, device=dev)
+        for name, shape, tab, norm in (("", plain, None, gain), ("vokelix: ", turned, wide, None)):
+            hbm(f"{name}decay_attention (retention), {m} x {length}", 5 * t * heads * d * 2,
+                lambda: ho.decay_attention(shape, x, off, decay, tab, norm, state, None, None, 0, spans, length, o2),
+                "all launches; q, k, v, gate, result")
+    del x, state
+
+    # ---- residual stream, activation, logits
+    for t in (64, rows):
+        x32, w32, y = rnd(t, width, dtype=torch.float32), torch.ones(width, device=dev), rnd(t, width)
+        norm = ho.TanhNorm(0.5, w32, w32)
+        hbm(f"tanh_norm with a bias, {t} rows", t * width * 12, lambda: ho.tanh_norm(x32, norm, y=y, bias=w32))
+        hbm(f"vokelix: post_norm, {t} rows", t * width * 12, lambda: ho.post_norm(x32, 1e-6, y=y, w_post=w32, alpha=1.0))
+        up, bias = rnd(t, ff), torch.zeros(ff, device=dev)
+        hbm(f"xielu, {t} rows", t * ff * 4, lambda: ho.xielu(up, bias, 0.8, 1.2))
+        gu = rnd(t, ff // 3 * 4)
+        hbm(f"vokelix: silu_and_mul, {t} rows", t * ff // 3 * 2 * 6, lambda: ho.silu_and_mul(gu))
+        del gu, up, x32
+    logits = rnd(64, 151936)
+    hbm("softcap, 64 rows of 151936", logits.numel() * 6, lambda: ho.softcap(logits, 30.0, 2.0))
+    return out
+
+
 def engine_points(models):
     points = []
     for size, batch, prompt, new in (("0.6b", 64, 1024, 64), ("8b", 64, 1024, 64), ("8b", 16, 4096, 64)):
@@ -738,6 +863,12 @@ def run_dogetar(args):
     """Dogetar beside Qwen3 and Vokelix, as ``run_hybrid``."""
     points = [] if args.hybrid_kernels_only else engine_points(("dogetar", "qwen3", "vokelix"))
     print(json.dumps({"dogetar_engine": points, "dogetar_kernels": dogetar_kernels()}))
+
+
+def run_tulurax(args):
+    """Tulurax beside Qwen3 and Vokelix, as ``run_hybrid``."""
+    points = [] if args.hybrid_kernels_only else engine_points(("tulurax", "qwen3", "vokelix"))
+    print(json.dumps({"tulurax_engine": points, "tulurax_kernels": tulurax_kernels()}))
 
 
 # ------------------------------------------------------------------------------------------ decode curve
@@ -839,7 +970,9 @@ def main():
                     help="Vokelix beside Qwen3 and Merilorn at equal sizes: engine throughput and every kernel, printed as JSON")
     ap.add_argument("--dogetar", action="store_true",
                     help="Dogetar beside Qwen3 and Vokelix at equal sizes: engine throughput and every kernel, printed as JSON")
-    ap.add_argument("--hybrid-kernels-only", action="store_true", help="with --hybrid, --vokelix or --dogetar: the kernels alone")
+    ap.add_argument("--tulurax", action="store_true",
+                    help="Tulurax beside Qwen3 and Vokelix at equal sizes: engine throughput and every kernel, printed as JSON")
+    ap.add_argument("--hybrid-kernels-only", action="store_true", help="with --hybrid, --vokelix, --dogetar or --tulurax: the kernels alone")
     ap.add_argument("--e2e", action="store_true",
                     help="end-to-end decode through the engine (random-init Qwen3, HIP-graph decode) instead "
                          "of the kernel benchmark")
@@ -862,9 +995,10 @@ def main():
     if args.e2e:
         run_e2e(args)
         return
-    if args.hybrid or args.vokelix or args.dogetar:
-        (run_dogetar if args.dogetar else run_vokelix if args.vokelix else run_hybrid)(args)
-        return
+    for chosen, run in ((args.hybrid, run_hybrid), (args.vokelix, run_vokelix), (args.dogetar, run_dogetar), (args.tulurax, run_tulurax)):
+        if chosen:
+            run(args)
+            return
     from infer_amd import ops, workloads
     dev = torch.device("cuda:0")
     if args.decode_curve:
