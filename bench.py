@@ -742,13 +742,13 @@ def tulurax_kernels(width=4096, ff=18432):
         talk, sink = rnd(heads, heads), torch.randn(heads, device=dev)
         for b, seen in ((64, 4096), (64, 1024), (16, 4096)):
             nblk = b * seen // bs
-            keys, values = rnd(nblk, kv_heads, bs, d), rnd(nblk, kv_heads, bs, d)
+            keys, values = rnd(nblk, kv_heads, bs // 32, d // 32, 32, 32), rnd(nblk, kv_heads, bs // 32, d, 32)
             tables = torch.randperm(nblk, device=dev).to(torch.int32).view(b, -1)
             lens, o, qx = torch.full((b,), seen, dtype=torch.int32, device=dev), torch.empty((b, heads * d), dtype=bf, device=dev), rnd(b, heads, d)
             moved = b * seen * kv_heads * 2 * d * 2
             hbm(f"talking_attention decode, {heads} heads, {b} x {seen}", moved,
                 lambda: ho.talking_attention(s, qx, keys, values, talk, tables, lens, o), "all launches; keys and values")
-            cache = torch.cat((values, keys), -1)
+            cache = rnd(nblk, kv_heads, bs, 2 * d)
             hbm(f"vokelix: grouped_attention decode, {heads} heads, {b} x {seen}", moved,
                 lambda: ho.grouped_attention(qx, cache, tables, lens, 0.09, d, o, sink, qx[:, :, 0].contiguous()))
             del cache, keys, values
@@ -769,11 +769,12 @@ def tulurax_kernels(width=4096, ff=18432):
         for heads, kv in ((16, 8), (16, 16), (32, 8)) if m == 8 else ((16, 8),):
             s = ho.TalkShape(heads, kv, d, d, 0.09, 1e-6)
             talk, q, at = rnd(heads, heads), rnd(t, heads * d), torch.empty((t, heads * d), dtype=bf, device=dev)
-            keys, values = rnd(blocks, kv, bs, d), rnd(blocks, kv, bs, d)
+            keys, values = rnd(blocks, kv, bs // 32, d // 32, 32, 32), rnd(blocks, kv, bs // 32, d, 32)
             mfma(f"talking_prefill, {heads} heads of {kv} keys, {m} x {length}", (4 * heads * d + 2 * heads * heads) * pairs, BF16_PEAK_TFLOPS,
-                 lambda: ho.talking_prefill(s, q, keys, values, talk, tables, seqs, cu, cu, length, at),
+                 lambda: ho.talking_prefill(s, q, keys, values, talk, tables, seqs, cu, cu, length, at,
+                                            max_score=s.max_score(length)),
                  "both launches; each product counted once")
-            dense = torch.cat((values, keys), -1).transpose(1, 2).reshape(-1, kv, 2 * d).contiguous()
+            dense = rnd(t, kv, 2 * d)
             zero, sink = torch.zeros(t, heads, dtype=bf, device=dev), torch.zeros(heads, device=dev)
             mfma(f"vokelix: grouped_prefill, {heads} heads of {kv} keys, {m} x {length}", 4 * heads * d * pairs, BF16_PEAK_TFLOPS,
                  lambda: ho.grouped_prefill(q, dense[:, :, d:], dense[:, :, :d], sink, zero, at, cu, cu, length, heads, d, d, 0.09))
@@ -788,10 +789,11 @@ def tulurax_kernels(width=4096, ff=18432):
     # ---- front end
     heads = 16
     s = ho.TalkShape(heads, kv_heads, d, d, 0.09, 1e-6, True, 0.1, 8192)
-    keys, values, cache = rnd(nblk, kv_heads, bs, d), rnd(nblk, kv_heads, bs, d), rnd(nblk, kv_heads, bs, 2 * d)
+    keys, values = rnd(nblk, kv_heads, bs // 32, d // 32, 32, 32), rnd(nblk, kv_heads, bs // 32, d, 32)
+    cache = rnd(nblk, kv_heads, bs, 2 * d)
     table, ones = yarn_rotary_table(64, 8192, 1e6, None, dev), torch.ones(heads * d, device=dev)
     for t in (64, rows):
-        pos, slots = torch.randint(0, 8192, (t,), device=dev), torch.randperm(nblk * bs, device=dev)[:t].to(torch.int32)
+        pos, slots = torch.randint(0, 8192, (t,), device=dev), torch.arange(t, device=dev, dtype=torch.int32)
         x, split = rnd(t, (heads + 2 * kv_heads) * d), t if t == 64 else 0
         qx, moved = rnd(max(split, 1), heads, d), t * 2 * (2 * heads + 4 * kv_heads) * d
         hbm(f"unit_head_front, {t} rows", moved,

@@ -55,20 +55,23 @@ class GroupedPages:
         return torch.zeros(num_blocks, self.kv_heads, block_size, self.row, dtype=self.dtype, device=device)
 
 
-class SplitPages:
-    """A key of ``key_row`` and a value of ``value_row`` elements per token and key/value head, in pages of their own: for kernels that
-    read the one without the other."""
-
-    def __init__(self, kv_heads: int, key_row: int, value_row: int, dtype: torch.dtype):
-        self.kv_heads, self.rows, self.dtype = kv_heads, {"keys": key_row, "values": value_row}, dtype
-
-    def block_bytes(self, block_size: int) -> int:
-        return block_size * self.kv_heads * sum(self.rows.values()) * self.dtype.itemsize
-
+class TilePages:
+    """Keys and values per token and key/value head in pages of their own, in tiles of 32 tokens that matrix operands read as they lie:
+    keys of ``key_row`` entries as ``[tile][key_row / 32][token][32]``, values transposed, ``[tile][value_row][token]``."""
+    TOKENS = 32
     slot_bytes = 0
 
+    def __init__(self, kv_heads: int, key_row: int, value_row: int, dtype: torch.dtype):
+        assert key_row % 32 == value_row % 32 == 0
+        self.kv_heads, self.key_row, self.value_row, self.dtype = kv_heads, key_row, value_row, dtype
+
+    def block_bytes(self, block_size: int) -> int:
+        return block_size * self.kv_heads * (self.key_row + self.value_row) * self.dtype.itemsize
+
     def allocate(self, num_blocks: int, num_slots: int, block_size: int, device):
-        return {name: torch.zeros(num_blocks, self.kv_heads, block_size, row, dtype=self.dtype, device=device) for name, row in self.rows.items()}
+        tiles = (num_blocks, self.kv_heads, block_size // self.TOKENS)
+        return {"keys": torch.zeros(*tiles, self.key_row // 32, self.TOKENS, 32, dtype=self.dtype, device=device),
+                "values": torch.zeros(*tiles, self.value_row, self.TOKENS, dtype=self.dtype, device=device)}
 
 
 class SharedStorage:

@@ -1,12 +1,13 @@
 // Front end of attention with heads of their own norms, for gfx950 (MI355X): per token the biases of the projections, an RMS norm over
 // every head's query and key (with or without a weight) and over its value (without), rotary positions (entry i turns with entry
 // i + half), a factor of the query that grows with the position, and the append of one key and one value per key/value head: to
-// pages of [value | key] rows (row_attention.hip) or to pages of keys and pages of values (talking_attention.hip).
+// pages of [value | key] rows (row_attention.hip) or to pages of tiles (tile_pages.h).
 //
 // A head may have two maps: two queries and two keys beside one value.  Each map is a vector of its own here.  The cached
 // row is [value | key of map 1 | key of map 2], and a query that goes to the row kernels is padded to the length of both keys,
 // with zeros where the other map's key stands.
 #include "elem.h"
+#include "tile_pages.h"
 
 namespace {
 
@@ -21,7 +22,9 @@ struct HeadFrontArgs {
     const float* table; int64_t max_pos;   // [max_pos][half][cos, sin]
     const int64_t* positions;
     const int32_t* slots;
-    T* keys; T* values; int key_row, value_row;              // [blocks][kv_heads][block_size][..]: distance of two tokens' rows
+    T* keys; T* values; int key_row, value_row;              // [blocks][kv_heads][block_size][..]: elements per token
+    bool tiles;                                              // tile_pages.h, or a token's entries one behind the other
+    bool values_apart;                                       // value_tiles_kernel has the values
     int block_size, key_pad, vdim_pad; int64_t num_slots;
     T* qx; int64_t qx_rows;                // rows below qx_rows: q to qx[row][head][map][key_pad], others in place
 };
@@ -44,27 +47,41 @@ template <class T>
 __device__ __forceinline__ Slot<T> slot_of(const HeadFrontArgs<T>& a, int64_t slot) {
     const int64_t kh = (int64_t)a.block_size * a.key_row, vh = (int64_t)a.block_size * a.value_row;
     if (slot < 0 || slot >= a.num_slots) return {nullptr, nullptr, kh, vh};
-    const int64_t block = slot / a.block_size, row = block * a.kv_heads * a.block_size + (slot - block * a.block_size);
-    return {a.keys + row * a.key_row, a.values + row * a.value_row, kh, vh};
+    const int64_t block = slot / a.block_size;
+    const int off = (int)(slot - block * a.block_size), in_tile = a.tiles ? off % kTileTokens : 0;
+    const int64_t row = block * a.kv_heads * a.block_size + off - in_tile;
+    return {a.keys + row * a.key_row + tile_key_entry(in_tile, 0), a.values + row * a.value_row + tile_value_entry(in_tile, 0), kh, vh};
 }
 
-// where vector i (queries first, then keys, then normed values) of a token comes from and goes to; to == nullptr: nowhere
+// where vector i (queries first, then keys, then values unless they are copied as they are) of a token comes from and goes to; to == nullptr: nowhere
 template <class T>
-struct Place { int from, size; T* to; const float* weight; bool norm, rotated; float factor; };
+struct Place {
+    int from, size; T* to; const float* weight; bool norm, rotated; float factor;
+    bool key_tile, value_tile;
+    __device__ __forceinline__ T* at(int d) const { return to + (key_tile ? tile_key_entry(0, d) : value_tile ? tile_value_entry(0, d) : d); }
+    __device__ __forceinline__ void store(int d, const float (&x)[8]) const {
+        if (!value_tile) {
+            store_elems<8>(at(d), x);                        // eight entries are neighbours in a tile, too
+        } else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) *at(d + e) = (T)x[e];
+        }
+    }
+};
 template <class T>
 __device__ __forceinline__ Place<T> place_of(const HeadFrontArgs<T>& a, T* pr, const Slot<T>& s, T* qx, float factor, int i) {
     const int nq = a.heads * a.maps, nk = a.kv_heads * a.maps;
     if (i < nq) {
         const int from = a.q_off + i * a.dim;
-        return {from, a.dim, qx ? qx + (int64_t)i * a.key_pad + i % a.maps * a.dim : pr + from, a.q_norm, a.norm_qk, true, factor};
+        return {from, a.dim, qx ? qx + (int64_t)i * a.key_pad + i % a.maps * a.dim : pr + from, a.q_norm, a.norm_qk, true, factor, false, false};
     }
     i -= nq;
-    if (i < nk) return {a.k_off + i * a.dim, a.dim, s.key ? s.key + i / a.maps * s.key_head + i % a.maps * a.dim : nullptr, a.k_norm, a.norm_qk, true, 1.f};
+    if (i < nk) return {a.k_off + i * a.dim, a.dim, s.key ? s.key + i / a.maps * s.key_head + i % a.maps * a.dim : nullptr, a.k_norm, a.norm_qk, true, 1.f, a.tiles, false};
     i -= nk;
-    return {a.v_off + i * a.vdim, a.vdim, s.value ? s.value + i * s.value_head : nullptr, nullptr, true, false, 1.f};
+    return {a.v_off + i * a.vdim, a.vdim, s.value ? s.value + i * s.value_head : nullptr, nullptr, a.norm_v, false, 1.f, false, a.tiles};
 }
 template <class T>
-__host__ __device__ __forceinline__ int num_vectors(const HeadFrontArgs<T>& a) { return (a.heads + a.kv_heads) * a.maps + (a.norm_v ? a.kv_heads : 0); }
+__host__ __device__ __forceinline__ int num_vectors(const HeadFrontArgs<T>& a) { return (a.heads + a.kv_heads) * a.maps + ((a.norm_v || a.tiles) && !a.values_apart ? a.kv_heads : 0); }
 
 template <class T>
 __device__ __forceinline__ float query_factor(const HeadFrontArgs<T>& a, int64_t pos) {
@@ -74,7 +91,7 @@ __device__ __forceinline__ float query_factor(const HeadFrontArgs<T>& a, int64_t
 // values that are stored as they are
 template <class T, int N>
 __device__ __forceinline__ void copy_values(const HeadFrontArgs<T>& a, const T* pr, const Slot<T>& s) {
-    if (!s.value || a.norm_v) return;
+    if (!s.value || a.norm_v || a.tiles) return;
     for (int i = threadIdx.x; i < a.kv_heads * a.vdim / N; i += 256) {
         float v[N];
         load_biased(a, pr, a.v_off + N * i, v);
@@ -88,8 +105,15 @@ template <class T>
 __device__ __forceinline__ void fill_padding(const HeadFrontArgs<T>& a, const Slot<T>& s, T* qx) {
     const int used = a.maps * a.dim, pad = a.key_pad - used, vpad = a.vdim_pad - a.vdim;
     if (s.key) {
-        for (int i = threadIdx.x; i < a.kv_heads * pad; i += 256) s.key[i / pad * s.key_head + used + i % pad] = (T)0.f;
-        for (int i = threadIdx.x; i < a.kv_heads * vpad; i += 256) s.value[i / vpad * s.value_head + a.vdim + i % vpad] = (T)0.f;
+        for (int i = threadIdx.x; i < a.kv_heads * pad; i += 256) {
+            const int d = used + i % pad;
+            s.key[i / pad * s.key_head + (a.tiles ? tile_key_entry(0, d) : d)] = (T)0.f;
+        }
+        if (!a.values_apart)
+            for (int i = threadIdx.x; i < a.kv_heads * vpad; i += 256) {
+                const int d = a.vdim + i % vpad;
+                s.value[i / vpad * s.value_head + (a.tiles ? tile_value_entry(0, d) : d)] = (T)0.f;
+            }
     }
     if (qx) {
         const int rest = a.key_pad - a.dim;
@@ -139,7 +163,7 @@ __global__ void __launch_bounds__(256) head_front_kernel(HeadFrontArgs<T> a) {
         const int i = tid / LANES + j * (256 / LANES);
         const Place<T> p = place_of(a, pr, slot, qx, factor, i < total ? i : 0);
         const bool in = c < p.size;
-        if (a.norm_qk || a.norm_v) {
+        if (a.norm_qk || a.norm_v) {                              // entries behind the size are zero
             float s = 0.f;
 #pragma unroll
             for (int e = 0; e < 8; ++e) s += x[j][e] * x[j][e];
@@ -165,7 +189,7 @@ __global__ void __launch_bounds__(256) head_front_kernel(HeadFrontArgs<T> a) {
                 if (turned && p.rotated) x[j][e] = x[j][e] * turn[2 * e] + (low ? -y : y) * turn[2 * e + 1];
             }
         }
-        if (in && i < total && p.to) store_elems<8>(p.to + c, x[j]);
+        if (in && i < total && p.to) p.store(c, x[j]);
     }
     fill_padding(a, slot, qx);
 }
@@ -206,14 +230,73 @@ __global__ void __launch_bounds__(256) head_front_any_kernel(HeadFrontArgs<T> a)
                 load_biased(a, pr, p.from + d + a.half, v);
                 v[0] *= p.weight ? r * p.weight[d + a.half] : r;
                 const float co = cs[2 * d], si = cs[2 * d + 1];
-                p.to[d + a.half] = (T)(v[0] * co + u[0] * si);
+                *p.at(d + a.half) = (T)(v[0] * co + u[0] * si);
                 u[0] = u[0] * co - v[0] * si;
             }
-            p.to[at] = (T)u[0];
+            *p.at(at) = (T)u[0];
         }
     }
     copy_values<T, 1>(a, pr, slot);
     fill_padding(a, slot, qx);
+}
+
+// Values of 32 consecutive tokens to tiles, where those of eight neighbouring tokens are one store.  Eight threads per token, NC chunks
+// of eight entries each.
+template <class T, int NC>
+__global__ void __launch_bounds__(256) value_tiles_kernel(HeadFrontArgs<T> a, int64_t n) {
+    constexpr int kRow = 64 * NC + 8;                            // entries of a token in LDS
+    __shared__ __attribute__((aligned(16))) T tile[32 * kRow];
+    __shared__ int64_t slot[32];
+    const int64_t t0 = (int64_t)blockIdx.x * 32;
+    const int tid = threadIdx.x, r = tid / 8, h = blockIdx.y;
+    const bool have = t0 + r < n;
+    const T* pr = a.proj + (t0 + (have ? r : 0)) * a.proj_stride + a.v_off + h * a.vdim;
+    if (tid < 32) {
+        const int64_t s = t0 + tid < n ? a.slots[t0 + tid] : -1;
+        slot[tid] = s < a.num_slots ? s : -1;
+    }
+    float x[NC][8], sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < NC; ++j) {
+        const int c = 8 * (tid % 8) + 64 * j;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[j][e] = 0.f;
+        if (c < a.vdim) load_elems<8>(pr + c, x[j]);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum += x[j][e] * x[j][e];
+    }
+#pragma unroll
+    for (int m = 4; m >= 1; m >>= 1) sum += __shfl_xor(sum, m, 64);
+    const float f = a.norm_v ? rsqrtf(sum / (float)a.vdim + a.eps) : 1.f;
+#pragma unroll
+    for (int j = 0; j < NC; ++j) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[j][e] *= f;
+        store_elems<8>(tile + r * kRow + 8 * (tid % 8) + 64 * j, x[j]);
+    }
+    __syncthreads();
+    // runs of neighbouring tokens that do not leave a group of eight, taken in turn by 256 / vdim_pad sets of threads
+    const int sets = 256 / a.vdim_pad, set = tid / a.vdim_pad, v = tid % a.vdim_pad;
+    if (set >= sets) return;
+    for (int first = 0, run = 0; first < 32; ++run) {
+        const int64_t s = slot[first];
+        int count = 1;
+        while (first + count < 32 && (s + count) % 8 != 0 && slot[first + count] == s + count) ++count;
+        if (s >= 0 && run % sets == set) {
+            const int64_t block = s / a.block_size;
+            const int off = (int)(s - block * a.block_size), in_tile = off % kTileTokens;
+            T* to = a.values + ((block * a.kv_heads + h) * a.block_size + off - in_tile) * a.value_row + tile_value_entry(in_tile, v);
+            if (count == 8) {
+                float y[8];
+#pragma unroll
+                for (int e = 0; e < 8; ++e) y[e] = (float)tile[(first + e) * kRow + v];
+                store_elems<8>(to, y);
+            } else {
+                for (int e = 0; e < count; ++e) to[e] = tile[(first + e) * kRow + v];
+            }
+        }
+        first += count;
+    }
 }
 
 template <class T, int LANES>
@@ -229,12 +312,19 @@ bool launch_vec(const HeadFrontArgs<T>& a, int64_t n, hipStream_t st) {
 }
 
 template <class T>
-int launch(const HeadFrontArgs<T>& a, int64_t n, hipStream_t st) {
+int launch(HeadFrontArgs<T> a, int64_t n, hipStream_t st) {
     const bool vec = a.dim % 8 == 0 && a.vdim % 8 == 0 && a.half % 8 == 0 && a.q_off % 8 == 0 && a.k_off % 8 == 0 && a.v_off % 8 == 0 &&
                      a.proj_stride % 8 == 0 && ptr_aligned(a.proj, 16) && ptr_aligned(a.keys, 16) && ptr_aligned(a.values, 16) && ptr_aligned(a.qx, 16) &&
                      ptr_aligned(a.bias, 16) && ptr_aligned(a.q_norm, 16) && ptr_aligned(a.k_norm, 16) && ptr_aligned(a.table, 16);
     bool done = false;
-    const int longest = a.norm_v && a.vdim > a.dim ? a.vdim : a.dim;
+    if (vec && a.tiles && a.vdim <= 256 && n >= 64 && a.kv_heads <= 65535) {
+        const dim3 grid((unsigned)((n + 31) / 32), (unsigned)a.kv_heads), block(256);
+        if (a.vdim <= 64) hipLaunchKernelGGL((value_tiles_kernel<T, 1>), grid, block, 0, st, a, n);
+        else if (a.vdim <= 128) hipLaunchKernelGGL((value_tiles_kernel<T, 2>), grid, block, 0, st, a, n);
+        else hipLaunchKernelGGL((value_tiles_kernel<T, 4>), grid, block, 0, st, a, n);
+        a.values_apart = true;
+    }
+    const int longest = (a.norm_v || a.tiles) && !a.values_apart && a.vdim > a.dim ? a.vdim : a.dim;
     if (vec) {
         if (longest <= 32) done = launch_vec<T, 4>(a, n, st);
         else if (longest <= 64) done = launch_vec<T, 8>(a, n, st);
@@ -283,7 +373,7 @@ extern "C" int infer_head_front(int elem, void* proj, int64_t proj_stride, int64
         const int row = (int)(key_pad + vdim_pad);
         const HeadFrontArgs<T> a{(T*)proj, proj_stride, (int)q_off, (int)k_off, (int)v_off, (int)heads, (int)kv_heads, (int)maps, (int)dim,
                                  (int)vdim, (int)(rot_dims / 2), bias, q_norm, k_norm, eps, q_norm != nullptr, false, 0.f, 0.0, table, max_pos,
-                                 positions, slots, (T*)cache + vdim_pad, (T*)cache, row, row, (int)block_size, (int)key_pad, (int)vdim_pad,
+                                 positions, slots, (T*)cache + vdim_pad, (T*)cache, row, row, false, false, (int)block_size, (int)key_pad, (int)vdim_pad,
                                  num_slots, (T*)qx, qx_rows};
         return run(a, n, stream);
     };
@@ -297,14 +387,14 @@ extern "C" int infer_unit_head_front(int elem, void* proj, int64_t proj_stride, 
                                      double temp_every, const int64_t* positions, const int32_t* slots, void* keys, void* values,
                                      int64_t block_size, int64_t key_pad, int64_t vdim_pad, int64_t num_slots, void* qx, int64_t qx_rows,
                                      int64_t n, void* stream) {
-    if (n < 0 || !sizes_valid(heads, kv_heads, 1, dim, vdim, q_off, k_off, v_off, 0, block_size, key_pad, vdim_pad) || !(temp_every >= 0.0))
+    if (n < 0 || !sizes_valid(heads, kv_heads, 1, dim, vdim, q_off, k_off, v_off, 0, block_size, key_pad, vdim_pad) || !(temp_every >= 0.0) || block_size % kTileTokens || key_pad % 32 || vdim_pad % 32)
         return INFER_KV_EINVAL;
     if (n == 0) return INFER_KV_OK;
     auto go = [&](auto zero) {
         using T = decltype(zero);
         const HeadFrontArgs<T> a{(T*)proj, proj_stride, (int)q_off, (int)k_off, (int)v_off, (int)heads, (int)kv_heads, 1, (int)dim, (int)vdim, 0,
                                  nullptr, nullptr, nullptr, eps, true, norm_values != 0, temp_coef, temp_every, nullptr, 1, positions, slots,
-                                 (T*)keys, (T*)values, (int)key_pad, (int)vdim_pad, (int)block_size, (int)key_pad, (int)vdim_pad, num_slots,
+                                 (T*)keys, (T*)values, (int)key_pad, (int)vdim_pad, true, false, (int)block_size, (int)key_pad, (int)vdim_pad, num_slots,
                                  (T*)qx, qx_rows};
         return run(a, n, stream);
     };

@@ -1,4 +1,4 @@
-// Attention whose heads mix their softmax weights, query row by query row over pages of keys and pages of values, for gfx950 (MI355X).
+// Attention whose heads mix their softmax weights, query row by query row over pages of tiles (tile_pages.h), for gfx950 (MI355X).
 //
 //     w_h(j) = e^{s_h(j)} / (1 + sum_j' e^{s_h(j')}) ,   o_h = c sum_j (sum_g T[h][g] w_g(j)) v_j
 //
@@ -14,21 +14,18 @@
 //   talk_scores_any_kernel, talk_values_any_kernel   the same for any size and element type
 #include "elem.h"
 #include "pieces.h"
+#include "tile_pages.h"
 
 namespace {
 
-typedef short i16x4 __attribute__((ext_vector_type(4)));
-typedef short i16x8 __attribute__((ext_vector_type(8)));
-typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
-
-constexpr int kTile = 32;
+constexpr int kTile = kTileTokens;
 constexpr int kWaves = 4;
 constexpr float kLow = -1e30f;            // a maximum before any key was seen; finite, since hidden scores are -inf
 
 template <class T>
 struct TalkArgs {
     const T* qx;                          // [rows][heads][key_pad]
-    const T* keys; const T* values;       // [blocks][kv_heads][block_size][key_pad], .. [vdim_pad]
+    const T* keys; const T* values;       // [blocks][kv_heads][tiles of block_size tokens], key_pad and vdim_pad entries per token
     int key_pad, vdim_pad;
     const int32_t* bt; int64_t bt_stride; int table_cols, block_size, num_blocks;
     const int32_t* row_seq;               // block-table row of each query row; nullptr: the query row itself
@@ -78,6 +75,13 @@ __device__ __forceinline__ float log_denominator(const TalkArgs<T>& a, int row, 
     for (int s = 0; s < used; ++s) sum += ml[s * next + 1] * exp2f(ml[s * next] - m);
     return m + log2f(sum);
 }
+// where the tile of a key begins, in tokens of all blocks of one head; the key's place in it
+template <class T>
+__device__ __forceinline__ int64_t tile_of(const TalkArgs<T>& a, const int32_t* bt, int kvh, int key, int& token) {
+    const int col = key / a.block_size, off = key - col * a.block_size;
+    token = off % kTile;
+    return ((int64_t)block_id(a, bt, col) * a.kv_heads + kvh) * a.block_size + off - token;
+}
 __device__ __forceinline__ void join_max_sum(float& m, float& l, float m2, float l2) {
     const float top = fmaxf(m, m2);
     l = l * exp2f(m - top) + l2 * exp2f(m2 - top);
@@ -99,12 +103,12 @@ __global__ void __launch_bounds__(256) talk_scores_any_kernel(TalkArgs<T> a) {
     for (int i = 0; i < NC; ++i) q[i] = lane + 64 * i < a.key_pad ? (float)qr[lane + 64 * i] * a.scale_log2 : 0.f;
     float m = kLow, l = 0.f;
     for (int key = wave; key < len; key += kWaves) {
-        const int col = key / a.block_size;
-        const T* kr = a.keys + (((int64_t)block_id(a, bt, col) * a.kv_heads + kvh) * a.block_size + (key - col * a.block_size)) * a.key_pad;
+        int token;
+        const T* kr = a.keys + tile_of(a, bt, kvh, key, token) * a.key_pad;
         float s = 0.f;
 #pragma unroll
         for (int i = 0; i < NC; ++i)
-            if (lane + 64 * i < a.key_pad) s += q[i] * (float)kr[lane + 64 * i];
+            if (lane + 64 * i < a.key_pad) s += q[i] * (float)kr[tile_key_entry(token, lane + 64 * i)];
         s = wave_sum(s);
         if (lane == 0) out[key] = s;
         join_max_sum(m, l, s, 1.f);
@@ -150,11 +154,11 @@ __global__ void __launch_bounds__(256) talk_values_any_kernel(TalkArgs<T> a, int
         __syncthreads();
         const int count = len - k0 < 256 ? len - k0 : 256;
         for (int k = part; k < count; k += parts) {
-            const int key = k0 + k, col = key / a.block_size;
-            const T* vr = a.values + (((int64_t)block_id(a, bt, col) * a.kv_heads + kvh) * a.block_size + (key - col * a.block_size)) * a.vdim_pad;
+            int token;
+            const T* vr = a.values + tile_of(a, bt, kvh, k0 + k, token) * a.vdim_pad;
 #pragma unroll
             for (int i = 0; i < COLS; ++i)
-                if (c + lanes * i < a.vdim) o[i] += p[k] * (float)vr[c + lanes * i];
+                if (c + lanes * i < a.vdim) o[i] += p[k] * (float)vr[tile_value_entry(token, c + lanes * i)];
         }
     }
 #pragma unroll
@@ -235,22 +239,20 @@ __global__ void __launch_bounds__(256) talk_scores_kernel(TalkArgs<__bf16> a) {
             if (32 * j < a.key_pad) q[i][j] = *reinterpret_cast<const bf16x8_t*>(a.qx + at * a.key_pad + 32 * j + 8 * g);
         }
     }
-    int k_off[2][KS];                                 // k-steps behind the size repeat the first one, which meets zeros
+    int k_step[KS];                                   // k-steps behind the size repeat the first one, which meets zeros
 #pragma unroll
-    for (int x = 0; x < 2; ++x)
-#pragma unroll
-        for (int j = 0; j < KS; ++j) k_off[x][j] = (16 * x + n) * a.key_pad + (32 * j < a.key_pad ? 32 * j : 0) + 8 * g;
+    for (int j = 0; j < KS; ++j) k_step[j] = tile_key_entry(0, 32 * j < a.key_pad ? 32 * j : 0);
     float m[MT], l[MT];
 #pragma unroll
     for (int i = 0; i < MT; ++i) { m[i] = kLow; l[i] = 0.f; }
     bf16x8_t kf[2][KS];
     TileWalk walk(a, bt, u.t0 + wave);
     auto fetch = [&]() {
-        const __bf16* src = a.keys + walk.next(a, bt, u.kvh) * kTile * a.key_pad;
+        const __bf16* src = a.keys + walk.next(a, bt, u.kvh) * kTile * a.key_pad + tile_key_entry(n, 8 * g);
 #pragma unroll
         for (int x = 0; x < 2; ++x)
 #pragma unroll
-            for (int j = 0; j < KS; ++j) kf[x][j] = *reinterpret_cast<const bf16x8_t*>(src + k_off[x][j]);
+            for (int j = 0; j < KS; ++j) kf[x][j] = *reinterpret_cast<const bf16x8_t*>(src + k_step[j] + tile_key_entry(16 * x, 0));
     };
     if (u.t0 + wave < u.t1) fetch();
     for (int t = u.t0 + wave; t < u.t1; t += kWaves) {
@@ -305,22 +307,45 @@ __global__ void __launch_bounds__(256) talk_scores_kernel(TalkArgs<__bf16> a) {
     }
 }
 
-__host__ __device__ constexpr int value_pitch(int nt) { return 32 * nt + 16; }      // bytes of a value in LDS
-
-// Every wavefront has tiles of its own:
+// Every wavefront has tiles of its own and reads their values straight into operands:
 //   P'^T[key, head] = W^T[key, g] . T^T[g, head]     weights of all heads g as two bf16 pieces each (2^-17), KH k-steps of 32 heads
-//   O^T[v, head]   += V^T[v, key] . P'^T[key, head]  values transposed by LDS, in a buffer of the wavefront's own
+//   O^T[v, head]   += V^T[v, key] . P'^T[key, head]
 // Row r of tile x of the first product is key 8 (r / 4) + 4 x + r % 4, so that a lane's eight results are the eight consecutive keys
 // that the second product wants from it.
 template <int MT, int KH, int NT>
 __global__ void __launch_bounds__(256) talk_values_kernel(TalkArgs<__bf16> a) {
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
     __shared__ float lse[32 * KH];
-    constexpr int kPitch = value_pitch(NT);
     const Unit<MT> u(a);
     if (!u.exists || (u.t0 >= u.t1 && (a.splits > 1 || u.len > 0))) return;       // the merge knows which splits are empty
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, n = lane & 15;
     const int32_t* bt = table_of(a, u.row);
+    int v_tile[NT];                                   // value tiles behind the size repeat the first one and are not stored
+#pragma unroll
+    for (int v = 0; v < NT; ++v) v_tile[v] = tile_value_entry(0, 16 * v < a.vdim_pad ? 16 * v : 0);
+    bf16x8_t vf[NT];
+    float sreg[KH][2][8];
+    const float* src_s[KH][8];
+#pragma unroll
+    for (int s = 0; s < KH; ++s)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const int from = 32 * s + 8 * g + e;
+            src_s[s][e] = a.scores + ((int64_t)u.row * a.heads + (from < a.heads ? from : a.heads - 1)) * a.key_cap + 8 * (n >> 2) + (n & 3);
+        }
+    TileWalk walk(a, bt, u.t0 + wave);
+    auto fetch = [&](int t) {
+        const __bf16* src = a.values + walk.next(a, bt, u.kvh) * kTile * a.vdim_pad + tile_value_entry(8 * g, n);
+#pragma unroll
+        for (int s = 0; s < KH; ++s)
+#pragma unroll
+            for (int x = 0; x < 2; ++x)
+#pragma unroll
+                for (int e = 0; e < 8; ++e) sreg[s][x][e] = src_s[s][e][(int64_t)t * kTile + 4 * x];
+#pragma unroll
+        for (int v = 0; v < NT; ++v) vf[v] = *reinterpret_cast<const bf16x8_t*>(src + v_tile[v]);
+    };
+    if (u.t0 + wave < u.t1) fetch(u.t0 + wave);
     const int used = used_splits(a, u.len);
     if (tid < 32 * KH) lse[tid] = tid < a.heads ? log_denominator(a, u.row, tid, used) : INFINITY;     // no such head: weight zero
     bf16x8_t tf[MT][KH];
@@ -335,52 +360,18 @@ __global__ void __launch_bounds__(256) talk_values_kernel(TalkArgs<__bf16> a) {
             }
     __syncthreads();
     float den[KH][8];
-    const float* src_s[KH][8];
 #pragma unroll
     for (int s = 0; s < KH; ++s)
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-            const int from = 32 * s + 8 * g + e;
-            den[s][e] = lse[from];
-            src_s[s][e] = a.scores + ((int64_t)u.row * a.heads + (from < a.heads ? from : a.heads - 1)) * a.key_cap + 8 * (n >> 2) + (n & 3);
-        }
-    // chunk i of this lane: 16 bytes of a value row; surplus ones repeat the tile's last
-    unsigned char* buf = lds + wave * kTile * kPitch;
-    const int per_row = a.vdim_pad / 8, chunks = kTile * per_row;
-    int c_row[NT], c_col[NT];
-#pragma unroll
-    for (int i = 0; i < NT; ++i) {
-        const int c = lane + 64 * i < chunks ? lane + 64 * i : chunks - 1;
-        c_row[i] = c / per_row;
-        c_col[i] = c - c_row[i] * per_row;
-    }
-    u32x4_t vreg[NT];
-    float sreg[KH][2][8];
-    TileWalk walk(a, bt, u.t0 + wave);
-    auto fetch = [&](int t) {
-        const int last = u.len - 1 - t * kTile;       // values behind the last one repeat it; their weights are zero
-        const __bf16* src = a.values + walk.next(a, bt, u.kvh) * kTile * a.vdim_pad;
-#pragma unroll
-        for (int i = 0; i < NT; ++i)
-            vreg[i] = *reinterpret_cast<const u32x4_t*>(src + (c_row[i] < last ? c_row[i] : last) * a.vdim_pad + 8 * c_col[i]);
-#pragma unroll
-        for (int s = 0; s < KH; ++s)
-#pragma unroll
-            for (int x = 0; x < 2; ++x)
-#pragma unroll
-                for (int e = 0; e < 8; ++e) sreg[s][x][e] = src_s[s][e][(int64_t)t * kTile + 4 * x];
-    };
+        for (int e = 0; e < 8; ++e) den[s][e] = lse[32 * s + 8 * g + e];
     f32x4_t acc[MT][NT];
 #pragma unroll
     for (int i = 0; i < MT; ++i)
 #pragma unroll
         for (int v = 0; v < NT; ++v) acc[i][v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    if (u.t0 + wave < u.t1) fetch(u.t0 + wave);
     for (int t = u.t0 + wave; t < u.t1; t += kWaves) {
-#pragma unroll
-        for (int i = 0; i < NT; ++i) *reinterpret_cast<u32x4_t*>(buf + c_row[i] * kPitch + 16 * c_col[i]) = vreg[i];
         f32x4_t mixed[MT][2];
-        const int left = u.len - t * kTile - 8 * (n >> 2) - (n & 3);
+        const int left = u.len - t * kTile;
 #pragma unroll
         for (int x = 0; x < 2; ++x) {
 #pragma unroll
@@ -389,7 +380,8 @@ __global__ void __launch_bounds__(256) talk_values_kernel(TalkArgs<__bf16> a) {
             for (int s = 0; s < KH; ++s) {
                 float w[8];
 #pragma unroll
-                for (int e = 0; e < 8; ++e) w[e] = 4 * x < left ? __builtin_amdgcn_exp2f(sreg[s][x][e] - den[s][e]) : 0.f;
+                for (int e = 0; e < 8; ++e)
+                    w[e] = 8 * (n >> 2) + 4 * x + (n & 3) < left ? __builtin_amdgcn_exp2f(sreg[s][x][e] - den[s][e]) : 0.f;
                 bf16x8_t wf[2];
                 split_frags<2>(w, wf);
 #pragma unroll
@@ -398,26 +390,22 @@ __global__ void __launch_bounds__(256) talk_values_kernel(TalkArgs<__bf16> a) {
                     for (int k = 1; k >= 0; --k) mixed[i][x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[k], tf[i][s], mixed[i][x], 0, 0, 0);
             }
         }
-        if (t + kWaves < u.t1) fetch(t + kWaves);
         bf16x8_t pb[MT];
 #pragma unroll
         for (int i = 0; i < MT; ++i)
 #pragma unroll
             for (int e = 0; e < 8; ++e) pb[i][e] = (__bf16)mixed[i][e >> 2][e & 3];
-        // a wavefront's own LDS operations happen in order; the compiler has to keep them so
-        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-        __builtin_amdgcn_wave_barrier();
-        const unsigned char* vr = buf + (8 * g + (n >> 2)) * kPitch + (n & 3) * 8;
+        if (left < kTile)                             // values behind the last one may be anything
 #pragma unroll
-        for (int v = 0; v < NT; ++v) {
-            const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 32 * v));
-            const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 32 * v + 4 * kPitch));
-            const bf16x8_t vt = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+            for (int v = 0; v < NT; ++v)
 #pragma unroll
-            for (int i = 0; i < MT; ++i) acc[i][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pb[i], acc[i][v], 0, 0, 0);
-        }
-        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-        __builtin_amdgcn_wave_barrier();
+                for (int e = 0; e < 8; ++e)
+                    if (8 * g + e >= left) vf[v][e] = (__bf16)0.f;
+#pragma unroll
+        for (int v = 0; v < NT; ++v)
+#pragma unroll
+            for (int i = 0; i < MT; ++i) acc[i][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[v], pb[i], acc[i][v], 0, 0, 0);
+        if (t + kWaves < u.t1) fetch(t + kWaves);
     }
     // ---- the wavefronts' sums, 16 heads at a time; columns behind the size are never stored
     f32x4_t* red = reinterpret_cast<f32x4_t*>(lds);   // [kWaves][NT][64]
@@ -485,7 +473,7 @@ int launch_any(const TalkArgs<T>& a, hipStream_t st) {
 
 template <int MT, int KH, int NT>
 int launch_values(const TalkArgs<__bf16>& a, dim3 grid, hipStream_t st) {
-    const size_t lds = (size_t)kWaves * kTile * value_pitch(NT);       // also holds the final sums
+    const size_t lds = (size_t)kWaves * NT * 64 * sizeof(f32x4_t);     // the wavefronts' sums
     auto kernel = &talk_values_kernel<MT, KH, NT>;
     if (lds > 64 * 1024) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);

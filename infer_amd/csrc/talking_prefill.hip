@@ -1,38 +1,37 @@
 // Attention whose heads mix their softmax weights (talking_attention.hip), for long prompt portions, for gfx950 (MI355X).  bf16 in, float32
-// accumulate, keys and values straight from their pages.
+// accumulate; keys and values go straight from their pages (tile_pages.h) into operands.
 //
 //     w_h(i, j) = e^{s_h(i, j)} / (1 + sum_j' e^{s_h(i, j')}) ,   o_h(i) = c sum_j (sum_g T[h][g] w_g(i, j)) v_j
 //
 // A running rescale does not commute with the mixture, so denominators come first, and the scores are computed twice instead of passing
 // through memory:
-//   talk_lse_kernel   log2 of every (head, query)'s denominator.  A wavefront owns 64 queries of a head and reads keys straight into operands.
+//   talk_lse_kernel   log2 of every (head, query)'s denominator; a wavefront owns 64 queries of a head
 //   talk_mix_kernel   a workgroup of eight wavefronts owns 16 QT queries and ALL heads, UH heads per wavefront, and walks the keys in
 //                     steps of 32:
 //       S^T[key, query] = K[key, :] . q^T           per wavefront its heads; weights e^{S - lse} go to LDS as two bf16 pieces each
 //                                                   (2^-17), one record [head][piece] per (query, key)
 //       P'^T[key, h]    = W^T[key, g] . T^T[g, h]    per wavefront 2 QT queries, the pieces side by side along k; to LDS as bf16
-//       O^T[v, query]  += V^T[v, key] . P'^T[key, query]      per wavefront its heads; values transposed by a buffer of its own in LDS
+//       O^T[v, query]  += V^T[v, key] . P'^T[key, query]      per wavefront its heads
 //                     Nothing is rescaled: what is added up is final.
 // Row r of tile x of the first two products is key 8 (r / 4) + 4 x + r % 4, so that a lane's eight results are eight consecutive keys.
 #include "elem.h"
 #include "pieces.h"
+#include "tile_pages.h"
 
 namespace {
 
-typedef short i16x4 __attribute__((ext_vector_type(4)));
-typedef short i16x8 __attribute__((ext_vector_type(8)));
-typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
 typedef uint32_t u32x2_t __attribute__((ext_vector_type(2)));
 
-constexpr int kStep = 32;
+constexpr int kStep = kTileTokens;
 constexpr int kLseWaves = 4, kLseQ = 64;  // queries per wavefront
 constexpr int kMixWaves = 8;
 constexpr float kLow = -1e30f;            // a maximum before any key was seen; finite, since hidden scores are -inf
 constexpr float kLazy = 8.f;              // log2 units by which a sum's terms may exceed one before it is rescaled
+constexpr float kBound = 100.f;           // log2 units: powers of scores below it add up in a float as they are
 
 struct TalkPrefillArgs {
     const __bf16* q; int64_t q_stride;    // [token][head * dim]
-    const __bf16* keys; const __bf16* values;                 // [blocks][kv_heads][block_size][key_pad], .. [vdim_pad]
+    const __bf16* keys; const __bf16* values;                 // tile_pages.h
     int key_pad, vdim_pad;
     const int32_t* bt; int64_t bt_stride; int table_cols, block_size, num_blocks;
     const int32_t* seqs; const int32_t* cu_q; const int32_t* cu_k;
@@ -72,19 +71,28 @@ struct PageWalk {
     }
 };
 
-// Workgroups go to the eight dies round-robin; die k works through the k-th contiguous eighth of the units.
-__device__ __forceinline__ unsigned unit_of(unsigned id, unsigned total) {
-    const unsigned die = id & 7u, per_die = total >> 3, extra = total & 7u;
-    return die * per_die + (die < extra ? die : extra) + (id >> 3);
+// Workgroups go to the eight dies round-robin.  A die works on its own share of `pairs`, on the late query blocks, which see the most
+// keys, first.  False: no such pair.
+__device__ __forceinline__ bool place_of_block(unsigned id, int pairs, int qblocks, int& pair, int& qblk) {
+    const int die = (int)(id & 7u), i = (int)(id >> 3), per_die = (pairs + 7) / 8;
+    pair = die * per_die + i % per_die;
+    qblk = qblocks - 1 - i / per_die;
+    return pair < pairs;
 }
 
-template <int KS>
+// An operand at an address that all lanes share plus a byte offset of each
+__device__ __forceinline__ bf16x8_t load_operand(const __bf16* base, unsigned lane_bytes) {
+    return *reinterpret_cast<const bf16x8_t*>(reinterpret_cast<const char*>(base) + lane_bytes);
+}
+
+// BOUNDED: all scores are below kBound, so that their powers need no maximum.
+template <int KS, bool BOUNDED>
 __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefillArgs a) {
     constexpr int U = kLseQ / 16;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, n = lane & 15;
-    const unsigned wg = unit_of(blockIdx.x, gridDim.x);
-    const int qblk = a.qblocks - 1 - (int)(wg % a.qblocks);      // late blocks see the most keys: first
-    const int b = (int)((wg / a.qblocks) % a.nseq), h = (int)(wg / ((unsigned)a.qblocks * a.nseq));
+    int pair, qblk;
+    if (!place_of_block(blockIdx.x, a.nseq * a.heads, a.qblocks, pair, qblk)) return;
+    const int b = pair / a.heads, h = pair - b * a.heads;
     const int q_beg = a.cu_q[b], sq = a.cu_q[b + 1] - q_beg, sk = a.cu_k[b + 1] - a.cu_k[b], shift = sk - sq;
     const int q0 = (qblk * kLseWaves + wave) * kLseQ;
     if (q0 >= sq) return;
@@ -96,7 +104,7 @@ __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefill
     for (int u = 0; u < U; ++u) {
         const int qi = q0 + 16 * u + n < sq ? q0 + 16 * u + n : sq - 1;
         limit[u] = qi + shift;
-        m[u] = kLow;
+        m[u] = BOUNDED ? 0.f : kLow;
         l[u] = 0.f;
         const __bf16* qp = a.q + (int64_t)(q_beg + qi) * a.q_stride + (int64_t)h * a.dim + 8 * g;
 #pragma unroll
@@ -105,12 +113,11 @@ __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefill
             if (32 * j + 8 * g < a.dim) q[u][j] = *reinterpret_cast<const bf16x8_t*>(qp + 32 * j);
         }
     }
-    int k_off[2][KS];                                 // k-steps behind the size repeat the first one, which meets zeros
+    int k_step[KS];                                   // k-steps behind the size repeat the first one, which meets zeros
 #pragma unroll
-    for (int x = 0; x < 2; ++x)
-#pragma unroll
-        for (int j = 0; j < KS; ++j) k_off[x][j] = (8 * (n >> 2) + 4 * x + (n & 3)) * a.key_pad + (32 * j < a.key_pad ? 32 * j : 0) + 8 * g;
+    for (int j = 0; j < KS; ++j) k_step[j] = tile_key_entry(0, 32 * j < a.key_pad ? 32 * j : 0);
     const int64_t head_at = (int64_t)(h / (a.heads / a.kv_heads)) * a.block_size * a.key_pad;
+    const unsigned k_lane = 2u * (unsigned)tile_key_entry(8 * (n >> 2) + (n & 3), 8 * g);
     PageWalk walk(a, b);
     bf16x8_t kf[2][KS];
     auto fetch = [&]() {
@@ -118,7 +125,7 @@ __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefill
 #pragma unroll
         for (int x = 0; x < 2; ++x)
 #pragma unroll
-            for (int j = 0; j < KS; ++j) kf[x][j] = *reinterpret_cast<const bf16x8_t*>(src + k_off[x][j]);
+            for (int j = 0; j < KS; ++j) kf[x][j] = load_operand(src + k_step[j] + tile_key_entry(4 * x, 0), k_lane);
     };
     fetch();
     for (int s = 0; s < steps; ++s) {
@@ -146,19 +153,22 @@ __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefill
                 for (int i = 0; i < 8; ++i)
                     if (i > rel) sv[i] = -INFINITY;
             }
-            float mx = sv[0];
+            if constexpr (BOUNDED) {
 #pragma unroll
-            for (int i = 1; i < 8; ++i) mx = fmaxf(mx, sv[i]);
-            mx *= a.scale_log2;
-            const bool grow = mx > m[u] + kLazy;
-            if (__any(grow)) {
-                l[u] *= grow ? __builtin_amdgcn_exp2f(m[u] - mx) : 1.f;
-                m[u] = grow ? mx : m[u];
+                for (int i = 0; i < 8; ++i) l[u] += __builtin_amdgcn_exp2f(sv[i] * a.scale_log2);
+            } else {
+                float mx = sv[0];
+#pragma unroll
+                for (int i = 1; i < 8; ++i) mx = fmaxf(mx, sv[i]);
+                mx *= a.scale_log2;
+                const bool grow = mx > m[u] + kLazy;
+                if (__any(grow)) {
+                    l[u] *= grow ? __builtin_amdgcn_exp2f(m[u] - mx) : 1.f;
+                    m[u] = grow ? mx : m[u];
+                }
+#pragma unroll
+                for (int i = 0; i < 8; ++i) l[u] += __builtin_amdgcn_exp2f(__builtin_fmaf(sv[i], a.scale_log2, -m[u]));
             }
-            float sum = 0.f;
-#pragma unroll
-            for (int i = 0; i < 8; ++i) sum += __builtin_amdgcn_exp2f(__builtin_fmaf(sv[i], a.scale_log2, -m[u]));
-            l[u] += sum;
         }
     }
 #pragma unroll
@@ -175,22 +185,36 @@ __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefill
     }
 }
 
-// byte addresses of LDS records that lanes reach with a stride of 128 and more
-__device__ __forceinline__ int spread(int addr) { return addr ^ (((addr >> 7) & 7) << 4); }
+// LDS addresses of what belongs to query q: lanes with 16 consecutive queries meet all banks
+__device__ __forceinline__ int spread(int q, int addr) { return addr ^ ((q & 15) << 4); }
+template <int HP>
+__device__ __forceinline__ int mixed_place(int q, int slot, int g) { return (q * HP + (slot ^ (q & (HP - 1)))) * 64 + 16 * (g ^ ((q >> 2) & 3)); }
 
+// A value that the compiler takes for a new one: what is computed from it is not kept in registers over the whole loop.
+__device__ __forceinline__ int renewed(int x) {
+    asm volatile("" : "+v"(x));
+    return x;
+}
+
+// SHARE: the heads of a wavefront have one key/value head.
 template <int KS, int VT, int UH, int QT, bool SHARE>
 __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefillArgs a) {
     constexpr int HP = kMixWaves * UH, Q = 16 * QT;              // head slots, queries
     constexpr int kRec = 4 * HP;                                 // bytes of a record: every head's weight in two pieces
     constexpr int KP = UH == 4 ? 2 : 1, RT = UH == 4 ? 2 : 1;    // k-steps and head tiles of the mixture
-    constexpr int kVRow = 32 * VT, kVBuf = kStep * kVRow;        // bytes of a value; units of 32 bytes are permuted by row
+    constexpr int UK = SHARE ? 1 : UH, UW = UH / UK;             // key heads of a wavefront, query heads of each
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
     unsigned char* wbuf = lds;                                   // [Q][32 keys][kRec]
     unsigned char* pbuf = wbuf + Q * kStep * kRec;               // [Q][HP][32 keys] bf16
+    bf16x8_t* talk = reinterpret_cast<bf16x8_t*>(pbuf + Q * HP * 2 * kStep);       // [KP][RT][64]
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, n = lane & 15;
-    unsigned char* vbuf = pbuf + Q * HP * 2 * kStep + wave * kVBuf;
-    const unsigned wg = a.nseq >= 8 ? unit_of(blockIdx.x, gridDim.x) : blockIdx.x;
-    const int qblk = a.qblocks - 1 - (int)(wg % a.qblocks), b = (int)(wg / a.qblocks);
+    int b, qblk;
+    if (a.nseq % 8 == 0) {                                       // a sequence belongs to one die, whose second-level cache has its keys
+        if (!place_of_block(blockIdx.x, a.nseq, a.qblocks, b, qblk)) return;
+    } else {
+        b = (int)(blockIdx.x % (unsigned)a.nseq);
+        qblk = a.qblocks - 1 - (int)(blockIdx.x / (unsigned)a.nseq);
+    }
     const int q_beg = a.cu_q[b], sq = a.cu_q[b + 1] - q_beg, sk = a.cu_k[b + 1] - a.cu_k[b], shift = sk - sq;
     const int q0 = qblk * Q;
     if (q0 >= sq) return;
@@ -200,19 +224,21 @@ __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefill
 
     bf16x8_t q[UH][QT][KS];
     float lse[UH][QT];
-    int limit[QT], hd[UH];
-    int64_t k_head[UH], v_head[UH];
+    int limit[QT];
+    int64_t k_head[UK], v_head[UK];
 #pragma unroll
     for (int u = 0; u < UH; ++u) {
-        hd[u] = wave * UH + u < a.heads ? wave * UH + u : a.heads - 1;       // a surplus slot repeats the last head and meets zeros in T
-        k_head[u] = (int64_t)(hd[u] / group) * a.block_size * a.key_pad;
-        v_head[u] = (int64_t)(hd[u] / group) * a.block_size * a.vdim_pad;
+        const int h = wave * UH + u < a.heads ? wave * UH + u : a.heads - 1;         // a surplus slot repeats the last head and meets zeros in T
+        if (u % UW == 0) {
+            k_head[u / UW] = (int64_t)(h / group) * a.block_size * a.key_pad;
+            v_head[u / UW] = (int64_t)(h / group) * a.block_size * a.vdim_pad;
+        }
 #pragma unroll
         for (int t = 0; t < QT; ++t) {
             const int qi = q0 + 16 * t + n < sq ? q0 + 16 * t + n : sq - 1;
             limit[t] = qi + shift;
-            lse[u][t] = a.lse[(int64_t)hd[u] * a.tokens + q_beg + qi];
-            const __bf16* qp = a.q + (int64_t)(q_beg + qi) * a.q_stride + (int64_t)hd[u] * a.dim + 8 * g;
+            lse[u][t] = a.lse[(int64_t)h * a.tokens + q_beg + qi];
+            const __bf16* qp = a.q + (int64_t)(q_beg + qi) * a.q_stride + (int64_t)h * a.dim + 8 * g;
 #pragma unroll
             for (int j = 0; j < KS; ++j) {
                 q[u][t][j] = bf16x8_t{};
@@ -221,32 +247,17 @@ __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefill
         }
     }
     // T^T: entry i of lane (g, n) is column (head) 16 s + 4 g + i / 2 of row (head) 16 r + n, once for either piece
-    bf16x8_t talk[KP][RT];
+    for (int i = tid; i < KP * RT * 64; i += 64 * kMixWaves) {
+        const int s = i / (64 * RT), r = i / 64 % RT, to = 16 * r + i % 16;
+        bf16x8_t x;
 #pragma unroll
-    for (int s = 0; s < KP; ++s)
-#pragma unroll
-        for (int r = 0; r < RT; ++r)
-#pragma unroll
-            for (int i = 0; i < 8; ++i) {
-                const int from = 16 * s + 4 * g + i / 2, to = 16 * r + n;
-                talk[s][r][i] = from < HP && from < a.heads && to < a.heads ? a.talk[(int64_t)to * a.heads + from] : (__bf16)0.f;
-            }
-    for (int i = tid; i < Q * kStep * kRec / 16; i += 64 * kMixWaves) reinterpret_cast<u32x4_t*>(wbuf)[i] = u32x4_t{0u, 0u, 0u, 0u};
-
-    const int k_row = (8 * (n >> 2) + (n & 3)) * a.key_pad + 8 * g;
-    int k_step[KS];
-#pragma unroll
-    for (int j = 0; j < KS; ++j) k_step[j] = 32 * j < a.key_pad ? 32 * j : 0;            // surplus steps meet zeros in q
-    // chunk i of this lane: 16 bytes of a value row; surplus ones repeat the tile's last
-    const int per_row = a.vdim_pad / 8, chunks = kStep * per_row;
-    int c_row[VT], c_col[VT];
-#pragma unroll
-    for (int i = 0; i < VT; ++i) {
-        const int c = lane + 64 * i < chunks ? lane + 64 * i : chunks - 1;
-        c_row[i] = c / per_row;
-        c_col[i] = c - c_row[i] * per_row;
+        for (int e = 0; e < 8; ++e) {
+            const int from = 16 * s + 4 * (i % 64 / 16) + e / 2;
+            x[e] = from < HP && from < a.heads && to < a.heads ? a.talk[(int64_t)to * a.heads + from] : (__bf16)0.f;
+        }
+        talk[i] = x;
     }
-    auto v_place = [&](int row, int byte) { return row * kVRow + (byte ^ ((row & (VT - 1)) * 32)); };
+    for (int i = tid; i < Q * kStep * kRec / 16; i += 64 * kMixWaves) reinterpret_cast<u32x4_t*>(wbuf)[i] = u32x4_t{0u, 0u, 0u, 0u};
 
     f32x4_t acc[UH][QT][VT];
 #pragma unroll
@@ -257,150 +268,148 @@ __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefill
             for (int v = 0; v < VT; ++v) acc[u][t][v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 
     PageWalk walk(a, b);
-    bf16x8_t kf[2][KS];
-    u32x4_t vreg[VT];
-    auto fetch_k = [&](int64_t tile, int u) {
-        const __bf16* src = a.keys + tile * kStep * a.key_pad + k_head[u] + k_row;
+    const unsigned k_lane = 2u * (unsigned)tile_key_entry(8 * (n >> 2) + (n & 3), 8 * g), v_lane = 2u * (unsigned)tile_value_entry(8 * g, n);
+    bf16x8_t kf[KS];
+    // half x of the keys of head uk; k-steps behind the size repeat the first one, which meets zeros in q
+    auto fetch_k = [&](int64_t tile, int uk, int x) {
+        const __bf16* src = a.keys + tile * kStep * a.key_pad + k_head[uk] + tile_key_entry(4 * x, 0);
 #pragma unroll
-        for (int x = 0; x < 2; ++x)
-#pragma unroll
-            for (int j = 0; j < KS; ++j) kf[x][j] = *reinterpret_cast<const bf16x8_t*>(src + 4 * x * a.key_pad + k_step[j]);
+        for (int j = 0; j < KS; ++j) kf[j] = load_operand(src + tile_key_entry(0, 32 * j < a.key_pad ? 32 * j : 0), k_lane);
     };
-    auto fetch_v = [&](int64_t tile, int u, int last) {          // values behind the last one repeat it; their weights are zero
-        const __bf16* src = a.values + tile * kStep * a.vdim_pad + v_head[u];
-#pragma unroll
-        for (int i = 0; i < VT; ++i) vreg[i] = *reinterpret_cast<const u32x4_t*>(src + (c_row[i] < last ? c_row[i] : last) * a.vdim_pad + 8 * c_col[i]);
+    constexpr int kRing = 4;                                     // value operands under way
+    bf16x8_t vf[kRing];
+    // operand i of the step: tile i % VT of head i / VT; tiles behind the size repeat the first one and are not stored
+    auto fetch_v = [&](int64_t tile, int i) {
+        const int v = i % VT;
+        vf[i % kRing] = load_operand(a.values + tile * kStep * a.vdim_pad + v_head[i / VT] + tile_value_entry(0, 16 * v < a.vdim_pad ? 16 * v : 0), v_lane);
     };
     int64_t tile = walk.next(a);
-    fetch_k(tile, 0);
-    __syncthreads();                                             // the zero fill
+    fetch_k(tile, 0, 0);
+    const int w_fixed = spread(n, (n * kStep + 8 * g) * kRec + wave * UH * 4);
+    __syncthreads();                                             // the zero fill and T
     for (int s = 0; s < steps; ++s) {
-        const int tok0 = s * kStep, last = sk - 1 - tok0;
+        const int tok0 = s * kStep, left = sk - tok0;
         const int64_t here = tile;
-        if (s + 1 < steps) tile = walk.next(a);
+        if (s + 1 < steps) tile = walk.next(a);                  // the last step requests its own keys again
         if (live) {
-            // ---- scores and weights
-            f32x4_t sc[UH][QT][2];
+            // ---- scores and weights, half of the keys of a key head at a time
+            const int w_base = renewed(w_fixed);
 #pragma unroll
-            for (int u = 0; u < UH; ++u) {
+            for (int i = 0; i < 2 * UK; ++i) {
+                const int uk = i / 2, x = i % 2;
+                f32x4_t sc[UW][QT];
 #pragma unroll
-                for (int t = 0; t < QT; ++t)
+                for (int w = 0; w < UW; ++w)
 #pragma unroll
-                    for (int x = 0; x < 2; ++x) sc[u][t][x] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-                if (!SHARE && u > 0) fetch_k(here, u);
+                    for (int t = 0; t < QT; ++t) {
+                        sc[w][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                for (int j = 0; j < KS; ++j)
+                        for (int j = 0; j < KS; ++j) sc[w][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j], q[uk * UW + w][t][j], sc[w][t], 0, 0, 0);
+                    }
+                if (i + 1 < 2 * UK) fetch_k(here, (i + 1) / 2, (i + 1) % 2);
+                else fetch_k(tile, 0, 0);
 #pragma unroll
-                    for (int x = 0; x < 2; ++x)
+                for (int t = 0; t < QT; ++t) {
+                    uint32_t w4[UW][4];
 #pragma unroll
-                        for (int t = 0; t < QT; ++t) sc[u][t][x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[x][j], q[u][t][j], sc[u][t][x], 0, 0, 0);
-            }
-            fetch_v(here, 0, last);
-            fetch_k(tile, 0);                                    // of the next step; the last one's repeats its own
+                    for (int w = 0; w < UW; ++w) {
+                        float p[4];
 #pragma unroll
-            for (int t = 0; t < QT; ++t) {
-                uint32_t w[UH][8];
+                        for (int e = 0; e < 4; ++e) p[e] = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[w][t][e], a.scale_log2, -lse[uk * UW + w][t]));
+                        if (tok0 + kStep - 1 > q0 + 16 * t + shift) {
+                            const int rel = limit[t] - tok0 - 8 * g - 4 * x;
 #pragma unroll
-                for (int u = 0; u < UH; ++u) {
-                    float p[8];
+                            for (int e = 0; e < 4; ++e)
+                                if (e > rel) p[e] = 0.f;
+                        }
 #pragma unroll
-                    for (int i = 0; i < 8; ++i) p[i] = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[u][t][i >> 2][i & 3], a.scale_log2, -lse[u][t]));
-                    if (tok0 + kStep - 1 > q0 + 16 * t + shift) {
-                        const int rel = limit[t] - tok0 - 8 * g;
-#pragma unroll
-                        for (int i = 0; i < 8; ++i)
-                            if (i > rel) p[i] = 0.f;
+                        for (int e = 0; e < 4; ++e) w4[w][e] = round_pack(head(p[e]), p[e] - head(p[e]));
                     }
 #pragma unroll
-                    for (int i = 0; i < 8; ++i) w[u][i] = round_pack(head(p[i]), p[i] - head(p[i]));
-                }
-#pragma unroll
-                for (int i = 0; i < 8; ++i) {
-                    unsigned char* to = wbuf + spread(((16 * t + n) * kStep + 8 * g + i) * kRec + wave * UH * 4);
-                    if constexpr (UH == 4) *reinterpret_cast<u32x4_t*>(to) = u32x4_t{w[0][i], w[1][i], w[2][i], w[3][i]};
-                    else if constexpr (UH == 2) *reinterpret_cast<u32x2_t*>(to) = u32x2_t{w[0][i], w[1][i]};
-                    else *reinterpret_cast<uint32_t*>(to) = w[0][i];
+                    for (int e = 0; e < 4; ++e) {
+                        unsigned char* to = wbuf + (w_base ^ ((4 * x + e) * kRec)) + t * (16 * kStep * kRec) + uk * UW * 4;
+                        if constexpr (UW == 4) *reinterpret_cast<u32x4_t*>(to) = u32x4_t{w4[0][e], w4[1][e], w4[2][e], w4[3][e]};
+                        else if constexpr (UW == 2) *reinterpret_cast<u32x2_t*>(to) = u32x2_t{w4[0][e], w4[1][e]};
+                        else *reinterpret_cast<uint32_t*>(to) = w4[0][e];
+                    }
                 }
             }
+#pragma unroll
+            for (int i = 0; i < kRing; ++i) fetch_v(here, i);
         }
         __syncthreads();
         // ---- the mixture, for queries 2 QT wave and on
+        {
+            const int g = renewed(lane >> 4), n = renewed(lane & 15);
+            bf16x8_t tf[KP][RT];
 #pragma unroll
-        for (int k = 0; k < 2 * QT; ++k) {
-            const int qi = 2 * QT * wave + k;
-            f32x4_t mixed[RT][2];
+            for (int y = 0; y < KP; ++y)
 #pragma unroll
-            for (int x = 0; x < 2; ++x) {
+                for (int r = 0; r < RT; ++r) tf[y][r] = talk[(y * RT + r) * 64 + lane];
 #pragma unroll
-                for (int r = 0; r < RT; ++r) mixed[r][x] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-                const int rec = (qi * kStep + 8 * (n >> 2) + 4 * x + (n & 3)) * kRec;
+            for (int k = 0; k < 2 * QT; ++k) {
+                const int qi = 2 * QT * wave + k;
+                f32x4_t mixed[RT][2];
 #pragma unroll
-                for (int y = 0; y < KP; ++y) {
-                    const bf16x8_t wf = *reinterpret_cast<const bf16x8_t*>(wbuf + spread(rec + 64 * y + 16 * (UH == 1 ? g & 1 : g)));
+                for (int x = 0; x < 2; ++x) {
 #pragma unroll
-                    for (int r = 0; r < RT; ++r) mixed[r][x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, talk[y][r], mixed[r][x], 0, 0, 0);
+                    for (int r = 0; r < RT; ++r) mixed[r][x] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+                    const int rec = (qi * kStep + 8 * (n >> 2) + 4 * x + (n & 3)) * kRec;
+#pragma unroll
+                    for (int y = 0; y < KP; ++y) {
+                        const bf16x8_t wf = *reinterpret_cast<const bf16x8_t*>(wbuf + spread(qi, rec + 64 * y + 16 * (UH == 1 ? g & 1 : g)));
+#pragma unroll
+                        for (int r = 0; r < RT; ++r) mixed[r][x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, tf[y][r], mixed[r][x], 0, 0, 0);
+                    }
                 }
-            }
 #pragma unroll
-            for (int r = 0; r < RT; ++r) {
-                bf16x8_t p;
+                for (int r = 0; r < RT; ++r) {
+                    bf16x8_t p;
 #pragma unroll
-                for (int i = 0; i < 8; ++i) p[i] = (__bf16)mixed[r][i >> 2][i & 3];
-                const int to = 16 * r + n;
-                if (HP >= 16 || to < HP) *reinterpret_cast<bf16x8_t*>(pbuf + (qi * HP + (to ^ (qi & (HP - 1)))) * 64 + 16 * g) = p;
+                    for (int i = 0; i < 8; ++i) p[i] = (__bf16)mixed[r][i >> 2][i & 3];
+                    const int to = 16 * r + n;
+                    if (HP >= 16 || to < HP) *reinterpret_cast<bf16x8_t*>(pbuf + mixed_place<HP>(qi, to, g)) = p;
+                }
             }
         }
         __syncthreads();
         // ---- weighted sum of the values
         if (live) {
+            const int g = renewed(lane >> 4), n = renewed(lane & 15);
 #pragma unroll
-            for (int u = 0; u < UH; ++u) {
-                if (!SHARE || u == 0) {
+            for (int uk = 0; uk < UK; ++uk) {
+                bf16x8_t pb[UW][QT];
 #pragma unroll
-                    for (int i = 0; i < VT; ++i) *reinterpret_cast<u32x4_t*>(vbuf + v_place(c_row[i], 16 * c_col[i])) = vreg[i];
-                    // a wavefront's own LDS operations happen in order; the compiler has to keep them so
-                    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-                    __builtin_amdgcn_wave_barrier();
-                    if (!SHARE && u + 1 < UH) fetch_v(here, u + 1, last);
-                }
-                bf16x8_t pb[SHARE ? UH : 1][QT];
-                if (!SHARE || u == 0)
+                for (int w = 0; w < UW; ++w)
 #pragma unroll
-                    for (int w = 0; w < (SHARE ? UH : 1); ++w)
-#pragma unroll
-                        for (int t = 0; t < QT; ++t) {
-                            const int qi = 16 * t + n, slot = wave * UH + (SHARE ? w : u);
-                            pb[w][t] = *reinterpret_cast<const bf16x8_t*>(pbuf + (qi * HP + (slot ^ (qi & (HP - 1)))) * 64 + 16 * g);
-                        }
-                if (SHARE && u > 0) continue;
+                    for (int t = 0; t < QT; ++t) pb[w][t] = *reinterpret_cast<const bf16x8_t*>(pbuf + mixed_place<HP>(16 * t + n, wave * UH + uk * UW + w, g));
 #pragma unroll
                 for (int v = 0; v < VT; ++v) {
-                    const int row = 8 * g + (n >> 2), at = 32 * v + (n & 3) * 8;
-                    const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vbuf + v_place(row, at)));
-                    const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vbuf + v_place(row + 4, at)));
-                    const bf16x8_t vt = __builtin_bit_cast(bf16x8_t, (i16x8)__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+                    const int i = uk * VT + v;
+                    bf16x8_t x = vf[i % kRing];
+                    if (left < kStep)                            // values behind the last one may be anything
 #pragma unroll
-                    for (int w = 0; w < (SHARE ? UH : 1); ++w)
+                        for (int e = 0; e < 8; ++e)
+                            if (8 * g + e >= left) x[e] = (__bf16)0.f;
 #pragma unroll
-                        for (int t = 0; t < QT; ++t) {
-                            f32x4_t& o = acc[SHARE ? w : u][t][v];
-                            o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pb[w][t], o, 0, 0, 0);
-                        }
+                    for (int w = 0; w < UW; ++w)
+#pragma unroll
+                        for (int t = 0; t < QT; ++t) acc[uk * UW + w][t][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, pb[w][t], acc[uk * UW + w][t][v], 0, 0, 0);
+                    if (i + kRing < UK * VT) fetch_v(here, i + kRing);
                 }
-                __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-                __builtin_amdgcn_wave_barrier();
             }
         }
     }
     if (!live) return;
 #pragma unroll
     for (int u = 0; u < UH; ++u) {
-        if (wave * UH + u >= a.heads) continue;
+        const int h = wave * UH + u;
+        if (h >= a.heads) continue;
 #pragma unroll
         for (int t = 0; t < QT; ++t) {
             const int qi = q0 + 16 * t + n;
             if (qi >= sq) continue;
-            __bf16* o = a.out + (int64_t)(q_beg + qi) * a.out_stride + (int64_t)hd[u] * a.vdim + 4 * g;
+            __bf16* o = a.out + (int64_t)(q_beg + qi) * a.out_stride + (int64_t)h * a.vdim + 4 * g;
 #pragma unroll
             for (int v = 0; v < VT; ++v) {
                 if (16 * v + 4 * g >= a.vdim) continue;
@@ -414,11 +423,12 @@ __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefill
 }
 
 template <int KS>
-int launch_lse(TalkPrefillArgs a, int64_t max_seqlen_q, hipStream_t st) {
-    const int64_t per = kLseQ * kLseWaves, qblocks = (max_seqlen_q + per - 1) / per, total = qblocks * a.nseq * a.heads;
+int launch_lse(TalkPrefillArgs a, int64_t max_seqlen_q, bool bounded, hipStream_t st) {
+    const int64_t per = kLseQ * kLseWaves, qblocks = (max_seqlen_q + per - 1) / per, total = ((int64_t)a.nseq * a.heads + 7) / 8 * 8 * qblocks;
     if (total > 0x7fffffff) return INFER_KV_EINVAL;
     a.qblocks = (int)qblocks;
-    hipLaunchKernelGGL((talk_lse_kernel<KS>), dim3((unsigned)total), dim3(64 * kLseWaves), 0, st, a);
+    if (bounded) hipLaunchKernelGGL((talk_lse_kernel<KS, true>), dim3((unsigned)total), dim3(64 * kLseWaves), 0, st, a);
+    else hipLaunchKernelGGL((talk_lse_kernel<KS, false>), dim3((unsigned)total), dim3(64 * kLseWaves), 0, st, a);
     return (int)hipGetLastError();
 }
 
@@ -428,7 +438,7 @@ int launch_mix(TalkPrefillArgs a, int64_t max_seqlen_q, hipStream_t st) {
     if (total > 0x7fffffff) return INFER_KV_EINVAL;
     a.qblocks = (int)qblocks;
     auto kernel = &talk_mix_kernel<KS, VT, UH, QT, SHARE>;
-    constexpr size_t lds = (size_t)16 * QT * kStep * kMixWaves * UH * (4 + 2) + (size_t)kMixWaves * kStep * 32 * VT;
+    constexpr size_t lds = (size_t)16 * QT * kStep * kMixWaves * UH * (4 + 2) + (UH == 4 ? 4 : 1) * 1024;
     static_assert(lds <= 160 * 1024, "LDS of a compute unit");
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return (int)e;
@@ -437,21 +447,24 @@ int launch_mix(TalkPrefillArgs a, int64_t max_seqlen_q, hipStream_t st) {
 }
 
 template <int KS, int VT>
-int launch(const TalkPrefillArgs& a, int64_t max_seqlen_q, hipStream_t st) {
-    const int rc = launch_lse<KS>(a, max_seqlen_q, st);
+int launch(const TalkPrefillArgs& a, int64_t max_seqlen_q, bool bounded, hipStream_t st) {
+    const int rc = launch_lse<KS>(a, max_seqlen_q, bounded, st);
     if (rc) return rc;
     const int group = a.heads / a.kv_heads;
-    if (a.heads <= 8) return launch_mix<KS, VT, 1, 2, true>(a, max_seqlen_q, st);
-    if (a.heads <= 16) return group % 2 == 0 ? launch_mix<KS, VT, 2, 1, true>(a, max_seqlen_q, st) : launch_mix<KS, VT, 2, 1, false>(a, max_seqlen_q, st);
+    // twice the queries per workgroup where that leaves one for every compute unit
+    const bool many = (max_seqlen_q + 63) / 64 * a.nseq >= 256, some = (max_seqlen_q + 31) / 32 * a.nseq >= 256;
+    if (a.heads <= 8) return many ? launch_mix<KS, VT, 1, 4, true>(a, max_seqlen_q, st) : launch_mix<KS, VT, 1, 2, true>(a, max_seqlen_q, st);
+    if (a.heads <= 16 && group % 2 == 0)
+        return some ? launch_mix<KS, VT, 2, 2, true>(a, max_seqlen_q, st) : launch_mix<KS, VT, 2, 1, true>(a, max_seqlen_q, st);
+    if (a.heads <= 16) return some ? launch_mix<KS, VT, 2, 2, false>(a, max_seqlen_q, st) : launch_mix<KS, VT, 2, 1, false>(a, max_seqlen_q, st);
     return group % 4 == 0 ? launch_mix<KS, VT, 4, 1, true>(a, max_seqlen_q, st) : launch_mix<KS, VT, 4, 1, false>(a, max_seqlen_q, st);
 }
 
 }  // namespace
 
 // 1 if the sizes are served
-extern "C" int infer_talking_prefill_supported(int64_t heads, int64_t dim, int64_t vdim, int64_t block_size) {
-    return heads >= 1 && heads <= 32 && dim >= 8 && dim <= 128 && dim % 8 == 0 && vdim >= 8 && vdim <= 128 && vdim % 8 == 0 && block_size >= kStep &&
-           block_size % kStep == 0;
+extern "C" int infer_talking_prefill_supported(int64_t heads, int64_t dim, int64_t vdim) {
+    return heads >= 1 && heads <= 32 && dim >= 8 && dim <= 128 && dim % 8 == 0 && vdim >= 8 && vdim <= 128 && vdim % 8 == 0;
 }
 
 extern "C" int infer_talking_prefill(const void* q, int64_t q_stride, const void* keys, const void* values, int64_t key_pad,
@@ -459,13 +472,13 @@ extern "C" int infer_talking_prefill(const void* q, int64_t q_stride, const void
                                      int64_t block_size, int64_t num_blocks, const int32_t* seqs, const int32_t* cu_q,
                                      const int32_t* cu_k, int64_t num_seqs, int64_t tokens, int64_t max_seqlen_q, int64_t heads,
                                      int64_t kv_heads, int64_t dim, int64_t vdim, float scale, const void* talk, float out_scale,
-                                     void* out, int64_t out_stride, float* workspace, int64_t workspace_floats, void* stream) {
-    if (!infer_talking_prefill_supported(heads, dim, vdim, block_size)) return INFER_KV_EUNSUPPORTED;
+                                     float max_score, void* out, int64_t out_stride, float* workspace, int64_t workspace_floats, void* stream) {
+    if (!infer_talking_prefill_supported(heads, dim, vdim)) return INFER_KV_EUNSUPPORTED;
     if (num_seqs < 0 || max_seqlen_q < 0 || tokens < 0 || num_seqs > 0x7fffffff || max_seqlen_q > 0x7fffffff || max_seqlen_q > tokens) return INFER_KV_EINVAL;
     if (num_seqs == 0 || max_seqlen_q == 0) return INFER_KV_OK;
     if (!q || !keys || !values || !block_table || !seqs || !cu_q || !cu_k || !talk || !out || kv_heads < 1 || heads % kv_heads ||
         q_stride < heads * dim || out_stride < heads * vdim || key_pad != (dim + 31) / 32 * 32 || vdim_pad != (vdim + 31) / 32 * 32 ||
-        block_size > (1 << 20) || table_cols < 1 || table_cols * block_size > 0x7fffffff || bt_stride < table_cols || num_blocks < 1 ||
+        block_size < kStep || block_size % kStep || block_size > (1 << 20) || table_cols < 1 || table_cols * block_size > 0x7fffffff || bt_stride < table_cols || num_blocks < 1 ||
         num_blocks > 0x7fffffff || !(scale > 0.f))
         return INFER_KV_EINVAL;
     if (q_stride % 8 || out_stride % 4 || !ptr_aligned(q, 16) || !ptr_aligned(keys, 16) || !ptr_aligned(values, 16) || !ptr_aligned(out, 8))
@@ -475,6 +488,7 @@ extern "C" int infer_talking_prefill(const void* q, int64_t q_stride, const void
                             bt_stride, (int)table_cols, (int)block_size, (int)num_blocks, seqs, cu_q, cu_k, (int)heads, (int)kv_heads, (int)dim,
                             (int)vdim, (int)num_seqs, 0, scale * kLog2e, (const __bf16*)talk, out_scale, (__bf16*)out, out_stride, workspace, tokens};
     hipStream_t st = (hipStream_t)stream;
-    if (dim <= 64) return vdim <= 64 ? launch<2, 4>(a, max_seqlen_q, st) : launch<2, 8>(a, max_seqlen_q, st);
-    return vdim <= 64 ? launch<4, 4>(a, max_seqlen_q, st) : launch<4, 8>(a, max_seqlen_q, st);
+    const bool bounded = max_score * kLog2e <= kBound;
+    if (dim <= 64) return vdim <= 64 ? launch<2, 4>(a, max_seqlen_q, bounded, st) : launch<2, 8>(a, max_seqlen_q, bounded, st);
+    return vdim <= 64 ? launch<4, 4>(a, max_seqlen_q, bounded, st) : launch<4, 8>(a, max_seqlen_q, bounded, st);
 }

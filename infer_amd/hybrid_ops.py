@@ -4,6 +4,7 @@ checks on the host, then one call into ``libinfer_kv.so`` on torch's current str
 from __future__ import annotations
 
 import ctypes
+import math
 from dataclasses import dataclass
 from functools import lru_cache
 
@@ -590,17 +591,25 @@ class TalkShape:
     def vdim_pad(self) -> int:
         return -(-self.vdim // 32) * 32
 
+    def max_score(self, positions: int) -> float:
+        """A bound of the scores at the first ``positions`` positions, with some room for rounding: queries and keys have the root mean
+        square one (or less)."""
+        temp = 1.0
+        if self.temp_every > 0:
+            temp = max(1.0, abs(1.0 + self.temp_coef * math.log(positions // self.temp_every + 1.0)))
+        return 1.05 * abs(self.scale) * self.dim * temp
+
 
 def _talk_pages(s: TalkShape, keys, values, dtype):
-    """(blocks, block size) of checked pages."""
+    """(blocks, block size) of checked pages (``cache.TilePages``)."""
     assert keys.dtype == values.dtype == dtype and keys.is_contiguous() and values.is_contiguous() and keys.shape[:3] == values.shape[:3]
-    assert keys.shape[1] == s.kv_heads and keys.shape[3] == s.key_pad and values.shape[3] == s.vdim_pad
-    return keys.shape[0], keys.shape[2]
+    assert keys.shape[1] == s.kv_heads and tuple(keys.shape[3:]) == (s.key_pad // 32, 32, 32) and tuple(values.shape[3:]) == (s.vdim_pad, 32)
+    return keys.shape[0], 32 * keys.shape[2]
 
 
 def unit_head_front(s: TalkShape, proj, offsets, positions, slots, keys, values, qx, qx_rows: int) -> None:
-    """Norms per head, the temperature of the queries and the append of keys [blocks, kv_heads, block_size, key_pad] and values
-    [blocks, kv_heads, block_size, vdim_pad]; ``qx`` [>= qx_rows, heads, key_pad]."""
+    """Norms per head, the temperature of the queries and the append of keys and values to pages of tiles; ``qx``
+    [>= qx_rows, heads, key_pad]."""
     n = proj.shape[0]
     blocks, bs = _talk_pages(s, keys, values, proj.dtype)
     cols = max(offsets[0] + s.heads * s.dim, offsets[1] + s.kv_heads * s.dim, offsets[2] + s.kv_heads * s.vdim)
@@ -652,14 +661,15 @@ def talking_attention(s: TalkShape, qx, keys, values, talk, block_table, ctx, ou
         _lib.check(rc, "talking_attention")
 
 
-def talking_prefill_supported(s: TalkShape, block_size: int) -> bool:
+def talking_prefill_supported(s: TalkShape) -> bool:
     """Whether the kernels for whole portions serve these sizes."""
-    return bool(_lib.load().infer_talking_prefill_supported(s.heads, s.dim, s.vdim, block_size))
+    return bool(_lib.load().infer_talking_prefill_supported(s.heads, s.dim, s.vdim))
 
 
-def talking_prefill(s: TalkShape, q, keys, values, talk, block_table, seqs, cu_q, cu_k, max_seqlen_q: int, out) -> None:
+def talking_prefill(s: TalkShape, q, keys, values, talk, block_table, seqs, cu_q, cu_k, max_seqlen_q: int, out, max_score=None) -> None:
     """Whole portions: ``q`` [tokens, heads * dim] (behind ``unit_head_front``) are the last tokens of the sequences in block-table rows
-    ``seqs``, whose numbers of keys ``cu_k`` sums up; ``out`` [tokens, heads * vdim], all bf16."""
+    ``seqs``, whose numbers of keys ``cu_k`` sums up; ``out`` [tokens, heads * vdim], all bf16.  ``max_score``: no score is larger
+    (None: nobody knows); a small bound spares the search for maxima."""
     blocks, bs = _talk_pages(s, keys, values, torch.bfloat16)
     assert q.dtype == out.dtype == talk.dtype == torch.bfloat16 and q.shape[0] == out.shape[0]
     assert talk.is_contiguous() and tuple(talk.shape) == (s.heads, s.heads)
@@ -673,8 +683,9 @@ def talking_prefill(s: TalkShape, q, keys, values, talk, block_table, seqs, cu_q
     rc = _lib.load().infer_talking_prefill(
         q.data_ptr(), _rows(q, s.heads * s.dim), keys.data_ptr(), values.data_ptr(), s.key_pad, s.vdim_pad, block_table.data_ptr(),
         max(block_table.stride(0), cols), cols, bs, blocks, seqs.data_ptr(), cu_q.data_ptr(), cu_k.data_ptr(), seqs.numel(), tokens,
-        int(max_seqlen_q), s.heads, s.kv_heads, s.dim, s.vdim, float(s.scale), talk.data_ptr(), float(s.out_scale), out.data_ptr(),
-        _rows(out, s.heads * s.vdim), ws.data_ptr(), ws.numel(), _stream_ptr(q))
+        int(max_seqlen_q), s.heads, s.kv_heads, s.dim, s.vdim, float(s.scale), talk.data_ptr(), float(s.out_scale),
+        float("inf") if max_score is None else float(max_score), out.data_ptr(), _rows(out, s.heads * s.vdim), ws.data_ptr(), ws.numel(),
+        _stream_ptr(q))
     _lib.check(rc, "talking_prefill")
 
 

@@ -1,4 +1,4 @@
-"""Attention whose heads mix their softmax weights before these meet the values (talking heads), over pages of keys and pages of values:
+"""Attention whose heads mix their softmax weights before these meet the values (talking heads), over pages of tiles:
 a part of a ``Mixer``.
 
 Queries and keys are divided by their root mean square per head, optionally values too; queries may have a temperature that grows with
@@ -10,7 +10,7 @@ import torch
 from torch import nn
 
 from . import hybrid_ops
-from .cache import SplitPages
+from .cache import TilePages
 from .context import get_context
 
 
@@ -37,8 +37,8 @@ class TalkingAttention(nn.Module):
         s = self.shape
         return {"q": s.heads * s.dim, "k": s.kv_heads * s.dim, "v": s.kv_heads * s.vdim}
 
-    def cache_spec(self) -> SplitPages:
-        return SplitPages(self.shape.kv_heads, self.shape.key_pad, self.shape.vdim_pad, self.dtype)
+    def cache_spec(self) -> TilePages:
+        return TilePages(self.shape.kv_heads, self.shape.key_pad, self.shape.vdim_pad, self.dtype)
 
     def finish_loading(self, max_position: int) -> None:
         pass
@@ -46,7 +46,7 @@ class TalkingAttention(nn.Module):
     def forward(self, proj: torch.Tensor, offset: dict, bias, pages: dict, out: torch.Tensor) -> None:
         plan, s, keys, values = get_context().step, self.shape, pages["keys"], pages["values"]
         n = proj.shape[0]
-        dense = self.dtype == torch.bfloat16 and hybrid_ops.talking_prefill_supported(s, keys.shape[2])
+        dense = self.dtype == torch.bfloat16 and hybrid_ops.talking_prefill_supported(s)
         split = plan.dense_row if dense else n                 # rows from here on belong to long portions
         qx = torch.empty((split, s.heads, s.key_pad), dtype=proj.dtype, device=proj.device)
         hybrid_ops.unit_head_front(s, proj, [offset[name] for name in "qkv"], plan.positions, plan.slot_mapping, keys, values, qx, split)
@@ -55,4 +55,4 @@ class TalkingAttention(nn.Module):
                                          row_seq=None if plan.row_seq is None else plan.row_seq[:split], max_keys=plan.max_keys)
         if split < n:
             hybrid_ops.talking_prefill(s, proj[split:, offset["q"]:], keys, values, self.talk, plan.block_tables, plan.dense_seqs, plan.dense_cu_q,
-                                       plan.dense_cu_k, plan.dense_max_q, out[split:])
+                                       plan.dense_cu_k, plan.dense_max_q, out[split:], max_score=s.max_score(plan.max_keys))

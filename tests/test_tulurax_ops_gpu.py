@@ -92,23 +92,46 @@ def test_scaled_softcap(gpu, dtype):
     close(ho.softcap(dev(x, dtype), 7.5, 0.3), 7.5 * np.tanh(0.3 * x / 7.5), 1e-6)
 
 
+# ------------------------------------------------------------------ pages
+def to_pages(keys, values):
+    """[blocks, kv_heads, block_size, entries] each, in tiles of 32 tokens as the kernels keep them."""
+    b, h, bs, n = keys.shape
+    k = keys.reshape(b, h, bs // 32, 32, n // 32, 32).transpose(0, 1, 2, 4, 3, 5)
+    v = values.reshape(b, h, bs // 32, 32, -1).transpose(0, 1, 2, 4, 3)
+    return k, v
+
+
+def from_pages(keys, values):
+    """The entries of every slot, [blocks * block_size, kv_heads, entries]."""
+    b, h, tiles, steps = keys.shape[:4]
+    k = keys.transpose(0, 2, 4, 1, 3, 5).reshape(b * tiles * 32, h, steps * 32)
+    return k, values.transpose(0, 2, 4, 1, 3).reshape(b * tiles * 32, h, -1)
+
+
 # ------------------------------------------------------------------ front end
 @BOTH
 @pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(6, 2, 24, 16), (3, 1, 10, 7), (16, 2, 128, 128), (32, 8, 64, 128), (8, 1, 64, 32), (2, 1, 200, 40),
                                                      (2, 2, 40, 200), (40, 8, 128, 96), (5, 5, 9, 300), (1, 1, 8, 8)])
 @pytest.mark.parametrize("temp,norm_values", [((0.7, 32), True), ((0.5, 1), False), (None, True)])
-def test_unit_head_front(gpu, dtype, heads, kv_heads, dim, vdim, temp, norm_values):
+@pytest.mark.parametrize("n", [9, 150])
+def test_unit_head_front(gpu, dtype, heads, kv_heads, dim, vdim, temp, norm_values, n):
     rng = np.random.default_rng(heads * dim)
-    n, bs, nblk, qx_rows, eps = 9, 32, 3, 4, 1e-2
+    bs, nblk, qx_rows, eps = 64, 4, 4, 1e-2
     s = ho.TalkShape(heads, kv_heads, dim, vdim, 1.0, eps, norm_values, *((temp[0], temp[1]) if temp else ()))
     off = [8, 8 + -(-heads * dim // 8) * 8]
     off.append(off[1] + -(-kv_heads * dim // 8) * 8)
     cols = -(-(off[2] + kv_heads * vdim + 5) // 8) * 8
     x = rounded(rng.standard_normal((n, cols)) * .2, dtype)
     pos = np.array([0, 30, 31, 32, 62, 63, 64, 1000, 70000])                                        # around where the factor changes
-    slots = np.array([5, 31, 32, -1, 64, 95, 200, 0, 33], np.int32)                                  # one padding row, one outside the pool
-    keys = torch.full((nblk, kv_heads, bs, s.key_pad), 7.0, dtype=dtype, device=gpu)
-    values = torch.full((nblk, kv_heads, bs, s.vdim_pad), 7.0, dtype=dtype, device=gpu)
+    slots = np.array([5, 31, 32, -1, 64, 95, 300, 0, 33], np.int32)                                  # one padding row, one outside the pool
+    if n > 9:                                                    # runs of tokens that start and end inside of tiles and groups of eight
+        runs = [np.arange(101, 134), np.arange(192, 256), np.arange(66, 77), np.arange(134, 167)]
+        slots = np.concatenate([slots] + runs).astype(np.int32)
+        assert len(slots) == n
+        pos = np.concatenate([pos, rng.integers(0, 5000, n - 9)])
+    shape = nblk, kv_heads, bs // 32
+    keys = torch.full((*shape, s.key_pad // 32, 32, 32), 7.0, dtype=dtype, device=gpu)
+    values = torch.full((*shape, s.vdim_pad, 32), 7.0, dtype=dtype, device=gpu)
     qx = torch.full((qx_rows, heads, s.key_pad), float("nan"), dtype=dtype, device=gpu)
     proj = dev(x, dtype)
     ho.unit_head_front(s, proj, off, dev(pos, torch.int64), dev(slots, torch.int32), keys, values, qx, qx_rows)
@@ -129,8 +152,7 @@ def test_unit_head_front(gpu, dtype, heads, kv_heads, dim, vdim, temp, norm_valu
         close(proj[r, off[0]:off[0] + width], q[r].ravel(), t)
     left = np.r_[0:off[0], off[0] + width:cols]
     assert np.array_equal(host(proj[:qx_rows]), x[:qx_rows]) and np.array_equal(host(proj)[:, left], x[:, left])
-    for pages, want, size in ((keys, k, dim), (values, v, vdim)):
-        got = host(pages).transpose(0, 2, 1, 3).reshape(nblk * bs, kv_heads, -1)
+    for got, want, size in zip(from_pages(host(keys), host(values)), (k, v), (dim, vdim)):
         for i, slot in enumerate(slots):
             if 0 <= slot < nblk * bs:
                 close(torch.tensor(got[slot, :, :size]), want[i], t)
@@ -158,7 +180,7 @@ class Pages:
                 for pages, data, size in ((keys, self.k[i], s.dim), (values, self.v[i], s.vdim)):
                     pages[block, :, :m] = 0.0
                     pages[block, :, :m, :size] = data[b * bs:b * bs + m].transpose(1, 0, 2)
-        self.pages, self.tables = (dev(keys, dtype), dev(values, dtype)), dev(tables, torch.int32)
+        self.pages, self.tables = tuple(dev(p, dtype) for p in to_pages(keys, values)), dev(tables, torch.int32)
 
 
 def one_query(s, talk, q, k, v):
@@ -230,7 +252,7 @@ def test_scores_beyond_what_exponentials_hold_and_below_the_sink(gpu, dtype, siz
     p.pages[0].zero_()
     for b in range(4):
         m = min(32, n - 32 * b)
-        p.pages[0][p.tables[0, b], :, :m] = dev(k[32 * b:32 * b + m].transpose(1, 0, 2), dtype)
+        p.pages[0][p.tables[0, b], :, 0, 0, :m] = dev(k[32 * b:32 * b + m].transpose(1, 0, 2), dtype)
     q = rounded(np.broadcast_to(key * size / (0.5 * key @ key), (1, 4, 32)), dtype)
     talk = mixing(rng, 4, dtype)
     want = one_query(s, talk, q[0], k, p.v[0])
@@ -288,11 +310,12 @@ def test_rows_run_in_turns_when_their_scores_are_many(gpu, dtype, monkeypatch):
                                                      (12, 3, 64, 128), (16, 4, 128, 64), (32, 8, 128, 128), (20, 20, 48, 56), (24, 2, 128, 96),
                                                      (30, 10, 64, 64), (32, 32, 128, 128), (17, 1, 128, 128)])
 @pytest.mark.parametrize("bs", [32, 96])
-def test_talking_prefill(gpu, heads, kv_heads, dim, vdim, bs):
+@pytest.mark.parametrize("bounded", [True, False])
+def test_talking_prefill(gpu, heads, kv_heads, dim, vdim, bs, bounded):
     """Portions behind a cached prefix; keys at the edges of what a query sees stand out, rows nobody sees are NaN."""
     rng, bf = np.random.default_rng(dim + heads), torch.bfloat16
     s = ho.TalkShape(heads, kv_heads, dim, vdim, 0.2, 0.0, out_scale=0.6)
-    assert ho.talking_prefill_supported(s, bs)
+    assert ho.talking_prefill_supported(s)
     lens, new = [130, 250, 64, 333], [130, 77, 64, 200]
     p = Pages(rng, lens, s, bs, bf)
     seqs = [2, 0, 3, 1]
@@ -305,7 +328,7 @@ def test_talking_prefill(gpu, heads, kv_heads, dim, vdim, bs):
     wide = torch.full((total, heads * vdim + 8), 9.0, dtype=bf, device=gpu)
     out = wide[:, :heads * vdim]
     ho.talking_prefill(s, proj[:, 8:], *p.pages, dev(talk, bf), p.tables, dev(seqs, torch.int32), dev(cu_q, torch.int32), dev(cu_k, torch.int32),
-                       max(new), out)
+                       max(new), out, max_score=20.0 if bounded else None)
     assert (wide[:, heads * vdim:] == 9.0).all()
     for j, i in enumerate(seqs):
         for t in range(0, new[i], 1 if heads <= 12 else 3):
@@ -313,24 +336,31 @@ def test_talking_prefill(gpu, heads, kv_heads, dim, vdim, bs):
             close(out[r], one_query(s, talk, q[r], p.k[i][:seen], p.v[i][:seen]).ravel(), 2e-2)
 
 
-def test_prefill_and_rows_agree(gpu):
-    """Eight sequences and more take another order of workgroups."""
+@pytest.mark.parametrize("heads,lens", [(8, [70, 64, 200, 33, 96, 5, 61, 300, 129]), (12, [70, 64, 200, 33, 96, 5, 61, 300]), (6, [700] * 40), (16, [470] * 24),
+                                        (14, [500] * 17), (32, [100] * 8)])
+def test_prefill_and_rows_agree(gpu, heads, lens):
+    """Eight sequences take another order of workgroups; many workgroups have more queries each."""
     rng, bf = np.random.default_rng(5), torch.bfloat16
-    s = ho.TalkShape(8, 2, 64, 64, 0.1, 0.0)
-    lens = [70, 64, 200, 33, 96, 5, 61, 300, 129]
+    s = ho.TalkShape(heads, 2, 64, 64, 0.1, 0.0)
     p = Pages(rng, lens, s, 32, bf)
     cu = np.cumsum([0] + lens)
-    q = dev(rms_norm(rng.standard_normal((cu[-1], 8, 64)), 1.0, 0.0), bf)
-    talk = dev(mixing(rng, 8, bf), bf)
-    a, b = (torch.empty((int(cu[-1]), 512), dtype=bf, device=gpu) for _ in range(2))
-    ho.talking_prefill(s, q.view(-1, 512), *p.pages, talk, p.tables, torch.arange(9, dtype=torch.int32, device=gpu), dev(cu, torch.int32),
-                       dev(cu, torch.int32), max(lens), a)
+    q = dev(rms_norm(rng.standard_normal((cu[-1], heads, 64)), 1.0, 0.0), bf)
+    talk = dev(mixing(rng, heads, bf), bf)
+    a, b = (torch.empty((int(cu[-1]), heads * 64), dtype=bf, device=gpu) for _ in range(2))
+    ho.talking_prefill(s, q.view(-1, heads * 64), *p.pages, talk, p.tables, torch.arange(len(lens), dtype=torch.int32, device=gpu), dev(cu, torch.int32),
+                       dev(cu, torch.int32), max(lens), a, max_score=s.max_score(max(lens)))
     ctx = np.concatenate([np.arange(1, n + 1) for n in lens])
-    row_seq = np.repeat(np.arange(9), lens)
-    ho.talking_attention(s, q, *p.pages, talk, p.tables, dev(ctx, torch.int32), b, row_seq=dev(row_seq, torch.int32), max_keys=300)
+    row_seq = np.repeat(np.arange(len(lens)), lens)
+    ho.talking_attention(s, q, *p.pages, talk, p.tables, dev(ctx, torch.int32), b, row_seq=dev(row_seq, torch.int32), max_keys=max(lens))
     close(a, host(b), 1.5e-2)
 
 
 def test_what_the_prompt_kernels_do_not_serve(gpu):
-    for heads, dim, vdim, bs in ((33, 64, 64, 32), (8, 136, 64, 32), (8, 64, 136, 32), (8, 20, 64, 32), (8, 64, 12, 32), (8, 64, 64, 48)):
-        assert not ho.talking_prefill_supported(ho.TalkShape(heads, heads, dim, vdim, 1.0, 0.0), bs)
+    for heads, dim, vdim in ((33, 64, 64), (8, 136, 64), (8, 64, 136), (8, 20, 64), (8, 64, 12)):
+        assert not ho.talking_prefill_supported(ho.TalkShape(heads, heads, dim, vdim, 1.0, 0.0))
+
+
+def test_a_bound_of_the_scores():
+    s = ho.TalkShape(2, 2, 16, 16, 0.5, 0.0, True, 3.0, 40)
+    assert s.max_score(39) == pytest.approx(1.05 * 8.0) and s.max_score(40) == pytest.approx(1.05 * 8.0 * (1 + 3 * np.log(2)))
+    assert ho.TalkShape(2, 2, 16, 16, 0.5, 0.0).max_score(10 ** 6) == pytest.approx(1.05 * 8.0)
