@@ -14,6 +14,8 @@
 //       O^T[v, query]  += V^T[v, key] . P'^T[key, query]      per wavefront its heads
 //                     Nothing is rescaled: what is added up is final.
 // Row r of tile x of the first two products is key 8 (r / 4) + 4 x + r % 4, so that a lane's eight results are eight consecutive keys.
+#include <type_traits>
+
 #include "elem.h"
 #include "pieces.h"
 #include "tile_pages.h"
@@ -45,14 +47,15 @@ struct TalkPrefillArgs {
 
 // The tiles of 32 keys of a sequence, one behind the other; a tile lies in one block, whose id is looked up one block ahead.
 struct PageWalk {
-    const int32_t* bt;
+    typedef const __attribute__((address_space(4))) int32_t* Table;       // nobody writes it meanwhile: scalar loads
+    Table bt;
     int tiles_per_block, col, in_block, id, next_id;
     __device__ __forceinline__ int lookup(const TalkPrefillArgs& a, int c) const {
         const int b = bt[c < a.table_cols ? c : a.table_cols - 1];
         return b < 0 ? 0 : (b >= a.num_blocks ? a.num_blocks - 1 : b);
     }
     __device__ __forceinline__ PageWalk(const TalkPrefillArgs& a, int seq) {
-        bt = a.bt + (int64_t)a.seqs[seq] * a.bt_stride;
+        bt = (Table)(uintptr_t)(a.bt + (int64_t)a.seqs[seq] * a.bt_stride);
         tiles_per_block = a.block_size / kStep;
         col = in_block = 0;
         id = lookup(a, 0);
@@ -287,7 +290,8 @@ __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefill
     fetch_k(tile, 0, 0);
     const int w_fixed = spread(n, (n * kStep + 8 * g) * kRec + wave * UH * 4);
     __syncthreads();                                             // the zero fill and T
-    for (int s = 0; s < steps; ++s) {
+    auto step = [&](auto masked, int s) {
+        constexpr bool MASKED = decltype(masked)::value;         // a query does not see all keys of the step
         const int tok0 = s * kStep, left = sk - tok0;
         const int64_t here = tile;
         if (s + 1 < steps) tile = walk.next(a);                  // the last step requests its own keys again
@@ -297,42 +301,44 @@ __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefill
 #pragma unroll
             for (int i = 0; i < 2 * UK; ++i) {
                 const int uk = i / 2, x = i % 2;
-                f32x4_t sc[UW][QT];
+                // two score tiles at a time: of two heads, or of two query tiles
+                constexpr int GW = UW >= 2 ? 2 : 1, GT = UW >= 2 || QT == 1 ? 1 : 2;
 #pragma unroll
-                for (int w = 0; w < UW; ++w)
+                for (int w0 = 0; w0 < UW; w0 += GW)
 #pragma unroll
-                    for (int t = 0; t < QT; ++t) {
-                        sc[w][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+                    for (int t0 = 0; t0 < QT; t0 += GT) {
+                        f32x4_t sc[GW][GT];
 #pragma unroll
-                        for (int j = 0; j < KS; ++j) sc[w][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j], q[uk * UW + w][t][j], sc[w][t], 0, 0, 0);
-                    }
-                if (i + 1 < 2 * UK) fetch_k(here, (i + 1) / 2, (i + 1) % 2);
-                else fetch_k(tile, 0, 0);
+                        for (int w = 0; w < GW; ++w)
 #pragma unroll
-                for (int t = 0; t < QT; ++t) {
-                    uint32_t w4[UW][4];
+                            for (int t = 0; t < GT; ++t) sc[w][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                    for (int w = 0; w < UW; ++w) {
-                        float p[4];
+                        for (int j = 0; j < KS; ++j)
 #pragma unroll
-                        for (int e = 0; e < 4; ++e) p[e] = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[w][t][e], a.scale_log2, -lse[uk * UW + w][t]));
-                        if (tok0 + kStep - 1 > q0 + 16 * t + shift) {
-                            const int rel = limit[t] - tok0 - 8 * g - 4 * x;
+                            for (int w = 0; w < GW; ++w)
 #pragma unroll
-                            for (int e = 0; e < 4; ++e)
-                                if (e > rel) p[e] = 0.f;
+                                for (int t = 0; t < GT; ++t)
+                                    sc[w][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j], q[uk * UW + w0 + w][t0 + t][j], sc[w][t], 0, 0, 0);
+                        if (w0 + GW == UW && t0 + GT == QT && i + 1 < 2 * UK) fetch_k(here, (i + 1) / 2, (i + 1) % 2);   // these are used up
+#pragma unroll
+                        for (int t = 0; t < GT; ++t) {
+                            uint32_t pieces[GW][4];
+#pragma unroll
+                            for (int w = 0; w < GW; ++w)
+#pragma unroll
+                                for (int e = 0; e < 4; ++e) {
+                                    float p = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[w][t][e], a.scale_log2, -lse[uk * UW + w0 + w][t0 + t]));
+                                    if (MASKED && e > limit[t0 + t] - tok0 - 8 * g - 4 * x) p = 0.f;
+                                    pieces[w][e] = round_pack(head(p), p - head(p));
+                                }
+#pragma unroll
+                            for (int e = 0; e < 4; ++e) {
+                                unsigned char* to = wbuf + (w_base ^ ((4 * x + e) * kRec)) + (t0 + t) * (16 * kStep * kRec) + (uk * UW + w0) * 4;
+                                if constexpr (GW == 2) *reinterpret_cast<u32x2_t*>(to) = u32x2_t{pieces[0][e], pieces[1][e]};
+                                else *reinterpret_cast<uint32_t*>(to) = pieces[0][e];
+                            }
                         }
-#pragma unroll
-                        for (int e = 0; e < 4; ++e) w4[w][e] = round_pack(head(p[e]), p[e] - head(p[e]));
                     }
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        unsigned char* to = wbuf + (w_base ^ ((4 * x + e) * kRec)) + t * (16 * kStep * kRec) + uk * UW * 4;
-                        if constexpr (UW == 4) *reinterpret_cast<u32x4_t*>(to) = u32x4_t{w4[0][e], w4[1][e], w4[2][e], w4[3][e]};
-                        else if constexpr (UW == 2) *reinterpret_cast<u32x2_t*>(to) = u32x2_t{w4[0][e], w4[1][e]};
-                        else *reinterpret_cast<uint32_t*>(to) = w4[0][e];
-                    }
-                }
             }
 #pragma unroll
             for (int i = 0; i < kRing; ++i) fetch_v(here, i);
@@ -348,6 +354,7 @@ __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefill
                 for (int r = 0; r < RT; ++r) tf[y][r] = talk[(y * RT + r) * 64 + lane];
 #pragma unroll
             for (int k = 0; k < 2 * QT; ++k) {
+                if (UH == 4) __builtin_amdgcn_sched_barrier(0);  // one at a time: registers
                 const int qi = 2 * QT * wave + k;
                 f32x4_t mixed[RT][2];
 #pragma unroll
@@ -387,7 +394,7 @@ __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefill
                 for (int v = 0; v < VT; ++v) {
                     const int i = uk * VT + v;
                     bf16x8_t x = vf[i % kRing];
-                    if (left < kStep)                            // values behind the last one may be anything
+                    if constexpr (MASKED)                        // values behind the last one may be anything
 #pragma unroll
                         for (int e = 0; e < 8; ++e)
                             if (8 * g + e >= left) x[e] = (__bf16)0.f;
@@ -396,10 +403,18 @@ __global__ void __launch_bounds__(64 * kMixWaves, 2) talk_mix_kernel(TalkPrefill
 #pragma unroll
                         for (int t = 0; t < QT; ++t) acc[uk * UW + w][t][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, pb[w][t], acc[uk * UW + w][t][v], 0, 0, 0);
                     if (i + kRing < UK * VT) fetch_v(here, i + kRing);
+                    if (i + kRing == UK * VT) {                  // the next step's first keys take the place of the last values
+                        __builtin_amdgcn_sched_barrier(0);
+                        fetch_k(tile, 0, 0);
+                    }
                 }
             }
         }
-    }
+    };
+    const int whole = (q0 + shift + 1) / kStep;                  // steps that the first query sees all of
+    int s = 0;
+    for (; s < whole; ++s) step(std::false_type{}, s);
+    for (; s < steps; ++s) step(std::true_type{}, s);
     if (!live) return;
 #pragma unroll
     for (int u = 0; u < UH; ++u) {
