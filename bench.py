@@ -742,7 +742,7 @@ def tulurax_kernels(width=4096, ff=18432):
         talk, sink = rnd(heads, heads), torch.randn(heads, device=dev)
         for b, seen in ((64, 4096), (64, 1024), (16, 4096)):
             nblk = b * seen // bs
-            keys, values = rnd(nblk, kv_heads, bs // 32, d // 32, 32, 32), rnd(nblk, kv_heads, bs // 32, d, 32)
+            keys, values = rnd(nblk, kv_heads, bs // 32, d // 8, 32, 8), rnd(nblk, kv_heads, bs // 32, d // 16, 4, 16, 8)
             tables = torch.randperm(nblk, device=dev).to(torch.int32).view(b, -1)
             lens, o, qx = torch.full((b,), seen, dtype=torch.int32, device=dev), torch.empty((b, heads * d), dtype=bf, device=dev), rnd(b, heads, d)
             moved = b * seen * kv_heads * 2 * d * 2
@@ -769,9 +769,9 @@ def tulurax_kernels(width=4096, ff=18432):
         for heads, kv in ((16, 8), (16, 16), (32, 8)) if m == 8 else ((16, 8),):
             s = ho.TalkShape(heads, kv, d, d, 0.09, 1e-6)
             talk, q, at = rnd(heads, heads), rnd(t, heads * d), torch.empty((t, heads * d), dtype=bf, device=dev)
-            keys, values = rnd(blocks, kv, bs // 32, d // 32, 32, 32), rnd(blocks, kv, bs // 32, d, 32)
+            keys, values = rnd(blocks, kv, bs // 32, d // 8, 32, 8), rnd(blocks, kv, bs // 32, d // 16, 4, 16, 8)
             mfma(f"talking_prefill, {heads} heads of {kv} keys, {m} x {length}", (4 * heads * d + 2 * heads * heads) * pairs, BF16_PEAK_TFLOPS,
-                 lambda: ho.talking_prefill(s, q, keys, values, talk, tables, seqs, cu, cu, length, at,
+                 lambda: ho.talking_prefill(s, q, keys, values, talk, tables, seqs, cu, cu, length, length, at,
                                             max_score=s.max_score(length)),
                  "both launches; each product counted once")
             dense = rnd(t, kv, 2 * d)
@@ -789,7 +789,7 @@ def tulurax_kernels(width=4096, ff=18432):
     # ---- front end
     heads = 16
     s = ho.TalkShape(heads, kv_heads, d, d, 0.09, 1e-6, True, 0.1, 8192)
-    keys, values = rnd(nblk, kv_heads, bs // 32, d // 32, 32, 32), rnd(nblk, kv_heads, bs // 32, d, 32)
+    keys, values = rnd(nblk, kv_heads, bs // 32, d // 8, 32, 8), rnd(nblk, kv_heads, bs // 32, d // 16, 4, 16, 8)
     cache = rnd(nblk, kv_heads, bs, 2 * d)
     table, ones = yarn_rotary_table(64, 8192, 1e6, None, dev), torch.ones(heads * d, device=dev)
     for t in (64, rows):

@@ -526,8 +526,9 @@ int infer_xielu(int elem, const void* x, int64_t x_stride, const float* bias, fl
                 int64_t out_stride, int64_t n_rows, int64_t cols, void* stream);
 
 /* Talking-heads attention: softmax weights (one added to every denominator) of all heads are mixed by talk [heads][heads] before they
- * meet the values, w'_h = sum_g talk[h][g] w_g.  Pages of tiles of 32 tokens: keys [blocks][kv_heads][tile][key_pad / 32][token][32], values
- * [blocks][kv_heads][tile][vdim_pad][token]; both sizes are padded with zeros to 32 elements, block_size is a multiple of 32.
+ * meet the values, w'_h = sum_g talk[h][g] w_g.  Pages of tiles of 32 tokens: keys [blocks][kv_heads][tile][key_pad / 8][token][8], values
+ * [blocks][kv_heads][tile][vdim_pad / 16][token / 8][16][8 tokens]; both sizes are padded with zeros to 32 elements, block_size is a
+ * multiple of 32.
  *
  * infer_unit_head_front: as infer_head_front for these pages; q, k and (norm_values) v of every head are divided by their root mean
  * square (eps), q is multiplied by 1 + temp_coef ln(floor((position + 1) / temp_every) + 1) (temp_every 0: by one).
@@ -535,8 +536,8 @@ int infer_xielu(int elem, const void* x, int64_t x_stride, const float* bias, fl
  * row_seq[r] (NULL: r); ctx is at most max_keys.  out [rows][heads * vdim], multiplied by out_scale.  Between its kernels the scores
  * are in the workspace (infer_talking_attention_workspace_floats).
  * infer_talking_prefill: whole portions, bf16 (infer_talking_prefill_supported): q [tokens][head][dim], rows cu_q[s] .. cu_q[s + 1] are
- * the last tokens of the sequence in block-table row seqs[s], which has cu_k[s + 1] - cu_k[s] keys; no score
- * exceeds max_score (infinity: no bound is known); workspace of heads * tokens floats. */
+ * the last tokens of the sequence in block-table row seqs[s], which has cu_k[s + 1] - cu_k[s] (at most
+ * max_keys) keys; no score exceeds max_score (infinity: no bound is known); workspace: infer_talking_prefill_workspace_floats. */
 int infer_unit_head_front(int elem, void* proj, int64_t proj_stride, int64_t heads, int64_t kv_heads, int64_t dim,
                           int64_t vdim, int64_t q_off, int64_t k_off, int64_t v_off, float eps, int norm_values,
                           float temp_coef, double temp_every, const int64_t* positions, const int32_t* slots, void* keys,
@@ -553,12 +554,14 @@ int infer_talking_attention(int elem, const void* qx, const void* keys, const vo
                             int64_t splits, int64_t max_keys, void* out, int64_t out_stride, int64_t vdim,
                             float* workspace, int64_t workspace_floats, void* stream);
 int infer_talking_prefill_supported(int64_t heads, int64_t dim, int64_t vdim);
+int64_t infer_talking_prefill_workspace_floats(int64_t heads, int64_t vdim, int64_t num_seqs, int64_t tokens,
+                                               int64_t max_seqlen_q, int64_t max_keys);
 int infer_talking_prefill(const void* q, int64_t q_stride, const void* keys, const void* values, int64_t key_pad,
                           int64_t vdim_pad, const int32_t* block_table, int64_t bt_stride, int64_t table_cols,
                           int64_t block_size, int64_t num_blocks, const int32_t* seqs, const int32_t* cu_q,
-                          const int32_t* cu_k, int64_t num_seqs, int64_t tokens, int64_t max_seqlen_q, int64_t heads,
-                          int64_t kv_heads, int64_t dim, int64_t vdim, float scale, const void* talk, float out_scale,
-                          float max_score, void* out, int64_t out_stride, float* workspace, int64_t workspace_floats,
+                          const int32_t* cu_k, int64_t num_seqs, int64_t tokens, int64_t max_seqlen_q, int64_t max_keys,
+                          int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, float scale, const void* talk,
+                          float out_scale, float max_score, void* out, int64_t out_stride, float* workspace, int64_t workspace_floats,
                           void* stream);
 
 /* Selective state space: S <- e^{a dt} S + dt B x^T, y = S^T C + D x per head, dt = softplus(. + dt_bias), a = -e^{a_log}; x, B and C

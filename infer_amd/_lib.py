@@ -92,8 +92,9 @@ SIGNATURES = {
     "infer_talking_attention": (_c.c_int, [_c.c_int, _vp, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i64, _i64, _vp, _vp, _i64,
                                            _i64, _i64, _f32, _vp, _f32, _i64, _i64, _vp, _i64, _i64, _vp, _i64, _vp]),
     "infer_talking_prefill_supported": (_c.c_int, [_i64, _i64, _i64]),
+    "infer_talking_prefill_workspace_floats": (_i64, [_i64, _i64, _i64, _i64, _i64, _i64]),
     "infer_talking_prefill": (_c.c_int, [_vp, _i64, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _i64,
-                                         _i64, _i64, _i64, _i64, _i64, _f32, _vp, _f32, _f32, _vp, _i64, _vp, _i64, _vp]),
+                                         _i64, _i64, _i64, _i64, _i64, _i64, _f32, _vp, _f32, _f32, _vp, _i64, _vp, _i64, _vp]),
     "infer_head_front": (_c.c_int, [_c.c_int, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _vp,
                                     _vp, _f32, _vp, _i64, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp, _i64,
                                     _i64, _vp]),

@@ -57,7 +57,7 @@ class GroupedPages:
 
 class TilePages:
     """Keys and values per token and key/value head in pages of their own, in tiles of 32 tokens that matrix operands read as they lie:
-    keys of ``key_row`` entries as ``[tile][key_row / 32][token][32]``, values transposed, ``[tile][value_row][token]``."""
+    keys of ``key_row`` entries as ``[tile][key_row / 8][token][8]``, values as ``[tile][value_row / 16][token / 8][16][8 tokens]``."""
     TOKENS = 32
     slot_bytes = 0
 
@@ -70,8 +70,8 @@ class TilePages:
 
     def allocate(self, num_blocks: int, num_slots: int, block_size: int, device):
         tiles = (num_blocks, self.kv_heads, block_size // self.TOKENS)
-        return {"keys": torch.zeros(*tiles, self.key_row // 32, self.TOKENS, 32, dtype=self.dtype, device=device),
-                "values": torch.zeros(*tiles, self.value_row, self.TOKENS, dtype=self.dtype, device=device)}
+        return {"keys": torch.zeros(*tiles, self.key_row // 8, self.TOKENS, 8, dtype=self.dtype, device=device),
+                "values": torch.zeros(*tiles, self.value_row // 16, 4, 16, 8, dtype=self.dtype, device=device)}
 
 
 class SharedStorage:

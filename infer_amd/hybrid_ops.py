@@ -603,7 +603,8 @@ class TalkShape:
 def _talk_pages(s: TalkShape, keys, values, dtype):
     """(blocks, block size) of checked pages (``cache.TilePages``)."""
     assert keys.dtype == values.dtype == dtype and keys.is_contiguous() and values.is_contiguous() and keys.shape[:3] == values.shape[:3]
-    assert keys.shape[1] == s.kv_heads and tuple(keys.shape[3:]) == (s.key_pad // 32, 32, 32) and tuple(values.shape[3:]) == (s.vdim_pad, 32)
+    assert keys.shape[1] == s.kv_heads and tuple(keys.shape[3:]) == (s.key_pad // 8, 32, 8)
+    assert tuple(values.shape[3:]) == (s.vdim_pad // 16, 4, 16, 8)
     return keys.shape[0], 32 * keys.shape[2]
 
 
@@ -666,9 +667,10 @@ def talking_prefill_supported(s: TalkShape) -> bool:
     return bool(_lib.load().infer_talking_prefill_supported(s.heads, s.dim, s.vdim))
 
 
-def talking_prefill(s: TalkShape, q, keys, values, talk, block_table, seqs, cu_q, cu_k, max_seqlen_q: int, out, max_score=None) -> None:
+def talking_prefill(s: TalkShape, q, keys, values, talk, block_table, seqs, cu_q, cu_k, max_seqlen_q: int, max_keys: int, out,
+                    max_score=None) -> None:
     """Whole portions: ``q`` [tokens, heads * dim] (behind ``unit_head_front``) are the last tokens of the sequences in block-table rows
-    ``seqs``, whose numbers of keys ``cu_k`` sums up; ``out`` [tokens, heads * vdim], all bf16.  ``max_score``: no score is larger
+    ``seqs``, whose numbers of keys (at most ``max_keys``) ``cu_k`` sums up; ``out`` [tokens, heads * vdim], all bf16.  ``max_score``: no score is larger
     (None: nobody knows); a small bound spares the search for maxima."""
     blocks, bs = _talk_pages(s, keys, values, torch.bfloat16)
     assert q.dtype == out.dtype == talk.dtype == torch.bfloat16 and q.shape[0] == out.shape[0]
@@ -679,11 +681,13 @@ def talking_prefill(s: TalkShape, q, keys, values, talk, block_table, seqs, cu_q
     assert cu_q.numel() == cu_k.numel() == seqs.numel() + 1
     _require_gpu(q, keys, values, talk, block_table, seqs, cu_q, cu_k, out)
     tokens, cols = q.shape[0], block_table.shape[1]
-    ws = torch.empty(s.heads * tokens, dtype=torch.float32, device=q.device)
-    rc = _lib.load().infer_talking_prefill(
+    lib = _lib.load()
+    ws = torch.empty(lib.infer_talking_prefill_workspace_floats(s.heads, s.vdim, seqs.numel(), tokens, int(max_seqlen_q), int(max_keys)),
+                     dtype=torch.float32, device=q.device)
+    rc = lib.infer_talking_prefill(
         q.data_ptr(), _rows(q, s.heads * s.dim), keys.data_ptr(), values.data_ptr(), s.key_pad, s.vdim_pad, block_table.data_ptr(),
         max(block_table.stride(0), cols), cols, bs, blocks, seqs.data_ptr(), cu_q.data_ptr(), cu_k.data_ptr(), seqs.numel(), tokens,
-        int(max_seqlen_q), s.heads, s.kv_heads, s.dim, s.vdim, float(s.scale), talk.data_ptr(), float(s.out_scale),
+        int(max_seqlen_q), int(max_keys), s.heads, s.kv_heads, s.dim, s.vdim, float(s.scale), talk.data_ptr(), float(s.out_scale),
         float("inf") if max_score is None else float(max_score), out.data_ptr(), _rows(out, s.heads * s.vdim), ws.data_ptr(), ws.numel(),
         _stream_ptr(q))
     _lib.check(rc, "talking_prefill")

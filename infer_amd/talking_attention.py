@@ -55,4 +55,4 @@ class TalkingAttention(nn.Module):
                                          row_seq=None if plan.row_seq is None else plan.row_seq[:split], max_keys=plan.max_keys)
         if split < n:
             hybrid_ops.talking_prefill(s, proj[split:, offset["q"]:], keys, values, self.talk, plan.block_tables, plan.dense_seqs, plan.dense_cu_q,
-                                       plan.dense_cu_k, plan.dense_max_q, out[split:], max_score=s.max_score(plan.max_keys))
+                                       plan.dense_cu_k, plan.dense_max_q, plan.dense_max_k, out[split:], max_score=s.max_score(plan.max_keys))

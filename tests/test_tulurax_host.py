@@ -188,9 +188,9 @@ def test_a_layer_keeps_pages_of_keys_pages_of_values_and_a_state(tmp_path):
     layout = TuluraxForCausalLM(cfg).cache_layout(64)
     assert isinstance(layout, LayeredLayout) and len(layout.layers) == 3
     storage = layout.allocate(5, 2, "cpu")
-    assert storage[0]["left"]["keys"].shape == (5, 2, 2, 1, 32, 32) and storage[0]["left"]["values"].shape == (5, 2, 2, 32, 32)
-    assert storage[1]["left"]["keys"].shape == (5, 5, 2, 1, 32, 32) and storage[1]["left"]["values"].shape == (5, 5, 2, 64, 32)
-    assert storage[2]["left"]["keys"].shape == (5, 1, 2, 2, 32, 32) and storage[2]["left"]["values"].dtype == torch.bfloat16
+    assert storage[0]["left"]["keys"].shape == (5, 2, 2, 4, 32, 8) and storage[0]["left"]["values"].shape == (5, 2, 2, 2, 4, 16, 8)
+    assert storage[1]["left"]["keys"].shape == (5, 5, 2, 4, 32, 8) and storage[1]["left"]["values"].shape == (5, 5, 2, 4, 4, 16, 8)
+    assert storage[2]["left"]["keys"].shape == (5, 1, 2, 8, 32, 8) and storage[2]["left"]["values"].dtype == torch.bfloat16
     assert storage[0]["right"]["state"].shape == (2, 3, 32, 32) and storage[0]["right"]["state"].dtype == torch.float32
     assert layout.block_bytes == sum(t.numel() * 2 for s in storage for t in s["left"].values()) // 5
     assert layout.slot_bytes == sum(s["right"]["state"].numel() * 4 for s in storage) // 2

@@ -96,16 +96,16 @@ def test_scaled_softcap(gpu, dtype):
 def to_pages(keys, values):
     """[blocks, kv_heads, block_size, entries] each, in tiles of 32 tokens as the kernels keep them."""
     b, h, bs, n = keys.shape
-    k = keys.reshape(b, h, bs // 32, 32, n // 32, 32).transpose(0, 1, 2, 4, 3, 5)
-    v = values.reshape(b, h, bs // 32, 32, -1).transpose(0, 1, 2, 4, 3)
+    k = keys.reshape(b, h, bs // 32, 32, n // 8, 8).transpose(0, 1, 2, 4, 3, 5)
+    v = values.reshape(b, h, bs // 32, 4, 8, -1, 16).transpose(0, 1, 2, 5, 3, 6, 4)
     return k, v
 
 
 def from_pages(keys, values):
     """The entries of every slot, [blocks * block_size, kv_heads, entries]."""
-    b, h, tiles, steps = keys.shape[:4]
-    k = keys.transpose(0, 2, 4, 1, 3, 5).reshape(b * tiles * 32, h, steps * 32)
-    return k, values.transpose(0, 2, 4, 1, 3).reshape(b * tiles * 32, h, -1)
+    b, h, tiles, groups = keys.shape[:4]
+    k = keys.transpose(0, 2, 4, 1, 3, 5).reshape(b * tiles * 32, h, groups * 8)
+    return k, values.transpose(0, 2, 4, 6, 1, 3, 5).reshape(b * tiles * 32, h, -1)
 
 
 # ------------------------------------------------------------------ front end
@@ -130,8 +130,8 @@ def test_unit_head_front(gpu, dtype, heads, kv_heads, dim, vdim, temp, norm_valu
         assert len(slots) == n
         pos = np.concatenate([pos, rng.integers(0, 5000, n - 9)])
     shape = nblk, kv_heads, bs // 32
-    keys = torch.full((*shape, s.key_pad // 32, 32, 32), 7.0, dtype=dtype, device=gpu)
-    values = torch.full((*shape, s.vdim_pad, 32), 7.0, dtype=dtype, device=gpu)
+    keys = torch.full((*shape, s.key_pad // 8, 32, 8), 7.0, dtype=dtype, device=gpu)
+    values = torch.full((*shape, s.vdim_pad // 16, 4, 16, 8), 7.0, dtype=dtype, device=gpu)
     qx = torch.full((qx_rows, heads, s.key_pad), float("nan"), dtype=dtype, device=gpu)
     proj = dev(x, dtype)
     ho.unit_head_front(s, proj, off, dev(pos, torch.int64), dev(slots, torch.int32), keys, values, qx, qx_rows)
@@ -252,7 +252,7 @@ def test_scores_beyond_what_exponentials_hold_and_below_the_sink(gpu, dtype, siz
     p.pages[0].zero_()
     for b in range(4):
         m = min(32, n - 32 * b)
-        p.pages[0][p.tables[0, b], :, 0, 0, :m] = dev(k[32 * b:32 * b + m].transpose(1, 0, 2), dtype)
+        p.pages[0][p.tables[0, b], :, 0, :, :m] = dev(k[32 * b:32 * b + m].reshape(m, 2, 4, 8).transpose(1, 2, 0, 3), dtype)
     q = rounded(np.broadcast_to(key * size / (0.5 * key @ key), (1, 4, 32)), dtype)
     talk = mixing(rng, 4, dtype)
     want = one_query(s, talk, q[0], k, p.v[0])
@@ -266,7 +266,7 @@ def test_scores_beyond_what_exponentials_hold_and_below_the_sink(gpu, dtype, siz
         out = torch.empty((n, 128), dtype=dtype, device=gpu)
         rows = np.broadcast_to(q.reshape(1, -1), (n, 128))
         cu = dev([0, n], torch.int32)
-        ho.talking_prefill(s, dev(rows, dtype), *p.pages, dev(talk, dtype), p.tables, dev([0], torch.int32), cu, cu, n, out)
+        ho.talking_prefill(s, dev(rows, dtype), *p.pages, dev(talk, dtype), p.tables, dev([0], torch.int32), cu, cu, n, n, out)
         for t in (0, 1, 31, 32, 99):
             close(out[t], one_query(s, talk, q[0], k[:t + 1], p.v[0][:t + 1]).ravel(), 2e-2)
 
@@ -328,7 +328,7 @@ def test_talking_prefill(gpu, heads, kv_heads, dim, vdim, bs, bounded):
     wide = torch.full((total, heads * vdim + 8), 9.0, dtype=bf, device=gpu)
     out = wide[:, :heads * vdim]
     ho.talking_prefill(s, proj[:, 8:], *p.pages, dev(talk, bf), p.tables, dev(seqs, torch.int32), dev(cu_q, torch.int32), dev(cu_k, torch.int32),
-                       max(new), out, max_score=20.0 if bounded else None)
+                       max(new), max(lens), out, max_score=20.0 if bounded else None)
     assert (wide[:, heads * vdim:] == 9.0).all()
     for j, i in enumerate(seqs):
         for t in range(0, new[i], 1 if heads <= 12 else 3):
@@ -348,7 +348,7 @@ def test_prefill_and_rows_agree(gpu, heads, lens):
     talk = dev(mixing(rng, heads, bf), bf)
     a, b = (torch.empty((int(cu[-1]), heads * 64), dtype=bf, device=gpu) for _ in range(2))
     ho.talking_prefill(s, q.view(-1, heads * 64), *p.pages, talk, p.tables, torch.arange(len(lens), dtype=torch.int32, device=gpu), dev(cu, torch.int32),
-                       dev(cu, torch.int32), max(lens), a, max_score=s.max_score(max(lens)))
+                       dev(cu, torch.int32), max(lens), max(lens), a, max_score=s.max_score(max(lens)))
     ctx = np.concatenate([np.arange(1, n + 1) for n in lens])
     row_seq = np.repeat(np.arange(len(lens)), lens)
     ho.talking_attention(s, q, *p.pages, talk, p.tables, dev(ctx, torch.int32), b, row_seq=dev(row_seq, torch.int32), max_keys=max(lens))
