@@ -24,7 +24,7 @@ struct HeadFrontArgs {
     const int32_t* slots;
     T* keys; T* values; int key_row, value_row;              // [blocks][kv_heads][block_size][..]: elements per token
     bool tiles;                                              // tile_pages.h, or a token's entries one behind the other
-    bool values_apart;                                       // value_tiles_kernel has the values
+    bool apart;                                              // fill_tiles_kernel has keys and values
     int block_size, key_pad, vdim_pad; int64_t num_slots;
     T* qx; int64_t qx_rows;                // rows below qx_rows: q to qx[row][head][map][key_pad], others in place
 };
@@ -81,7 +81,9 @@ __device__ __forceinline__ Place<T> place_of(const HeadFrontArgs<T>& a, T* pr, c
     return {a.v_off + i * a.vdim, a.vdim, s.value ? s.value + i * s.value_head : nullptr, nullptr, a.norm_v, false, 1.f, false, a.tiles};
 }
 template <class T>
-__host__ __device__ __forceinline__ int num_vectors(const HeadFrontArgs<T>& a) { return (a.heads + a.kv_heads) * a.maps + ((a.norm_v || a.tiles) && !a.values_apart ? a.kv_heads : 0); }
+__host__ __device__ __forceinline__ int num_vectors(const HeadFrontArgs<T>& a) {
+    return (a.heads + (a.apart ? 0 : a.kv_heads)) * a.maps + ((a.norm_v || a.tiles) && !a.apart ? a.kv_heads : 0);
+}
 
 template <class T>
 __device__ __forceinline__ float query_factor(const HeadFrontArgs<T>& a, int64_t pos) {
@@ -104,16 +106,15 @@ __device__ __forceinline__ void copy_values(const HeadFrontArgs<T>& a, const T* 
 template <class T>
 __device__ __forceinline__ void fill_padding(const HeadFrontArgs<T>& a, const Slot<T>& s, T* qx) {
     const int used = a.maps * a.dim, pad = a.key_pad - used, vpad = a.vdim_pad - a.vdim;
-    if (s.key) {
+    if (s.key && !a.apart) {
         for (int i = threadIdx.x; i < a.kv_heads * pad; i += 256) {
             const int d = used + i % pad;
             s.key[i / pad * s.key_head + (a.tiles ? tile_key_entry(0, d) : d)] = (T)0.f;
         }
-        if (!a.values_apart)
-            for (int i = threadIdx.x; i < a.kv_heads * vpad; i += 256) {
-                const int d = a.vdim + i % vpad;
-                s.value[i / vpad * s.value_head + (a.tiles ? tile_value_entry(0, d) : d)] = (T)0.f;
-            }
+        for (int i = threadIdx.x; i < a.kv_heads * vpad; i += 256) {
+            const int d = a.vdim + i % vpad;
+            s.value[i / vpad * s.value_head + (a.tiles ? tile_value_entry(0, d) : d)] = (T)0.f;
+        }
     }
     if (qx) {
         const int rest = a.key_pad - a.dim;
@@ -240,17 +241,18 @@ __global__ void __launch_bounds__(256) head_front_any_kernel(HeadFrontArgs<T> a)
     fill_padding(a, slot, qx);
 }
 
-// Values of 32 consecutive tokens to tiles, where those of eight neighbouring tokens are one store.  Eight threads per token, NC chunks
-// of eight entries each.
+// Keys or values of one head of 32 consecutive tokens to tiles, with neighbouring tokens in one store or in neighbouring lanes.  No biases,
+// rotation or second map.  Eight threads per token, NC chunks of eight entries each.  blockIdx.y: heads of keys, then of values.
 template <class T, int NC>
-__global__ void __launch_bounds__(256) value_tiles_kernel(HeadFrontArgs<T> a, int64_t n) {
+__global__ void __launch_bounds__(256) fill_tiles_kernel(HeadFrontArgs<T> a, int64_t n) {
     constexpr int kRow = 64 * NC + 8;                            // entries of a token in LDS
     __shared__ __attribute__((aligned(16))) T tile[32 * kRow];
     __shared__ int64_t slot[32];
     const int64_t t0 = (int64_t)blockIdx.x * 32;
-    const int tid = threadIdx.x, r = tid / 8, h = blockIdx.y;
-    const bool have = t0 + r < n;
-    const T* pr = a.proj + (t0 + (have ? r : 0)) * a.proj_stride + a.v_off + h * a.vdim;
+    const bool is_key = (int)blockIdx.y < a.kv_heads, norm = is_key ? a.norm_qk : a.norm_v;
+    const int tid = threadIdx.x, r = tid / 8, h = is_key ? blockIdx.y : blockIdx.y - a.kv_heads;
+    const int size = is_key ? a.dim : a.vdim, pad = is_key ? a.key_pad : a.vdim_pad;
+    const T* pr = a.proj + (t0 + r < n ? t0 + r : t0) * a.proj_stride + (is_key ? a.k_off : a.v_off) + h * size;
     if (tid < 32) {
         const int64_t s = t0 + tid < n ? a.slots[t0 + tid] : -1;
         slot[tid] = s < a.num_slots ? s : -1;
@@ -261,13 +263,13 @@ __global__ void __launch_bounds__(256) value_tiles_kernel(HeadFrontArgs<T> a, in
         const int c = 8 * (tid % 8) + 64 * j;
 #pragma unroll
         for (int e = 0; e < 8; ++e) x[j][e] = 0.f;
-        if (c < a.vdim) load_elems<8>(pr + c, x[j]);
+        if (c < size) load_elems<8>(pr + c, x[j]);
 #pragma unroll
         for (int e = 0; e < 8; ++e) sum += x[j][e] * x[j][e];
     }
 #pragma unroll
     for (int m = 4; m >= 1; m >>= 1) sum += __shfl_xor(sum, m, 64);
-    const float f = a.norm_v ? rsqrtf(sum / (float)a.vdim + a.eps) : 1.f;
+    const float f = norm ? rsqrtf(sum / (float)size + a.eps) : 1.f;
 #pragma unroll
     for (int j = 0; j < NC; ++j) {
 #pragma unroll
@@ -275,17 +277,36 @@ __global__ void __launch_bounds__(256) value_tiles_kernel(HeadFrontArgs<T> a, in
         store_elems<8>(tile + r * kRow + 8 * (tid % 8) + 64 * j, x[j]);
     }
     __syncthreads();
-    // runs of neighbouring tokens that do not leave a group of eight, taken in turn by 256 / vdim_pad sets of threads
-    const int sets = 256 / a.vdim_pad, set = tid / a.vdim_pad, v = tid % a.vdim_pad;
+    // the tile of a slot, from the start of the pages, and the slot's place in it
+    auto place = [&](int64_t s, int& token) {
+        const int64_t block = s / a.block_size;
+        const int off = (int)(s - block * a.block_size);
+        token = off % kTileTokens;
+        return ((block * a.kv_heads + h) * a.block_size + off - token) * pad;
+    };
+    if (is_key) {
+        const int64_t s = slot[tid % 32];
+        if (s < 0) return;
+        int token;
+        T* to = a.keys + place(s, token);
+        for (int d = tid / 32 * 8; d < pad; d += 64) {
+            float y[8];
+            load_elems<8>(tile + tid % 32 * kRow + d, y);
+            store_elems<8>(to + tile_key_entry(token, d), y);
+        }
+        return;
+    }
+    // runs of neighbouring tokens that do not leave a group of eight, taken in turn by 256 / pad sets of threads
+    const int sets = 256 / pad, set = tid / pad, v = tid % pad;
     if (set >= sets) return;
     for (int first = 0, run = 0; first < 32; ++run) {
         const int64_t s = slot[first];
         int count = 1;
         while (first + count < 32 && (s + count) % 8 != 0 && slot[first + count] == s + count) ++count;
         if (s >= 0 && run % sets == set) {
-            const int64_t block = s / a.block_size;
-            const int off = (int)(s - block * a.block_size), in_tile = off % kTileTokens;
-            T* to = a.values + ((block * a.kv_heads + h) * a.block_size + off - in_tile) * a.value_row + tile_value_entry(in_tile, v);
+            int token;
+            T* to = a.values + place(s, token);
+            to += tile_value_entry(token, v);
             if (count == 8) {
                 float y[8];
 #pragma unroll
@@ -317,14 +338,15 @@ int launch(HeadFrontArgs<T> a, int64_t n, hipStream_t st) {
                      a.proj_stride % 8 == 0 && ptr_aligned(a.proj, 16) && ptr_aligned(a.keys, 16) && ptr_aligned(a.values, 16) && ptr_aligned(a.qx, 16) &&
                      ptr_aligned(a.bias, 16) && ptr_aligned(a.q_norm, 16) && ptr_aligned(a.k_norm, 16) && ptr_aligned(a.table, 16);
     bool done = false;
-    if (vec && a.tiles && a.vdim <= 256 && n >= 64 && a.kv_heads <= 65535) {
-        const dim3 grid((unsigned)((n + 31) / 32), (unsigned)a.kv_heads), block(256);
-        if (a.vdim <= 64) hipLaunchKernelGGL((value_tiles_kernel<T, 1>), grid, block, 0, st, a, n);
-        else if (a.vdim <= 128) hipLaunchKernelGGL((value_tiles_kernel<T, 2>), grid, block, 0, st, a, n);
-        else hipLaunchKernelGGL((value_tiles_kernel<T, 4>), grid, block, 0, st, a, n);
-        a.values_apart = true;
+    if (vec && a.tiles && a.key_pad <= 256 && a.vdim_pad <= 256 && n >= 64 && a.kv_heads <= 32767) {
+        const dim3 grid((unsigned)((n + 31) / 32), (unsigned)(2 * a.kv_heads)), block(256);
+        const int pad = a.key_pad > a.vdim_pad ? a.key_pad : a.vdim_pad;
+        if (pad <= 64) hipLaunchKernelGGL((fill_tiles_kernel<T, 1>), grid, block, 0, st, a, n);
+        else if (pad <= 128) hipLaunchKernelGGL((fill_tiles_kernel<T, 2>), grid, block, 0, st, a, n);
+        else hipLaunchKernelGGL((fill_tiles_kernel<T, 4>), grid, block, 0, st, a, n);
+        a.apart = true;
     }
-    const int longest = (a.norm_v || a.tiles) && !a.values_apart && a.vdim > a.dim ? a.vdim : a.dim;
+    const int longest = (a.norm_v || a.tiles) && !a.apart && a.vdim > a.dim ? a.vdim : a.dim;
     if (vec) {
         if (longest <= 32) done = launch_vec<T, 4>(a, n, st);
         else if (longest <= 64) done = launch_vec<T, 8>(a, n, st);

@@ -232,13 +232,14 @@ __global__ void __launch_bounds__(256) talk_scores_kernel(TalkArgs<__bf16> a) {
     for (int i = 0; i < MT; ++i) {
         const int h = u.head0 + 16 * i + n;
         const int64_t at = (int64_t)u.row * a.heads + (h < u.head_end ? h : u.head0);
-        to[i] = h < u.head_end ? a.scores + at * a.key_cap + 4 * g : nullptr;
+        to[i] = h < u.head_end ? a.scores + at * a.key_cap + 8 * g : nullptr;
 #pragma unroll
         for (int j = 0; j < KS; ++j) {
             q[i][j] = bf16x8_t{};
             if (32 * j < a.key_pad) q[i][j] = *reinterpret_cast<const bf16x8_t*>(a.qx + at * a.key_pad + 32 * j + 8 * g);
         }
     }
+    const int k_lane = tile_key_entry(tile_row_token(n, 0), 8 * g);
     int k_step[KS];                                   // k-steps behind the size repeat the first one, which meets zeros
 #pragma unroll
     for (int j = 0; j < KS; ++j) k_step[j] = tile_key_entry(0, 32 * j < a.key_pad ? 32 * j : 0);
@@ -248,11 +249,11 @@ __global__ void __launch_bounds__(256) talk_scores_kernel(TalkArgs<__bf16> a) {
     bf16x8_t kf[2][KS];
     TileWalk walk(a, bt, u.t0 + wave);
     auto fetch = [&]() {
-        const __bf16* src = a.keys + walk.next(a, bt, u.kvh) * kTile * a.key_pad + tile_key_entry(n, 8 * g);
+        const __bf16* src = a.keys + walk.next(a, bt, u.kvh) * kTile * a.key_pad + k_lane;
 #pragma unroll
         for (int x = 0; x < 2; ++x)
 #pragma unroll
-            for (int j = 0; j < KS; ++j) kf[x][j] = *reinterpret_cast<const bf16x8_t*>(src + k_step[j] + tile_key_entry(16 * x, 0));
+            for (int j = 0; j < KS; ++j) kf[x][j] = *reinterpret_cast<const bf16x8_t*>(src + k_step[j] + tile_key_entry(tile_row_token(0, x), 0));
     };
     if (u.t0 + wave < u.t1) fetch();
     for (int t = u.t0 + wave; t < u.t1; t += kWaves) {
@@ -266,17 +267,17 @@ __global__ void __launch_bounds__(256) talk_scores_kernel(TalkArgs<__bf16> a) {
                 for (int j = 0; j < KS; ++j) s[i][x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[x][j], q[i][j], s[i][x], 0, 0, 0);
             }
         if (t + kWaves < u.t1) fetch();
-        const int left = u.len - t * kTile - 4 * g;   // of this lane's keys 16 x + e those below `left` exist
+        const int left = u.len - t * kTile - 8 * g;   // of this lane's keys 4 x + e those below `left` exist
 #pragma unroll
         for (int i = 0; i < MT; ++i) {
             float top = m[i];
 #pragma unroll
             for (int x = 0; x < 2; ++x) {
                 s[i][x] *= a.scale_log2;
-                if (to[i]) *reinterpret_cast<f32x4_t*>(to[i] + (int64_t)t * kTile + 16 * x) = s[i][x];
+                if (to[i]) *reinterpret_cast<f32x4_t*>(to[i] + (int64_t)t * kTile + 4 * x) = s[i][x];
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
-                    if (16 * x + e >= left) s[i][x][e] = -INFINITY;
+                    if (4 * x + e >= left) s[i][x][e] = -INFINITY;
                     top = fmaxf(top, s[i][x][e]);
                 }
             }
@@ -310,8 +311,7 @@ __global__ void __launch_bounds__(256) talk_scores_kernel(TalkArgs<__bf16> a) {
 // Every wavefront has tiles of its own and reads their values straight into operands:
 //   P'^T[key, head] = W^T[key, g] . T^T[g, head]     weights of all heads g as two bf16 pieces each (2^-17), KH k-steps of 32 heads
 //   O^T[v, head]   += V^T[v, key] . P'^T[key, head]
-// Row r of tile x of the first product is key 8 (r / 4) + 4 x + r % 4, so that a lane's eight results are the eight consecutive keys
-// that the second product wants from it.
+// A lane's eight results of the first product are the eight consecutive keys that the second one wants from it (tile_row_token).
 template <int MT, int KH, int NT>
 __global__ void __launch_bounds__(256) talk_values_kernel(TalkArgs<__bf16> a) {
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
@@ -331,7 +331,7 @@ __global__ void __launch_bounds__(256) talk_values_kernel(TalkArgs<__bf16> a) {
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
             const int from = 32 * s + 8 * g + e;
-            src_s[s][e] = a.scores + ((int64_t)u.row * a.heads + (from < a.heads ? from : a.heads - 1)) * a.key_cap + 8 * (n >> 2) + (n & 3);
+            src_s[s][e] = a.scores + ((int64_t)u.row * a.heads + (from < a.heads ? from : a.heads - 1)) * a.key_cap + tile_row_token(n, 0);
         }
     TileWalk walk(a, bt, u.t0 + wave);
     auto fetch = [&](int t) {
@@ -381,7 +381,7 @@ __global__ void __launch_bounds__(256) talk_values_kernel(TalkArgs<__bf16> a) {
                 float w[8];
 #pragma unroll
                 for (int e = 0; e < 8; ++e)
-                    w[e] = 8 * (n >> 2) + 4 * x + (n & 3) < left ? __builtin_amdgcn_exp2f(sreg[s][x][e] - den[s][e]) : 0.f;
+                    w[e] = tile_row_token(n, x) < left ? __builtin_amdgcn_exp2f(sreg[s][x][e] - den[s][e]) : 0.f;
                 bf16x8_t wf[2];
                 split_frags<2>(w, wf);
 #pragma unroll

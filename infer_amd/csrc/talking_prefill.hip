@@ -5,7 +5,7 @@
 //
 // A running rescale does not commute with the mixture, so denominators come first, and the scores are computed twice instead of passing
 // through memory:
-//   talk_lse_kernel   log2 of every (head, query)'s denominator; a wavefront owns 64 queries of a head
+//   talk_lse_kernel   log2 of every (head, query)'s denominator; a wavefront owns 16 U queries of a head
 //   talk_mix_kernel   a workgroup of eight wavefronts owns 16 QT queries and ALL heads, UH heads per wavefront, and walks the keys in
 //                     steps of 32:
 //       S^T[key, query] = K[key, :] . q^T           per wavefront its heads; weights e^{S - lse} go to LDS as two bf16 pieces each
@@ -15,7 +15,7 @@
 //                     Nothing is rescaled: what is added up is final, and the keys of a few queries can be split over workgroups, whose
 //                     sums talk_sum_kernel adds up.  Between the barriers that enclose the mixture a wavefront computes the scores
 //                     of the next step and the sums of this one, the two wavefronts of a vector unit in opposite order.
-// Row r of tile x of the first two products is key 8 (r / 4) + 4 x + r % 4, so that a lane's eight results are eight consecutive keys.
+// A lane's eight results of the first two products are those of eight consecutive keys (tile_row_token).
 #include <type_traits>
 
 #include "elem.h"
@@ -27,7 +27,7 @@ namespace {
 typedef uint32_t u32x2_t __attribute__((ext_vector_type(2)));
 
 constexpr int kStep = kTileTokens;
-constexpr int kLseWaves = 4, kLseQ = 64;  // queries per wavefront
+constexpr int kLseWaves = 4;
 constexpr int kMixWaves = 8;
 constexpr float kLow = -1e30f;            // a maximum before any key was seen; finite, since hidden scores are -inf
 constexpr float kLazy = 8.f;              // log2 units by which a sum's terms may exceed one before it is rescaled
@@ -94,9 +94,9 @@ __device__ __forceinline__ bf16x8_t load_operand(const __bf16* base, unsigned la
 }
 
 // BOUNDED: all scores are below kBound, so that their powers need no maximum.
-template <int KS, bool BOUNDED>
+template <int KS, int U, bool BOUNDED>
 __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefillArgs a) {
-    constexpr int U = kLseQ / 16;
+    constexpr int kLseQ = 16 * U;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, n = lane & 15;
     int pair, qblk;
     if (!place_of_block(blockIdx.x, a.nseq * a.heads, a.qblocks, pair, qblk)) return;
@@ -125,7 +125,7 @@ __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefill
 #pragma unroll
     for (int j = 0; j < KS; ++j) k_step[j] = tile_key_entry(0, 32 * j < a.key_pad ? 32 * j : 0);
     const int64_t head_at = (int64_t)(h / (a.heads / a.kv_heads)) * a.block_size * a.key_pad;
-    const unsigned k_lane = 2u * (unsigned)tile_key_entry(8 * (n >> 2) + (n & 3), 8 * g);
+    const unsigned k_lane = 2u * (unsigned)tile_key_entry(tile_row_token(n, 0), 8 * g);
     PageWalk walk(a, b);
     bf16x8_t kf[2][KS];
     auto fetch = [&]() {
@@ -133,7 +133,7 @@ __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefill
 #pragma unroll
         for (int x = 0; x < 2; ++x)
 #pragma unroll
-            for (int j = 0; j < KS; ++j) kf[x][j] = load_operand(src + k_step[j] + tile_key_entry(4 * x, 0), k_lane);
+            for (int j = 0; j < KS; ++j) kf[x][j] = load_operand(src + k_step[j] + tile_key_entry(tile_row_token(0, x), 0), k_lane);
     };
     fetch();
     for (int s = 0; s < steps; ++s) {
@@ -193,8 +193,15 @@ __global__ void __launch_bounds__(64 * kLseWaves, 2) talk_lse_kernel(TalkPrefill
     }
 }
 
-// LDS addresses of what belongs to query q: lanes with 16 consecutive queries meet all banks
-__device__ __forceinline__ int spread(int q, int addr) { return addr ^ ((q & 15) << 4); }
+// Address in LDS of byte `at` of the record of (query q, key token), REC bytes long.  Lanes that write (16 queries, one key) and lanes
+// that read (16 keys of tile_row_token, one query) meet all banks.  For the second eight of 16 queries the halves of every 16 bytes
+// are swapped (`swapped`).  What a query, a key and `at` contribute is independent.
+template <int REC>
+__device__ __forceinline__ int record_place(int q, int token, int at) {
+    const int low = REC == 128 ? (token & 3) | (token >> 1 & 4) : REC == 64 ? (token >> 1 & 1) | (token >> 2 & 2) : token >> 3 & 1;
+    return (q * kStep + token) * REC + at ^ (low << 4) ^ ((q & 15) << 4) ^ (q & 8);
+}
+__device__ __forceinline__ bool swapped(int q) { return q & 8; }
 template <int HP>
 __device__ __forceinline__ int mixed_place(int q, int slot, int g) { return (q * HP + (slot ^ (q & (HP - 1)))) * 64 + 16 * (g ^ ((q >> 2) & 3)); }
 
@@ -214,7 +221,7 @@ __global__ void __launch_bounds__(64 * kMixWaves) __attribute__((amdgpu_waves_pe
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
     unsigned char* wbuf = lds;                                   // [Q][32 keys][kRec]
     unsigned char* pbuf = wbuf + Q * kStep * kRec;               // [Q][HP][32 keys] bf16
-    bf16x8_t* talk = reinterpret_cast<bf16x8_t*>(pbuf + Q * HP * 2 * kStep);       // [KP][RT][64]
+    bf16x8_t* talk = reinterpret_cast<bf16x8_t*>(pbuf + Q * HP * 2 * kStep);       // [2][KP][RT][64]
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, n = lane & 15;
     int b, qblk;
     const int split = blockIdx.y;
@@ -256,13 +263,14 @@ __global__ void __launch_bounds__(64 * kMixWaves) __attribute__((amdgpu_waves_pe
             }
         }
     }
-    // T^T: entry i of lane (g, n) is column (head) 16 s + 4 g + i / 2 of row (head) 16 r + n, once for either piece
-    for (int i = tid; i < KP * RT * 64; i += 64 * kMixWaves) {
-        const int s = i / (64 * RT), r = i / 64 % RT, to = 16 * r + i % 16;
+    // T^T: entry i of lane (g, n) is column (head) 16 s + 4 g + i / 2 of row (head) 16 r + n, once for either piece; behind it the same
+    // for records whose halves are swapped
+    for (int i = tid; i < 2 * KP * RT * 64; i += 64 * kMixWaves) {
+        const int s = i / (64 * RT) % KP, r = i / 64 % RT, to = 16 * r + i % 16;
         bf16x8_t x;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-            const int from = 16 * s + 4 * (i % 64 / 16) + e / 2;
+            const int from = 16 * s + 4 * (i % 64 / 16) + (i < KP * RT * 64 ? e : e ^ 4) / 2;
             x[e] = from < HP && from < a.heads && to < a.heads ? a.talk[(int64_t)to * a.heads + from] : (__bf16)0.f;
         }
         talk[i] = x;
@@ -277,11 +285,11 @@ __global__ void __launch_bounds__(64 * kMixWaves) __attribute__((amdgpu_waves_pe
             for (int v = 0; v < VT; ++v) acc[u][t][v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 
     PageWalk walk(a, b, s0);
-    const unsigned k_lane = 2u * (unsigned)tile_key_entry(8 * (n >> 2) + (n & 3), 8 * g), v_lane = 2u * (unsigned)tile_value_entry(8 * g, n);
+    const unsigned k_lane = 2u * (unsigned)tile_key_entry(tile_row_token(n, 0), 8 * g), v_lane = 2u * (unsigned)tile_value_entry(8 * g, n);
     bf16x8_t kf[KS];
     // half x of the keys of head uk; k-steps behind the size repeat the first one, which meets zeros in q
     auto fetch_k = [&](int64_t tile, int uk, int x) __attribute__((always_inline)) {
-        const __bf16* src = a.keys + tile * kStep * a.key_pad + k_head[uk] + tile_key_entry(4 * x, 0);
+        const __bf16* src = a.keys + tile * kStep * a.key_pad + k_head[uk] + tile_key_entry(tile_row_token(0, x), 0);
 #pragma unroll
         for (int j = 0; j < KS; ++j) kf[j] = load_operand(src + tile_key_entry(0, 32 * j < a.key_pad ? 32 * j : 0), k_lane);
     };
@@ -292,7 +300,7 @@ __global__ void __launch_bounds__(64 * kMixWaves) __attribute__((amdgpu_waves_pe
         const int v = i % VT;
         vf[i % kRing] = load_operand(a.values + tile * kStep * a.vdim_pad + v_head[i / VT] + tile_value_entry(0, 16 * v < a.vdim_pad ? 16 * v : 0), v_lane);
     };
-    const int w_fixed = spread(n, (n * kStep + 8 * g) * kRec + wave * UH * 4);
+    const int w_fixed = record_place<kRec>(n, 8 * g, wave * UH * 4);
     const int whole = (q0 + shift + 1) / kStep;                  // steps of which the first query sees every key
 
     // scores and weights of step s, half of the keys of a key head at a time; its first keys are in kf
@@ -334,7 +342,7 @@ __global__ void __launch_bounds__(64 * kMixWaves) __attribute__((amdgpu_waves_pe
                             }
 #pragma unroll
                         for (int e = 0; e < 4; ++e) {
-                            unsigned char* to = wbuf + (w_base ^ ((4 * x + e) * kRec)) + (t0 + t) * (16 * kStep * kRec) + (uk * UW + w0) * 4;
+                            unsigned char* to = wbuf + (w_base ^ record_place<kRec>(0, 4 * x + e, (uk * UW + w0) * 4)) + (t0 + t) * (16 * kStep * kRec);
                             if constexpr (GW == 2) *reinterpret_cast<u32x2_t*>(to) = u32x2_t{pieces[0][e], pieces[1][e]};
                             else *reinterpret_cast<uint32_t*>(to) = pieces[0][e];
                         }
@@ -349,20 +357,19 @@ __global__ void __launch_bounds__(64 * kMixWaves) __attribute__((amdgpu_waves_pe
 #pragma unroll
         for (int y = 0; y < KP; ++y)
 #pragma unroll
-            for (int r = 0; r < RT; ++r) tf[y][r] = talk[(y * RT + r) * 64 + lane];
+            for (int r = 0; r < RT; ++r) tf[y][r] = talk[((swapped(2 * QT * wave) ? KP : 0) + y) * RT * 64 + r * 64 + lane];
 #pragma unroll
         for (int k = 0; k < 2 * QT; ++k) {
-            if (UH * QT == 4) __builtin_amdgcn_sched_barrier(0);  // one at a time: registers
+            if (UH == 4) __builtin_amdgcn_sched_barrier(0);      // one query at a time: registers
             const int qi = 2 * QT * wave + k;
             f32x4_t mixed[RT][2];
 #pragma unroll
             for (int x = 0; x < 2; ++x) {
 #pragma unroll
                 for (int r = 0; r < RT; ++r) mixed[r][x] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-                const int rec = (qi * kStep + 8 * (n >> 2) + 4 * x + (n & 3)) * kRec;
 #pragma unroll
                 for (int y = 0; y < KP; ++y) {
-                    const bf16x8_t wf = *reinterpret_cast<const bf16x8_t*>(wbuf + spread(qi, rec + 64 * y + 16 * (UH == 1 ? g & 1 : g)));
+                    const bf16x8_t wf = *reinterpret_cast<const bf16x8_t*>(wbuf + record_place<kRec>(qi, tile_row_token(n, x), 64 * y + 16 * (UH == 1 ? g & 1 : g) ^ (qi & 8)));
 #pragma unroll
                     for (int r = 0; r < RT; ++r) mixed[r][x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, tf[y][r], mixed[r][x], 0, 0, 0);
                 }
@@ -427,10 +434,8 @@ __global__ void __launch_bounds__(64 * kMixWaves) __attribute__((amdgpu_waves_pe
         else fetch_k(tile1, 0, 0);
         __syncthreads();
         auto step = [&](auto masked, int s) __attribute__((always_inline)) {
-            __builtin_amdgcn_sched_barrier(0);
             mix();
             __syncthreads();
-            __builtin_amdgcn_sched_barrier(0);
             if constexpr (SUMS_FIRST) {
                 sums(masked, s, tile, tile1);
                 if (!decltype(masked)::value || s + 1 < steps) scores(masked, s + 1, tile1);
@@ -511,14 +516,20 @@ void plan(int64_t heads, int64_t num_seqs, int64_t max_seqlen_q, int64_t max_key
     if (splits < 1) splits = 1;
 }
 
-template <int KS>
-int launch_lse(TalkPrefillArgs a, int64_t max_seqlen_q, bool bounded, hipStream_t st) {
-    const int64_t per = kLseQ * kLseWaves, qblocks = (max_seqlen_q + per - 1) / per, total = ((int64_t)a.nseq * a.heads + 7) / 8 * 8 * qblocks;
+template <int KS, int U>
+int launch_lse_of(TalkPrefillArgs a, int64_t max_seqlen_q, bool bounded, hipStream_t st) {
+    const int64_t per = 16 * U * kLseWaves, qblocks = (max_seqlen_q + per - 1) / per, total = ((int64_t)a.nseq * a.heads + 7) / 8 * 8 * qblocks;
     if (total > 0x7fffffff) return INFER_KV_EINVAL;
     a.qblocks = (int)qblocks;
-    if (bounded) hipLaunchKernelGGL((talk_lse_kernel<KS, true>), dim3((unsigned)total), dim3(64 * kLseWaves), 0, st, a);
-    else hipLaunchKernelGGL((talk_lse_kernel<KS, false>), dim3((unsigned)total), dim3(64 * kLseWaves), 0, st, a);
+    if (bounded) hipLaunchKernelGGL((talk_lse_kernel<KS, U, true>), dim3((unsigned)total), dim3(64 * kLseWaves), 0, st, a);
+    else hipLaunchKernelGGL((talk_lse_kernel<KS, U, false>), dim3((unsigned)total), dim3(64 * kLseWaves), 0, st, a);
     return (int)hipGetLastError();
+}
+template <int KS>
+int launch_lse(const TalkPrefillArgs& a, int64_t max_seqlen_q, bool bounded, hipStream_t st) {
+    // few queries: more wavefronts with fewer of them each
+    if ((max_seqlen_q + 63) / 64 * a.nseq * a.heads < 2048) return launch_lse_of<KS, 2>(a, max_seqlen_q, bounded, st);
+    return launch_lse_of<KS, 4>(a, max_seqlen_q, bounded, st);
 }
 
 template <int KS, int VT, int UH, int QT, bool SHARE>
@@ -527,7 +538,7 @@ int launch_mix(TalkPrefillArgs a, int64_t max_seqlen_q, hipStream_t st) {
     if (total > 0x7fffffff) return INFER_KV_EINVAL;
     a.qblocks = (int)qblocks;
     auto kernel = &talk_mix_kernel<KS, VT, UH, QT, SHARE>;
-    constexpr size_t lds = (size_t)16 * QT * kStep * kMixWaves * UH * (4 + 2) + (UH == 4 ? 4 : 1) * 1024;
+    constexpr size_t lds = (size_t)16 * QT * kStep * kMixWaves * UH * (4 + 2) + (UH == 4 ? 4 : 1) * 2048;
     static_assert(lds <= 160 * 1024, "LDS of a compute unit");
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return (int)e;

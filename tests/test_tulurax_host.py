@@ -196,47 +196,71 @@ def test_a_layer_keeps_pages_of_keys_pages_of_values_and_a_state(tmp_path):
     assert layout.slot_bytes == sum(s["right"]["state"].numel() * 4 for s in storage) // 2
 
 
-# ------------------------------------------------------------------ LDS of the prompt kernel
-@pytest.mark.parametrize("per_wave,tiles", [(1, 2), (2, 1), (4, 1)])
+# ------------------------------------------------------------------ index arithmetic of the kernels
+def row_token(r, x):
+    return 8 * (r >> 2) + 4 * x + (r & 3)
+
+
+def key_entry(token, d):
+    return (d >> 3) * 256 + ((token >> 2 & 1) * 16 + (token >> 3) * 4 + (token & 3)) * 8 + (d & 7)
+
+
+def value_entry(token, v):
+    return (v >> 4) * 512 + (token >> 3) * 128 + (v & 15) * 8 + (token & 7)
+
+
+def test_tiles_hold_every_entry_and_operands_lie_in_a_row():
+    for entry in (key_entry, value_entry):
+        assert sorted(entry(t, d) for t in range(32) for d in range(64)) == list(range(2048))
+        assert all(entry(t, d) == entry(t, 0) + entry(0, d) for t in range(32) for d in range(64))
+    for x in range(2):                                           # lane (g, n): row n, entries 8 g + e of a k-step
+        lanes = [key_entry(row_token(n, x), 8 * g) for g in range(4) for n in range(16)]
+        assert lanes == [256 * g + 128 * x + 8 * n for g in range(4) for n in range(16)]
+    assert [value_entry(8 * g, n) for g in range(4) for n in range(16)] == [8 * i for i in range(64)]
+    for g in range(4):
+        assert [row_token(r, x) for x in range(2) for r in range(4 * g, 4 * g + 4)] == list(range(8 * g, 8 * g + 8))
+
+
+def record_place(rec, q, token, at):
+    low = (token & 3) | (token >> 1 & 4) if rec == 128 else (token >> 1 & 1) | (token >> 2 & 2) if rec == 64 else token >> 3 & 1
+    return ((q * 32 + token) * rec + at) ^ (low << 4) ^ ((q & 15) << 4) ^ (q & 8)
+
+
+@pytest.mark.parametrize("per_wave,tiles", [(1, 2), (1, 4), (2, 1), (2, 2), (4, 1)])
 def test_records_of_the_prompt_kernel_have_places_of_their_own(per_wave, tiles):
     """Every (query, key, head) has one word, written once and read back at the same address; the mixed weights likewise."""
     heads, queries = 8 * per_wave, 16 * tiles
-    rec = 4 * heads
-
-    def spread(addr):
-        return addr ^ (((addr >> 7) & 7) << 4)
-
-    words = {}
+    rec, words = 4 * heads, {}
     for q in range(queries):
         for key in range(32):
             for wave in range(8):
-                base = spread((q * 32 + key) * rec + wave * per_wave * 4)
-                assert base % (4 * per_wave) == 0 and 0 <= base and base + 4 * per_wave <= queries * 32 * rec
-                for u in range(per_wave):
-                    words[base + 4 * u] = (q, key, wave * per_wave + u)
-    assert len(words) == queries * 32 * heads
+                for u in range(per_wave):                        # as the kernel puts the address together
+                    fixed = record_place(rec, q % 16, key // 8 * 8, wave * per_wave * 4)
+                    words[(fixed ^ record_place(rec, 0, key % 8, 4 * u)) + q // 16 * (16 * 32 * rec)] = (q, key, wave * per_wave + u)
+    assert len(words) == queries * 32 * heads and max(words) + 4 == queries * 32 * rec
     for q in range(queries):
         for key in range(32):
-            for unit in range(rec // 16):                        # 16-byte reads hold four consecutive heads
-                base = spread((q * 32 + key) * rec + 16 * unit)
-                assert [words[base + 4 * i] for i in range(4)] == [(q, key, 4 * unit + i) for i in range(4)]
-    places = {(q * heads + (h ^ (q & (heads - 1)))) * 64 for q in range(queries) for h in range(heads)}
-    assert len(places) == queries * heads and max(places) + 64 <= queries * heads * 64
+            for unit in range(rec // 16):                        # a 16-byte read holds four heads, two by two in either order
+                base = record_place(rec, q, key, 16 * unit ^ (q & 8))
+                assert base % 16 == 0
+                order = (2, 3, 0, 1) if q & 8 else (0, 1, 2, 3)
+                assert [words[base + 4 * i] for i in range(4)] == [(q, key, 4 * unit + i) for i in order]
+    for wave in range(8):                                        # the queries that a wavefront mixes have one order
+        assert len({q & 8 for q in range(2 * tiles * wave, 2 * tiles * (wave + 1))}) == 1
+    places = {(q * heads + (h ^ (q & (heads - 1)))) * 64 + 16 * (g ^ (q >> 2 & 3)) for q in range(queries) for h in range(heads) for g in range(4)}
+    assert len(places) == queries * heads * 4 and max(places) + 16 == queries * heads * 64
 
 
-@pytest.mark.parametrize("vt", [4, 8])
-def test_permuted_values_have_places_of_their_own(vt):
-    row_bytes = 32 * vt
-    place = {row * row_bytes + (16 * c ^ ((row & (vt - 1)) * 32)): (row, c) for row in range(32) for c in range(2 * vt)}
-    assert len(place) == 64 * vt and max(place) + 16 <= 32 * row_bytes
-    for row in range(32):
-        for v in range(vt):
-            for piece in range(4):                               # an eight-byte read lies in one 16-byte unit
-                at = row * row_bytes + ((32 * v + 8 * piece) ^ ((row & (vt - 1)) * 32))
-                assert place[at // 16 * 16] == (row, 2 * v + piece // 2)
-
-
-def test_rows_of_the_score_tiles_give_every_lane_consecutive_keys():
-    for g in range(4):
-        keys = [8 * (r // 4) + 4 * x + r % 4 for x in range(2) for r in range(4 * g, 4 * g + 4)]
-        assert keys == list(range(8 * g, 8 * g + 8))
+@pytest.mark.parametrize("per_wave", [1, 2, 4])
+def test_lanes_meet_all_banks(per_wave):
+    """128 bytes a clock: writes of 16 lanes (one key, 16 queries), reads of eight lanes (eight keys, one query)."""
+    rec = 32 * per_wave
+    size = 8 if per_wave > 1 else 4
+    for key in range(32):
+        banks = [(record_place(rec, q, key, 0) + b) % 128 // 4 for q in range(16) for b in range(0, size, 4)]
+        assert len(set(banks)) == len(banks)
+    for q in range(16):
+        for x in range(2):
+            for r0 in (0, 8):
+                units = {record_place(rec, q, row_token(r, x), q & 8) % 128 // 16 for r in range(r0, r0 + 8)}
+                assert len(units) == 8

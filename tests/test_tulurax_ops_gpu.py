@@ -93,10 +93,13 @@ def test_scaled_softcap(gpu, dtype):
 
 
 # ------------------------------------------------------------------ pages
+KEY_ORDER = np.array([8 * (r // 4) + 4 * x + r % 4 for x in range(2) for r in range(16)])      # of a tile's tokens, for keys
+
+
 def to_pages(keys, values):
     """[blocks, kv_heads, block_size, entries] each, in tiles of 32 tokens as the kernels keep them."""
     b, h, bs, n = keys.shape
-    k = keys.reshape(b, h, bs // 32, 32, n // 8, 8).transpose(0, 1, 2, 4, 3, 5)
+    k = keys.reshape(b, h, bs // 32, 32, n // 8, 8)[:, :, :, KEY_ORDER].transpose(0, 1, 2, 4, 3, 5)
     v = values.reshape(b, h, bs // 32, 4, 8, -1, 16).transpose(0, 1, 2, 5, 3, 6, 4)
     return k, v
 
@@ -104,7 +107,7 @@ def to_pages(keys, values):
 def from_pages(keys, values):
     """The entries of every slot, [blocks * block_size, kv_heads, entries]."""
     b, h, tiles, groups = keys.shape[:4]
-    k = keys.transpose(0, 2, 4, 1, 3, 5).reshape(b * tiles * 32, h, groups * 8)
+    k = keys[:, :, :, :, np.argsort(KEY_ORDER)].transpose(0, 2, 4, 1, 3, 5).reshape(b * tiles * 32, h, groups * 8)
     return k, values.transpose(0, 2, 4, 6, 1, 3, 5).reshape(b * tiles * 32, h, -1)
 
 
@@ -252,7 +255,9 @@ def test_scores_beyond_what_exponentials_hold_and_below_the_sink(gpu, dtype, siz
     p.pages[0].zero_()
     for b in range(4):
         m = min(32, n - 32 * b)
-        p.pages[0][p.tables[0, b], :, 0, :, :m] = dev(k[32 * b:32 * b + m].reshape(m, 2, 4, 8).transpose(1, 2, 0, 3), dtype)
+        tile = np.zeros((1, 2, 32, 32))
+        tile[0, :, :m] = k[32 * b:32 * b + m].transpose(1, 0, 2)
+        p.pages[0][p.tables[0, b]] = dev(to_pages(tile, tile)[0][0], dtype)
     q = rounded(np.broadcast_to(key * size / (0.5 * key @ key), (1, 4, 32)), dtype)
     talk = mixing(rng, 4, dtype)
     want = one_query(s, talk, q[0], k, p.v[0])
