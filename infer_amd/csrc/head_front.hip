@@ -338,7 +338,9 @@ int launch(HeadFrontArgs<T> a, int64_t n, hipStream_t st) {
                      a.proj_stride % 8 == 0 && ptr_aligned(a.proj, 16) && ptr_aligned(a.keys, 16) && ptr_aligned(a.values, 16) && ptr_aligned(a.qx, 16) &&
                      ptr_aligned(a.bias, 16) && ptr_aligned(a.q_norm, 16) && ptr_aligned(a.k_norm, 16) && ptr_aligned(a.table, 16);
     bool done = false;
-    if (vec && a.tiles && a.key_pad <= 256 && a.vdim_pad <= 256 && n >= 64 && a.kv_heads <= 32767) {
+    // portions fill whole tiles; the rows of a decode batch belong to as many pages, and the main kernel writes them
+    const bool portions = a.qx_rows < n ? n >= 64 : n >= 2048;
+    if (vec && a.tiles && a.key_pad <= 256 && a.vdim_pad <= 256 && portions && a.kv_heads <= 32767) {
         const dim3 grid((unsigned)((n + 31) / 32), (unsigned)(2 * a.kv_heads)), block(256);
         const int pad = a.key_pad > a.vdim_pad ? a.key_pad : a.vdim_pad;
         if (pad <= 64) hipLaunchKernelGGL((fill_tiles_kernel<T, 1>), grid, block, 0, st, a, n);

@@ -342,9 +342,10 @@ def test_talking_prefill(gpu, heads, kv_heads, dim, vdim, bs, bounded):
 
 
 @pytest.mark.parametrize("heads,lens", [(8, [70, 64, 200, 33, 96, 5, 61, 300, 129]), (12, [70, 64, 200, 33, 96, 5, 61, 300]), (6, [700] * 40), (16, [470] * 24),
-                                        (14, [500] * 17), (32, [100] * 8)])
+                                        (14, [500] * 17), (32, [100] * 8), (8, [1100]), (10, [650, 40, 330]), (16, [900, 40]), (32, [1030])])
 def test_prefill_and_rows_agree(gpu, heads, lens):
-    """Eight sequences take another order of workgroups; many workgroups have more queries each."""
+    """Eight sequences take another order of workgroups; many workgroups have more queries each; few queries of many keys are
+    split over workgroups, of which short sequences leave some without keys."""
     rng, bf = np.random.default_rng(5), torch.bfloat16
     s = ho.TalkShape(heads, 2, 64, 64, 0.1, 0.0)
     p = Pages(rng, lens, s, 32, bf)
