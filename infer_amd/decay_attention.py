@@ -1,9 +1,9 @@
 """Linear attention with a constant decay per head: a recurrent layer with a ``[dim, vdim]`` float32 state per head and
 neither softmax nor denominator.
 
-``DecayHeads`` is a part of a ``Mixer``, ``DecayAttention`` a layer of its own with its projections; the state is an argument.  What stands in front of and behind the recurrence are
-parameters: silu on q, k and v or a rotary embedding of q and k; a norm over each head or over all heads together,
-with or without a weight; a sigmoid or silu output gate."""
+``DecayHeads`` is a part of a ``Mixer``, ``DecayAttention`` a layer of its own with its projections; the state is an
+argument.  What stands in front of and behind the recurrence are parameters: silu on q, k and v or a rotary embedding of
+q and k; a norm over each head or over all heads together, with or without a weight; a sigmoid or silu output gate."""
 from __future__ import annotations
 
 import torch
